@@ -111,8 +111,11 @@ class LlamaEngine:
                                  48, 64, 96, 128, max_batch)
                                 if b <= max_batch})
         self._dummy_slot = -1
-        # opt-in: capture the top-k/top-p tail in-graph (see _samp_class)
-        self._GRAPH_TOPK = _os.environ.get("OLLAMAMQ_GRAPH_TOPK") == "1"
+        if _os.environ.get("OLLAMAMQ_GRAPH_TOPK") == "1":
+            raise RuntimeError(
+                "in-graph top-k/top-p sampling is switched off: a captured "
+                "torch.topk over the full vocabulary has faulted the GPU "
+                "and its cause is not known; unset OLLAMAMQ_GRAPH_TOPK")
 
     # -- submission --------------------------------------------------------
     def submit(self, prompt: List[int], params: GenParams,
@@ -404,23 +407,19 @@ class LlamaEngine:
 
     def _samp_class(self, seqs) -> int:
         """0 = all greedy (argmax tail), 1 = temperature-only mix (Gumbel
-        tail — exact), 2 = top-k/top-p present.
+        tail — exact), 3 = top-k/top-p present.
 
-        Class 2 is captured ONLY behind OLLAMAMQ_GRAPH_TOPK=1: the
-        candidate tail (torch.topk over [B, 128256] + filters) is clean
-        in isolation (tools/repro_tail.py: 3000 mutated replays) and on
-        tiny models, but faults under real multi-graph 8B serving with
-        or without the fused chain (tools/repro_sampled.py WORKLOAD=topk)
-        — an unresolved interaction between the captured topk and the
-        serving graph set.  Until root-caused, top-k/p rows sample on the
-        host (exact, full vocabulary) with the forward still graphed."""
+        Class 3 is never captured: the candidate tail (torch.topk over
+        [B, 128256] + filters) faulted the GPU inside the serving graph
+        set and the cause is not known.  Those rows sample on the host
+        (exact, full vocabulary) with the forward still graphed."""
         k = 0
         for s in seqs:
             p = s.params
             if p.temperature > 0:
                 if (p.top_k or 0) > 0 or (p.top_p if p.top_p else 1.0) \
                         < 1.0:
-                    return 2 if self._GRAPH_TOPK else 3
+                    return 3
                 k = 1
         return k
 
@@ -451,8 +450,6 @@ class LlamaEngine:
             "lens": torch.zeros(B, dtype=torch.int32, device=dev),
             "temps": torch.zeros(B, dtype=torch.float32, device=dev),
             "seeds": torch.zeros(B, dtype=torch.int64, device=dev),
-            "topk": torch.zeros(B, dtype=torch.int64, device=dev),
-            "topp": torch.ones(B, dtype=torch.float32, device=dev),
             # 1 for live rows, 0 for bucket padding: the in-graph
             # advance applies it so pad rows never grow their dummy slot
             "adv": torch.ones(B, dtype=torch.int32, device=dev),
@@ -496,23 +493,13 @@ class LlamaEngine:
                 [getattr(s, "noise_seed", 1234) for s in seqs]
                 + [0] * pad,
                 dtype=torch.int64).to(self.dev, non_blocking=True))
-        if entry["klass"] == 2:
-            bufs["topk"].copy_(torch.tensor(
-                [s.params.top_k or 0 for s in seqs] + [0] * pad,
-                dtype=torch.int64).to(self.dev, non_blocking=True))
-            bufs["topp"].copy_(torch.tensor(
-                [s.params.top_p if s.params.top_p else 1.0
-                 for s in seqs] + [1.0] * pad,
-                dtype=torch.float32).to(self.dev, non_blocking=True))
 
     def _graph_tail(self, entry, logits):
         """The in-graph sampling tail: class 0 = greedy argmax; class 1 =
         exact Gumbel-max temperature sampling (kernels.hip sample_gumbel,
         greedy rows ride the same kernel with T<=0), noise keyed by
         (per-seq seed, kv length) so replays draw fresh randomness with
-        no host RNG; class 2 = per-row top-k/top-p over the top-256
-        candidates (capturable torch ops), then exact Gumbel-max on the
-        filtered set.
+        no host RNG.
 
         This MUST also run once EAGERLY in the pre-capture warmup: the
         samplers cache split-scratch buffers (ops/hip.py _scratch), and a
@@ -525,26 +512,6 @@ class LlamaEngine:
             from ..ops import hip as _hip
             return _hip.sample_gumbel(logits, bufs["temps"],
                                       bufs["seeds"], bufs["lens"])
-        if entry["klass"] == 2:
-            from ..ops import hip as _hip
-            C = min(256, logits.shape[1])
-            v, idx = torch.topk(logits.float(), C, dim=-1)
-            t = bufs["temps"].clamp(min=1e-6).unsqueeze(1)
-            p = torch.softmax(v / t, dim=-1)
-            ar = torch.arange(C, device=logits.device)
-            kk = torch.where(bufs["topk"] > 0,
-                             bufs["topk"].clamp(max=C),
-                             torch.full_like(bufs["topk"], C))
-            keep = ar.unsqueeze(0) < kk.unsqueeze(1)
-            cum = p.cumsum(dim=-1)
-            keep &= (cum - p) < bufs["topp"].unsqueeze(1)
-            keep[:, 0] = True
-            # greedy rows bypass the (garbage) filter math
-            keep |= (bufs["temps"] <= 0).unsqueeze(1)
-            vm = v.masked_fill(~keep, float("-inf")).bfloat16()
-            ci = _hip.sample_gumbel(vm.contiguous(), bufs["temps"],
-                                    bufs["seeds"], bufs["lens"])
-            return idx.gather(1, ci.long().unsqueeze(1)).squeeze(1).int()
         return ops.sample(logits, 0.0, 0, 1.0, None).int()
 
     def _graph_replay(self, entry):
@@ -599,13 +566,13 @@ class LlamaEngine:
         """Pre-capture the decode graphs for EVERY (bucket, sampling
         class) at load time — a capture costs ~150 ms and ~75 MB, and a
         LAZY capture mid-serving stalls every in-flight stream for that
-        long (a 50%-sampled stress wave against lazy class-1/2 capture
+        long (a 50%-sampled stress wave against lazy class-1 capture
         timed out 189 of 303 requests before this).  With bucketing the
         set is small and fixed; load time pays ~5-10 s once."""
         if not self.use_graphs:
             return
         if classes is None:
-            classes = (0, 1, 2) if self._GRAPH_TOPK else (0, 1)
+            classes = (0, 1)
         sizes = [b for b in (sizes or self._buckets)
                  if 0 < b <= self.max_batch]
         for b in sorted(set(sizes)):
