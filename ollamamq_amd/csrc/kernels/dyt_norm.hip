@@ -1,0 +1,333 @@
+// gfx950 elementwise steps of blocks built on dynamic tanh (DyT):
+//
+//   x' = x + post(y)            residual sum, fp32
+//   h  = pre(x')                DyT: tanh(alpha * x) * w + b
+//   out[t] = h[t] + (h[t-1] - h[t]) * mix      token shift (optional)
+//
+// DyT has no row statistics, so the whole chain between two matrix products
+// is one pass over the row, and split-K partial sums of the product that
+// made y are folded on the way in.  With token shift a sequence's last h is
+// its state; a portion's first row reads it (zero at position 0) and the
+// same thread writes the portion's last h, so the read and the write are
+// ordered without a second launch.
+//
+// Also here: PolyNorm, and the RMS norm of a latent with its append to the
+// paged pool.
+#include "tile_mma.h"
+
+struct DyT {
+    const float* w;
+    const float* b;
+    float alpha;
+};
+
+// |x| small: odd series (relative error below 4e-7 up to 0.25); else from
+// exp(-2|x|)
+DEV float tanh_fast(float x) {
+    const float a = fabsf(x), x2 = x * x;
+    const float e = __expf(-2.f * a);
+    const float big = copysignf((1.f - e) * __builtin_amdgcn_rcpf(1.f + e),
+                                x);
+    const float ser = x * (1.f + x2 * (-1.f / 3.f + x2 * (2.f / 15.f
+                           + x2 * (-17.f / 315.f))));
+    return a < 0.25f ? ser : big;
+}
+template <typename T> DEV float tanh_of(float x) {
+    if constexpr (sizeof(T) == 4) return tanhf(x);
+    else return tanh_fast(x);
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void k_dyt(
+    float* __restrict__ x_out,          // [n, W] or null
+    T* __restrict__ h_out,              // [n, W]
+    const float* __restrict__ x_in,     // [T, W], or null: embedding rows
+    const T* __restrict__ embed, const int* __restrict__ tokens,
+    const T* __restrict__ y,            // [T, W] or null
+    const float* __restrict__ y_part,   // [n_part, T, W] instead of y
+    int n_part,
+    DyT post, DyT pre,
+    const float* __restrict__ mix,      // null: no token shift
+    float* __restrict__ prev,           // [slots, W]
+    const int* __restrict__ slot, const int* __restrict__ pos,
+    const int* __restrict__ row_seq,    // null: every row its own sequence
+    const int* __restrict__ cu_q,
+    const int64_t* __restrict__ rows,   // null, or the rows to compute
+    int n, int T_in, int W, int strip)
+{
+    const int c = (blockIdx.y * 256 + threadIdx.x) * VEC;
+    if (c >= W) return;
+    float pw[VEC], pb[VEC], qw[VEC], qb[VEC], mx[VEC];
+    const bool has_y = y != nullptr || y_part != nullptr;
+    if (has_y) { ldv<VEC>(post.w + c, qw); ldv<VEC>(post.b + c, qb); }
+    ldv<VEC>(pre.w + c, pw);
+    ldv<VEC>(pre.b + c, pb);
+    if (mix) ldv<VEC>(mix + c, mx);
+
+    auto load_x = [&](int r, float* x) {
+        if (x_in) ldv<VEC>(x_in + (int64_t)r * W + c, x);
+        else ldv<VEC>(embed + (int64_t)tokens[r] * W + c, x);
+        if (!has_y) return;
+        float v[VEC];
+        if (y) ldv<VEC>(y + (int64_t)r * W + c, v);
+        else {
+            ldv<VEC>(y_part + (int64_t)r * W + c, v);
+            for (int s = 1; s < n_part; s++) {
+                float u[VEC];
+                ldv<VEC>(y_part + ((int64_t)s * T_in + r) * W + c, u);
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) v[i] += u[i];
+            }
+        }
+        #pragma unroll
+        for (int i = 0; i < VEC; i++)
+            x[i] += tanh_of<T>(post.alpha * v[i]) * qw[i] + qb[i];
+    };
+    auto norm = [&](const float* x, float* h) {
+        #pragma unroll
+        for (int i = 0; i < VEC; i++)
+            h[i] = tanh_of<T>(pre.alpha * x[i]) * pw[i] + pb[i];
+    };
+
+    const int r0 = blockIdx.x * strip;
+    const int r1 = min(r0 + strip, n);
+    float hp[VEC];
+    for (int o = r0; o < r1; ++o) {
+        const int r = rows ? (int)rows[o] : o;
+        float x[VEC], h[VEC];
+        load_x(r, x);
+        if (x_out) stv<VEC>(x_out + (int64_t)o * W + c, x);
+        norm(x, h);
+        if (!mix) {
+            stv<VEC>(h_out + (int64_t)o * W + c, h);
+            continue;
+        }
+        const int s = row_seq ? row_seq[r] : r;
+        const int first = row_seq ? cu_q[s] : r;
+        if (r == first) {
+            float* st = prev + (int64_t)slot[r] * W + c;
+            if (pos[r] == 0) {
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) hp[i] = 0.f;
+            } else ldv<VEC>(st, hp);
+            const int last = row_seq ? cu_q[s + 1] - 1 : r;
+            if (last == r) stv<VEC>(st, h);
+            else {
+                float xl[VEC], hl[VEC];
+                load_x(last, xl);
+                norm(xl, hl);
+                stv<VEC>(st, hl);
+            }
+        } else if (o == r0) {
+            float xl[VEC];
+            load_x(r - 1, xl);
+            norm(xl, hp);
+        }
+        float out[VEC];
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) {
+            out[i] = h[i] + (hp[i] - h[i]) * mx[i];
+            hp[i] = h[i];
+        }
+        stv<VEC>(h_out + (int64_t)o * W + c, out);
+    }
+}
+
+template <typename T>
+static int dyt_launch(
+    void* x_out, void* h_out, const void* x_in, const void* embed,
+    const void* tokens, const void* y, const void* y_part, int n_part,
+    DyT post, DyT pre, const void* mix, void* prev, const void* slot,
+    const void* pos, const void* row_seq, const void* cu_q,
+    const void* rows, int n, int T_in, int W, hipStream_t stream)
+{
+    const bool v4 = W % 4 == 0;
+    const int per = 256 * (v4 ? 4 : 1);
+    const int cols = (W + per - 1) / per;
+    // longer strips save the second evaluation of a strip's predecessor
+    int strip = 1;
+    while (strip < 8 && (int64_t)n * cols / (strip * 2) >= 2048) strip *= 2;
+    dim3 grid((n + strip - 1) / strip, cols);
+    #define DYT_GO(V)                                                      \
+        k_dyt<T, V><<<grid, 256, 0, stream>>>(                             \
+            (float*)x_out, (T*)h_out, (const float*)x_in,                  \
+            (const T*)embed, (const int*)tokens, (const T*)y,              \
+            (const float*)y_part, n_part, post, pre, (const float*)mix,    \
+            (float*)prev, (const int*)slot, (const int*)pos,               \
+            (const int*)row_seq, (const int*)cu_q, (const int64_t*)rows,   \
+            n, T_in, W, strip)
+    if (v4) DYT_GO(4); else DYT_GO(1);
+    #undef DYT_GO
+    return (int)hipGetLastError();
+}
+
+extern "C" int dyt_residual(
+    int f32, void* x_out, void* h_out, const void* x_in, const void* embed,
+    const void* tokens, const void* y, const void* y_part, int n_part,
+    const void* post_w, const void* post_b, float post_alpha,
+    const void* pre_w, const void* pre_b, float pre_alpha,
+    const void* mix, void* prev, const void* slot, const void* pos,
+    const void* row_seq, const void* cu_q, const void* rows,
+    int n, int T_in, int W, hipStream_t stream)
+{
+    DyT post{(const float*)post_w, (const float*)post_b, post_alpha};
+    DyT pre{(const float*)pre_w, (const float*)pre_b, pre_alpha};
+    auto go = f32 ? dyt_launch<float> : dyt_launch<bf16>;
+    return go(x_out, h_out, x_in, embed, tokens, y, y_part, n_part, post,
+              pre, mix, prev, slot, pos, row_seq, cu_q, rows, n, T_in, W,
+              stream);
+}
+
+// ---------------------------------------------------------------------------
+// PolyNorm: out = a z/rms(z) + b z^2/rms(z^2) + c z^3/rms(z^3) + e, the rms
+// over the row.  One block per row; rows up to NV*256*VEC stay in registers
+// between the two passes (NV == 0: the second pass reads again).
+// ---------------------------------------------------------------------------
+template <typename T, int VEC, int NV>
+__global__ __launch_bounds__(256) void k_polynorm(
+    T* __restrict__ out, const T* __restrict__ z,
+    const float* __restrict__ z_part, int n_part, int64_t part_stride,
+    float ca, float cb, float cc, float ce, int F, float eps)
+{
+    const int64_t row = blockIdx.x;
+    const int tid = threadIdx.x;
+    __shared__ float red[3][4];
+    auto load = [&](int c, float* v) {
+        if (z) { ldv<VEC>(z + row * F + c, v); return; }
+        ldv<VEC>(z_part + row * F + c, v);
+        for (int s = 1; s < n_part; s++) {
+            float u[VEC];
+            ldv<VEC>(z_part + s * part_stride + row * F + c, u);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) v[i] += u[i];
+        }
+    };
+    float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+    auto stat = [&](const float* v) {
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) {
+            const float p = v[i] * v[i];
+            s1 += p;
+            s2 += p * p;
+            s3 += p * p * p;
+        }
+    };
+    float keep[NV > 0 ? NV : 1][VEC];
+    if constexpr (NV > 0) {
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int c = (j * 256 + tid) * VEC;
+            if (c < F) { load(c, keep[j]); stat(keep[j]); }
+        }
+    } else {
+        for (int c = tid * VEC; c < F; c += 256 * VEC) {
+            float v[VEC];
+            load(c, v);
+            stat(v);
+        }
+    }
+    s1 = wave_sum(s1); s2 = wave_sum(s2); s3 = wave_sum(s3);
+    if ((tid & 63) == 0) {
+        red[0][tid >> 6] = s1; red[1][tid >> 6] = s2; red[2][tid >> 6] = s3;
+    }
+    __syncthreads();
+    const float inv = 1.f / F;
+    auto scale = [&](int k, float coef) {
+        const float s = (red[k][0] + red[k][1]) + (red[k][2] + red[k][3]);
+        return coef / sqrtf(s * inv + eps);
+    };
+    const float a = scale(0, ca), b = scale(1, cb), g = scale(2, cc);
+    auto emit = [&](int c, const float* v) {
+        float o[VEC];
+        #pragma unroll
+        for (int i = 0; i < VEC; i++)
+            o[i] = v[i] * (a + v[i] * (b + v[i] * g)) + ce;
+        stv<VEC>(out + row * F + c, o);
+    };
+    if constexpr (NV > 0) {
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int c = (j * 256 + tid) * VEC;
+            if (c < F) emit(c, keep[j]);
+        }
+    } else {
+        for (int c = tid * VEC; c < F; c += 256 * VEC) {
+            float v[VEC];
+            load(c, v);
+            emit(c, v);
+        }
+    }
+}
+
+extern "C" int polynorm(
+    int f32, void* out, const void* z, const void* z_part, int n_part,
+    float ca, float cb, float cc, float ce, int T_rows, int F, float eps,
+    hipStream_t stream)
+{
+    const int64_t ps = (int64_t)T_rows * F;
+    #define PN_GO(T, V, NV)                                                \
+        k_polynorm<T, V, NV><<<T_rows, 256, 0, stream>>>(                  \
+            (T*)out, (const T*)z, (const float*)z_part, n_part, ps,        \
+            ca, cb, cc, ce, F, eps)
+    #define PN_TYPE(T)                                                     \
+        do {                                                               \
+            if (F % 8) PN_GO(T, 1, 0);                                     \
+            else if (F <= 2048) PN_GO(T, 8, 1);                            \
+            else if (F <= 4096) PN_GO(T, 8, 2);                            \
+            else if (F <= 8192) PN_GO(T, 8, 4);                            \
+            else if (F <= 16384) PN_GO(T, 8, 8);                           \
+            else PN_GO(T, 8, 0);                                           \
+        } while (0)
+    if (f32) PN_TYPE(float); else PN_TYPE(bf16);
+    #undef PN_TYPE
+    #undef PN_GO
+    return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// Latent append: c = rmsnorm(d) * w into pool[page][offset][R].  One wave
+// per token.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void k_latent_append(
+    T* __restrict__ pool, const T* __restrict__ d, int64_t ds,
+    const float* __restrict__ w, const int* __restrict__ slot,
+    const int* __restrict__ pos, const int* __restrict__ ptab,
+    int T_rows, int R, int psz, int maxp, float eps)
+{
+    const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
+    if (t >= T_rows) return;
+    const T* src = d + (int64_t)t * ds;
+    float s = 0.f;
+    for (int i = lane; i < R; i += 64) {
+        const float v = ldf(src + i);
+        s += v * v;
+    }
+    s = wave_sum(s);
+    const float r = 1.f / sqrtf(s / R + eps);
+    const int p = pos[t];
+    const int pg = ptab[(int64_t)slot[t] * maxp + p / psz];
+    T* dst = pool + ((int64_t)pg * psz + p % psz) * R;
+    for (int i = lane; i < R; i += 64)
+        stf(dst + i, ldf(src + i) * r * w[i]);
+}
+
+extern "C" int latent_append(
+    int f32, void* pool, const void* d, int64_t ds, const void* w,
+    const void* slot, const void* pos, const void* ptab, int T_rows, int R,
+    int psz, int maxp, float eps, hipStream_t stream)
+{
+    const int g = (T_rows + 3) / 4;
+    if (f32)
+        k_latent_append<float><<<g, 256, 0, stream>>>(
+            (float*)pool, (const float*)d, ds, (const float*)w,
+            (const int*)slot, (const int*)pos, (const int*)ptab, T_rows, R,
+            psz, maxp, eps);
+    else
+        k_latent_append<bf16><<<g, 256, 0, stream>>>(
+            (bf16*)pool, (const bf16*)d, ds, (const float*)w,
+            (const int*)slot, (const int*)pos, (const int*)ptab, T_rows, R,
+            psz, maxp, eps);
+    return (int)hipGetLastError();
+}

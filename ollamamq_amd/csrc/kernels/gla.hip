@@ -1,0 +1,522 @@
+// gfx950 gated linear attention: per head a [D, V] fp32 state with
+//   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,
+// alpha_t = sigmoid(z_t)^(1/tau) per key channel, z = a2 u + b from the
+// low-rank projection u.  The recurrence is fp32 throughout, on the fp32
+// matrix cores in chunks, in both element types of the surrounding model.
+//
+// * k_gla_step: a token at a time (decode, portions of a few tokens), with
+//   the head norm and the output gate in the same kernel.
+// * k_gla_prep / k_gla_scan / k_gla_out: chunks of 64 tokens.  With b the
+//   running sum of log alpha inside a chunk,
+//     o_i = (q_i e^{b_i}) S_0 + sum_{j<=i} (sum_d q_id k_jd e^{b_id-b_jd}) v_j
+//     S'  = diag(e^{b_64}) S_0 + sum_j (k_j e^{b_64-b_j}) v_j^T.
+//   prep makes the three decayed factors for all chunks at once; scan walks
+//   a sequence's chunks with the state in registers.  No exponent is ever
+//   positive: sums are kept per 16-token part, and a pair of parts is joined
+//   by the decay across the parts between them.
+// A sequence starts where its position is 0: the state is then taken as
+// zero and whatever the slot held is ignored.
+#include "tile_mma.h"
+
+struct GlaIn {            // one row of the fused projection
+    int64_t ld;           // row stride
+    int oq, ok, ov, og, ou;   // column offsets of q, k, v, gate, low rank
+    int rank;
+};
+
+DEV float log_alpha(float z, float inv_tau) {
+    return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau;
+}
+DEV float silu(float x) { return x / (1.f + expf(-x)); }
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void k_gla_step(
+    T* __restrict__ out,                // [T, H*V]
+    const T* __restrict__ p, GlaIn in,
+    const T* __restrict__ a2, const float* __restrict__ a2_b,
+    const float* __restrict__ norm_w,
+    float* __restrict__ state,          // [slots, H, D, V]
+    const int* __restrict__ slot, const int* __restrict__ pos,
+    const int* __restrict__ spans,      // [n, 2] first row, rows; null: 1 row
+    int H, int D, int V, float scale, float inv_tau, float eps)
+{
+    const int h = blockIdx.y, tid = threadIdx.x;
+    const int t0 = spans ? spans[blockIdx.x * 2] : blockIdx.x;
+    const int nt = spans ? spans[blockIdx.x * 2 + 1] : 1;
+    const int nv = V / VEC;             // threads across a state row
+    const int RG = 256 / nv;            // state rows in flight
+    const int vt = tid % nv, rg = tid / nv;
+    const bool live = rg < RG;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    float* q_s = sm;                    // [D]
+    float* k_s = q_s + D;
+    float* a_s = k_s + D;
+    float* o_s = a_s + D;               // [RG][V]
+    float* r_s = o_s + RG * V;          // [4]
+    float* S = state + ((int64_t)slot[t0] * H + h) * D * V + vt * VEC;
+    bool fresh = pos[t0] == 0;
+    for (int t = t0; t < t0 + nt; ++t) {
+        const T* row = p + (int64_t)t * in.ld;
+        for (int d = tid; d < D; d += 256) {
+            const int c = h * D + d;
+            q_s[d] = ldf(row + in.oq + c) * scale;
+            k_s[d] = ldf(row + in.ok + c);
+            float z = a2_b[c];
+            for (int r = 0; r < in.rank; r++)
+                z += ldf(a2 + (int64_t)c * in.rank + r)
+                     * ldf(row + in.ou + r);
+            a_s[d] = expf(log_alpha(z, inv_tau));
+        }
+        __syncthreads();
+        if (live) {
+            float v[VEC], acc[VEC] = {};
+            ldv<VEC>(row + in.ov + h * V + vt * VEC, v);
+            #pragma unroll 8
+            for (int d = rg; d < D; d += RG) {
+                float s[VEC];
+                if (fresh) {
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) s[i] = k_s[d] * v[i];
+                } else {
+                    ldv<VEC>(S + (int64_t)d * V, s);
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++)
+                        s[i] = a_s[d] * s[i] + k_s[d] * v[i];
+                }
+                stv<VEC>(S + (int64_t)d * V, s);
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) acc[i] += q_s[d] * s[i];
+            }
+            stv<VEC>(o_s + rg * V + vt * VEC, acc);
+        }
+        fresh = false;
+        __syncthreads();
+        float sq = 0.f;
+        for (int c = tid; c < V; c += 256) {
+            float o = 0.f;
+            for (int r = 0; r < RG; r++) o += o_s[r * V + c];
+            o_s[c] = o;                 // only this thread reads column c
+            sq += o * o;
+        }
+        sq = wave_sum(sq);
+        if ((tid & 63) == 0) r_s[tid >> 6] = sq;
+        __syncthreads();
+        const float ms = ((r_s[0] + r_s[1]) + (r_s[2] + r_s[3])) / V;
+        const float rs = 1.f / sqrtf(ms + eps);
+        for (int c = tid; c < V; c += 256)
+            stf(out + ((int64_t)t * H + h) * V + c,
+                o_s[c] * rs * norm_w[c]
+                    * silu(ldf(row + in.og + h * V + c)));
+        __syncthreads();
+    }
+}
+
+static bool gla_sizes_ok(int D, int V, int rank)
+{
+    return D >= 1 && D <= 512 && V >= 1 && rank >= 1 && rank <= 256
+           && (V % 4 == 0 ? V <= 1024 : V <= 256);
+}
+
+extern "C" int gla_step(
+    int f32, void* out, const void* p, int64_t ld, int oq, int ok, int ov,
+    int og, int ou, int rank, const void* a2, const void* a2_b,
+    const void* norm_w, void* state, const void* slot, const void* pos,
+    const void* spans, int n, int H, int D, int V, float scale,
+    float inv_tau, float eps, hipStream_t stream)
+{
+    if (!gla_sizes_ok(D, V, rank)) return (int)hipErrorInvalidValue;
+    // a vector load of v needs aligned columns
+    const bool v4 = V % 4 == 0 && ov % 4 == 0 && ld % 4 == 0;
+    if (!v4 && V > 256) return (int)hipErrorInvalidValue;
+    GlaIn in{ld, oq, ok, ov, og, ou, rank};
+    const int rg = 256 / (v4 ? V / 4 : V);
+    const int lds = (3 * D + rg * V + 4) * 4;
+    dim3 grid(n, H);
+    #define GS_GO(T, VV)                                                   \
+        k_gla_step<T, VV><<<grid, 256, lds, stream>>>(                     \
+            (T*)out, (const T*)p, in, (const T*)a2, (const float*)a2_b,    \
+            (const float*)norm_w, (float*)state, (const int*)slot,         \
+            (const int*)pos, (const int*)spans, H, D, V, scale, inv_tau,   \
+            eps)
+    if (f32) { if (v4) GS_GO(float, 4); else GS_GO(float, 1); }
+    else { if (v4) GS_GO(bf16, 4); else GS_GO(bf16, 1); }
+    #undef GS_GO
+    return (int)hipGetLastError();
+}
+
+// ---- chunks --------------------------------------------------------------
+#define CH 64             // tokens of a chunk
+#define SUB 16            // tokens of a part
+#define DB 32             // key channels of a prep pass
+#define DS (DB + 1)       // LDS row stride
+// largest sum of decay inside a part for which the part's own triangle may
+// be factored (e^{b_i} e^{-b_j}); beyond it the pairs are taken one by one
+#define SAFE 40.f
+
+// scratch per (chunk, head): qd [64][Dp], kd^T [Dp][64], A [64][64], eb [Dp]
+DEV int64_t gla_unit(int Dp) {
+    return (int64_t)2 * CH * Dp + CH * CH + Dp;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void k_gla_prep(
+    float* __restrict__ scr, const T* __restrict__ p, GlaIn in,
+    const T* __restrict__ a2, const float* __restrict__ a2_b,
+    const int* __restrict__ chunks,     // [n, 2] first row, rows
+    int H, int D, int Dp, float scale, float inv_tau)
+{
+    const int h = blockIdx.y, tid = threadIdx.x;
+    const int lane = tid & 63, w = tid >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    const int t0 = chunks[blockIdx.x * 2], n = chunks[blockIdx.x * 2 + 1];
+    float* qd = scr + ((int64_t)blockIdx.x * H + h) * gla_unit(Dp);
+    float* kdt = qd + CH * Dp;
+    float* Ao = kdt + CH * Dp;
+    float* eb = Ao + CH * CH;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    float* q_s = sm;                    // [64][DS] scaled q
+    float* k_s = q_s + CH * DS;
+    float* b_s = k_s + CH * DS;         // running log decay inside a part
+    float* qe_s = b_s + CH * DS;        // q e^{b}
+    float* ke_s = qe_s + CH * DS;       // k e^{part total - b}
+    float* et_s = ke_s + CH * DS;       // [4][DB] e^{part total}
+    float* u_s = et_s + 4 * DB;         // [64][rank]
+
+    for (int i = tid; i < CH * in.rank; i += 256) {
+        const int t = i / in.rank;
+        u_s[i] = t < n ? ldf(p + (int64_t)(t0 + t) * in.ld + in.ou
+                             + i % in.rank) : 0.f;
+    }
+    // this wave's tiles of A: its own diagonal, and of the six tiles below
+    // it (1,0) (2,1) (3,2) (2,0) (3,1) (3,0) numbers w and w + 4
+    const int ti[6] = {1, 2, 3, 2, 3, 3}, tj[6] = {0, 1, 2, 0, 1, 0};
+    f32x4 diag = {}, off[2] = {};
+
+    for (int d0 = 0; d0 < Dp; d0 += DB) {
+        __syncthreads();
+        for (int i = tid; i < CH * DB; i += 256) {
+            const int t = i / DB, d = i % DB;
+            const bool on = t < n && d0 + d < D;
+            const T* row = p + (int64_t)(t0 + t) * in.ld + h * D + d0 + d;
+            q_s[t * DS + d] = on ? ldf(row + in.oq) * scale : 0.f;
+            k_s[t * DS + d] = on ? ldf(row + in.ok) : 0.f;
+            float la = 0.f;
+            if (on) {
+                const int c = h * D + d0 + d;
+                float z = a2_b[c];
+                const T* wr = a2 + (int64_t)c * in.rank;
+                for (int r = 0; r < in.rank; r++)
+                    z += ldf(wr + r) * u_s[t * in.rank + r];
+                la = log_alpha(z, inv_tau);
+            }
+            b_s[t * DS + d] = la;
+        }
+        __syncthreads();
+        if (tid < 4 * DB) {
+            const int s = tid / DB, d = tid % DB;
+            float b = 0.f;
+            for (int t = s * SUB; t < (s + 1) * SUB; t++) {
+                b += b_s[t * DS + d];
+                b_s[t * DS + d] = b;
+                qe_s[t * DS + d] = q_s[t * DS + d] * expf(b);
+            }
+            for (int t = s * SUB; t < (s + 1) * SUB; t++)
+                ke_s[t * DS + d] = k_s[t * DS + d]
+                                   * expf(b - b_s[t * DS + d]);
+            et_s[s * DB + d] = expf(b);
+        }
+        __syncthreads();
+        // factors that meet the state
+        for (int i = tid; i < CH * DB; i += 256) {
+            const int t = i / DB, d = i % DB;
+            if (d0 + d < Dp) {
+                float f = qe_s[t * DS + d];
+                for (int s = 0; s < t / SUB; s++) f *= et_s[s * DB + d];
+                qd[t * Dp + d0 + d] = f;
+            }
+        }
+        for (int i = tid; i < CH * DB; i += 256) {
+            const int d = i / CH, t = i % CH;
+            if (d0 + d < Dp) {
+                float f = ke_s[t * DS + d];
+                for (int s = t / SUB + 1; s < 4; s++) f *= et_s[s * DB + d];
+                kdt[(d0 + d) * CH + t] = f;
+            }
+        }
+        if (tid < DB && d0 + tid < Dp)
+            eb[d0 + tid] = et_s[tid] * et_s[DB + tid]
+                           * et_s[2 * DB + tid] * et_s[3 * DB + tid];
+        // tiles below the diagonal
+        #pragma unroll
+        for (int x = 0; x < 2; x++) {
+            const int id = w + x * 4;
+            if (id >= 6) continue;
+            const int I = ti[id], J = tj[id];
+            for (int d = g; d < DB; d += 4) {
+                float a = qe_s[(I * SUB + lr) * DS + d];
+                for (int s = J + 1; s < I; s++) a *= et_s[s * DB + d];
+                off[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    a, ke_s[(J * SUB + lr) * DS + d], off[x], 0, 0, 0);
+            }
+        }
+        // the part's own triangle
+        float mn = 0.f;
+        for (int d = lane; d < DB; d += 64)
+            mn = fminf(mn, b_s[(w * SUB + SUB - 1) * DS + d]);
+        const bool safe = wave_max(-mn) < SAFE;
+        if (safe) {
+            for (int d = g; d < DB; d += 4) {
+                const int o = (w * SUB + lr) * DS + d;
+                diag = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    qe_s[o], k_s[o] * expf(-b_s[o]), diag, 0, 0, 0);
+            }
+        } else {
+            // lane: column lr (the key), rows g*4 + i (the query)
+            for (int d = 0; d < DB; d++) {
+                const int oj = (w * SUB + lr) * DS + d;
+                const float kj = k_s[oj], bj = b_s[oj];
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int oi = (w * SUB + g * 4 + i) * DS + d;
+                    diag[i] += q_s[oi] * kj
+                               * expf(fminf(b_s[oi] - bj, 0.f));
+                }
+            }
+        }
+    }
+    #pragma unroll
+    for (int i = 0; i < 4; i++)
+        Ao[(w * SUB + g * 4 + i) * CH + w * SUB + lr] =
+            lr <= g * 4 + i ? diag[i] : 0.f;
+    #pragma unroll
+    for (int x = 0; x < 2; x++) {
+        const int id = w + x * 4;
+        if (id >= 6) continue;
+        #pragma unroll
+        for (int i = 0; i < 4; i++)
+            Ao[(ti[id] * SUB + g * 4 + i) * CH + tj[id] * SUB + lr] =
+                off[x][i];
+    }
+}
+
+// NS: 16-row state tiles per wave (D <= 64 * NS); VC: 16-column tiles
+template <typename T, int NS, int VC>
+__global__ __launch_bounds__(256) void k_gla_scan(
+    float* __restrict__ o,              // [rows, H, V]
+    const float* __restrict__ scr, const T* __restrict__ p, GlaIn in,
+    float* __restrict__ state,
+    const int* __restrict__ slot, const int* __restrict__ pos,
+    const int* __restrict__ chunks,     // [n, 2]
+    const int* __restrict__ seqs,       // [m, 2] first chunk, chunks
+    int row_base,                       // first row of o
+    int H, int D, int Dp, int V)
+{
+    constexpr int W = VC * 16, WS = W + (W % 64 == 16 ? 0 : 16);
+    const int h = blockIdx.y, v0 = blockIdx.z * W, tid = threadIdx.x;
+    const int lane = tid & 63, w = tid >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    const int c0 = seqs[blockIdx.x * 2], nc = seqs[blockIdx.x * 2 + 1];
+    const int first = chunks[c0 * 2];
+    float* St = state + ((int64_t)slot[first] * H + h) * D * V;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    float* S_s = sm;                    // [Dp][WS]
+    float* v_s = S_s + Dp * WS;         // [64][WS]
+
+    f32x4 S[NS][VC];
+    const bool fresh = pos[first] == 0;
+    #pragma unroll
+    for (int x = 0; x < NS; x++)
+        #pragma unroll
+        for (int c = 0; c < VC; c++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int d = (w + x * 4) * 16 + g * 4 + i;
+                const int v = v0 + c * 16 + lr;
+                S[x][c][i] = (fresh || d >= D || v >= V)
+                                 ? 0.f : St[(int64_t)d * V + v];
+            }
+
+    for (int ci = c0; ci < c0 + nc; ++ci) {
+        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
+        const float* qd = scr + ((int64_t)ci * H + h) * gla_unit(Dp);
+        const float* kdt = qd + CH * Dp;
+        const float* A = kdt + CH * Dp;
+        const float* eb = A + CH * CH;
+        for (int i = tid; i < CH * W; i += 256) {
+            const int t = i / W, c = i % W;
+            v_s[t * WS + c] = (t < n && v0 + c < V)
+                ? ldf(p + (int64_t)(t0 + t) * in.ld + in.ov + h * V + v0 + c)
+                : 0.f;
+        }
+        #pragma unroll
+        for (int x = 0; x < NS; x++) {
+            const int d0 = (w + x * 4) * 16;
+            if (d0 < Dp)
+                #pragma unroll
+                for (int c = 0; c < VC; c++)
+                    #pragma unroll
+                    for (int i = 0; i < 4; i++)
+                        S_s[(d0 + g * 4 + i) * WS + c * 16 + lr] =
+                            S[x][c][i];
+        }
+        __syncthreads();
+        // o tile of this wave's 16 tokens; a lane's k runs in fours, the
+        // same for both operands
+        f32x4 acc[VC] = {};
+        const float* qr = qd + (w * 16 + lr) * Dp + g * 4;
+        for (int d = 0; d < Dp; d += 16) {
+            const f32x4 a = *reinterpret_cast<const f32x4*>(qr + d);
+            #pragma unroll
+            for (int e = 0; e < 4; e++)
+                #pragma unroll
+                for (int c = 0; c < VC; c++)
+                    acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                        a[e], S_s[(d + g * 4 + e) * WS + c * 16 + lr],
+                        acc[c], 0, 0, 0);
+        }
+        const float* Ar = A + (w * 16 + lr) * CH + g * 4;
+        for (int j = 0; j <= w; j++) {
+            const f32x4 a = *reinterpret_cast<const f32x4*>(Ar + j * 16);
+            #pragma unroll
+            for (int e = 0; e < 4; e++)
+                #pragma unroll
+                for (int c = 0; c < VC; c++)
+                    acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                        a[e], v_s[(j * 16 + g * 4 + e) * WS + c * 16 + lr],
+                        acc[c], 0, 0, 0);
+        }
+        #pragma unroll
+        for (int c = 0; c < VC; c++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int t = w * 16 + g * 4 + i, v = v0 + c * 16 + lr;
+                if (t < n && v < V)
+                    o[((int64_t)(t0 - row_base + t) * H + h) * V + v] =
+                        acc[c][i];
+            }
+        // state
+        #pragma unroll
+        for (int x = 0; x < NS; x++) {
+            const int d0 = (w + x * 4) * 16;
+            if (d0 >= Dp) continue;
+            const f32x4 e4 = *reinterpret_cast<const f32x4*>(
+                eb + d0 + g * 4);
+            #pragma unroll
+            for (int c = 0; c < VC; c++) S[x][c] *= e4;
+            const float* kr = kdt + (d0 + lr) * CH + g * 4;
+            #pragma unroll
+            for (int t = 0; t < CH; t += 16) {
+                const f32x4 a = *reinterpret_cast<const f32x4*>(kr + t);
+                #pragma unroll
+                for (int e = 0; e < 4; e++)
+                    #pragma unroll
+                    for (int c = 0; c < VC; c++)
+                        S[x][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                            a[e], v_s[(t + g * 4 + e) * WS + c * 16 + lr],
+                            S[x][c], 0, 0, 0);
+            }
+        }
+        __syncthreads();
+    }
+    #pragma unroll
+    for (int x = 0; x < NS; x++)
+        #pragma unroll
+        for (int c = 0; c < VC; c++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int d = (w + x * 4) * 16 + g * 4 + i;
+                const int v = v0 + c * 16 + lr;
+                if (d < D && v < V) St[(int64_t)d * V + v] = S[x][c][i];
+            }
+}
+
+// head norm and gate, one wave per (token, head)
+template <typename T>
+__global__ __launch_bounds__(256) void k_gla_out(
+    T* __restrict__ out, const float* __restrict__ o,
+    const T* __restrict__ p, GlaIn in, const float* __restrict__ norm_w,
+    int row_base, int64_t n, int H, int V, float eps)
+{
+    const int64_t u = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
+    if (u >= n) return;
+    const int64_t t = u / H;
+    const int h = (int)(u % H);
+    const float* src = o + u * V;
+    float sq = 0.f;
+    for (int c = lane; c < V; c += 64) sq += src[c] * src[c];
+    const float rs = 1.f / sqrtf(wave_sum(sq) / V + eps);
+    const T* gr = p + (row_base + t) * in.ld + in.og + h * V;
+    T* dst = out + ((row_base + t) * H + h) * V;
+    for (int c = lane; c < V; c += 64)
+        stf(dst + c, src[c] * rs * norm_w[c] * silu(ldf(gr + c)));
+}
+
+extern "C" int64_t gla_scratch_floats(int n_chunks, int H, int D)
+{
+    const int Dp = (D + 15) & ~15;
+    return (int64_t)n_chunks * H * (2 * CH * Dp + CH * CH + Dp);
+}
+
+// Portions of whole sequences in chunks of 64 rows.  chunks int32 [n, 2]
+// (first row, rows), a sequence's chunks in a run; seqs int32 [m, 2] (first
+// chunk, chunks).  Rows row_base .. row_base + rows - 1 are covered.
+extern "C" int gla_chunks(
+    int f32, void* out, void* scr, void* o_scr, const void* p, int64_t ld,
+    int oq, int ok, int ov, int og, int ou, int rank, const void* a2,
+    const void* a2_b, const void* norm_w, void* state, const void* slot,
+    const void* pos, const void* chunks, int n_chunks, const void* seqs,
+    int n_seqs, int row_base, int rows, int H, int D, int V, float scale,
+    float inv_tau, float eps, hipStream_t stream)
+{
+    if (!gla_sizes_ok(D, V, rank)) return (int)hipErrorInvalidValue;
+    GlaIn in{ld, oq, ok, ov, og, ou, rank};
+    const int Dp = (D + 15) & ~15;
+    const int lds_a = (5 * CH * DS + 4 * DB + CH * rank) * 4;
+    // wider column tiles re-read the factors less; narrow ones fill the chip
+    const int vc = (int64_t)n_seqs * H * ((V + 31) / 32) >= 256 ? 2 : 1;
+    const int ws = vc == 1 ? 16 : 48;
+    const int lds_b = (Dp + CH) * ws * 4;
+    if (lds_a > 160 * 1024 || lds_b > 160 * 1024)
+        return (int)hipErrorInvalidValue;
+    dim3 ga(n_chunks, H), gb(n_seqs, H, (V + vc * 16 - 1) / (vc * 16));
+    const int64_t units = (int64_t)rows * H;
+    const int gc = (int)((units + 3) / 4);
+    #define GC_SCAN(T, NS, VC)                                             \
+        do {                                                               \
+            (void)hipFuncSetAttribute(                                     \
+                (const void*)k_gla_scan<T, NS, VC>,                        \
+                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);   \
+            k_gla_scan<T, NS, VC><<<gb, 256, lds_b, stream>>>(             \
+                (float*)o_scr, (const float*)scr, (const T*)p, in,         \
+                (float*)state, (const int*)slot, (const int*)pos,          \
+                (const int*)chunks, (const int*)seqs, row_base, H, D, Dp,  \
+                V);                                                        \
+        } while (0)
+    #define GC_NS(T, VC)                                                   \
+        do {                                                               \
+            if (Dp <= 64) GC_SCAN(T, 1, VC);                               \
+            else if (Dp <= 128) GC_SCAN(T, 2, VC);                         \
+            else if (Dp <= 256) GC_SCAN(T, 4, VC);                         \
+            else GC_SCAN(T, 8, VC);                                        \
+        } while (0)
+    #define GC_TYPE(T)                                                     \
+        do {                                                               \
+            (void)hipFuncSetAttribute(                                     \
+                (const void*)k_gla_prep<T>,                                \
+                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);   \
+            k_gla_prep<T><<<ga, 256, lds_a, stream>>>(                     \
+                (float*)scr, (const T*)p, in, (const T*)a2,                \
+                (const float*)a2_b, (const int*)chunks, H, D, Dp, scale,   \
+                inv_tau);                                                  \
+            if (vc == 1) GC_NS(T, 1); else GC_NS(T, 2);                    \
+            k_gla_out<T><<<gc, 256, 0, stream>>>(                          \
+                (T*)out, (const float*)o_scr, (const T*)p, in,             \
+                (const float*)norm_w, row_base, units, H, V, eps);         \
+        } while (0)
+    if (f32) GC_TYPE(float); else GC_TYPE(bf16);
+    #undef GC_TYPE
+    #undef GC_NS
+    #undef GC_SCAN
+    return (int)hipGetLastError();
+}

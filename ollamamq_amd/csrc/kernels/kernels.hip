@@ -39,6 +39,15 @@ DEV void load8f(const bf16* p, float* out) {
     out[4] = fc.x; out[5] = fc.y; out[6] = fd.x; out[7] = fd.y;
 }
 
+DEV void load8f(const float* p, float* out) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    const float4 b = *reinterpret_cast<const float4*>(p + 4);
+    out[0] = a.x; out[1] = a.y; out[2] = a.z; out[3] = a.w;
+    out[4] = b.x; out[5] = b.y; out[6] = b.z; out[7] = b.w;
+}
+DEV float tof(float x) { return x; }
+DEV float tof(bf16 x) { return bf2f(x); }
+
 DEV void store8bf(bf16* p, const float* in) {
     bf162* v = reinterpret_cast<bf162*>(p);
     v[0] = __float22bfloat162_rn(make_float2(in[0], in[1]));
@@ -484,15 +493,16 @@ extern "C" int swiglu_bf16(void* out, const void* gu, int T, int F,
 }
 
 // ---------------------------------------------------------------------------
-// Greedy sampler: per-row argmax over the vocab, bf16 logits.
+// Greedy sampler: per-row argmax over the vocab, bf16 or fp32 logits.
 // One 256-thread block per row; ties resolve to the LOWEST index (matches
 // torch.argmax on the reference path).
 // ---------------------------------------------------------------------------
+template <typename T>
 __global__ __launch_bounds__(256) void k_argmax(
-    int* __restrict__ out, const bf16* __restrict__ logits, int V)
+    int* __restrict__ out, const T* __restrict__ logits, int V)
 {
     const int row = blockIdx.x;
-    const bf16* lr = logits + (int64_t)row * V;
+    const T* lr = logits + (int64_t)row * V;
     float best = -3.0e38f;
     int bidx = 0;
     for (int i = threadIdx.x * 8; i < V; i += blockDim.x * 8) {
@@ -506,7 +516,7 @@ __global__ __launch_bounds__(256) void k_argmax(
                 }
         } else {
             for (int e = i; e < V; e++) {
-                const float v = bf2f(lr[e]);
+                const float v = tof(lr[e]);
                 if (v > best || (v == best && e < bidx)) { best = v; bidx = e; }
             }
         }
@@ -536,13 +546,14 @@ __global__ __launch_bounds__(256) void k_argmax(
 // serialize ~V/2048 load rounds each (measured 45 us at V=128256).
 // Stage 1: (B, SP) blocks scan V/SP slices; stage 2: one wave per row
 // combines SP partials.  Global indices keep lowest-index tie-breaking.
+template <typename T>
 __global__ __launch_bounds__(256) void k_argmax_part(
     float* __restrict__ pb, int* __restrict__ pi,
-    const bf16* __restrict__ logits, int V, int seg)
+    const T* __restrict__ logits, int V, int seg)
 {
     const int row = blockIdx.x, slice = blockIdx.y;
     const int lo = slice * seg, hi = min(V, lo + seg);
-    const bf16* lr = logits + (int64_t)row * V;
+    const T* lr = logits + (int64_t)row * V;
     float best = -3.0e38f;
     int bidx = 0;
     for (int i = lo + threadIdx.x * 8; i < hi; i += blockDim.x * 8) {
@@ -556,7 +567,7 @@ __global__ __launch_bounds__(256) void k_argmax_part(
                 }
         } else {
             for (int e = i; e < hi; e++) {
-                const float v = bf2f(lr[e]);
+                const float v = tof(lr[e]);
                 if (v > best || (v == best && e < bidx)) { best = v; bidx = e; }
             }
         }
@@ -600,21 +611,34 @@ __global__ __launch_bounds__(256) void k_argmax_comb(
     if (lane == 0) out[row] = bidx;
 }
 
-extern "C" int argmax_bf16(void* out, const void* logits, int B, int V,
-                            void* pb, void* pi, int SP, hipStream_t stream)
+template <typename T>
+static int argmax_go(void* out, const void* logits, int B, int V,
+                     void* pb, void* pi, int SP, hipStream_t stream)
 {
     if (SP > 1 && pb != nullptr) {
         int seg = (V / SP + 2047) & ~2047;          // 256-thread x8 rounds
         while ((int64_t)(SP - 1) * seg >= V) SP--;  // drop empty slices
         dim3 grid(B, SP);
-        k_argmax_part<<<grid, 256, 0, stream>>>(
-            (float*)pb, (int*)pi, (const bf16*)logits, V, seg);
+        k_argmax_part<T><<<grid, 256, 0, stream>>>(
+            (float*)pb, (int*)pi, (const T*)logits, V, seg);
         k_argmax_comb<<<(B + 3) / 4, 256, 0, stream>>>(
             (int*)out, (const float*)pb, (const int*)pi, B, SP);
     } else {
-        k_argmax<<<B, 256, 0, stream>>>((int*)out, (const bf16*)logits, V);
+        k_argmax<T><<<B, 256, 0, stream>>>((int*)out, (const T*)logits, V);
     }
     return (int)hipGetLastError();
+}
+
+extern "C" int argmax_bf16(void* out, const void* logits, int B, int V,
+                            void* pb, void* pi, int SP, hipStream_t stream)
+{
+    return argmax_go<bf16>(out, logits, B, V, pb, pi, SP, stream);
+}
+
+extern "C" int argmax_f32(void* out, const void* logits, int B, int V,
+                          void* pb, void* pi, int SP, hipStream_t stream)
+{
+    return argmax_go<float>(out, logits, B, V, pb, pi, SP, stream);
 }
 
 // ---------------------------------------------------------------------

@@ -1,0 +1,706 @@
+// gfx950 latent attention: a paged pool caches one latent row of R values
+// per token, keys and values are linear maps of it (k = W_uk c, v = W_uv c,
+// per head).  Two exact ways to attend, chosen per sequence by the caller:
+//
+// * absorbed (decode, short portions): q' = W_uk^T q makes the score
+//   q' . c, so all heads share the cached row — the pool is read once per
+//   token of context.  k_latent_attn streams the pool with the (token,
+//   head) rows on the matrix cores and returns the weighted latent per row,
+//   which k_head_gemm maps through W_uv.
+// * expanded (long portions): k and v of the whole context are made with
+//   one matrix product each, then k_flash is an ordinary causal flash
+//   attention with free key and value widths.
+#include "tile_mma.h"
+
+#define NEG (-3.0e38f)
+
+template <typename T> DEV float exp_of(float x) {
+    if constexpr (sizeof(T) == 4) return expf(x);
+    else return __expf(x);
+}
+
+// ---------------------------------------------------------------------------
+// out[t][h][n] = sum_k x[t*xs + h*K + k] * w[h][n][k]
+// Grid (n / 64, t / (16*MT), H); a wave makes 16 n x 16*MT tokens.  The
+// product is transposed (A = w) so a lane stores four consecutive n.
+// ---------------------------------------------------------------------------
+template <typename T, int MT>
+__global__ __launch_bounds__(256) void k_head_gemm(
+    T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ w,
+    int T_rows, int H, int N, int K, int64_t xs)
+{
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    const int h = blockIdx.z;
+    const int n0 = (blockIdx.x * 4 + wid) * 16;
+    const int t0 = blockIdx.y * 16 * MT;
+    if (n0 >= N) return;
+    const T* wr = w + ((int64_t)h * N + min(n0 + lr, N - 1)) * K;
+    const T* xr[MT];
+    #pragma unroll
+    for (int m = 0; m < MT; m++)
+        xr[m] = x + (int64_t)min(t0 + m * 16 + lr, T_rows - 1) * xs
+                + (int64_t)h * K;
+    f32x4 acc[MT] = {};
+    const bool vec = K % 8 == 0 && xs % 8 == 0;
+    for (int k0 = 0; k0 < K; k0 += 32) {
+        const int k = k0 + g * 8;
+        Frag<T> a, b[MT];
+        if (vec) {
+            const bool in = k < K;
+            a = in ? frag8(wr + k) : frag_zero<T>();
+            #pragma unroll
+            for (int m = 0; m < MT; m++)
+                b[m] = in ? frag8(xr[m] + k) : frag_zero<T>();
+        } else {
+            a = frag_guard(wr, k, K);
+            #pragma unroll
+            for (int m = 0; m < MT; m++) b[m] = frag_guard(xr[m], k, K);
+        }
+        #pragma unroll
+        for (int m = 0; m < MT; m++) acc[m] = mma(a, b[m], acc[m]);
+    }
+    #pragma unroll
+    for (int m = 0; m < MT; m++) {
+        const int t = t0 + m * 16 + lr;
+        if (t >= T_rows) continue;
+        T* o = out + ((int64_t)t * H + h) * N + n0 + g * 4;
+        if (N % 4 == 0 && n0 + g * 4 + 4 <= N) {
+            float v[4] = {acc[m][0], acc[m][1], acc[m][2], acc[m][3]};
+            stv<4>(o, v);
+        } else
+            for (int i = 0; i < 4; i++)
+                if (n0 + g * 4 + i < N) stf(o + i, acc[m][i]);
+    }
+}
+
+extern "C" int head_gemm(int f32, void* out, const void* x, const void* w,
+                         int T_rows, int H, int N, int K, int64_t xs,
+                         hipStream_t stream)
+{
+    const bool wide = T_rows > 16;
+    dim3 grid((N + 63) / 64, (T_rows + (wide ? 31 : 15)) / (wide ? 32 : 16),
+              H);
+    #define HG_GO(T, M)                                                    \
+        k_head_gemm<T, M><<<grid, 256, 0, stream>>>(                       \
+            (T*)out, (const T*)x, (const T*)w, T_rows, H, N, K, xs)
+    if (f32) { if (wide) HG_GO(float, 2); else HG_GO(float, 1); }
+    else { if (wide) HG_GO(bf16, 2); else HG_GO(bf16, 1); }
+    #undef HG_GO
+    return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// Absorbed attention over the paged latent pool.
+//
+// Rows are (token, head) pairs, row = token * H + head; a work item is up to
+// M = 16*MT consecutive rows of one sequence, and grid.y cuts its context
+// into segments (exact merge in k_latent_combine).  Per KT-key chunk, staged
+// once into LDS for all rows:
+//   S^T[key, row] = C q'^T      key tiles dealt over the four waves
+//   online softmax              16 lanes a row, fp32
+//   O^T[r, row]  += C^T P^T     latent columns dealt over the four waves
+// NT: 16-wide latent column tiles per wave (R <= 64 * NT).
+// ---------------------------------------------------------------------------
+template <typename T, int MT, int KT, int NT>
+__global__ __launch_bounds__(256) void k_latent_attn(
+    T* __restrict__ out,               // [rows, R]      (split == 1)
+    float* __restrict__ o_part,        // [split, rows, R]
+    float* __restrict__ ml_part,       // [split, rows, 2]
+    const T* __restrict__ q,           // [rows, R]
+    const T* __restrict__ pool,        // [pages, psz, R]
+    const int* __restrict__ ptab, const int* __restrict__ slot,
+    const int* __restrict__ pos,
+    const int* __restrict__ items,     // [n, 2] first row, rows; null: decode
+    int per_seq,                       // decode: items per sequence
+    int H, int R, int psz, int maxp, float scale, int64_t rows_total,
+    int split)
+{
+    constexpr int M = 16 * MT;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    int row0, n_rows;
+    if (items) {
+        row0 = items[blockIdx.x * 2];
+        n_rows = items[blockIdx.x * 2 + 1];
+    } else {
+        const int j = blockIdx.x % per_seq;
+        row0 = (blockIdx.x / per_seq) * H + j * M;
+        n_rows = min(M, H - j * M);
+    }
+    const int tok0 = row0 / H, tok1 = (row0 + n_rows - 1) / H;
+    const int kv_len = pos[tok1] + 1;
+    const int* pt = ptab + (int64_t)slot[tok0] * maxp;
+    const int n_chunks = (kv_len + KT - 1) / KT;
+    const int c_lo = (int)((int64_t)blockIdx.y * n_chunks / split);
+    const int c_hi = (int)((int64_t)(blockIdx.y + 1) * n_chunks / split);
+
+    const int Rp = (R + 31) & ~31;
+    const int cs = Rp + 16 / (int)sizeof(T);      // LDS row strides
+    constexpr int SS = KT + 4, PS = KT + 16 / (int)sizeof(T);
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    T* q_s = reinterpret_cast<T*>(smem);          // [M][cs]
+    T* c_s = q_s + M * cs;                        // [KT][cs]
+    T* p_s = c_s + KT * cs;                       // [M][PS]
+    float* s_s = reinterpret_cast<float*>(p_s + M * PS);   // [M][SS]
+    float* m_s = s_s + M * SS;                    // [M] running max
+    float* l_s = m_s + M;                         // [M] running sum
+    float* f_s = l_s + M;                         // [M] this chunk's rescale
+    int* lim_s = reinterpret_cast<int*>(f_s + M); // [M] visible keys
+
+    const bool vec = R % 8 == 0;
+    // rows of the chunk or of q, zero beyond R
+    auto stage = [&](T* dst, const T* src_row, int c8) {
+        const int k = c8 * 8;
+        Frag<T> v;
+        if (src_row == nullptr) v = frag_zero<T>();
+        else if (vec) v = k < R ? frag8(src_row + k) : frag_zero<T>();
+        else v = frag_guard(src_row, k, R);
+        *reinterpret_cast<Frag<T>*>(dst + k) = v;
+    };
+    const int n8 = Rp / 8;
+    for (int u = tid; u < M * n8; u += 256) {
+        const int r = u / n8;
+        stage(q_s + r * cs,
+              r < n_rows ? q + (int64_t)(row0 + r) * R : nullptr, u % n8);
+    }
+    if (tid < M) {
+        m_s[tid] = NEG;
+        l_s[tid] = 0.f;
+        lim_s[tid] = tid < n_rows ? pos[(row0 + tid) / H] + 1 : 0;
+    }
+    f32x4 acc[MT][NT] = {};
+    __syncthreads();               // a segment may hold no chunk at all
+
+    for (int ch = c_lo; ch < c_hi; ++ch) {
+        const int base = ch * KT;
+        for (int u = tid; u < KT * n8; u += 256) {
+            const int k = u / n8, key = base + k;
+            stage(c_s + k * cs,
+                  key < kv_len
+                      ? pool + ((int64_t)pt[key / psz] * psz + key % psz) * R
+                      : nullptr,
+                  u % n8);
+        }
+        __syncthreads();
+        #pragma unroll
+        for (int i = 0; i < (MT * KT / 16 + 3) / 4; i++) {
+            const int id = wid + i * 4;
+            if (id < MT * KT / 16) {
+                const int mt = id / (KT / 16), kt = id % (KT / 16);
+                f32x4 s = {};
+                const T* ar = c_s + (kt * 16 + lr) * cs + g * 8;
+                const T* br = q_s + (mt * 16 + lr) * cs + g * 8;
+                for (int k = 0; k < Rp; k += 32)
+                    s = mma(frag8(ar + k), frag8(br + k), s);
+                const int row = mt * 16 + lr, k0 = kt * 16 + g * 4;
+                #pragma unroll
+                for (int e = 0; e < 4; e++)
+                    s[e] = base + k0 + e < lim_s[row] ? s[e] * scale : NEG;
+                *reinterpret_cast<f32x4*>(s_s + row * SS + k0) = s;
+            }
+        }
+        __syncthreads();
+        // 16 lanes a row, KT/16 keys a lane
+        #pragma unroll
+        for (int mt = 0; mt < MT; mt++) {
+            const int row = mt * 16 + wid * 4 + g;
+            constexpr int KL = KT / 16;
+            float s[KL], mx = NEG;
+            #pragma unroll
+            for (int j = 0; j < KL; j++) {
+                s[j] = s_s[row * SS + lr + j * 16];
+                mx = fmaxf(mx, s[j]);
+            }
+            #pragma unroll
+            for (int o = 8; o; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
+            const float m_old = m_s[row], m_new = fmaxf(m_old, mx);
+            float sum = 0.f;
+            #pragma unroll
+            for (int j = 0; j < KL; j++) {
+                const float p = s[j] > NEG ? exp_of<T>(s[j] - m_new) : 0.f;
+                sum += p;
+                stf(p_s + row * PS + lr + j * 16, p);
+            }
+            #pragma unroll
+            for (int o = 8; o; o >>= 1) sum += __shfl_xor(sum, o, 64);
+            if (lr == 0) {
+                const float f = exp_of<T>(m_old - m_new);
+                f_s[row] = f;
+                l_s[row] = l_s[row] * f + sum;
+                m_s[row] = m_new;
+            }
+        }
+        __syncthreads();
+        float f[MT];
+        #pragma unroll
+        for (int mt = 0; mt < MT; mt++) f[mt] = f_s[mt * 16 + lr];
+        #pragma unroll
+        for (int n = 0; n < NT; n++) {
+            const int col = (n * 4 + wid) * 16 + lr;
+            if ((n * 4 + wid) * 16 < Rp) {
+                #pragma unroll
+                for (int mt = 0; mt < MT; mt++) acc[mt][n] *= f[mt];
+                #pragma unroll
+                for (int k = 0; k < KT; k += 32) {
+                    Frag<T> a;
+                    #pragma unroll
+                    for (int e = 0; e < 8; e++) {
+                        const int key = k + g * 8 + e;
+                        if constexpr (KT >= 32)
+                            frag_set(a, e, ldf(c_s + key * cs + col));
+                        else
+                            frag_set(a, e, key < KT
+                                     ? ldf(c_s + key * cs + col) : 0.f);
+                    }
+                    #pragma unroll
+                    for (int mt = 0; mt < MT; mt++) {
+                        const T* br = p_s + (mt * 16 + lr) * PS + k + g * 8;
+                        Frag<T> b;
+                        if (KT >= 32 || g < 2) b = frag8(br);
+                        else b = frag_zero<T>();
+                        acc[mt][n] = mma(a, b, acc[mt][n]);
+                    }
+                }
+            }
+        }
+        __syncthreads();
+    }
+
+    #pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const int row = mt * 16 + lr;
+        if (row >= n_rows) continue;
+        const int64_t gr = row0 + row;
+        const float l = l_s[row];
+        const float inv = split > 1 ? 1.f : (l > 0.f ? 1.f / l : 0.f);
+        #pragma unroll
+        for (int n = 0; n < NT; n++) {
+            const int c0 = (n * 4 + wid) * 16 + g * 4;
+            #pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (c0 + i < R) {
+                    const float v = acc[mt][n][i] * inv;
+                    if (split > 1)
+                        o_part[((int64_t)blockIdx.y * rows_total + gr) * R
+                               + c0 + i] = v;
+                    else stf(out + gr * R + c0 + i, v);
+                }
+        }
+        if (split > 1 && wid == 0 && g == 0) {
+            float* d = ml_part
+                + ((int64_t)blockIdx.y * rows_total + gr) * 2;
+            d[0] = m_s[row];
+            d[1] = l;
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(128) void k_latent_combine(
+    T* __restrict__ out, const float* __restrict__ o_part,
+    const float* __restrict__ ml, int64_t row_base, int64_t rows_total,
+    int R, int split)
+{
+    const int64_t row = row_base + blockIdx.x;
+    float m = NEG;
+    for (int s = 0; s < split; s++)
+        m = fmaxf(m, ml[(s * rows_total + row) * 2]);
+    float l = 0.f;
+    for (int s = 0; s < split; s++) {
+        const float* d = ml + (s * rows_total + row) * 2;
+        l += d[1] * exp_of<T>(d[0] - m);
+    }
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+    for (int i = threadIdx.x; i < R; i += 128) {
+        float v = 0.f;
+        for (int s = 0; s < split; s++)
+            v += o_part[(s * rows_total + row) * R + i]
+                 * exp_of<T>(ml[(s * rows_total + row) * 2] - m);
+        stf(out + row * R + i, v * inv);
+    }
+}
+
+static int latent_lds(int M, int KT, int R, int esz)
+{
+    const int cs = ((R + 31) & ~31) + 16 / esz;
+    return (M + KT) * cs * esz + M * (KT + 16 / esz) * esz
+           + M * (KT + 4) * 4 + 4 * M * 4;
+}
+
+template <typename T, int MT, int KT, int NT>
+static int latent_go(
+    void* out, void* op, void* mp, const void* q, const void* pool,
+    const void* ptab, const void* slot, const void* pos, const void* items,
+    int n_items, int per_seq, int H, int R, int psz, int maxp, float scale,
+    int64_t rows_total, int split, hipStream_t stream)
+{
+    const int lds = latent_lds(16 * MT, KT, R, sizeof(T));
+    static bool once = false;
+    if (!once) {
+        (void)hipFuncSetAttribute(
+            (const void*)k_latent_attn<T, MT, KT, NT>,
+            hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        once = true;
+    }
+    k_latent_attn<T, MT, KT, NT><<<dim3(n_items, split), 256, lds, stream>>>(
+        (T*)out, (float*)op, (float*)mp, (const T*)q, (const T*)pool,
+        (const int*)ptab, (const int*)slot, (const int*)pos,
+        (const int*)items, per_seq, H, R, psz, maxp, scale, rows_total,
+        split);
+    return (int)hipGetLastError();
+}
+
+// rows of an item: 16 * latent_mt(f32, H, R)
+extern "C" int latent_mt(int f32, int H, int R)
+{
+    const int esz = f32 ? 4 : 2;
+    if (H > 16 && latent_lds(32, 32, R, esz) <= 160 * 1024 && R <= 512)
+        return 2;
+    return 1;
+}
+
+// items: int32 [n_items, 2] (first row, rows <= 16 * latent_mt), each within
+// one sequence; null with per_seq = ceil(H / rows) for a decode batch.
+extern "C" int latent_attn(
+    int f32, void* out, void* o_part, void* ml_part, const void* q,
+    const void* pool, const void* ptab, const void* slot, const void* pos,
+    const void* items, int n_items, int per_seq, int H, int R, int psz,
+    int maxp, float scale, int64_t rows_total, int64_t row_base,
+    int64_t rows_here, int split, hipStream_t stream)
+{
+    const int esz = f32 ? 4 : 2;
+    const int mt = latent_mt(f32, H, R);
+    const int budget = 80 * 1024;            // two blocks a CU if possible
+    int kt = 64;
+    if (latent_lds(16 * mt, 64, R, esz) > budget) kt = 32;
+    if (latent_lds(16 * mt, kt, R, esz) > 160 * 1024) kt = 16;
+    if (latent_lds(16 * mt, kt, R, esz) > 160 * 1024 || R > 1024)
+        return (int)hipErrorInvalidValue;
+    int err = (int)hipErrorInvalidValue;
+    #define LA(T, M, K, N)                                                 \
+        err = latent_go<T, M, K, N>(                                       \
+            out, o_part, ml_part, q, pool, ptab, slot, pos, items,         \
+            n_items, per_seq, H, R, psz, maxp, scale, rows_total, split,   \
+            stream)
+    #define LA_N(T, M, K)                                                  \
+        do {                                                               \
+            if (R <= 128) LA(T, M, K, 2);                                  \
+            else if (R <= 512) LA(T, M, K, 8);                             \
+            else LA(T, 1, K, 16);                                          \
+        } while (0)
+    #define LA_K(T, M)                                                     \
+        do {                                                               \
+            if (kt == 64) LA_N(T, M, 64);                                  \
+            else if (kt == 32) LA_N(T, M, 32);                             \
+            else LA_N(T, M, 16);                                           \
+        } while (0)
+    #define LA_T(T)                                                        \
+        do { if (mt == 2) LA_K(T, 2); else LA_K(T, 1); } while (0)
+    if (f32) LA_T(float); else LA_T(bf16);
+    #undef LA_T
+    #undef LA_K
+    #undef LA_N
+    #undef LA
+    if (err || split == 1) return err;
+    if (f32)
+        k_latent_combine<float><<<(int)rows_here, 128, 0, stream>>>(
+            (float*)out, (const float*)o_part, (const float*)ml_part,
+            row_base, rows_total, R, split);
+    else
+        k_latent_combine<bf16><<<(int)rows_here, 128, 0, stream>>>(
+            (bf16*)out, (const float*)o_part, (const float*)ml_part,
+            row_base, rows_total, R, split);
+    return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// Causal flash attention with free key width (<= 32*DT) and value width
+// (<= 16*VT), contiguous keys [kv, H, D] and TRANSPOSED values [H, V, kv]
+// (the caller's matrix product writes them that way).
+//
+// Block: four waves of NQ 16-query tiles.  S^T = K Q^T puts a query on a
+// lane, so its softmax state is two scalars after two cross-lane steps; P
+// never leaves registers: the PV product may take keys in any order as long
+// as both operands agree, so V^T fragments are read in the order in which
+// the lanes already hold P.
+// ---------------------------------------------------------------------------
+template <typename T, int DT, int VT, int NQ>
+__global__ __launch_bounds__(256) void k_flash(
+    T* __restrict__ out,               // [T, H, V]
+    const T* __restrict__ q,           // [T, ..] row stride qs, head h at h*D
+    const T* __restrict__ k,           // [kv, H*D]
+    const T* __restrict__ vt,          // [H*V, kv_ld]
+    const int* __restrict__ tiles,     // [n, 4] q row, pos, rows, kv offset
+    int H, int D, int V, int64_t qs, int64_t kv_ld, float scale)
+{
+    constexpr int KT = 64;
+    constexpr int PAD = 16 / sizeof(T);
+    constexpr int KS = DT * 32 + PAD, VS = KT + PAD;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    const int h = blockIdx.x;
+    const int* tl = tiles + (int64_t)(gridDim.y - 1 - blockIdx.y) * 4;
+    const int q0 = tl[0], pos0 = tl[1], rows = tl[2];
+    const int64_t kv0 = tl[3];
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    T* k_s = reinterpret_cast<T*>(smem);          // [KT][KS]
+    T* v_s = k_s + KT * KS;                       // [VT*16][VS]
+
+    const bool vec = D % 8 == 0 && qs % 8 == 0;
+    Frag<T> qf[NQ][DT];
+    int qpos[NQ];
+    #pragma unroll
+    for (int n = 0; n < NQ; n++) {
+        const int r = (wid * NQ + n) * 16 + lr;
+        qpos[n] = pos0 + r;
+        const T* qr = q + (int64_t)(q0 + min(r, rows - 1)) * qs
+                      + (int64_t)h * D;
+        #pragma unroll
+        for (int d = 0; d < DT; d++) {
+            const int c = d * 32 + g * 8;
+            if (vec) qf[n][d] = c < D ? frag8(qr + c) : frag_zero<T>();
+            else qf[n][d] = frag_guard(qr, c, D);
+        }
+    }
+    const T* kh = k + kv0 * H * D + (int64_t)h * D;
+    const T* vh = vt + (int64_t)h * V * kv_ld + kv0;
+    const int kv_len = pos0 + rows;
+    const int n_chunks = (kv_len + KT - 1) / KT;
+
+    constexpr int NK = DT;                        // 8-element pieces a thread
+    constexpr int NV = VT / 2;
+    Frag<T> kp[NK], vp[NV];
+    auto load = [&](int base) {
+        #pragma unroll
+        for (int j = 0; j < NK; j++) {
+            const int u = tid + j * 256;
+            const int key = u / (DT * 4), c = (u % (DT * 4)) * 8;
+            const T* src = kh + (int64_t)(base + key) * H * D;
+            if (vec) kp[j] = c < D ? frag8(src + c) : frag_zero<T>();
+            else kp[j] = frag_guard(src, c, D);
+        }
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int u = tid + j * 256;
+            const int v = u >> 3, c = (u & 7) * 8;
+            vp[j] = v < V ? frag8(vh + (int64_t)v * kv_ld + base + c)
+                          : frag_zero<T>();
+        }
+    };
+    auto store = [&]() {
+        #pragma unroll
+        for (int j = 0; j < NK; j++) {
+            const int u = tid + j * 256;
+            *reinterpret_cast<Frag<T>*>(
+                k_s + (u / (DT * 4)) * KS + (u % (DT * 4)) * 8) = kp[j];
+        }
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int u = tid + j * 256;
+            *reinterpret_cast<Frag<T>*>(v_s + (u >> 3) * VS + (u & 7) * 8)
+                = vp[j];
+        }
+    };
+
+    float m[NQ], l[NQ];
+    f32x4 o[NQ][VT] = {};
+    #pragma unroll
+    for (int n = 0; n < NQ; n++) { m[n] = NEG; l[n] = 0.f; }
+
+    load(0);
+    for (int ch = 0; ch < n_chunks; ++ch) {
+        const int base = ch * KT;
+        store();
+        __syncthreads();
+        if (ch + 1 < n_chunks) load(base + KT);
+        f32x4 s[NQ][4] = {};
+        #pragma unroll
+        for (int kt = 0; kt < 4; kt++) {
+            const T* ar = k_s + (kt * 16 + lr) * KS + g * 8;
+            #pragma unroll
+            for (int d = 0; d < DT; d++) {
+                const Frag<T> a = frag8(ar + d * 32);
+                #pragma unroll
+                for (int n = 0; n < NQ; n++)
+                    s[n][kt] = mma(a, qf[n][d], s[n][kt]);
+            }
+        }
+        const bool edge = base + KT > pos0 + 1;   // some query sees less
+        #pragma unroll
+        for (int n = 0; n < NQ; n++) {
+            float mx = NEG;
+            #pragma unroll
+            for (int kt = 0; kt < 4; kt++)
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    float v = s[n][kt][i] * scale;
+                    if (edge && base + kt * 16 + g * 4 + i > qpos[n])
+                        v = NEG;
+                    s[n][kt][i] = v;
+                    mx = fmaxf(mx, v);
+                }
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            // key 0 is visible to every query, so the maximum is finite
+            // from the first chunk on and masked scores give exp() == 0
+            const float mn = fmaxf(m[n], mx);
+            const float f = exp_of<T>(m[n] - mn);
+            float sum = 0.f;
+            #pragma unroll
+            for (int kt = 0; kt < 4; kt++)
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const float p = exp_of<T>(s[n][kt][i] - mn);
+                    s[n][kt][i] = p;
+                    sum += p;
+                }
+            sum += __shfl_xor(sum, 16, 64);
+            sum += __shfl_xor(sum, 32, 64);
+            l[n] = l[n] * f + sum;
+            m[n] = mn;
+            #pragma unroll
+            for (int v = 0; v < VT; v++) o[n][v] *= f;
+        }
+        #pragma unroll
+        for (int kp2 = 0; kp2 < 2; kp2++) {
+            Frag<T> b[NQ];
+            #pragma unroll
+            for (int n = 0; n < NQ; n++)
+                #pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    frag_set(b[n], e, s[n][kp2 * 2][e]);
+                    frag_set(b[n], e + 4, s[n][kp2 * 2 + 1][e]);
+                }
+            #pragma unroll
+            for (int v = 0; v < VT; v++) {
+                const T* ar = v_s + (v * 16 + lr) * VS + kp2 * 32 + g * 4;
+                const Frag<T> a = frag44(ar, ar + 16);
+                #pragma unroll
+                for (int n = 0; n < NQ; n++) o[n][v] = mma(a, b[n], o[n][v]);
+            }
+        }
+        __syncthreads();
+    }
+    #pragma unroll
+    for (int n = 0; n < NQ; n++) {
+        const int r = (wid * NQ + n) * 16 + lr;
+        if (r >= rows) continue;
+        const float inv = 1.f / l[n];
+        T* orow = out + ((int64_t)(q0 + r) * H + h) * V;
+        #pragma unroll
+        for (int v = 0; v < VT; v++) {
+            const int c = v * 16 + g * 4;
+            if (V % 4 == 0) {
+                if (c < V) {
+                    float w[4];
+                    #pragma unroll
+                    for (int i = 0; i < 4; i++) w[i] = o[n][v][i] * inv;
+                    stv<4>(orow + c, w);
+                }
+            } else
+                #pragma unroll
+                for (int i = 0; i < 4; i++)
+                    if (c + i < V) stf(orow + c + i, o[n][v][i] * inv);
+        }
+    }
+}
+
+template <typename T, int DT, int VT, int NQ>
+static int flash_go(void* out, const void* q, const void* k, const void* vt,
+                    const void* tiles, int n_tiles, int H, int D, int V,
+                    int64_t qs, int64_t kv_ld, float scale,
+                    hipStream_t stream)
+{
+    const int pad = 16 / sizeof(T);
+    const int lds = (64 * (DT * 32 + pad) + VT * 16 * (64 + pad))
+                    * (int)sizeof(T);
+    static bool once = false;
+    if (!once) {
+        (void)hipFuncSetAttribute(
+            (const void*)k_flash<T, DT, VT, NQ>,
+            hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        once = true;
+    }
+    k_flash<T, DT, VT, NQ><<<dim3(H, n_tiles), 256, lds, stream>>>(
+        (T*)out, (const T*)q, (const T*)k, (const T*)vt, (const int*)tiles,
+        H, D, V, qs, kv_ld, scale);
+    return (int)hipGetLastError();
+}
+
+// queries per tile; tiles: int32 [n, 4] (first q row, its position, rows,
+// first row of the sequence in k / vt); k and vt hold every sequence padded
+// to a multiple of 64 positions; D, V <= 256
+extern "C" int flash_rows(int f32) { return f32 ? 64 : 128; }
+
+extern "C" int flash_attn(
+    int f32, void* out, const void* q, const void* k, const void* vt,
+    const void* tiles, int n_tiles, int H, int D, int V, int64_t qs,
+    int64_t kv_ld, float scale, hipStream_t stream)
+{
+    if (D > 256 || V > 256) return (int)hipErrorInvalidValue;
+    int err;
+    #define FA(T, D_, V_, Q)                                               \
+        err = flash_go<T, D_, V_, Q>(out, q, k, vt, tiles, n_tiles, H, D,  \
+                                     V, qs, kv_ld, scale, stream)
+    #define FA_V(T, D_, Q)                                                 \
+        do {                                                               \
+            if (V <= 64) FA(T, D_, 4, Q);                                  \
+            else if (V <= 128) FA(T, D_, 8, Q);                            \
+            else FA(T, D_, 16, Q);                                         \
+        } while (0)
+    #define FA_D(T, Q)                                                     \
+        do {                                                               \
+            if (D <= 64) FA_V(T, 2, Q);                                    \
+            else if (D <= 128) FA_V(T, 4, Q);                              \
+            else FA_V(T, 8, Q);                                            \
+        } while (0)
+    if (f32) FA_D(float, 1); else FA_D(bf16, 2);
+    #undef FA_D
+    #undef FA_V
+    #undef FA
+    return err;
+}
+
+// Gather of several sequences' latents, 64 positions a block: groups
+// int32 [n, 3] (slot, first position, rows that exist); the rest is zero.
+template <typename T>
+__global__ __launch_bounds__(256) void k_latent_gather_groups(
+    T* __restrict__ out, const T* __restrict__ pool,
+    const int* __restrict__ ptab, const int* __restrict__ groups,
+    int R, int psz, int maxp)
+{
+    const int* gp = groups + (int64_t)blockIdx.x * 3;
+    const int* row = ptab + (int64_t)gp[0] * maxp;
+    const int base = gp[1], have = gp[2];
+    const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    for (int j = wid; j < 64; j += 4) {
+        T* dst = out + ((int64_t)blockIdx.x * 64 + j) * R;
+        if (j >= have) {
+            for (int i = lane; i < R; i += 64) stf(dst + i, 0.f);
+            continue;
+        }
+        const int p = base + j;
+        const T* src = pool + ((int64_t)row[p / psz] * psz + p % psz) * R;
+        if (R % 8 == 0)
+            for (int i = lane * 8; i < R; i += 512)
+                *reinterpret_cast<Frag<T>*>(dst + i) = frag8(src + i);
+        else
+            for (int i = lane; i < R; i += 64) dst[i] = src[i];
+    }
+}
+
+extern "C" int latent_gather(
+    int f32, void* out, const void* pool, const void* ptab,
+    const void* groups, int n, int R, int psz, int maxp, hipStream_t stream)
+{
+    if (f32)
+        k_latent_gather_groups<float><<<n, 256, 0, stream>>>(
+            (float*)out, (const float*)pool, (const int*)ptab,
+            (const int*)groups, R, psz, maxp);
+    else
+        k_latent_gather_groups<bf16><<<n, 256, 0, stream>>>(
+            (bf16*)out, (const bf16*)pool, (const int*)ptab,
+            (const int*)groups, R, psz, maxp);
+    return (int)hipGetLastError();
+}

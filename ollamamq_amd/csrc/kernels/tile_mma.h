@@ -1,0 +1,143 @@
+// Shared pieces of the kernels that run in bf16 and in true fp32: typed
+// loads and stores, wave reductions, and a 16x16 matrix-core tile whose
+// fragments look the same for both types.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <hip/hip_bf16.h>
+#include <cstdint>
+
+typedef __hip_bfloat16 bf16;
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4;
+typedef __attribute__((ext_vector_type(4))) float f32x4;
+
+#define DEV static __device__ __forceinline__
+
+DEV float ldf(const float* p) { return *p; }
+DEV float ldf(const bf16* p) { return __bfloat162float(*p); }
+DEV void stf(float* p, float v) { *p = v; }
+DEV void stf(bf16* p, float v) { *p = __float2bfloat16(v); }
+
+// VEC consecutive elements as floats; VEC is 1, 4 or 8 and the address is
+// aligned to VEC elements
+template <int VEC>
+DEV void ldv(const float* p, float* o) {
+    if constexpr (VEC == 1) o[0] = *p;
+    else {
+        #pragma unroll
+        for (int i = 0; i < VEC; i += 4) {
+            const f32x4 v = *reinterpret_cast<const f32x4*>(p + i);
+            o[i] = v[0]; o[i + 1] = v[1]; o[i + 2] = v[2]; o[i + 3] = v[3];
+        }
+    }
+}
+template <int VEC>
+DEV void ldv(const bf16* p, float* o) {
+    if constexpr (VEC == 1) o[0] = __bfloat162float(*p);
+    else if constexpr (VEC == 4) {
+        const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+        #pragma unroll
+        for (int i = 0; i < 4; i++) o[i] = (float)v[i];
+    } else {
+        const bf16x8 v = *reinterpret_cast<const bf16x8*>(p);
+        #pragma unroll
+        for (int i = 0; i < 8; i++) o[i] = (float)v[i];
+    }
+}
+template <int VEC>
+DEV void stv(float* p, const float* o) {
+    if constexpr (VEC == 1) *p = o[0];
+    else {
+        #pragma unroll
+        for (int i = 0; i < VEC; i += 4)
+            *reinterpret_cast<f32x4*>(p + i) =
+                f32x4{o[i], o[i + 1], o[i + 2], o[i + 3]};
+    }
+}
+template <int VEC>
+DEV void stv(bf16* p, const float* o) {
+    if constexpr (VEC == 1) *p = __float2bfloat16(o[0]);
+    else if constexpr (VEC == 4) {
+        bf16x4 v;
+        #pragma unroll
+        for (int i = 0; i < 4; i++) v[i] = (__bf16)o[i];
+        *reinterpret_cast<bf16x4*>(p) = v;
+    } else {
+        bf16x8 v;
+        #pragma unroll
+        for (int i = 0; i < 8; i++) v[i] = (__bf16)o[i];
+        *reinterpret_cast<bf16x8*>(p) = v;
+    }
+}
+
+DEV float wave_sum(float x) {
+    #pragma unroll
+    for (int o = 32; o; o >>= 1) x += __shfl_xor(x, o, 64);
+    return x;
+}
+DEV float wave_max(float x) {
+    #pragma unroll
+    for (int o = 32; o; o >>= 1) x = fmaxf(x, __shfl_xor(x, o, 64));
+    return x;
+}
+
+// ---- 16x16 tile, 32 deep -------------------------------------------------
+// A lane holds 8 elements of one row (A) or column (B): row/col = lane & 15,
+// k = (lane >> 4) * 8 + e.  bf16 is one mfma_16x16x32; fp32 is eight
+// mfma_16x16x4, one per element e: each takes k = {(lane >> 4) * 8 + e},
+// and over all e the 32 k's are covered once.  Any other assignment of k to
+// (lane group, e) gives the same product as long as A and B share it.
+// The result: col = lane & 15, row = (lane >> 4) * 4 + i.
+template <typename T> struct FragOf;
+template <> struct FragOf<bf16> { typedef bf16x8 type; };
+struct f32x8s { f32x4 lo, hi; };
+template <> struct FragOf<float> { typedef f32x8s type; };
+template <typename T> using Frag = typename FragOf<T>::type;
+
+DEV f32x4 mma(bf16x8 a, bf16x8 b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+DEV f32x4 mma(const f32x8s& a, const f32x8s& b, f32x4 c) {
+    #pragma unroll
+    for (int e = 0; e < 4; e++)
+        c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.lo[e], b.lo[e], c, 0, 0, 0);
+    #pragma unroll
+    for (int e = 0; e < 4; e++)
+        c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.hi[e], b.hi[e], c, 0, 0, 0);
+    return c;
+}
+
+DEV bf16x8 frag8(const bf16* p) { return *reinterpret_cast<const bf16x8*>(p); }
+DEV f32x8s frag8(const float* p) {
+    return {*reinterpret_cast<const f32x4*>(p),
+            *reinterpret_cast<const f32x4*>(p + 4)};
+}
+// two runs of four
+DEV bf16x8 frag44(const bf16* p, const bf16* q) {
+    const bf16x4 a = *reinterpret_cast<const bf16x4*>(p);
+    const bf16x4 b = *reinterpret_cast<const bf16x4*>(q);
+    return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+}
+DEV f32x8s frag44(const float* p, const float* q) {
+    return {*reinterpret_cast<const f32x4*>(p),
+            *reinterpret_cast<const f32x4*>(q)};
+}
+DEV void frag_set(bf16x8& f, int e, float v) { f[e] = (__bf16)v; }
+DEV void frag_set(f32x8s& f, int e, float v) {
+    if (e < 4) f.lo[e] = v; else f.hi[e - 4] = v;
+}
+// elements e with k0 + e < K; the rest are zero
+template <typename T>
+DEV Frag<T> frag_guard(const T* p, int k0, int K) {
+    Frag<T> f;
+    #pragma unroll
+    for (int e = 0; e < 8; e++)
+        frag_set(f, e, k0 + e < K ? ldf(p + k0 + e) : 0.f);
+    return f;
+}
+template <typename T> DEV Frag<T> frag_zero() {
+    Frag<T> f;
+    #pragma unroll
+    for (int e = 0; e < 8; e++) frag_set(f, e, 0.f);
+    return f;
+}

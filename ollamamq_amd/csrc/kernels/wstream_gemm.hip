@@ -625,6 +625,7 @@ __global__ __launch_bounds__(256) void k_wstream_combine_tiles(
     }
 }
 
+// y == null with ksplit > 1: the partial sums are the result
 extern "C" int wstream_gemm_bf16(
     void* y, void* part, const void* x, const void* wp, const void* bias,
     int M, int N, int K, int64_t xs, int ksplit, int depth, int xlds,
@@ -678,7 +679,7 @@ extern "C" int wstream_gemm_bf16(
                 (const bf16*)bias, M, N, K, xs, ksplit, nullptr, 0,
                 0.f, 0.f, nullptr, nullptr);
     }
-    if (ksplit > 1) {
+    if (ksplit > 1 && y != nullptr) {
         if (res_in || sq_parts) {
             k_wstream_combine_tiles<<<N / 32, 256, 0, stream>>>(
                 (bf16*)y, (const float*)part, (const bf16*)res_in,

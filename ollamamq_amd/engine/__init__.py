@@ -1,4 +1,5 @@
-from .kvcache import PagedKVCache
+from .kvcache import HybridCache, PagedKVCache, cache_for_model
 from .engine import LlamaEngine, Sequence, GenParams
 
-__all__ = ["PagedKVCache", "LlamaEngine", "Sequence", "GenParams"]
+__all__ = ["HybridCache", "PagedKVCache", "cache_for_model", "LlamaEngine",
+           "Sequence", "GenParams"]

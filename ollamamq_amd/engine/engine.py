@@ -217,6 +217,56 @@ class LlamaEngine:
         finally:
             self.kv.free_slot(slot)
 
+    # -- given tokens --------------------------------------------------------
+    def open_stream(self) -> Sequence:
+        """A sequence that is fed given tokens instead of generating."""
+        seq = Sequence(next(self._ids), [], GenParams())
+        seq.slot = self.kv.alloc_slot()
+        seq.state = "stream"
+        return seq
+
+    def close_stream(self, seq: Sequence) -> None:
+        if seq.slot >= 0:
+            self.kv.free_slot(seq.slot)
+            seq.slot, seq.state = -1, "done"
+
+    def feed(self, parts) -> torch.Tensor:
+        """Advance streams by given tokens in one batch: parts is a list of
+        (stream, tokens, wanted places among them).  Returns the logits at
+        the wanted places, in that order.  The batch runs as generation runs
+        it: single tokens take the (captured) decode step, portions of
+        prompts share one forward with them."""
+        vocab = self.model.cfg.vocab
+        for s, toks, want in parts:
+            if not toks or min(toks) < 0 or max(toks) >= vocab:
+                raise ValueError("a part needs tokens of the vocabulary")
+            if any(not 0 <= w < len(toks) for w in want):
+                raise ValueError("a wanted place is outside its tokens")
+        order = sorted(range(len(parts)), key=lambda i: len(parts[i][1]))
+        seqs = [parts[i][0] for i in order]
+        q_lens = [len(parts[i][1]) for i in order]
+        tokens = [t for i in order for t in parts[i][1]]
+        pos, first, at = [], {}, 0
+        for i, s, n in zip(order, seqs, q_lens):
+            done = self.kv.seq_lens[s.slot]
+            pos.extend(range(done, done + n))
+            first[i] = at
+            at += n
+        rows = [first[i] + w for i, p in enumerate(parts) for w in p[2]]
+        nd = sum(n == 1 for n in q_lens)
+        if nd == len(parts):
+            if self.use_graphs and nd <= self.max_batch:
+                for s in seqs:
+                    self.kv.ensure(s.slot, self.kv.seq_lens[s.slot] + 1)
+                logits = self._decode_forward_graphed(seqs, tokens, pos)
+            else:
+                logits = self._forward(seqs, tokens, pos, q_lens, "decode")
+            return logits[rows]
+        logits = self._forward(seqs, tokens, pos, q_lens,
+                               "mixed" if nd else "prefill", n_decode=nd,
+                               rows=rows or [at - 1])
+        return logits[:len(rows)]
+
     # -- internals ---------------------------------------------------------
     def _reap_cancelled(self):
         if any(s.cancelled for s in self.running):
@@ -305,7 +355,8 @@ class LlamaEngine:
                 if s.on_token:
                     s.on_token(int(tok), False)
 
-    def _build_meta(self, seqs, q_lens, mode, n_decode=0) -> AttnMeta:
+    def _build_meta(self, seqs, q_lens, mode, n_decode=0,
+                    rows=None) -> AttnMeta:
         dev = self.dev
         slot_ids = torch.tensor([s.slot for s in seqs], dtype=torch.int32,
                                 device=dev)
@@ -315,18 +366,23 @@ class LlamaEngine:
         for ql in q_lens:
             cu.append(cu[-1] + ql)
         cu_q = torch.tensor(cu, dtype=torch.int32, device=dev)
-        logits_idx = torch.tensor([c - 1 for c in cu[1:]], dtype=torch.long,
-                                  device=dev)
+        # default: every sequence's last token
+        logits_idx = torch.tensor(
+            [c - 1 for c in cu[1:]] if rows is None else rows,
+            dtype=torch.long, device=dev)
         return AttnMeta(
             mode=mode, slot_ids=slot_ids, seq_lens=seq_lens, cu_q=cu_q,
             logits_idx=logits_idx, max_q=max(q_lens),
             max_kv=int(max(self.kv.seq_lens[s.slot] for s in seqs)),
             n_decode=n_decode,
             window=getattr(self.model.cfg, "sliding_window", 0),
+            q_lens=list(q_lens),
+            kv_lens=[self.kv.seq_lens[s.slot] for s in seqs],
+            slots=[s.slot for s in seqs],
         )
 
     def _forward(self, seqs, token_list, pos_list, q_lens, mode,
-                 n_decode=0):
+                 n_decode=0, rows=None):
         dev = self.dev
         tokens = torch.tensor(token_list, dtype=torch.int32, device=dev)
         positions = torch.tensor(pos_list, dtype=torch.int32, device=dev)
@@ -335,7 +391,7 @@ class LlamaEngine:
             dtype=torch.int32, device=dev)
         for s, ql in zip(seqs, q_lens):
             self.kv.ensure(s.slot, self.kv.seq_lens[s.slot] + ql)
-        meta = self._build_meta(seqs, q_lens, mode, n_decode)
+        meta = self._build_meta(seqs, q_lens, mode, n_decode, rows)
         logits = self.model.forward(tokens, positions, self.kv, slot_per_tok,
                                     meta)
         return logits
@@ -430,6 +486,8 @@ class LlamaEngine:
         return self._buckets[-1]
 
     def _ensure_dummy(self) -> int:
+        if self.kv.scratch_slot is not None:
+            return self.kv.scratch_slot
         if self._dummy_slot < 0:
             self._dummy_slot = self.kv.alloc_slot()
             self.kv.ensure(self._dummy_slot, 1)
@@ -524,6 +582,14 @@ class LlamaEngine:
             # GPU suite) — flush pending frees first, then hold GC off.
             import gc
             gc.collect()
+            # the warmups really run: with recurrent state they must not
+            # advance the batch's sequences, so they work on the scratch slot
+            live = {}
+            if self.kv.scratch_slot is not None:
+                live = {k: bufs[k].clone() for k in ("slot", "pos", "lens")}
+                bufs["slot"].fill_(self.kv.scratch_slot)
+                bufs["pos"].zero_()
+                bufs["lens"].fill_(1)
             s = torch.cuda.Stream()
             s.wait_stream(torch.cuda.current_stream())
             with torch.cuda.stream(s):
@@ -534,6 +600,8 @@ class LlamaEngine:
                     # eager tail warmup — see _graph_tail docstring
                     self._graph_tail(entry, warm_logits)
             torch.cuda.current_stream().wait_stream(s)
+            for k, v in live.items():
+                bufs[k].copy_(v)
             torch.cuda.synchronize()
             gc.disable()
             try:

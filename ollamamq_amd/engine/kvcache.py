@@ -1,57 +1,53 @@
-"""Paged KV cache sized for 288 GB HBM3E per MI355X.
+"""Sequence memory sized for 288 GB HBM3E per MI355X: paged caches for
+attention and per-slot state for recurrent layers.
 
-Layout [L, n_pages, KVH, page_size, D]: one (page, kv-head) is a contiguous
-page_size*D*2B run (4 KiB at page=16, D=128), the unit the decode-attention
-kernel streams with wide vector loads.  Page tables are int32 per slot.
+SequenceCache owns what every model needs: sequence slots, the page pool's
+free list and the int32 page table per slot.  Its subclasses add storage:
+
+* PagedKVCache, layout [L, n_pages, KVH, page_size, D]: one (page, kv-head)
+  is a contiguous page_size*D*2B run (4 KiB at page=16, D=128), the unit the
+  decode-attention kernel streams with wide vector loads;
+* HybridCache: one store per layer run of a model that mixes mechanisms --
+  a paged pool with one latent row per token, and fp32 state per slot.
 
 The reference has no KV concept (its context handling is only plumbing the
 `num_ctx` option to Ollama, reference src/control.rs:804-806); the paged pool
-is this framework's realization of "model loaded with context N" — "load"
-allocates weights + this pool in HBM, "unload" frees them (SURVEY.md §2 C14).
+is this framework's realization of "model loaded with context N" -- "load"
+allocates weights + this pool in HBM, "unload" frees them.
 """
 from __future__ import annotations
 
-from typing import List
+from dataclasses import dataclass
+from typing import List, Optional, Tuple
 
 import torch
 
 
-class PagedKVCache:
-    def __init__(
-        self,
-        n_layers: int,
-        n_kv_heads: int,
-        head_dim: int,
-        page_size: int = 16,
-        n_pages: int = 1024,
-        max_slots: int = 64,
-        max_ctx: int = 8192,
-        device: str = "cpu",
-        dtype: torch.dtype = torch.float32,
-    ):
+class SequenceCache:
+    """Slots and pages.  `scratch` adds one slot row and one page that no
+    sequence ever gets: work that must not touch live state (graph warmups,
+    batch padding) runs there."""
+
+    scratch_slot: Optional[int] = None
+
+    def __init__(self, page_size: int, n_pages: int, max_slots: int,
+                 max_ctx: int, dev: torch.device, scratch: bool = False):
         self.page_size = page_size
-        self.head_dim = head_dim
-        self.n_kv_heads = n_kv_heads
         self.max_ctx = max_ctx
-        dev = torch.device(device)
-        shape = (n_layers, n_pages, n_kv_heads, page_size, head_dim)
-        self.k_pool = torch.zeros(shape, device=dev, dtype=dtype)
-        self.v_pool = torch.zeros(shape, device=dev, dtype=dtype)
         max_pages = (max_ctx + page_size - 1) // page_size
         self.page_table = torch.zeros(
-            (max_slots, max_pages), device=dev, dtype=torch.int32
+            (max_slots + scratch, max_pages), device=dev, dtype=torch.int32
         )
+        if scratch:
+            self.scratch_slot = max_slots
+            self.page_table[max_slots].fill_(n_pages)
         self._free_pages: List[int] = list(range(n_pages - 1, -1, -1))
         self._free_slots: List[int] = list(range(max_slots - 1, -1, -1))
         self._slot_pages: List[List[int]] = [[] for _ in range(max_slots)]
-        self.seq_lens = [0] * max_slots  # host-side truth
+        # host-side truth
+        self.seq_lens = [0] * (max_slots + scratch)
         self.max_slots = max_slots
         self.n_pages = n_pages
-
-    @classmethod
-    def for_model(cls, cfg, tp_size=1, **kw):
-        n_kv = max(1, cfg.n_kv_heads // tp_size)
-        return cls(cfg.n_layers, n_kv, cfg.head_dim, **kw)
 
     def free_page_count(self) -> int:
         return len(self._free_pages)
@@ -75,13 +71,93 @@ class PagedKVCache:
             raise RuntimeError(f"sequence exceeds max_ctx {self.max_ctx}")
         need = (new_len + self.page_size - 1) // self.page_size
         pages = self._slot_pages[slot]
+        had = len(pages)
+        if need - had > len(self._free_pages):
+            raise RuntimeError("KV cache: out of pages")
         while len(pages) < need:
-            if not self._free_pages:
-                raise RuntimeError("KV cache: out of pages")
-            p = self._free_pages.pop()
-            self.page_table[slot, len(pages)] = p
-            pages.append(p)
+            pages.append(self._free_pages.pop())
+        if need == had + 1:
+            self.page_table[slot, had] = pages[had]
+        elif need > had:
+            self.page_table[slot, had:need] = torch.tensor(
+                pages[had:], dtype=torch.int32)
         self.seq_lens[slot] = new_len
 
     def can_fit(self, extra_tokens: int) -> bool:
         return len(self._free_pages) * self.page_size >= extra_tokens
+
+
+class PagedKVCache(SequenceCache):
+    def __init__(
+        self,
+        n_layers: int,
+        n_kv_heads: int,
+        head_dim: int,
+        page_size: int = 16,
+        n_pages: int = 1024,
+        max_slots: int = 64,
+        max_ctx: int = 8192,
+        device: str = "cpu",
+        dtype: torch.dtype = torch.float32,
+    ):
+        dev = torch.device(device)
+        super().__init__(page_size, n_pages, max_slots, max_ctx, dev)
+        self.head_dim = head_dim
+        self.n_kv_heads = n_kv_heads
+        shape = (n_layers, n_pages, n_kv_heads, page_size, head_dim)
+        self.k_pool = torch.zeros(shape, device=dev, dtype=dtype)
+        self.v_pool = torch.zeros(shape, device=dev, dtype=dtype)
+
+    @classmethod
+    def for_model(cls, cfg, tp_size=1, **kw):
+        n_kv = max(1, cfg.n_kv_heads // tp_size)
+        return cls(cfg.n_layers, n_kv, cfg.head_dim, **kw)
+
+
+@dataclass(frozen=True)
+class RunStore:
+    """What one layer run keeps for a sequence: `latent` values per token in
+    the paged pool (0: nothing), and named fp32 tensors of fixed shape."""
+    latent: int = 0
+    state: Tuple[Tuple[str, Tuple[int, ...]], ...] = ()
+
+
+class HybridCache(SequenceCache):
+    """Storage for a model whose config lists a RunStore per layer run.
+
+    Slots are reused without clearing: a layer takes its state as zero
+    wherever a token's position is 0.
+    """
+
+    def __init__(
+        self,
+        stores: List[RunStore],
+        page_size: int = 16,
+        n_pages: int = 1024,
+        max_slots: int = 64,
+        max_ctx: int = 8192,
+        device: str = "cpu",
+        dtype: torch.dtype = torch.float32,
+    ):
+        dev = torch.device(device)
+        super().__init__(page_size, n_pages, max_slots, max_ctx, dev,
+                         scratch=True)
+        self.latent_pool = [
+            torch.zeros((n_pages + 1, page_size, s.latent), device=dev,
+                        dtype=dtype) if s.latent else None for s in stores]
+        self.state = [
+            {name: torch.zeros((max_slots + 1, *shape), device=dev,
+                               dtype=torch.float32)
+             for name, shape in s.state} for s in stores]
+
+    @classmethod
+    def for_model(cls, cfg, tp_size=1, **kw):
+        if tp_size != 1:
+            raise ValueError(f"{cfg.name}: no tensor parallelism")
+        return cls(cfg.run_stores(), **kw)
+
+
+def cache_for_model(cfg, tp_size=1, **kw) -> SequenceCache:
+    """The cache a model's config asks for."""
+    cls = HybridCache if hasattr(cfg, "run_stores") else PagedKVCache
+    return cls.for_model(cfg, tp_size=tp_size, **kw)

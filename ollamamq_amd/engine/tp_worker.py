@@ -38,9 +38,9 @@ import time
 import torch
 import torch.distributed as dist
 
-from ..models import LlamaModel, PRESETS
+from ..models import PRESETS, build_model
 from .engine import GenParams, LlamaEngine
-from .kvcache import PagedKVCache
+from .kvcache import cache_for_model
 from .tokenizer import ByteTokenizer
 from . import worker as worker_mod
 
@@ -73,18 +73,22 @@ class TPWorker(worker_mod.Worker):
         cfg = PRESETS.get(model)
         if cfg is None:
             return f"unknown model: {model}"
-        if cfg.n_heads % self.world or \
-                (cfg.n_kv_heads % self.world and self.world > cfg.n_kv_heads):
+        if self.world > 1 and hasattr(cfg, "run_stores"):
+            return f"model {model} has no tensor-parallel form"
+        if not hasattr(cfg, "run_stores") and (
+                cfg.n_heads % self.world or
+                (cfg.n_kv_heads % self.world
+                 and self.world > cfg.n_kv_heads)):
             return f"model {model} heads not divisible by TP={self.world}"
         ctx = min(num_ctx or self.default_ctx, cfg.max_ctx)
         try:
             if torch.cuda.is_available():
                 torch.cuda.set_device(self.gpu)
-            m = LlamaModel(cfg, device=self.device, dtype=self.dtype,
-                           seed=1234, tp_rank=self.rank, tp_size=self.world,
-                           fast_init=self.device != "cpu")
+            m = build_model(cfg, device=self.device, dtype=self.dtype,
+                            seed=1234, tp_rank=self.rank, tp_size=self.world,
+                            fast_init=self.device != "cpu")
             pages = (self.max_batch + 2) * ((ctx + 15) // 16 + 2)
-            kv = PagedKVCache.for_model(
+            kv = cache_for_model(
                 cfg, tp_size=self.world, n_pages=pages,
                 max_slots=self.max_batch + 2, max_ctx=ctx,
                 device=self.device, dtype=self.dtype)

@@ -34,9 +34,9 @@ from typing import Dict, Optional
 
 import torch
 
-from ..models import LlamaModel, PRESETS
+from ..models import PRESETS, build_model, register_checkpoint
 from .engine import GenParams, LlamaEngine
-from .kvcache import PagedKVCache
+from .kvcache import cache_for_model
 from .tokenizer import ByteTokenizer
 
 VERSION = "0.1.0-ollamamq-amd"
@@ -70,7 +70,9 @@ class Worker:
         if self.model_filter is not None:
             return list(self.model_filter)
         if self.device == "cpu":
-            return ["tiny", "tiny-cpu"]
+            return ["tiny", "tiny-cpu"] + [
+                n for n, c in PRESETS.items()
+                if getattr(c, "checkpoint", None)]
         return [n for n in PRESETS if n != "tiny-cpu"]
 
     def load(self, model: str, num_ctx: int = 0) -> Optional[str]:
@@ -89,10 +91,10 @@ class Worker:
             try:
                 if torch.cuda.is_available():
                     torch.cuda.set_device(self.gpu)
-                m = LlamaModel(cfg, device=self.device, dtype=self.dtype,
-                               seed=1234, fast_init=self.device != "cpu")
+                m = build_model(cfg, device=self.device, dtype=self.dtype,
+                                seed=1234, fast_init=self.device != "cpu")
                 pages = (self.max_batch + 2) * ((ctx + 15) // 16 + 2)
-                kv = PagedKVCache.for_model(
+                kv = cache_for_model(
                     cfg, n_pages=pages, max_slots=self.max_batch + 2,
                     max_ctx=ctx, device=self.device, dtype=self.dtype)
                 eng = LlamaEngine(m, kv, max_batch=self.max_batch)
@@ -570,16 +572,13 @@ class Conn:
             # Ollama tags/ps entry schema (name/model/size/digest/details)
             import hashlib
             cfg = PRESETS.get(m)
-            qd = cfg.n_heads * cfg.head_dim if cfg else 0
-            kvd = cfg.n_kv_heads * cfg.head_dim if cfg else 0
-            size = 2 * (cfg.vocab * cfg.hidden * 2 + cfg.n_layers *
-                        (cfg.hidden * (qd + 2 * kvd) + qd * cfg.hidden +
-                         3 * cfg.hidden * cfg.ffn)) if cfg else 0
+            size = cfg.weight_bytes() if cfg else 0
+            family = cfg.family if cfg else "llama"
             e = {"name": m, "model": m, "size": size,
                  "digest": hashlib.sha256(m.encode()).hexdigest(),
                  "modified_at": _now_iso(),
-                 "details": {"format": "safetensors", "family": "llama",
-                             "families": ["llama"], "parameter_size": m,
+                 "details": {"format": "safetensors", "family": family,
+                             "families": [family], "parameter_size": m,
                              "quantization_level": "BF16"}}
             if res:
                 e["size_vram"] = size
@@ -627,19 +626,14 @@ class Conn:
                 "modelfile": "",
                 "parameters": f"num_ctx {cfg.max_ctx}",
                 "template": "{{ .Prompt }}",
-                "details": {"format": "safetensors", "family": "llama",
-                            "families": ["llama"],
+                "details": {"format": "safetensors", "family": cfg.family,
+                            "families": [cfg.family],
                             "parameter_size": cfg.name,
                             "quantization_level": "BF16"},
                 "model_info": {
-                    "general.architecture": "llama",
-                    "llama.block_count": cfg.n_layers,
-                    "llama.embedding_length": cfg.hidden,
-                    "llama.context_length": cfg.max_ctx,
-                    "llama.feed_forward_length": cfg.ffn,
-                    "llama.attention.head_count": cfg.n_heads,
-                    "llama.attention.head_count_kv": cfg.n_kv_heads,
-                    "llama.vocab_size": cfg.vocab,
+                    "general.architecture": cfg.family,
+                    **{f"{cfg.family}.{k}": v
+                       for k, v in cfg.model_info().items()},
                 },
                 "capabilities": ["completion"],
             }
@@ -676,7 +670,13 @@ def main():
     ap.add_argument("--models", type=str, default=None,
                     help="comma list restricting this worker's advertised "
                          "models (fleet sharding for multi-model routing)")
+    ap.add_argument("--checkpoint", action="append", default=[],
+                    metavar="NAME=DIR",
+                    help="serve the checkpoint folder DIR (config.json, "
+                         "model.safetensors) as model NAME; repeatable")
     args = ap.parse_args()
+    for spec in args.checkpoint:
+        register_checkpoint(spec)
 
     w = Worker(args.gpu, max_batch=args.max_batch, default_ctx=args.max_ctx,
                models=args.models.split(",") if args.models else None)

@@ -65,6 +65,10 @@ def main():
                          "config 5).  Each worker advertises ONLY its "
                          "model, so /api/tags routing steers requests "
                          "(reference src/dispatcher.rs:599-620).")
+    ap.add_argument("--checkpoint", action="append", default=[],
+                    metavar="NAME=DIR",
+                    help="checkpoint folder DIR served as model NAME by the "
+                         "1-GPU workers; repeatable")
     args = ap.parse_args()
 
     if not os.path.exists(SERVER_BIN):
@@ -111,6 +115,8 @@ def main():
                    "--max-batch", str(args.max_batch)]
             if args.workers:
                 cmd += ["--models", model]
+            for spec in args.checkpoint:
+                cmd += ["--checkpoint", spec]
             procs.append(subprocess.Popen(cmd, env=env))
         else:
             cmd = [sys.executable, "-m", "torch.distributed.run",

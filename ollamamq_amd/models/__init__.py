@@ -1,3 +1,8 @@
 from .llama import LlamaConfig, LlamaModel, PRESETS
+from .rinitar import RinitarConfig, RinitarModel
+from .registry import (build_model, config_from_folder, model_class,
+                       register_checkpoint)
 
-__all__ = ["LlamaConfig", "LlamaModel", "PRESETS"]
+__all__ = ["LlamaConfig", "LlamaModel", "RinitarConfig", "RinitarModel",
+           "PRESETS", "build_model", "config_from_folder", "model_class",
+           "register_checkpoint"]

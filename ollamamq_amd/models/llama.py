@@ -46,6 +46,26 @@ class LlamaConfig:
     # high_freq_factor, original_max_ctx); None = plain RoPE
     rope_scaling: Optional[tuple] = None
 
+    family = "llama"
+
+    def weight_bytes(self) -> int:
+        """Size of the bf16 weights."""
+        return 2 * (self.vocab * self.hidden * 2 + self.n_layers * (
+            self.hidden * (self.q_dim + 2 * self.kv_dim)
+            + self.q_dim * self.hidden + 3 * self.hidden * self.ffn))
+
+    def model_info(self) -> dict:
+        """Architecture facts for /api/show."""
+        return {
+            "block_count": self.n_layers,
+            "embedding_length": self.hidden,
+            "context_length": self.max_ctx,
+            "feed_forward_length": self.ffn,
+            "attention.head_count": self.n_heads,
+            "attention.head_count_kv": self.n_kv_heads,
+            "vocab_size": self.vocab,
+        }
+
     @property
     def q_dim(self) -> int:
         return self.n_heads * self.head_dim

@@ -1,0 +1,338 @@
+"""Rinitar: blocks normed by dynamic tanh, mixing gated linear attention and
+position-free latent attention, with an optional loop over some layers.
+
+    x <- x + norm1b(mixer(shift(norm1(x))))
+    x <- x + norm2b(ff(norm2(x)))
+
+* every norm is a dynamic tanh (ops.DyT): no row statistics, so the step
+  between two matrix products -- norm, residual sum, norm, token shift -- is
+  one elementwise kernel (ops.dyt_residual);
+* mixers: "gla" keeps an fp32 [heads, dim, vdim] state per sequence
+  (ops.gla), "latent_attention" a paged row of kv_rank values per token
+  (ops.latent_attention);
+* feed-forward: one up projection with PolyNorm (ops.polynorm);
+* layers start..stop-1 may run several times with the same weights; every
+  run has its own cache and state, so memory is per run, weights per layer.
+
+The residual stream, norms, scores, decays and states are fp32.  A mixer's
+input projections are one matrix product.  On the GPU in bf16 the decode
+path streams packed copies of the weights (ops.pack_weight).
+"""
+from __future__ import annotations
+
+import os
+from dataclasses import dataclass, field
+from typing import List, Optional, Tuple
+
+import torch
+
+from ..ops import interface as ops
+from .checkpoint import CheckpointSource, RandomSource
+
+MIXER_KEYS = {
+    "gla": ("heads", "dim", "vdim", "tau"),
+    "latent_attention": ("heads", "dim", "vdim", "kv_rank", "scale"),
+}
+LOW_RANK = 16      # rank of a random model's decay projection
+
+
+@dataclass(frozen=True)
+class RinitarLayerSpec:
+    type: str
+    heads: int
+    dim: int
+    vdim: int
+    tau: float = 1.0          # gla
+    kv_rank: int = 0          # latent_attention
+    scale: float = 1.0
+    ff: Optional[int] = None  # None: no feed-forward
+
+    @classmethod
+    def from_json(cls, d: dict) -> "RinitarLayerSpec":
+        kind = d["type"]
+        if kind not in MIXER_KEYS:
+            raise ValueError(f"unknown mixer {kind!r}")
+        sizes = {k: d["mixer"][k] for k in MIXER_KEYS[kind]}
+        mlp = d.get("mlp")
+        if mlp and mlp.get("kind") != "dense":
+            raise ValueError(f"unknown feed-forward {mlp.get('kind')!r}")
+        return cls(type=kind, ff=mlp["ff"] if mlp else None, **sizes)
+
+
+@dataclass
+class RinitarConfig:
+    name: str
+    width: int
+    vocab: int
+    layers: List[RinitarLayerSpec]
+    eps: float = 1e-5
+    loop: Optional[Tuple[int, int, int]] = None   # start, stop, times
+    max_ctx: int = 131072                 # no positions: memory is the limit
+    checkpoint: Optional[str] = None      # folder with the weights
+
+    family = "rinitar"
+    sliding_window = 0
+
+    def __post_init__(self):
+        if self.loop is not None:
+            start, stop, times = self.loop
+            if not (0 <= start <= stop <= len(self.layers)) or times < 0:
+                raise ValueError(f"loop {self.loop} does not fit "
+                                 f"{len(self.layers)} layers")
+
+    @classmethod
+    def from_json(cls, d: dict, name: str = "rinitar",
+                  checkpoint: Optional[str] = None) -> "RinitarConfig":
+        lp = d.get("loop")
+        return cls(
+            name=name, width=d["width"], vocab=d["vocab"],
+            layers=[RinitarLayerSpec.from_json(e) for e in d["layers"]],
+            eps=d["norm"]["eps"],
+            loop=(lp["start"], lp["stop"], lp["times"]) if lp else None,
+            checkpoint=checkpoint)
+
+    @property
+    def runs(self) -> List[int]:
+        """Layer index of every layer run, in order."""
+        n = len(self.layers)
+        if self.loop is None:
+            return list(range(n))
+        start, stop, times = self.loop
+        return (list(range(start)) + list(range(start, stop)) * times
+                + list(range(stop, n)))
+
+    def run_stores(self):
+        """What each layer run keeps per sequence."""
+        from ..engine.kvcache import RunStore
+        out = []
+        for li in self.runs:
+            s = self.layers[li]
+            state = [("prev", (self.width,))]
+            if s.type == "gla":
+                state.append(("gla", (s.heads, s.dim, s.vdim)))
+            out.append(RunStore(latent=s.kv_rank, state=tuple(state)))
+        return out
+
+    def weight_bytes(self) -> int:
+        """Size of the bf16 weights."""
+        W, n = self.width, self.vocab * self.width
+        for s in self.layers:
+            qk, v = s.heads * s.dim, s.heads * s.vdim
+            if s.type == "gla":
+                n += W * (2 * qk + 3 * v + LOW_RANK) + qk * LOW_RANK
+            else:
+                n += W * (qk + s.kv_rank + v) + s.kv_rank * (qk + v)
+            n += 2 * W * (s.ff or 0)
+        return 2 * n
+
+    def model_info(self) -> dict:
+        """Architecture facts for /api/show."""
+        return {
+            "block_count": len(self.layers),
+            "block_runs": len(self.runs),
+            "embedding_length": self.width,
+            "context_length": self.max_ctx,
+            "feed_forward_length": max(s.ff or 0 for s in self.layers),
+            "attention.head_count": max(s.heads for s in self.layers),
+            "vocab_size": self.vocab,
+        }
+
+
+def _stack(width, vocab, gla, latent, pattern, **kw):
+    kinds = {"g": gla, "l": latent}
+    return dict(width=width, vocab=vocab,
+                layers=[kinds[c] for c in pattern], **kw)
+
+
+RINITAR_PRESETS = {
+    # small enough for CPU tests
+    "rinitar-tiny": RinitarConfig(name="rinitar-tiny", **_stack(
+        192, 320,
+        RinitarLayerSpec("gla", 3, 24, 40, tau=8.0, ff=288),
+        RinitarLayerSpec("latent_attention", 3, 16, 24, kv_rank=40,
+                         scale=0.21, ff=288),
+        "glgl", loop=(1, 3, 2), max_ctx=2048)),
+    # layers the size of an 8B model's: width 4096, equal parts of both
+    # mixers, one pass
+    "rinitar-8b": RinitarConfig(name="rinitar-8b", **_stack(
+        4096, 128256,
+        RinitarLayerSpec("gla", 16, 128, 256, tau=16.0, ff=14336),
+        RinitarLayerSpec("latent_attention", 32, 128, 128, kv_rank=512,
+                         scale=128 ** -0.5, ff=14336),
+        "gggl" * 10)),
+    # width 2048: a 1B-class stack
+    "rinitar-1b": RinitarConfig(name="rinitar-1b", **_stack(
+        2048, 128256,
+        RinitarLayerSpec("gla", 8, 128, 256, tau=16.0, ff=8192),
+        RinitarLayerSpec("latent_attention", 16, 128, 128, kv_rank=512,
+                         scale=128 ** -0.5, ff=8192),
+        "gggl" * 5)),
+}
+
+
+class RinitarLayer:
+    """One layer's resident weights."""
+
+    def __init__(self, spec: RinitarLayerSpec, width: int, eps: float,
+                 pre: str, get, put, norm):
+        self.spec = spec
+        s, W = spec, width
+        qk, v = s.heads * s.dim, s.heads * s.vdim
+        mix = pre + "mix."
+
+        def vec(name, n, **kw):
+            return put(get(name, (n,), **kw)).float()
+
+        self.norm1, self.norm1b = norm(pre + "norm1"), norm(pre + "norm1b")
+        self.shift = vec(pre + "shift", W, mean=0.3, spread=0.2)
+        if s.type == "gla":
+            a1 = get(mix + "a1", (None, W))
+            rank = a1.shape[0]
+            cols = [get(mix + "q", (qk, W)), get(mix + "k", (qk, W)),
+                    get(mix + "v", (v, W)), get(mix + "g", (v, W)), a1]
+            self.gla = ops.GlaWeights(
+                heads=s.heads, dim=s.dim, vdim=s.vdim, rank=rank,
+                offsets=(0, qk, 2 * qk, 2 * qk + v, 2 * qk + 2 * v),
+                a2=put(get(mix + "a2", (qk, rank))).contiguous(),
+                a2_b=vec(mix + "a2.b", qk, mean=2.0, spread=1.0),
+                norm=vec(mix + "norm", s.vdim, mean=1.0, spread=0.1),
+                tau=float(s.tau), eps=eps)
+        else:
+            R = s.kv_rank
+            cols = [get(mix + "q", (qk, W)), get(mix + "dkv", (R, W))]
+            self.dkv_norm = vec(mix + "dkv.norm", R, mean=1.0, spread=0.1)
+            uk = put(get(mix + "uk", (qk, R))).view(s.heads, s.dim, R)
+            uv = put(get(mix + "uv", (v, R))).view(s.heads, s.vdim, R)
+            self.latent = ops.LatentWeights(
+                uk=uk.contiguous(), uk_t=uk.transpose(1, 2).contiguous(),
+                uv=uv.contiguous(), scale=float(s.scale))
+        # the input projections are one product; zero rows fill it up to the
+        # 32-row tiles of the packed form
+        n = sum(c.shape[0] for c in cols)
+        if n % 32:
+            cols.append(torch.zeros(32 - n % 32, W, dtype=cols[0].dtype,
+                                    device=cols[0].device))
+        self.w_in = put(torch.cat(cols)).contiguous()
+        self.w_o = put(get(mix + "o", (W, v))).contiguous()
+        if s.ff:
+            self.norm2, self.norm2b = norm(pre + "norm2"), \
+                norm(pre + "norm2b")
+            self.w_up = put(get(pre + "mlp.up", (s.ff, W))).contiguous()
+            self.w_down = put(get(pre + "mlp.down", (W, s.ff))).contiguous()
+            self.act = tuple(get(pre + "mlp.act", (4,), mean=0.4,
+                                 spread=0.1).float().tolist())
+        # packed decode copies (GPU, bf16)
+        self.packs = {}
+
+    def matrices(self):
+        names = ["w_in", "w_o"] + (["w_up", "w_down"] if self.spec.ff else [])
+        return {n: getattr(self, n) for n in names}
+
+
+class RinitarModel:
+    """Holds weights only: caches and states live in engine.HybridCache."""
+
+    def __init__(self, cfg: RinitarConfig, device: str = "cpu",
+                 dtype: torch.dtype = torch.float32, seed: int = 1234,
+                 tp_rank: int = 0, tp_size: int = 1, process_group=None,
+                 fast_init: bool = False):
+        if tp_size != 1 or process_group is not None:
+            raise ValueError(f"{cfg.name}: no tensor parallelism")
+        self.cfg = cfg
+        self.device = torch.device(device)
+        self.dtype = dtype
+        self.tp_rank, self.tp_size, self.group = 0, 1, None
+        if cfg.checkpoint:
+            get = CheckpointSource(cfg.checkpoint)
+        else:
+            on_gpu = fast_init and self.device.type == "cuda"
+            get = RandomSource(seed, "cuda" if on_gpu else "cpu", LOW_RANK)
+
+        def put(t):
+            return t.to(device=self.device, dtype=dtype)
+
+        def norm(name):
+            W = cfg.width
+            alpha = get(name + ".alpha", (), mean=0.6, spread=0.05)
+            return ops.DyT(
+                get(name, (W,), mean=1.0, spread=0.1)
+                .to(self.device).float(),
+                get(name + ".b", (W,), spread=0.1).to(self.device).float(),
+                float(alpha))
+
+        self.embed = put(get("embed", (cfg.vocab, cfg.width),
+                             spread=1.0)).contiguous()
+        self.layers = [
+            RinitarLayer(s, cfg.width, cfg.eps, f"l{i}.", get, put, norm)
+            for i, s in enumerate(cfg.layers)]
+        self.final_norm = norm("final.norm")
+        self._pack_weights()
+
+    def _pack_weights(self):
+        if self.device.type != "cuda" or self.dtype != torch.bfloat16 \
+                or os.environ.get("OLLAMAMQ_NO_PACK") == "1":
+            return
+        free, _ = torch.cuda.mem_get_info(self.device)
+        if self.weight_bytes() > free * 0.45:
+            return
+        for layer in self.layers:
+            layer.packs = {n: ops.pack_weight(w)
+                           for n, w in layer.matrices().items()}
+
+    def weight_bytes(self) -> int:
+        n = self.embed.numel()
+        for layer in self.layers:
+            n += sum(w.numel() for w in layer.matrices().values())
+        return n * self.embed.element_size()
+
+    def _mixer(self, layer, run, h, cache, slot_ids, positions, meta):
+        p = ops.linear(h, layer.w_in, packed=layer.packs.get("w_in"))
+        s = layer.spec
+        if s.type == "gla":
+            o = ops.gla(p, layer.gla, cache.state[run]["gla"], slot_ids,
+                        positions, meta)
+        else:
+            qk = s.heads * s.dim
+            ops.latent_append(cache, run, p[:, qk:qk + s.kv_rank],
+                              layer.dkv_norm, slot_ids, positions,
+                              self.cfg.eps)
+            o = ops.latent_attention(p[:, :qk], cache, run, layer.latent,
+                                     slot_ids, positions, meta)
+        return ops.linear_parts(o, layer.w_o, layer.packs.get("w_o"))
+
+    def forward(
+        self,
+        tokens: torch.Tensor,      # [T] flat token ids
+        positions: torch.Tensor,   # [T] position of each token in its seq
+        kv_cache,                  # engine.kvcache.HybridCache
+        slot_ids: torch.Tensor,    # [T] slot of each token's sequence
+        attn_meta,                 # ops.AttnMeta
+        return_hidden: bool = False,
+    ) -> torch.Tensor:
+        """Logits (or final-norm hidden states) of the rows attn_meta
+        selects."""
+        meta, eps = attn_meta, self.cfg.eps
+        x = y = post = None
+        for run, li in enumerate(self.cfg.runs):
+            layer = self.layers[li]
+            shift = ops.TokenShift(layer.shift, kv_cache.state[run]["prev"],
+                                   slot_ids, positions, meta)
+            x, h = ops.dyt_residual(x, y, post, layer.norm1, shift,
+                                    embed=self.embed, tokens=tokens)
+            y = self._mixer(layer, run, h, kv_cache, slot_ids, positions,
+                            meta)
+            post = layer.norm1b
+            if layer.spec.ff:
+                x, h = ops.dyt_residual(x, y, post, layer.norm2,
+                                        embed=self.embed)
+                z = ops.linear_parts(h, layer.w_up, layer.packs.get("w_up"))
+                a = ops.polynorm(z, layer.act, eps)
+                y = ops.linear_parts(a, layer.w_down,
+                                     layer.packs.get("w_down"))
+                post = layer.norm2b
+        _, h = ops.dyt_residual(x, y, post, self.final_norm,
+                                embed=self.embed, tokens=tokens,
+                                rows=meta.logits_idx, need_x=False)
+        if return_hidden:
+            return h
+        return ops.linear(h, self.embed)

@@ -14,7 +14,7 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .interface import AttnMeta
+from .interface import AttnMeta, Partials
 
 _LIB_PATH = os.path.join(
     os.path.dirname(os.path.dirname(os.path.abspath(__file__))),
@@ -44,6 +44,7 @@ def _try_load():
                                     i, i, i, i, i, i, f, i64, vp]
     lib.swiglu_bf16.argtypes = [vp, vp, i, i, vp]
     lib.argmax_bf16.argtypes = [vp, vp, i, i, vp, vp, i, vp]
+    lib.argmax_f32.argtypes = lib.argmax_bf16.argtypes
     lib.decode_attn_bf16.argtypes = [vp, vp, vp, vp, vp, vp, vp, vp, vp,
                                      i, i, i, i, i, f, i64, i, i, i, vp,
                                      i, vp]
@@ -68,6 +69,27 @@ def _try_load():
     lib.wstream_qkv_rope_bf16.argtypes = [vp, vp, vp, vp, i, i, i, i64,
                                           vp, i, f, f, vp, vp, vp, vp,
                                           vp, vp, vp, i, i, i, i, i, vp]
+    lib.dyt_residual.argtypes = [i, vp, vp, vp, vp, vp, vp, vp, i,
+                                 vp, vp, f, vp, vp, f, vp, vp, vp, vp, vp,
+                                 vp, vp, i, i, i, vp]
+    lib.polynorm.argtypes = [i, vp, vp, vp, i, f, f, f, f, i, i, f, vp]
+    lib.latent_append.argtypes = [i, vp, vp, i64, vp, vp, vp, vp,
+                                  i, i, i, i, f, vp]
+    lib.latent_gather.argtypes = [i, vp, vp, vp, vp, i, i, i, i, vp]
+    lib.head_gemm.argtypes = [i, vp, vp, vp, i, i, i, i, i64, vp]
+    lib.latent_mt.argtypes = [i, i, i]
+    lib.latent_attn.argtypes = [i, vp, vp, vp, vp, vp, vp, vp, vp, vp,
+                                i, i, i, i, i, i, f, i64, i64, i64, i, vp]
+    lib.flash_rows.argtypes = [i]
+    lib.flash_attn.argtypes = [i, vp, vp, vp, vp, vp, i, i, i, i, i64, i64,
+                               f, vp]
+    lib.gla_step.argtypes = [i, vp, vp, i64, i, i, i, i, i, i, vp, vp, vp,
+                             vp, vp, vp, vp, i, i, i, i, f, f, f, vp]
+    lib.gla_chunks.argtypes = [i, vp, vp, vp, vp, i64, i, i, i, i, i, i,
+                               vp, vp, vp, vp, vp, vp, vp, i, vp, i, i, i,
+                               i, i, i, f, f, f, vp]
+    lib.gla_scratch_floats.argtypes = [i, i, i]
+    lib.gla_scratch_floats.restype = i64
     for fn in ("rmsnorm_residual_bf16", "rope_bf16", "kv_append_bf16",
                "paged_attn_bf16", "swiglu_bf16", "argmax_bf16",
                "decode_attn_bf16", "skinny_gemm_bf16",
@@ -712,6 +734,327 @@ def swiglu(gate_up):
     return out
 
 
+# ---------------------------------------------------------------------------
+# dynamic-tanh blocks, latent attention, gated linear attention: every kernel
+# exists for bf16 and for true fp32
+
+def _is_f32(t):
+    if t.dtype not in (torch.float32, torch.bfloat16):
+        raise TypeError(f"kernels take float32 or bfloat16, not {t.dtype}")
+    return int(t.dtype == torch.float32)
+
+
+def _i32(t):
+    return t if t.dtype == torch.int32 else t.int()
+
+
+def linear_parts(x, weight, packed=None):
+    """Decode: the weight-streaming product, left as split-K partial sums
+    where it splits (the next kernel folds them in)."""
+    M, K = x.shape
+    N = weight.shape[0]
+    if packed is not None and USE_WSTREAM and M <= 64 and N <= _WS_MAX_N \
+            and x.dtype == torch.bfloat16 and x.stride(1) == 1:
+        ks = int(_WS_KS) if _WS_KS else _wstream_ksplit(N, K)
+        if ks > 1:
+            part = torch.empty((ks, M, N), dtype=torch.float32,
+                               device=x.device)
+            xlds = (_WS_XLDS if M <= 32 and N * K * 2 > (64 << 20) else 0)
+            _check(_lib.wstream_gemm_bf16(
+                _p(None), _p(part), _p(x), _p(packed), _p(None), M, N, K,
+                x.stride(0), ks, _WS_DEPTH, xlds, _p(None), 0, 0.0, 0.0,
+                _p(None), _p(None), 0, _stream()), "wstream_gemm")
+            return Partials(part)
+    return linear(x, weight, packed=packed)
+
+
+def _row_seq(meta):
+    """Sequence index of every row of a varlen batch (cached on the meta)."""
+    t = getattr(meta, "_row_seq", None)
+    if t is None:
+        _, q_lens, _ = meta.layout()
+        t = torch.repeat_interleave(
+            torch.arange(len(q_lens), dtype=torch.int32),
+            torch.tensor(q_lens)).to(meta.slot_ids.device)
+        meta._row_seq = t
+    return t
+
+
+def dyt_residual(x, y, post, pre, shift, embed, tokens, rows, need_x):
+    parts = y.parts if isinstance(y, Partials) else None
+    yt = None if parts is not None else y
+    W = pre.w.shape[0]
+    if x is not None:
+        T_in = x.shape[0]
+        assert x.dtype == torch.float32 and x.is_contiguous()
+    else:
+        T_in = tokens.shape[0]
+    dtype = embed.dtype
+    assert yt is None or (yt.shape == (T_in, W) and yt.is_contiguous()
+                          and yt.dtype == dtype)
+    assert parts is None or parts.shape[1:] == (T_in, W)
+    n = T_in if rows is None else rows.shape[0]
+    h = torch.empty((n, W), dtype=dtype, device=pre.w.device)
+    if x is not None and y is None and rows is None:
+        x_out, write = x, None               # nothing to add
+    else:
+        x_out = write = (torch.empty((n, W), dtype=torch.float32,
+                                     device=pre.w.device)
+                         if need_x else None)
+    mix = prev = slot = pos = row_seq = cu = None
+    if shift is not None:
+        assert rows is None
+        mix, prev = shift.mix, shift.prev
+        slot, pos = _i32(shift.slot_ids), _i32(shift.positions)
+        if not shift.meta.one_each:
+            row_seq, cu = _row_seq(shift.meta), shift.meta.cu_q
+            assert cu.dtype == torch.int32
+    tok = None if tokens is None else _i32(tokens)
+    z = post if post is not None else pre
+    if n == 0:
+        return x_out, h
+    _check(_lib.dyt_residual(
+        _is_f32(h), _p(write), _p(h), _p(x), _p(embed), _p(tok), _p(yt),
+        _p(parts), 0 if parts is None else parts.shape[0],
+        _p(z.w), _p(z.b), z.alpha, _p(pre.w), _p(pre.b), pre.alpha,
+        _p(mix), _p(prev), _p(slot), _p(pos), _p(row_seq), _p(cu), _p(rows),
+        n, T_in, W, _stream()), "dyt_residual")
+    return x_out, h
+
+
+def polynorm(z, coef, eps):
+    parts = z.parts if isinstance(z, Partials) else None
+    T, F = (z if parts is None else parts[0]).shape
+    dtype = torch.bfloat16 if parts is not None else z.dtype
+    out = torch.empty((T, F), dtype=dtype, device=(
+        z if parts is None else parts).device)
+    assert parts is not None or z.is_contiguous()
+    _check(_lib.polynorm(
+        _is_f32(out), _p(out), _p(None if parts is not None else z),
+        _p(parts), 0 if parts is None else parts.shape[0], *coef, T, F,
+        float(eps), _stream()), "polynorm")
+    return out
+
+
+def latent_append(cache, run, d, weight, slot_ids, positions, eps):
+    T, R = d.shape
+    pool = cache.latent_pool[run]
+    assert d.stride(1) == 1 and pool.dtype == d.dtype and pool.shape[2] == R
+    _check(_lib.latent_append(
+        _is_f32(d), _p(pool), _p(d), d.stride(0), _p(weight),
+        _p(_i32(slot_ids)), _p(_i32(positions)), _p(cache.page_table), T, R,
+        cache.page_size, cache.page_table.shape[1], float(eps), _stream()),
+        "latent_append")
+
+
+def head_gemm(x, w, out):
+    """out[t, h] = w[h] @ x[t, h]; x [T, H, K] (rows may be strided)."""
+    T, H, K = x.shape
+    N = w.shape[1]
+    assert w.shape == (H, N, K) and w.is_contiguous() \
+        and out.shape == (T, H, N) and out.is_contiguous() \
+        and x.stride(2) == 1 and (H == 1 or x.stride(1) == K)
+    if T:
+        _check(_lib.head_gemm(_is_f32(x), _p(out), _p(x), _p(w), T, H, N, K,
+                              x.stride(0), _stream()), "head_gemm")
+    return out
+
+
+LATENT_MAX_R = 1024       # absorbed kernel: latent width
+FLASH_MAX = 256           # expanded kernel: key and value widths
+EXPAND_BYTES = 1 << 30    # expanded keys and values held at a time
+
+
+def _absorb_limit(H, D, V, R):
+    """Portions below this many tokens attend in latent space: the expanded
+    form pays R*(D+V) per key once, the absorbed one R+R instead of D+V per
+    (query, key)."""
+    if R > LATENT_MAX_R:
+        return 0
+    if max(D, V) > FLASH_MAX or 2 * R <= D + V:
+        return 1 << 62
+    return max(16, R * (D + V) // (2 * R - D - V))
+
+
+def _latent_plan(meta, H, D, V, R, f32, dev):
+    """Batch layout for one attention shape, shared by the layers that have
+    it: leading sequences attend in latent space, the rest expanded."""
+    key = f"_latent_{H}_{D}_{V}_{R}"
+    plan = getattr(meta, key, None)
+    if plan is not None:
+        return plan
+    slots, q_lens, kv_lens = meta.layout()
+    limit = _absorb_limit(H, D, V, R)
+    M = 16 * _lib.latent_mt(f32, H, R)
+    nd = meta.n_single
+    i, row, items = nd, nd, []
+    kv_absorbed = 0
+    while i < len(slots) and q_lens[i] < limit:
+        lo, hi = row * H, (row + q_lens[i]) * H
+        items += [(r, min(M, hi - r)) for r in range(lo, hi, M)]
+        kv_absorbed = max(kv_absorbed, kv_lens[i])
+        row += q_lens[i]
+        i += 1
+    n_absorbed = row
+    QT = _lib.flash_rows(f32)
+    esz = 4 if f32 else 2
+    groups = []            # (gather rows, tiles, padded keys) per batch
+    gather, tiles, kv0 = [], [], 0
+
+    def flush():
+        nonlocal gather, tiles, kv0
+        if tiles:
+            groups.append((
+                torch.tensor(gather, dtype=torch.int32).to(dev),
+                torch.tensor(tiles, dtype=torch.int32).to(dev), kv0))
+        gather, tiles, kv0 = [], [], 0
+
+    while i < len(slots):
+        n, kv = q_lens[i], kv_lens[i]
+        for b in range(0, kv, 64):
+            gather.append((slots[i], b, min(64, kv - b)))
+        for t in range(0, n, QT):
+            tiles.append((row + t, kv - n + t, min(QT, n - t), kv0))
+        row += n
+        kv0 += (kv + 63) // 64 * 64
+        i += 1
+        if kv0 * H * (D + V) * esz > EXPAND_BYTES:
+            flush()
+    flush()
+    dev_items = torch.tensor(items, dtype=torch.int32).to(dev) \
+        if items else None
+    plan = (n_absorbed, dev_items, kv_absorbed, groups)
+    setattr(meta, key, plan)
+    return plan
+
+
+def _latent_absorbed(o, q, cache, run, slots, pos, H, R, scale, items,
+                     n_items, per_seq, row0, rows, max_kv):
+    """One launch of the absorbed kernel over rows row0.. of q / o."""
+    f32 = _is_f32(q)
+    split = int(max(1, min(512 // n_items, (max_kv + 127) // 128, 32)))
+    op = ml = None
+    total = q.shape[0]
+    if split > 1:
+        op = torch.empty((split, total, R), dtype=torch.float32,
+                         device=q.device)
+        ml = torch.empty((split, total, 2), dtype=torch.float32,
+                         device=q.device)
+    pool = cache.latent_pool[run]
+    assert pool.dtype == q.dtype and pool.shape[2] == R
+    _check(_lib.latent_attn(
+        f32, _p(o), _p(op), _p(ml), _p(q), _p(pool), _p(cache.page_table),
+        _p(slots), _p(pos), _p(items), n_items, per_seq, H, R,
+        cache.page_size, cache.page_table.shape[1], float(scale), total,
+        row0, rows, split, _stream()), "latent_attn")
+
+
+def latent_attention(q, cache, run, w, slot_ids, positions, meta):
+    H, D, R = w.uk.shape
+    V = w.uv.shape[1]
+    T = q.shape[0]
+    f32 = _is_f32(q)
+    if R > LATENT_MAX_R and (max(D, V) > FLASH_MAX or meta.n_single):
+        raise ValueError(f"latent attention with rank {R}, head widths "
+                         f"{D}/{V}: no kernel")
+    out = torch.empty((T, H, V), dtype=q.dtype, device=q.device)
+    slots, pos = _i32(slot_ids), _i32(positions)
+    nd = meta.n_single
+    if meta.one_each:
+        n_abs, items, kv_abs, groups = T, None, 0, []
+    else:
+        n_abs, items, kv_abs, groups = _latent_plan(meta, H, D, V, R, f32,
+                                                    q.device)
+    if n_abs:
+        qa = q[:n_abs].unflatten(1, (H, D))
+        lat = torch.empty((n_abs, H, R), dtype=q.dtype, device=q.device)
+        head_gemm(qa, w.uk_t, lat)
+        lat = lat.view(n_abs * H, R)
+        o = torch.empty_like(lat)
+        if nd:
+            per = -(-H // (16 * _lib.latent_mt(f32, H, R)))
+            _latent_absorbed(o, lat, cache, run, slots, pos, H, R, w.scale,
+                             None, nd * per, per, 0, nd * H, meta.max_kv)
+        if items is not None:
+            _latent_absorbed(o, lat, cache, run, slots, pos, H, R, w.scale,
+                             items, items.shape[0], 1, nd * H,
+                             (n_abs - nd) * H, kv_abs)
+        head_gemm(o.view(n_abs, H, R), w.uv, out[:n_abs])
+    pool = cache.latent_pool[run]
+    for gather, tiles, kv in groups:
+        c = torch.empty((kv, R), dtype=q.dtype, device=q.device)
+        _check(_lib.latent_gather(
+            f32, _p(c), _p(pool), _p(cache.page_table), _p(gather),
+            gather.shape[0], R, cache.page_size, cache.page_table.shape[1],
+            _stream()), "latent_gather")
+        k = torch.nn.functional.linear(c, w.uk.view(H * D, R))
+        vt = torch.mm(w.uv.view(H * V, R), c.t())
+        _check(_lib.flash_attn(
+            f32, _p(out), _p(q), _p(k), _p(vt), _p(tiles), tiles.shape[0],
+            H, D, V, q.stride(0), kv, float(w.scale), _stream()),
+            "flash_attn")
+    return out.view(T, H * V)
+
+
+GLA_STEP_TOKENS = 4       # portions up to this walk token by token
+
+
+def _gla_plan(meta, dev):
+    plan = getattr(meta, "_gla_plan", None)
+    if plan is not None:
+        return plan
+    _, q_lens, _ = meta.layout()
+    nd = meta.n_single
+    i, row, spans = nd, nd, []
+    while i < len(q_lens) and q_lens[i] <= GLA_STEP_TOKENS:
+        spans.append((row, q_lens[i]))
+        row += q_lens[i]
+        i += 1
+    base, chunks, seqs = row, [], []
+    for n in q_lens[i:]:
+        seqs.append((len(chunks), (n + 63) // 64))
+        chunks += [(row + t, min(64, n - t)) for t in range(0, n, 64)]
+        row += n
+    t32 = lambda x: torch.tensor(x, dtype=torch.int32).to(dev) \
+        if x else None
+    plan = (t32(spans), t32(chunks), t32(seqs), base, row - base)
+    meta._gla_plan = plan
+    return plan
+
+
+def gla(p, w, state, slot_ids, positions, meta):
+    T = p.shape[0]
+    H, D, V = w.heads, w.dim, w.vdim
+    assert p.stride(1) == 1 and state.dtype == torch.float32 \
+        and state.shape[1:] == (H, D, V) and w.a2.dtype == p.dtype
+    assert max(w.offsets) + w.rank <= p.shape[1]
+    out = torch.empty((T, H * V), dtype=p.dtype, device=p.device)
+    slots, pos = _i32(slot_ids), _i32(positions)
+    f32 = _is_f32(p)
+    head = (_p(p), p.stride(0), *w.offsets, w.rank, _p(w.a2), _p(w.a2_b),
+            _p(w.norm), _p(state), _p(slots), _p(pos))
+    tail = (H, D, V, D ** -0.5, 1.0 / w.tau, float(w.eps), _stream())
+    nd = meta.n_single
+    if nd:
+        _check(_lib.gla_step(f32, _p(out), *head, _p(None), nd, *tail),
+               "gla_step")
+    if meta.one_each:
+        return out
+    spans, chunks, seqs, base, rows = _gla_plan(meta, p.device)
+    if spans is not None:
+        _check(_lib.gla_step(f32, _p(out), *head, _p(spans),
+                             spans.shape[0], *tail), "gla_step")
+    if chunks is not None:
+        nc = chunks.shape[0]
+        scr = torch.empty(_lib.gla_scratch_floats(nc, H, D),
+                          dtype=torch.float32, device=p.device)
+        o = torch.empty(rows * H * V, dtype=torch.float32, device=p.device)
+        _check(_lib.gla_chunks(
+            f32, _p(out), _p(scr), _p(o), *head, _p(chunks), nc, _p(seqs),
+            seqs.shape[0], base, rows, *tail), "gla_chunks")
+    return out
+
+
 def sample_gumbel(logits, temps, seeds, ctrs, noise=None, out=None):
     """Exact temperature sampling (Gumbel-max): token ~ softmax(l/T) per
     row; rows with temps<=0 are greedy argmax.  Counter-based noise from
@@ -746,8 +1089,12 @@ def sample(logits, temperature, top_k, top_p, generator=None):
         all_greedy = temperature <= 0
     if all_greedy:
         B, V = logits.shape
+        if V % 8 or not logits.is_contiguous():
+            return logits.argmax(-1)     # rows not aligned for the kernel
         out = torch.empty(B, dtype=torch.int32, device=logits.device)
-        l = logits if logits.dtype == torch.bfloat16 else logits.bfloat16()
+        f32 = logits.dtype == torch.float32
+        l = logits if f32 or logits.dtype == torch.bfloat16 \
+            else logits.bfloat16()
         # split-V: B blocks alone underfill the chip at decode batch sizes
         sp = min(32, max(1, 768 // max(1, B)))
         pb = pi = ctypes.c_void_p(0)
@@ -761,8 +1108,8 @@ def sample(logits, temperature, top_k, top_p, generator=None):
                                  device=logits.device))
                 _scratch[key] = t
             pb, pi = _p(t[0]), _p(t[1])
-        _check(_lib.argmax_bf16(_p(out), _p(l), B, V, pb, pi, sp,
-                                _stream()), "argmax")
+        fn = _lib.argmax_f32 if f32 else _lib.argmax_bf16
+        _check(fn(_p(out), _p(l), B, V, pb, pi, sp, _stream()), "argmax")
         return out.long()
     # stochastic host path.  When every stochastic row carries
     # 0 < top_k <= 256 the sampling is EXACT over the top-256 candidates

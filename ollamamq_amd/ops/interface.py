@@ -9,7 +9,7 @@ from __future__ import annotations
 
 import os
 from dataclasses import dataclass
-from typing import Optional
+from typing import List, NamedTuple, Optional, Union
 
 import torch
 
@@ -50,6 +50,77 @@ class AttnMeta:
     # sliding-window attention (Mistral-style): query at position p attends
     # keys [max(0, p - window + 1), p]; 0 = full causal
     window: int = 0
+    # host copies of the batch layout (None in a captured decode step):
+    # tokens per sequence and cached length per sequence
+    q_lens: Optional[List[int]] = None
+    kv_lens: Optional[List[int]] = None
+    slots: Optional[List[int]] = None
+
+    @property
+    def one_each(self) -> bool:
+        """Every sequence brings exactly one token."""
+        return self.mode == "decode"
+
+    @property
+    def n_single(self) -> int:
+        """Leading rows that are single tokens of their sequence."""
+        return (self.slot_ids.shape[0] if self.one_each
+                else self.n_decode if self.mode == "mixed" else 0)
+
+    def layout(self):
+        """(slots, tokens per sequence, cached lengths) as host lists."""
+        if self.q_lens is None:
+            cu = self.cu_q.tolist()
+            self.q_lens = [b - a for a, b in zip(cu, cu[1:])]
+            self.kv_lens = self.seq_lens.tolist()
+            self.slots = self.slot_ids.tolist()
+        return self.slots, self.q_lens, self.kv_lens
+
+
+class DyT(NamedTuple):
+    """Dynamic tanh: tanh(alpha * x) * w + b (w, b fp32)."""
+    w: torch.Tensor
+    b: torch.Tensor
+    alpha: float
+
+
+class TokenShift(NamedTuple):
+    """h[t] + (h[t-1] - h[t]) * mix; `prev` [slots, W] fp32 keeps every
+    sequence's last h between steps (zero at position 0)."""
+    mix: torch.Tensor
+    prev: torch.Tensor
+    slot_ids: torch.Tensor        # per token
+    positions: torch.Tensor       # per token
+    meta: AttnMeta
+
+
+class Partials(NamedTuple):
+    """A matrix product as [parts, rows, cols] fp32 partial sums; the
+    consumer folds them."""
+    parts: torch.Tensor
+
+
+class LatentWeights(NamedTuple):
+    """k = uk c, v = uv c per head; uk [H, D, R], uk_t [H, R, D] and
+    uv [H, V, R] are views or copies of the same values."""
+    uk: torch.Tensor
+    uk_t: torch.Tensor
+    uv: torch.Tensor
+    scale: float
+
+
+class GlaWeights(NamedTuple):
+    """Columns of the fused projection, and what the recurrence reads."""
+    heads: int
+    dim: int
+    vdim: int
+    rank: int
+    offsets: tuple                # columns of q, k, v, gate, low rank
+    a2: torch.Tensor              # [heads * dim, rank]
+    a2_b: torch.Tensor            # fp32
+    norm: torch.Tensor            # fp32 [vdim]
+    tau: float
+    eps: float
 
 
 def embedding(tokens: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
@@ -124,6 +195,68 @@ def pack_weight(w):
         if hip.available():
             return hip.pack_weight(w)
     return None
+
+
+def linear_parts(x, weight, packed=None) -> Union[torch.Tensor, Partials]:
+    """As linear, but a split product may come back as its partial sums."""
+    if _use_hip(x):
+        from . import hip
+        return hip.linear_parts(x, weight, packed)
+    return torch.nn.functional.linear(x, weight)
+
+
+def dyt_residual(x, y, post: Optional[DyT], pre: DyT,
+                 shift: Optional[TokenShift] = None, embed=None, tokens=None,
+                 rows=None, need_x=True):
+    """One pass between two matrix products: x' = x + post(y), h = pre(x'),
+    then the token shift.  x is fp32 [T, W], or None for the embedding rows
+    of `tokens`; y a tensor, Partials or None; `rows` selects the rows to
+    compute.  Returns (x', h)."""
+    if _use_hip(pre.w):
+        from . import hip
+        return hip.dyt_residual(x, y, post, pre, shift, embed, tokens, rows,
+                                need_x)
+    return ref.dyt_residual(x, y, post, pre, shift, embed, tokens, rows)
+
+
+def polynorm(z, coef, eps):
+    """a N(z) + b N(z^2) + c N(z^3) + e with coef = (a, b, c, e) and N the
+    division by the row's root mean square."""
+    t = z.parts if isinstance(z, Partials) else z
+    if _use_hip(t):
+        from . import hip
+        return hip.polynorm(z, coef, eps)
+    return ref.polynorm(z, coef, eps)
+
+
+def latent_append(cache, run, d, weight, slot_ids, positions, eps):
+    """RMS norm of d [T, R] and append to the run's paged latent pool."""
+    if _use_hip(d):
+        from . import hip
+        return hip.latent_append(cache, run, d, weight, slot_ids, positions,
+                                 eps)
+    return ref.latent_append(cache, run, d, weight, slot_ids, positions, eps)
+
+
+def latent_attention(q, cache, run, w: LatentWeights, slot_ids, positions,
+                     meta: AttnMeta):
+    """Causal softmax attention whose keys and values are linear in the
+    cached latent.  q [T, H*D] (rows may be strided) -> [T, H*V]."""
+    if _use_hip(q):
+        from . import hip
+        return hip.latent_attention(q, cache, run, w, slot_ids, positions,
+                                    meta)
+    return ref.latent_attention(q, cache, run, w, meta)
+
+
+def gla(p, w: GlaWeights, state, slot_ids, positions, meta: AttnMeta):
+    """Gated linear attention over the fused projection p [T, ...]; state
+    [slots, H, D, V] fp32 is read and advanced.  Head norm and output gate
+    included.  -> [T, H*V]."""
+    if _use_hip(p):
+        from . import hip
+        return hip.gla(p, w, state, slot_ids, positions, meta)
+    return ref.gla(p, w, state, meta)
 
 
 def swiglu(gate_up):

@@ -111,6 +111,87 @@ def swiglu(gate_up):
     return (torch.nn.functional.silu(g) * u).to(gate_up.dtype)
 
 
+def dyt_residual(x, y, post, pre, shift, embed, tokens, rows):
+    if x is None:
+        x = embed.index_select(0, tokens.long()).float()
+    if y is not None:
+        x = x + torch.tanh(post.alpha * y.float()) * post.w + post.b
+    if rows is not None:
+        x = x[rows]
+    h = torch.tanh(pre.alpha * x) * pre.w + pre.b
+    if shift is not None:
+        before = torch.roll(h, 1, 0)
+        slots, q_lens, _ = shift.meta.layout()
+        r = 0
+        for slot, n in zip(slots, q_lens):
+            before[r] = 0 if shift.positions[r] == 0 else shift.prev[slot]
+            shift.prev[slot] = h[r + n - 1]
+            r += n
+        h = h + (before - h) * shift.mix
+    return x, h.to(embed.dtype if embed is not None else pre.w.dtype)
+
+
+def polynorm(z, coef, eps):
+    f = z.float()
+    out = torch.full_like(f, coef[3])
+    for k in range(3):
+        p = f ** (k + 1)
+        out += coef[k] * p * torch.rsqrt(p.pow(2).mean(-1, True) + eps)
+    return out.to(z.dtype)
+
+
+def latent_append(cache, run, d, weight, slot_ids, positions, eps):
+    f = d.float()
+    c = f * torch.rsqrt(f.pow(2).mean(-1, True) + eps) * weight
+    ps = cache.page_size
+    pages = cache.page_table[slot_ids.long(), (positions // ps).long()]
+    pool = cache.latent_pool[run]
+    pool[pages.long(), (positions % ps).long()] = c.to(pool.dtype)
+
+
+def latent_attention(q, cache, run, w, meta):
+    H, D, R = w.uk.shape
+    T = q.shape[0]
+    pool = cache.latent_pool[run]
+    out = torch.empty(T, H, w.uv.shape[1], dtype=q.dtype, device=q.device)
+    r = 0
+    for slot, n, kv in zip(*meta.layout()):
+        pages = cache.page_table[slot, :-(-kv // cache.page_size)].long()
+        c = pool[pages].reshape(-1, R)[:kv].float()
+        k = torch.einsum("tr,hdr->htd", c, w.uk.float())
+        v = torch.einsum("tr,hvr->htv", c, w.uv.float())
+        qi = q[r:r + n].float().view(n, H, D).transpose(0, 1)
+        s = qi @ k.transpose(1, 2) * w.scale
+        ahead = torch.arange(kv)[None] > torch.arange(kv - n, kv)[:, None]
+        s.masked_fill_(ahead, float("-inf"))
+        out[r:r + n] = (torch.softmax(s, -1) @ v).transpose(0, 1)
+        r += n
+    return out.view(T, -1)
+
+
+def gla(p, w, state, meta):
+    T, H, D, V = p.shape[0], w.heads, w.dim, w.vdim
+    oq, ok, ov, og, ou = w.offsets
+    f = p.float()
+    q = f[:, oq:oq + H * D].view(T, H, D) * D ** -0.5
+    k = f[:, ok:ok + H * D].view(T, H, D)
+    v = f[:, ov:ov + H * V].view(T, H, V)
+    z = f[:, ou:ou + w.rank] @ w.a2.float().T + w.a2_b
+    a = torch.exp(torch.nn.functional.logsigmoid(z) / w.tau).view(T, H, D)
+    out = torch.empty(T, H, V)
+    r = 0
+    for slot, n, kv in zip(*meta.layout()):
+        S = state[slot] if kv > n else torch.zeros_like(state[slot])
+        for t in range(r, r + n):
+            S = a[t].unsqueeze(-1) * S + k[t].unsqueeze(-1) * v[t].unsqueeze(1)
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S
+        r += n
+    out = out * torch.rsqrt(out.pow(2).mean(-1, True) + w.eps) * w.norm
+    g = torch.nn.functional.silu(f[:, og:og + H * V]).view(T, H, V)
+    return (out * g).reshape(T, H * V).to(p.dtype)
+
+
 def sample(logits, temperature, top_k, top_p, generator=None):
     """Per-row sampling: greedy when temperature<=0, else temp/top-k/top-p.
 
