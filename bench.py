@@ -167,6 +167,107 @@ def run_stack(args):
         node.wait(timeout=30)
 
 
+def layer_stacks(width, n_layers=4):
+    """(name, config) pairs of `n_layers` layers with equal weights per
+    layer: the Llama layer's three feed-forward matrices against two wider
+    ones."""
+    import dataclasses
+    from ollamamq_amd.models import PRESETS
+    rin = PRESETS["rinitar-1b" if width <= 2048 else "rinitar-8b"]
+    gla = [s for s in rin.layers if s.type == "gla"][0]
+    lat = [s for s in rin.layers if s.type != "gla"][0]
+    llama = dataclasses.replace(
+        PRESETS["llama3-8b"], n_layers=n_layers, hidden=width, vocab=32000,
+        n_heads=width // 128, n_kv_heads=max(1, width // 512),
+        ffn=gla.ff * 2 // 3, name=f"llama-{width}")
+
+    def stack(name, layers):
+        return dataclasses.replace(rin, name=f"{name}-{width}",
+                                   width=width, vocab=32000,
+                                   layers=layers)
+    return [("llama", llama),
+            ("rinitar gla", stack("gla", [gla] * n_layers)),
+            ("rinitar latent", stack("latent", [lat] * n_layers)),
+            ("rinitar mixed", stack("mixed", [gla, lat] * (n_layers // 2)))]
+
+
+def run_layers(args):
+    """Throughput of the hybrid design's layers at the sizes of real models,
+    beside Llama layers of equal weight count: prefill of 2 x 2048 tokens in
+    one step, and decode of --users sequences after a prompt of
+    --prompt-len.  Both go through the engine."""
+    from ollamamq_amd.models import build_model
+    from ollamamq_amd.engine import (GenParams, LlamaEngine,
+                                     cache_for_model)
+    has_gpu = torch.cuda.is_available()
+    device = "cuda:0" if has_gpu else "cpu"
+    dtype = torch.bfloat16 if has_gpu else torch.float32
+
+    def sync():
+        if has_gpu:
+            torch.cuda.synchronize()
+
+    table = []
+    widths = [int(w) for w in args.layer_sizes.split(",")] if has_gpu \
+        else [256]
+    users = args.users if has_gpu else 2
+    p_len, d_len = (2048, args.prompt_len) if has_gpu else (32, 16)
+    for width in widths:
+        for name, cfg in layer_stacks(width):
+            model = build_model(cfg, device=device, dtype=dtype, seed=1,
+                                fast_init=has_gpu)
+            ctx = max(p_len, d_len + args.warmup + args.steps + 16) + 16
+            kv = cache_for_model(
+                cfg, n_pages=(users + 2) * (ctx // 16 + 2),
+                max_slots=users + 2, max_ctx=ctx, device=device, dtype=dtype)
+            eng = LlamaEngine(model, kv, max_batch=users,
+                              prefill_chunk=2 * p_len)
+            g = torch.Generator().manual_seed(7)
+
+            def prompt(n):
+                return torch.randint(0, cfg.vocab, (n,), generator=g).tolist()
+
+            times = []
+            for _ in range(4):
+                for _ in range(2):
+                    eng.submit(prompt(p_len), GenParams(max_tokens=0))
+                sync()
+                t0 = time.monotonic()
+                while eng.has_work():
+                    eng.step()
+                sync()
+                times.append(time.monotonic() - t0)
+            prefill = 2 * p_len / min(times[1:])
+            for _ in range(users):
+                eng.submit(prompt(d_len), GenParams(max_tokens=10 ** 9))
+            while eng.waiting:
+                eng.step()
+            for _ in range(args.warmup):
+                eng.step()
+            sync()
+            t0 = time.monotonic()
+            for _ in range(args.steps):
+                eng.step()
+            sync()
+            dt = time.monotonic() - t0
+            table.append({
+                "stack": name, "width": width,
+                "layers": 4,
+                "weights_mb": round(model.weight_bytes() / 2 ** 20),
+                "prefill_tokens_per_s": round(prefill),
+                "decode_tokens_per_s": round(users * args.steps / dt),
+                "decode_ms_per_step": round(dt / args.steps * 1e3, 3)})
+            print(json.dumps(table[-1]), file=sys.stderr, flush=True)
+            del eng, kv, model
+            if has_gpu:
+                torch.cuda.empty_cache()
+    print(json.dumps({
+        "metric": "layer_stack_tokens_per_sec", "unit": "tokens/s",
+        "dtype": "bf16" if has_gpu else "fp32", "data": "random weights",
+        "config": {"users": users, "prefill": f"2x{p_len}",
+                   "decode_prompt": d_len}, "results": table}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -182,7 +283,16 @@ def main():
                     help="benchmark through the full dispatcher stack "
                          "(HTTP + scheduler + UDS workers) instead of "
                          "the engine-only kernel metric")
+    ap.add_argument("--layers", action="store_true",
+                    help="prefill and decode throughput of Rinitar layer "
+                         "stacks beside Llama stacks of equal size")
+    ap.add_argument("--layer-sizes", type=str, default="2048,4096",
+                    help="widths for --layers, of 2048, 4096")
     args = ap.parse_args()
+
+    if args.layers:
+        run_layers(args)
+        return
 
     if args.stack:
         run_stack(args)

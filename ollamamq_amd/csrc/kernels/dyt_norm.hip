@@ -276,6 +276,7 @@ extern "C" int polynorm(
             else if (F <= 4096) PN_GO(T, 8, 2);                            \
             else if (F <= 8192) PN_GO(T, 8, 4);                            \
             else if (F <= 16384) PN_GO(T, 8, 8);                           \
+            else if (F <= 24576) PN_GO(T, 8, 12);                          \
             else PN_GO(T, 8, 0);                                           \
         } while (0)
     if (f32) PN_TYPE(float); else PN_TYPE(bf16);

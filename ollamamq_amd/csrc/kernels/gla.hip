@@ -43,17 +43,16 @@ __global__ __launch_bounds__(256) void k_gla_step(
     const int h = blockIdx.y, tid = threadIdx.x;
     const int t0 = spans ? spans[blockIdx.x * 2] : blockIdx.x;
     const int nt = spans ? spans[blockIdx.x * 2 + 1] : 1;
-    const int nv = V / VEC;             // threads across a state row
+    const int nv = min(V / VEC, 256);   // threads across a state row
     const int RG = 256 / nv;            // state rows in flight
-    const int vt = tid % nv, rg = tid / nv;
-    const bool live = rg < RG;
+    const int rg = tid / nv;
     extern __shared__ __attribute__((aligned(16))) float sm[];
     float* q_s = sm;                    // [D]
     float* k_s = q_s + D;
     float* a_s = k_s + D;
     float* o_s = a_s + D;               // [RG][V]
     float* r_s = o_s + RG * V;          // [4]
-    float* S = state + ((int64_t)slot[t0] * H + h) * D * V + vt * VEC;
+    float* Sh = state + ((int64_t)slot[t0] * H + h) * D * V;
     bool fresh = pos[t0] == 0;
     for (int t = t0; t < t0 + nt; ++t) {
         const T* row = p + (int64_t)t * in.ld;
@@ -68,7 +67,8 @@ __global__ __launch_bounds__(256) void k_gla_step(
             a_s[d] = expf(log_alpha(z, inv_tau));
         }
         __syncthreads();
-        if (live) {
+        for (int vt = rg < RG ? tid % nv : V; vt * VEC < V; vt += nv) {
+            float* S = Sh + vt * VEC;
             float v[VEC], acc[VEC] = {};
             ldv<VEC>(row + in.ov + h * V + vt * VEC, v);
             #pragma unroll 8
@@ -111,12 +111,6 @@ __global__ __launch_bounds__(256) void k_gla_step(
     }
 }
 
-static bool gla_sizes_ok(int D, int V, int rank)
-{
-    return D >= 1 && D <= 512 && V >= 1 && rank >= 1 && rank <= 256
-           && (V % 4 == 0 ? V <= 1024 : V <= 256);
-}
-
 extern "C" int gla_step(
     int f32, void* out, const void* p, int64_t ld, int oq, int ok, int ov,
     int og, int ou, int rank, const void* a2, const void* a2_b,
@@ -124,13 +118,14 @@ extern "C" int gla_step(
     const void* spans, int n, int H, int D, int V, float scale,
     float inv_tau, float eps, hipStream_t stream)
 {
-    if (!gla_sizes_ok(D, V, rank)) return (int)hipErrorInvalidValue;
     // a vector load of v needs aligned columns
     const bool v4 = V % 4 == 0 && ov % 4 == 0 && ld % 4 == 0;
-    if (!v4 && V > 256) return (int)hipErrorInvalidValue;
     GlaIn in{ld, oq, ok, ov, og, ou, rank};
-    const int rg = 256 / (v4 ? V / 4 : V);
-    const int lds = (3 * D + rg * V + 4) * 4;
+    const int nv = v4 ? V / 4 : V;
+    const int rg = nv < 256 ? 256 / nv : 1;
+    const int64_t lds = ((int64_t)3 * D + (int64_t)rg * V + 4) * 4;
+    if (D < 1 || V < 1 || rank < 1 || lds > 64 * 1024)
+        return (int)hipErrorInvalidValue;
     dim3 grid(n, H);
     #define GS_GO(T, VV)                                                   \
         k_gla_step<T, VV><<<grid, 256, lds, stream>>>(                     \
@@ -460,7 +455,7 @@ extern "C" int64_t gla_scratch_floats(int n_chunks, int H, int D)
 
 // Portions of whole sequences in chunks of 64 rows.  chunks int32 [n, 2]
 // (first row, rows), a sequence's chunks in a run; seqs int32 [m, 2] (first
-// chunk, chunks).  Rows row_base .. row_base + rows - 1 are covered.
+// chunk, chunks); D <= 512, rank <= 256.  Rows row_base .. row_base + rows - 1 are covered.
 extern "C" int gla_chunks(
     int f32, void* out, void* scr, void* o_scr, const void* p, int64_t ld,
     int oq, int ok, int ov, int og, int ou, int rank, const void* a2,
@@ -469,7 +464,8 @@ extern "C" int gla_chunks(
     int n_seqs, int row_base, int rows, int H, int D, int V, float scale,
     float inv_tau, float eps, hipStream_t stream)
 {
-    if (!gla_sizes_ok(D, V, rank)) return (int)hipErrorInvalidValue;
+    if (D < 1 || V < 1 || rank < 1 || D > 512 || rank > 256)
+        return (int)hipErrorInvalidValue;
     GlaIn in{ld, oq, ok, ov, og, ou, rank};
     const int Dp = (D + 15) & ~15;
     const int lds_a = (5 * CH * DS + 4 * DB + CH * rank) * 4;

@@ -152,21 +152,20 @@ RINITAR_PRESETS = {
         RinitarLayerSpec("latent_attention", 3, 16, 24, kv_rank=40,
                          scale=0.21, ff=288),
         "glgl", loop=(1, 3, 2), max_ctx=2048)),
-    # layers the size of an 8B model's: width 4096, equal parts of both
-    # mixers, one pass
+    # layers the size of an 8B and of a 1B model's, one pass, three
+    # recurrent layers for every attention layer
     "rinitar-8b": RinitarConfig(name="rinitar-8b", **_stack(
         4096, 128256,
-        RinitarLayerSpec("gla", 16, 128, 256, tau=16.0, ff=14336),
+        RinitarLayerSpec("gla", 16, 128, 256, tau=16.0, ff=21504),
         RinitarLayerSpec("latent_attention", 32, 128, 128, kv_rank=512,
-                         scale=128 ** -0.5, ff=14336),
-        "gggl" * 10)),
-    # width 2048: a 1B-class stack
+                         scale=128 ** -0.5, ff=21504),
+        "gggl" * 8)),
     "rinitar-1b": RinitarConfig(name="rinitar-1b", **_stack(
         2048, 128256,
-        RinitarLayerSpec("gla", 8, 128, 256, tau=16.0, ff=8192),
+        RinitarLayerSpec("gla", 8, 128, 256, tau=16.0, ff=12288),
         RinitarLayerSpec("latent_attention", 16, 128, 128, kv_rank=512,
-                         scale=128 ** -0.5, ff=8192),
-        "gggl" * 5)),
+                         scale=128 ** -0.5, ff=12288),
+        "gggl" * 4)),
 }
 
 
@@ -188,11 +187,12 @@ class RinitarLayer:
         if s.type == "gla":
             a1 = get(mix + "a1", (None, W))
             rank = a1.shape[0]
-            cols = [get(mix + "q", (qk, W)), get(mix + "k", (qk, W)),
-                    get(mix + "v", (v, W)), get(mix + "g", (v, W)), a1]
+            # values first, so that their rows stay aligned
+            cols = [get(mix + "v", (v, W)), get(mix + "g", (v, W)),
+                    get(mix + "q", (qk, W)), get(mix + "k", (qk, W)), a1]
             self.gla = ops.GlaWeights(
                 heads=s.heads, dim=s.dim, vdim=s.vdim, rank=rank,
-                offsets=(0, qk, 2 * qk, 2 * qk + v, 2 * qk + 2 * v),
+                offsets=(2 * v, 2 * v + qk, 0, v, 2 * v + 2 * qk),
                 a2=put(get(mix + "a2", (qk, rank))).contiguous(),
                 a2_b=vec(mix + "a2.b", qk, mean=2.0, spread=1.0),
                 norm=vec(mix + "norm", s.vdim, mean=1.0, spread=0.1),

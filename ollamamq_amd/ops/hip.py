@@ -997,16 +997,18 @@ def latent_attention(q, cache, run, w, slot_ids, positions, meta):
 
 
 GLA_STEP_TOKENS = 4       # portions up to this walk token by token
+GLA_CHUNK_MAX = (512, 256)   # key width and low rank the chunk kernels take
 
 
-def _gla_plan(meta, dev):
-    plan = getattr(meta, "_gla_plan", None)
+def _gla_plan(meta, dev, step_tokens):
+    key = f"_gla_plan_{step_tokens}"
+    plan = getattr(meta, key, None)
     if plan is not None:
         return plan
     _, q_lens, _ = meta.layout()
     nd = meta.n_single
     i, row, spans = nd, nd, []
-    while i < len(q_lens) and q_lens[i] <= GLA_STEP_TOKENS:
+    while i < len(q_lens) and q_lens[i] <= step_tokens:
         spans.append((row, q_lens[i]))
         row += q_lens[i]
         i += 1
@@ -1018,7 +1020,7 @@ def _gla_plan(meta, dev):
     t32 = lambda x: torch.tensor(x, dtype=torch.int32).to(dev) \
         if x else None
     plan = (t32(spans), t32(chunks), t32(seqs), base, row - base)
-    meta._gla_plan = plan
+    setattr(meta, key, plan)
     return plan
 
 
@@ -1040,7 +1042,9 @@ def gla(p, w, state, slot_ids, positions, meta):
                "gla_step")
     if meta.one_each:
         return out
-    spans, chunks, seqs, base, rows = _gla_plan(meta, p.device)
+    chunked = D <= GLA_CHUNK_MAX[0] and w.rank <= GLA_CHUNK_MAX[1]
+    spans, chunks, seqs, base, rows = _gla_plan(
+        meta, p.device, GLA_STEP_TOKENS if chunked else 1 << 62)
     if spans is not None:
         _check(_lib.gla_step(f32, _p(out), *head, _p(spans),
                              spans.shape[0], *tail), "gla_step")
