@@ -1,0 +1,747 @@
+"""The Rinitar design against a plain float64 statement of its equations
+(rinitar_oracle.py): every mechanism alone, then whole models fed in
+portions, in batches and through reused memory, then generation.
+
+The same tests run on the CPU and, in fp32 and bf16, on the GPU kernels.
+"""
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+from safetensors.torch import save_file
+
+import rinitar_oracle as oracle
+from ollamamq_amd.engine import (GenParams, HybridCache, LlamaEngine,
+                                 cache_for_model)
+from ollamamq_amd.engine.kvcache import RunStore
+from ollamamq_amd.engine.trace import make_engine
+from ollamamq_amd.models import (RinitarConfig, build_model,
+                                 config_from_folder)
+from ollamamq_amd.ops import interface as ops
+from ollamamq_amd.ops.interface import AttnMeta
+
+REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+F32, BF16, F64 = torch.float32, torch.bfloat16, torch.float64
+GPU = pytest.mark.gpu
+WHERE = [pytest.param(("cpu", F32), id="cpu"),
+         pytest.param(("cuda:0", F32), id="gpu-f32", marks=GPU),
+         pytest.param(("cuda:0", BF16), id="gpu-bf16", marks=GPU)]
+EXACT = WHERE[:2]
+where = pytest.mark.parametrize("where", WHERE)
+exact = pytest.mark.parametrize("where", EXACT)
+
+
+def tol(dtype, f32, bf16):
+    return bf16 if dtype == BF16 else f32
+
+
+def rel(got, want):
+    """Root mean square error over the root mean square of `want`."""
+    got, want = got.to("cpu", F64), want.to(F64)
+    return ((got - want).pow(2).mean() / want.pow(2).mean()).sqrt().item()
+
+
+def gla_layer(heads, dim, vdim, tau, ff=None):
+    return {"type": "gla", "mixer": {"heads": heads, "dim": dim,
+                                     "vdim": vdim, "tau": tau},
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def latent_layer(heads, dim, vdim, rank, scale, ff=None):
+    return {"type": "latent_attention",
+            "mixer": {"heads": heads, "dim": dim, "vdim": vdim,
+                      "kv_rank": rank, "scale": scale},
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def config(width, vocab, layers, loop=None, eps=1e-5):
+    return {"architecture": "Rinitar", "width": width, "vocab": vocab,
+            "layers": layers, "norm": {"eps": eps},
+            "loop": dict(zip(("start", "stop", "times"), loop))
+            if loop else None}
+
+
+MODELS = {
+    # both mixers, loop over a pair, unequal sizes everywhere
+    "mixed": config(128, 200, [
+        gla_layer(3, 24, 40, 4.0, 160),
+        latent_layer(5, 16, 24, 56, 0.31, 96),
+        gla_layer(2, 40, 16, 1.0),
+        latent_layer(2, 48, 32, 24, 0.1, 160)], loop=(1, 3, 2)),
+    # sizes that fit no tile: odd widths, one head, other eps
+    "odd": config(90, 131, [
+        latent_layer(1, 18, 10, 30, 0.5, 50),
+        gla_layer(1, 22, 14, 2.5, 70),
+        gla_layer(3, 9, 7, 16.0, 34)], loop=(0, 3, 1), eps=1e-3),
+    "only-gla": config(64, 96, [gla_layer(2, 64, 64, 16.0, 64),
+                                gla_layer(4, 16, 32, 8.0)]),
+    "only-latent": config(192, 96, [latent_layer(20, 64, 64, 128, 0.125, 128),
+                                    latent_layer(3, 72, 136, 40, 0.3)],
+                          loop=(1, 2, 3)),
+}
+A1_RANK = {"mixed": 8, "odd": 5, "only-gla": 16, "only-latent": 1}
+
+
+@pytest.fixture(scope="module")
+def models(tmp_path_factory):
+    out = {}
+    for name, cfg in MODELS.items():
+        d = tmp_path_factory.mktemp(name)
+        w = oracle.random_weights(cfg, seed=len(name), a1_rank=A1_RANK[name])
+        (d / "config.json").write_text(json.dumps(cfg))
+        save_file({k: t.contiguous() for k, t in w.items()},
+                  str(d / "model.safetensors"))
+        out[name] = (str(d), cfg, w)
+    return out
+
+
+_ORACLE = {}
+
+
+def expected(models, name, tokens):
+    key = (name, tuple(tokens))
+    if key not in _ORACLE:
+        _, cfg, w = models[name]
+        _ORACLE[key] = oracle.run(cfg, w, tokens)[0]
+    return _ORACLE[key]
+
+
+def tokens_for(name, n, seed=0):
+    g = torch.Generator().manual_seed(seed * 1000 + n)
+    return torch.randint(0, MODELS[name]["vocab"], (n,), generator=g).tolist()
+
+
+def run_portions(eng, tokens, portions, before=()):
+    """Feed one stream in portions; logits at every place."""
+    s = eng.open_stream()
+    got, at = [], 0
+    for n in portions:
+        part = tokens[at:at + n]
+        got.append(eng.feed([(s, part, list(range(len(part))))]).cpu())
+        at += n
+    assert at == len(tokens)
+    eng.close_stream(s)
+    return torch.cat(got)
+
+
+def model_tol(dtype):
+    return tol(dtype, 2e-5, 0.06)
+
+
+def cut(n, size):
+    return [size] * (n // size) + ([n % size] if n % size else [])
+
+
+# ---------------------------------------------------------------- mechanisms
+
+def dyt_params(W, g, dev):
+    w, b = 1 + 0.2 * torch.randn(W, generator=g), \
+        0.1 * torch.randn(W, generator=g)
+    alpha = 0.7 + 0.2 * float(torch.rand((), generator=g))
+    return ops.DyT(w.to(dev), b.to(dev), alpha)
+
+
+def o_dyt(x, p):
+    return oracle.dyt(x.to(F64), p.w.to("cpu", F64), p.b.to("cpu", F64),
+                      p.alpha)
+
+
+def meta_for(dev, slots, q_lens, kv_lens, n_decode=0):
+    cu = [0]
+    for n in q_lens:
+        cu.append(cu[-1] + n)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    mode = ("decode" if all(n == 1 for n in q_lens)
+            else "mixed" if n_decode else "prefill")
+    return AttnMeta(mode=mode, slot_ids=i32(slots), seq_lens=i32(kv_lens),
+                    cu_q=i32(cu), logits_idx=None, max_q=max(q_lens),
+                    max_kv=max(kv_lens), n_decode=n_decode)
+
+
+def rows_of(dev, slots, q_lens, kv_lens):
+    pos = [p for n, kv in zip(q_lens, kv_lens) for p in range(kv - n, kv)]
+    sl = [s for s, n in zip(slots, q_lens) for _ in range(n)]
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    return i32(sl), i32(pos)
+
+
+@where
+@pytest.mark.parametrize("W", [64, 90, 2100])
+def test_dyt_chain_and_small_arguments(where, W):
+    dev, dt = where
+    g = torch.Generator().manual_seed(W)
+    post, pre = dyt_params(W, g, dev), dyt_params(W, g, dev)
+    # magnitudes from 1e-4 to 30 pass every branch of the tanh
+    mag = torch.logspace(-4, 1.5, W)
+    x = torch.randn(9, W, generator=g) * mag
+    y = (torch.randn(9, W, generator=g) * mag.flip(0)).to(dt)
+    emb = torch.zeros(1, W, dtype=dt, device=dev)
+    xo, h = ops.dyt_residual(x.to(dev), y.to(dev), post, pre, embed=emb)
+    want_x = x.to(F64) + o_dyt(y, post)
+    assert rel(xo, want_x) < 1e-6
+    assert rel(h, o_dyt(want_x, pre)) < tol(dt, 1e-6, 4e-3)
+    small = (torch.randn(4, W, generator=g) * 1e-3)
+    flat = ops.DyT(pre.w, torch.zeros_like(pre.b), pre.alpha)
+    _, h = ops.dyt_residual(small.to(dev), None, None, flat, embed=emb)
+    assert rel(h, o_dyt(small, flat)) < tol(dt, 1e-6, 4e-3)
+    # selected rows only
+    pick = torch.tensor([7, 2, 2], device=dev)
+    _, h = ops.dyt_residual(x.to(dev), y.to(dev), post, pre, embed=emb,
+                            rows=pick, need_x=False)
+    assert rel(h, o_dyt(want_x, pre)[[7, 2, 2]]) < tol(dt, 1e-6, 4e-3)
+
+
+@where
+def test_token_shift_over_portions(where):
+    """A sequence's shift reaches across portions, starts from zero, and
+    ignores what its slot held before; neighbours in the batch stay out."""
+    dev, dt = where
+    W, n = 72, 37
+    g = torch.Generator().manual_seed(3)
+    pre = dyt_params(W, g, dev)
+    mix = torch.rand(W, generator=g)
+    emb = torch.randn(50, W, generator=g).to(BF16)
+    toks = [torch.randint(0, 50, (n,), generator=g) for _ in range(2)]
+    want = [oracle.token_shift(o_dyt(emb[t], pre), mix.to(F64)) for t in toks]
+    prev = torch.full((3, W), 9.0, device=dev)
+    e = emb.to(dt).to(dev)
+    got = [[], []]
+    at = [0, 0]
+    for lens in ((1, 2), (5, 1), (1, 1), (20, 3), (10, 30)):
+        kv = [a + b for a, b in zip(at, lens)]
+        meta = meta_for(dev, [2, 0], lens, kv)
+        sl, pos = rows_of(dev, [2, 0], lens, kv)
+        t = torch.cat([toks[i][at[i]:kv[i]] for i in (0, 1)]).int().to(dev)
+        _, h = ops.dyt_residual(
+            None, None, None, pre,
+            ops.TokenShift(mix.to(dev), prev, sl, pos, meta), embed=e,
+            tokens=t)
+        got[0].append(h[:lens[0]].cpu())
+        got[1].append(h[lens[0]:].cpu())
+        at = kv
+    for i in (0, 1):
+        assert rel(torch.cat(got[i]), want[i]) < tol(dt, 1e-6, 4e-3)
+
+
+@where
+@pytest.mark.parametrize("F", [34, 320, 5000, 17000, 30000])
+def test_polynorm(where, F):
+    dev, dt = where
+    g = torch.Generator().manual_seed(F)
+    z = (torch.randn(3, F, generator=g) * torch.tensor([[1e-3], [1.], [9.]])
+         ).to(dt)
+    coef = (0.7, -0.4, 0.2, 0.3)
+    got = ops.polynorm(z.to(dev), coef, 1e-4)
+    want = oracle.polynorm(z.to(F64), coef, 1e-4)
+    assert rel(got, want) < tol(dt, 2e-6, 4e-3)
+    if dev != "cpu" and dt == BF16:
+        parts = torch.randn(4, 3, F, generator=g)
+        got = ops.polynorm(ops.Partials(parts.to(dev)), coef, 1e-4)
+        want = oracle.polynorm(parts.to(F64).sum(0), coef, 1e-4)
+        assert rel(got, want) < 4e-3
+
+
+def latent_case(dev, dt, H, D, V, R, scale, kv, seed=0, slots=3):
+    g = torch.Generator().manual_seed(seed)
+    uk = (torch.randn(H, D, R, generator=g) / R ** 0.5).to(dt)
+    uv = (torch.randn(H, V, R, generator=g) / R ** 0.5).to(dt)
+    w = ops.LatentWeights(uk.to(dev), uk.transpose(1, 2).contiguous().to(dev),
+                          uv.to(dev), scale)
+    cache = HybridCache([RunStore(latent=R)], n_pages=3 * (kv // 16 + 2),
+                        max_slots=slots, max_ctx=kv + 16, device=dev,
+                        dtype=dt)
+    d = torch.randn(kv, R, generator=g).to(dt)
+    nw = 1 + 0.2 * torch.randn(R, generator=g)
+    return g, uk, uv, w, cache, d, nw
+
+
+def o_latent(d, nw, eps, uk, uv, q, scale):
+    c = oracle.unit_rms(d.to(F64), eps) * nw.to(F64)
+    out = []
+    for h in range(uk.shape[0]):
+        out.append(oracle.softmax_attention(
+            q[:, h].to(F64), c @ uk[h].to(F64).T, c @ uv[h].to(F64).T,
+            scale))
+    return torch.cat(out, -1)
+
+
+LATENT_SIZES = [(4, 32, 40, 88), (1, 18, 10, 30), (20, 64, 48, 128),
+                (3, 72, 136, 40), (2, 256, 256, 520), (2, 264, 40, 72)]
+
+
+@where
+@pytest.mark.parametrize("size", LATENT_SIZES, ids=str)
+@pytest.mark.parametrize("form", ["whole", "portions", "single"])
+def test_latent_attention(where, size, form):
+    """Whole prompts, portions and single tokens over a context whose length
+    is no multiple of anything, with pages handed out in a mixed order."""
+    dev, dt = where
+    H, D, V, R = size
+    kv = 150 if form == "single" else 333
+    scale = 1.3 * D ** -0.5
+    g, uk, uv, w, cache, d, nw = latent_case(dev, dt, H, D, V, R, scale, kv)
+    q = torch.randn(kv, H, D, generator=g).to(dt)
+    want = o_latent(d, nw, 1e-5, uk, uv, q, scale)
+    other, slot = cache.alloc_slot(), cache.alloc_slot()
+    cache.ensure(other, 40)
+    lens = {"whole": [kv], "single": [1] * kv,
+            "portions": [100, 2, 2, 31, 1, 64, 17, 16, 100]}[form]
+    got, at = [], 0
+    for n in lens:
+        cache.ensure(slot, at + n)
+        cache.ensure(other, min(kv, 40 + at))
+        meta = meta_for(dev, [slot], [n], [at + n])
+        sl, pos = rows_of(dev, [slot], [n], [at + n])
+        # strided rows, as the fused projection gives them
+        buf = torch.zeros(n, H * D + 8, dtype=dt)
+        buf[:, :H * D] = q[at:at + n].view(n, -1)
+        dbuf = d[at:at + n].to(dev)
+        ops.latent_append(cache, 0, dbuf, nw.to(dev), sl, pos, 1e-5)
+        got.append(ops.latent_attention(buf.to(dev)[:, :H * D], cache, 0, w,
+                                        sl, pos, meta).cpu())
+        at += n
+    assert rel(torch.cat(got), want) < tol(dt, 3e-6, 1.2e-2)
+
+
+@where
+@pytest.mark.parametrize("n", [1, 2, 40, 300])
+def test_latent_attention_finds_far_keys(where, n):
+    """One key stands out for each query: the first, the last, both sides of
+    page, chunk and tile borders.  Missing or shifting it shows."""
+    dev, dt = where
+    H, D, V, R, kv = 2, 32, 32, 64, 700
+    g, uk, uv, w, cache, d, nw = latent_case(dev, dt, H, D, V, R, 1.0, kv, 5)
+    c = oracle.unit_rms(d.to(F64), 1e-5) * nw.to(F64)
+    marks = [0, 1, 15, 16, 17, 31, 32, 63, 64, 65, 127, 128, 129, 255, 256,
+             399]
+    slot = cache.alloc_slot()
+    cache.ensure(slot, kv)
+    sl, pos = rows_of(dev, [slot], [kv], [kv])
+    ops.latent_append(cache, 0, d.to(dev), nw.to(dev), sl, pos, 1e-5)
+    meta = meta_for(dev, [slot], [n], [kv])
+    sl, pos = rows_of(dev, [slot], [n], [kv])
+    for j0 in range(0, len(marks), n):
+        q = torch.empty(n, H, D, dtype=F64)
+        aim = [marks[(j0 + i) % len(marks)] for i in range(n)]
+        if n > 1:
+            aim[-1] = kv - 1                 # its own key
+            aim[0] = kv - n
+        for i, j in enumerate(aim):
+            for h in range(H):
+                k = uk[h].to(F64) @ c[j]
+                q[i, h] = 30.0 * k / (k @ k)
+        q = q.to(dt)
+        got = ops.latent_attention(q.view(n, -1).to(dev), cache, 0, w, sl,
+                                   pos, meta).cpu()
+        for i, j in enumerate(aim):
+            i_abs = kv - n + i
+            k_all = [c[:i_abs + 1] @ uk[h].to(F64).T for h in range(H)]
+            want = []
+            for h in range(H):
+                p = torch.softmax(k_all[h] @ q[i, h].to(F64), 0)
+                assert p[j] > 0.5, "the aimed key must stand out"
+                want.append(p @ (c[:i_abs + 1] @ uv[h].to(F64).T))
+            assert rel(got[i], torch.cat(want)) < tol(dt, 1e-5, 5e-2), (i, j)
+
+
+def gla_case(dev, dt, T, H, D, V, tau, rank, seed, shift=1.0, spread=1.0):
+    g = torch.Generator().manual_seed(seed)
+    ld = 2 * H * D + 2 * H * V + rank
+    p = torch.randn(T, ld, generator=g).to(dt)
+    a2 = (spread * torch.randn(H * D, rank, generator=g) / rank ** 0.5).to(dt)
+    b = shift + spread * torch.randn(H * D, generator=g)
+    nw = 1 + 0.2 * torch.randn(V, generator=g)
+    hd, hv = H * D, H * V
+    off = (2 * hv, 2 * hv + hd, 0, hv, 2 * hv + 2 * hd)
+    w = ops.GlaWeights(H, D, V, rank, off, a2.to(dev), b.to(dev), nw.to(dev),
+                       tau, 1e-4)
+    f = p.to(F64)
+    q = f[:, off[0]:off[0] + hd].view(T, H, D) * D ** -0.5
+    k = f[:, off[1]:off[1] + hd].view(T, H, D)
+    v = f[:, :hv].view(T, H, V)
+    gate = f[:, hv:2 * hv]
+    eye = torch.eye(rank, dtype=F64)
+    alpha = oracle.gla_decay(f[:, off[4]:], eye, a2.to(F64), b.to(F64),
+                             tau).view(T, H, D)
+    outs, states = [], []
+    for h in range(H):
+        o, S = oracle.gla_scan(q[:, h], k[:, h], v[:, h], alpha[:, h])
+        outs.append(oracle.unit_rms(o, 1e-4) * nw.to(F64))
+        states.append(S)
+    want = torch.cat(outs, -1) * gate * torch.sigmoid(gate)
+    return p, w, want, torch.stack(states)
+
+
+GLA_SIZES = [(3, 24, 40, 8), (1, 22, 14, 5), (2, 128, 256, 16),
+             (2, 64, 64, 33), (1, 200, 20, 1), (2, 9, 7, 4)]
+
+
+@where
+@pytest.mark.parametrize("size", GLA_SIZES, ids=str)
+@pytest.mark.parametrize("cuts", [[150], [64, 64, 22], [1, 2, 63, 65, 5, 14],
+                                  [4, 3, 2, 1, 17, 123]], ids=str)
+def test_gla_portions_carry_the_state(where, size, cuts):
+    dev, dt = where
+    H, D, V, rank = size
+    T = sum(cuts)
+    p, w, want, last = gla_case(dev, dt, T, H, D, V, 4.0, rank, T + D)
+    state = torch.full((3, H, D, V), 7.0, device=dev)     # a used slot
+    got, at = [], 0
+    for n in cuts:
+        meta = meta_for(dev, [1], [n], [at + n])
+        sl, pos = rows_of(dev, [1], [n], [at + n])
+        got.append(ops.gla(p[at:at + n].to(dev), w, state, sl, pos,
+                           meta).cpu())
+        at += n
+    assert rel(torch.cat(got), want) < tol(dt, 1e-5, 6e-3)
+    assert rel(state[1], last) < 1e-5
+    assert bool((state[0] == 7).all() and (state[2] == 7).all())
+
+
+@where
+@pytest.mark.parametrize("tau,shift,spread", [
+    (1.0, 0.0, 12.0),      # some channels forget within a token
+    (1.0, -30.0, 1.0),     # all do: sums of decay far below exp's range
+    (64.0, 8.0, 1.0),      # nothing is forgotten
+    (1.0, 20.0, 25.0),     # both at once
+], ids=str)
+def test_gla_extreme_decay(where, tau, shift, spread):
+    """Chunked sums must neither overflow nor lose what a plain recurrence
+    keeps when channels forget at very different rates."""
+    dev, dt = where
+    p, w, want, last = gla_case(dev, dt, 200, 2, 48, 32, tau, 6, 11, shift,
+                                spread)
+    state = torch.zeros(1, 2, 48, 32, device=dev)
+    meta = meta_for(dev, [0], [200], [200])
+    sl, pos = rows_of(dev, [0], [200], [200])
+    got = ops.gla(p.to(dev), w, state, sl, pos, meta)
+    assert torch.isfinite(got).all() and torch.isfinite(state).all()
+    assert rel(got, want) < tol(dt, 3e-5, 6e-3)
+    assert rel(state[0], last) < 3e-5
+
+
+@where
+def test_gla_remembers_a_far_token(where):
+    """One loud key far back, asked for across chunk and portion borders in
+    channels that do not decay; everything else is quiet."""
+    dev, dt = where
+    T, H, D, V, rank = 330, 1, 32, 32, 4
+    for far in (0, 1, 15, 16, 63, 64, 130):
+        p, w, _, _ = gla_case(dev, dt, T, H, D, V, 64.0, rank, far,
+                              shift=12.0, spread=0.0)
+        hd, hv = H * D, H * V
+        f = p.clone()
+        f[:, 2 * hv + hd:2 * hv + 2 * hd] *= 0.01            # keys
+        f[:, 2 * hv:2 * hv + hd] = f[far, 2 * hv:2 * hv + hd]  # queries
+        f[far, 2 * hv + hd:2 * hv + 2 * hd] = \
+            f[far, 2 * hv:2 * hv + hd] * 3
+        f64 = f.to(F64)
+        q = f64[:, 2 * hv:2 * hv + hd] * D ** -0.5
+        k = f64[:, 2 * hv + hd:2 * hv + 2 * hd]
+        v = f64[:, :hv]
+        a = torch.sigmoid(w.a2_b.cpu().to(F64)) ** (1 / 64.0)
+        o, _ = oracle.gla_scan(q, k, v, a.expand(T, D))
+        cosine = torch.cosine_similarity(o[-1], v[far], dim=0)
+        assert cosine > 0.9, "the far token must stand out"
+        gate = f64[:, hv:2 * hv]
+        want = oracle.unit_rms(o, 1e-4) * w.norm.cpu().to(F64) * gate \
+            * torch.sigmoid(gate)
+        state = torch.zeros(1, H, D, V, device=dev)
+        got, at = [], 0
+        for n in (100, 2, 62, 1, 130, 1, 34):
+            meta = meta_for(dev, [0], [n], [at + n])
+            sl, pos = rows_of(dev, [0], [n], [at + n])
+            got.append(ops.gla(f[at:at + n].to(dev), w, state, sl, pos,
+                               meta).cpu())
+            at += n
+        assert rel(torch.cat(got), want) < tol(dt, 1e-5, 6e-3), far
+
+
+@GPU
+def test_argmax_of_fp32_logits_is_exact():
+    """Two logits that agree in bfloat16 are told apart."""
+    x = torch.full((5, 4096), -1.0)
+    win = [3, 4095, 0, 2048, 777]
+    for r, c in enumerate(win):
+        x[r, (c + 9) % 4096] = 1.0
+        x[r, c] = 1.0 + 1e-4
+    got = ops.sample(x.cuda(), 0.0, 0, 1.0)
+    assert got.tolist() == win
+
+
+# --------------------------------------------------------------- whole models
+
+@where
+@pytest.mark.parametrize("name", list(MODELS))
+def test_layers_and_logits_of_a_prompt(models, where, name):
+    dev, dt = where
+    toks = tokens_for(name, 140)
+    eng = make_engine(models[name][0], dt, 192, dev)
+    got = run_portions(eng, toks, [140])
+    assert rel(got, expected(models, name, toks)) < model_tol(dt)
+
+
+@where
+@pytest.mark.parametrize("name", list(MODELS))
+@pytest.mark.parametrize("size", [1, 2, 3, 17, 64, 65])
+def test_portions_agree_with_the_whole(models, where, name, size):
+    dev, dt = where
+    toks = tokens_for(name, 140)
+    eng = make_engine(models[name][0], dt, 192, dev)
+    got = run_portions(eng, toks, cut(140, size))
+    assert rel(got, expected(models, name, toks)) < model_tol(dt)
+
+
+@where
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+def test_mixed_batches_and_reused_memory(models, where, name):
+    """Four slots and just enough pages, seven requests of unequal length:
+    prompts' portions beside decoded tokens, pauses, freed pages and slots
+    taken over by the next request."""
+    dev, dt = where
+    g = torch.Generator().manual_seed(4)
+    reqs = [tokens_for(name, n, i) for i, n in
+            enumerate((90, 1, 33, 17, 64, 2, 50))]
+    eng = make_engine(models[name][0], dt, 96 + 48 + 64 + 64, dev)
+    waiting, live, got = list(range(7)), {}, {i: [] for i in range(7)}
+    at = [0] * 7
+    while waiting or live:
+        while waiting and len(live) < 4 and (
+                len(live) < 3 or eng.kv.free_page_count() >= 6):
+            i = waiting.pop(0)
+            live[i] = eng.open_stream()
+        parts, who = [], []
+        for i, s in live.items():
+            if torch.rand((), generator=g) < 0.2 and len(live) > 1:
+                continue                                  # left out this time
+            left = len(reqs[i]) - at[i]
+            n = min(left, [1, 1, 2, 5, 16, 31][
+                int(torch.randint(0, 6, (), generator=g))])
+            parts.append((s, reqs[i][at[i]:at[i] + n], list(range(n))))
+            who.append((i, n))
+        if not parts:
+            continue
+        out = eng.feed(parts).cpu()
+        for i, n in who:
+            got[i].append(out[:n])
+            out = out[n:]
+            at[i] += n
+            if at[i] == len(reqs[i]):
+                eng.close_stream(live.pop(i))
+    for i, toks in enumerate(reqs):
+        assert rel(torch.cat(got[i]), expected(models, name, toks)) \
+            < model_tol(dt), i
+    assert eng.kv.free_page_count() == eng.kv.n_pages
+
+
+@where
+def test_long_decoding(models, where):
+    dev, dt = where
+    toks = tokens_for("mixed", 300)
+    eng = make_engine(models["mixed"][0], dt, 320, dev)
+    got = run_portions(eng, toks, [7] + [1] * 293)
+    assert rel(got[200:], expected(models, "mixed", toks)[200:]) \
+        < model_tol(dt)
+
+
+@where
+def test_batch_neighbours_do_not_matter(models, where):
+    """A stream's logits beside others are those it has alone."""
+    dev, dt = where
+    name = "mixed"
+    toks, noise = tokens_for(name, 70), tokens_for(name, 70, 9)
+    want = run_portions(make_engine(models[name][0], dt, 256, dev), toks,
+                        [40, 1, 2, 20, 1, 1, 5])
+    eng = make_engine(models[name][0], dt, 256, dev)
+    a, b, c = (eng.open_stream() for _ in range(3))
+    got, at = [], 0
+    for i, n in enumerate([40, 1, 2, 20, 1, 1, 5]):
+        other = [(b, noise[2 * i:2 * i + 2], []),
+                 (c, noise[i:i + 1], [0])]
+        out = eng.feed([other[1], (a, toks[at:at + n], list(range(n))),
+                        other[0]])
+        got.append(out[1:].cpu())
+        at += n
+    assert rel(torch.cat(got), want) < tol(dt, 1e-5, 2e-2)
+
+
+@where
+def test_first_tokens(models, where):
+    """Sequences of one and two tokens, decoded from nothing and prefilled."""
+    dev, dt = where
+    for name in MODELS:
+        toks = tokens_for(name, 3)
+        want = expected(models, name, toks)
+        for cuts in ([1, 1, 1], [2, 1], [3], [1, 2]):
+            eng = make_engine(models[name][0], dt, 64, dev)
+            got = run_portions(eng, toks, cuts)
+            assert rel(got, want) < model_tol(dt), (name, cuts)
+
+
+def generate(eng, prompts, n):
+    seqs = [eng.seqs[eng.submit(p, GenParams(max_tokens=n))] for p in prompts]
+    for _ in range(2000):
+        if not eng.has_work():
+            break
+        eng.step()
+    assert not eng.has_work()
+    return [list(s.generated) for s in seqs]
+
+
+@exact
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+def test_greedy_generation(models, where, name):
+    """Through submit/step: admission, chunked prompts, mixed steps, the
+    pipelined decode, slots that are freed and taken again.  Every token is
+    the oracle's argmax (or a tie within rounding)."""
+    dev, dt = where
+    path, cfg, w = models[name]
+    rc = config_from_folder(path)
+    kv = cache_for_model(rc, n_pages=40, max_slots=3, max_ctx=160,
+                         device=dev, dtype=dt)
+    eng = LlamaEngine(build_model(rc, device=dev, dtype=dt), kv, max_batch=3,
+                      prefill_chunk=24)
+    prompts = [tokens_for(name, n, i) for i, n in enumerate((5, 61, 1, 30))]
+    out = generate(eng, prompts, 12)
+    for p, o in zip(prompts, out):
+        assert len(o) == 12
+        lg = oracle.run(cfg, w, p + o[:-1])[0][len(p) - 1:]
+        for step, tok in zip(lg, o):
+            assert step.max() - step[tok] < 1e-4
+    assert kv.free_page_count() == 40
+
+
+@GPU
+def test_graph_replay_equals_eager(models):
+    """Captured decode with batch padding and host work between replays
+    against the same steps without graphs."""
+    path = models["mixed"][0]
+    rc = config_from_folder(path)
+
+    def run(graphs):
+        kv = cache_for_model(rc, n_pages=64, max_slots=6, max_ctx=160,
+                             device="cuda:0", dtype=F32)
+        eng = LlamaEngine(build_model(rc, device="cuda:0", dtype=F32), kv,
+                          max_batch=6)
+        eng.use_graphs = eng.use_pipeline = graphs
+        if graphs:
+            eng.warm_graphs()
+        return generate(eng, [tokens_for("mixed", n, n) for n in
+                              (3, 20, 9, 14, 30)], 25)
+
+    assert run(True) == run(False)
+
+
+@where
+def test_preset_runs(where):
+    dev, dt = where
+    from ollamamq_amd.models import PRESETS
+    cfg = PRESETS["rinitar-tiny"]
+    kv = cache_for_model(cfg, n_pages=32, max_slots=2, max_ctx=128,
+                         device=dev, dtype=dt)
+    eng = LlamaEngine(build_model(cfg, device=dev, dtype=dt, seed=3), kv,
+                      max_batch=2)
+    out = generate(eng, [[1, 2, 3], [4] * 20], 5)
+    assert all(len(o) == 5 for o in out)
+    assert len(eng.embed([1, 2, 3])) == cfg.width
+
+
+# ------------------------------------------------------------ loading, runner
+
+def test_loop_order():
+    cfg = RinitarConfig.from_json(MODELS["mixed"])
+    assert cfg.runs == [0, 1, 2, 1, 2, 3] == oracle.layer_order(
+        MODELS["mixed"])
+    assert len(cfg.run_stores()) == 6
+
+
+def test_bad_checkpoints_are_refused(models, tmp_path):
+    path, cfg, w = models["odd"]
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    bad = dict(w)
+    bad["l1.mix.k"] = torch.zeros(3, 90, dtype=BF16)
+    save_file(bad, str(tmp_path / "model.safetensors"))
+    with pytest.raises(ValueError, match="l1.mix.k"):
+        build_model(config_from_folder(str(tmp_path)))
+    del bad["l1.mix.k"]
+    save_file(bad, str(tmp_path / "model.safetensors"))
+    with pytest.raises(KeyError, match="l1.mix.k"):
+        build_model(config_from_folder(str(tmp_path)))
+    other = json.loads(json.dumps(cfg))
+    other["layers"][0]["type"] = "something"
+    with pytest.raises(ValueError, match="something"):
+        RinitarConfig.from_json(other)
+    (tmp_path / "config.json").write_text('{"architecture": "Nothing"}')
+    with pytest.raises(ValueError, match="Nothing"):
+        config_from_folder(str(tmp_path))
+    with pytest.raises(ValueError, match="parallel"):
+        build_model(RinitarConfig.from_json(cfg), tp_size=2)
+
+
+@exact
+def test_trace_runner(models, where, tmp_path):
+    dev, _ = where
+    path = models["mixed"][0]
+    a, b = tokens_for("mixed", 30), tokens_for("mixed", 20, 1)
+    steps = [
+        {"step": 0, "entries": [{"id": "a", "tokens": a[:21], "want": [20]}],
+         "end": []},
+        {"step": 1, "entries": [{"id": "b", "tokens": b[:7], "want": [0, 6]},
+                                {"id": "a", "tokens": a[21:22],
+                                 "want": []}], "end": []},
+        {"step": 2, "entries": [{"id": "b", "tokens": b[7:8], "want": []}],
+         "end": []},
+        {"step": 3, "entries": [{"id": "b", "tokens": b[8:], "want": [11]},
+                                {"id": "a", "tokens": a[22:],
+                                 "want": [7, 3]}], "end": ["a", "b"]},
+        {"step": 4, "entries": [{"id": "a", "tokens": b, "want": [5]}],
+         "end": ["a"]},
+    ]
+    p = subprocess.run(
+        [os.path.join(REPO, "bin", "trace_run"), "--model", path, "--dtype",
+         "float32", "--out", str(tmp_path), "--max-tokens", "128",
+         "--device", dev], input="".join(json.dumps(s) + "\n"
+                                         for s in steps),
+        capture_output=True, text=True, timeout=240)
+    assert p.returncode == 0, p.stderr[-2000:]
+    done = [x for x in p.stdout.splitlines() if x.startswith("done")]
+    assert done == [f"done {i}" for i in range(5)]
+
+    def read(i):
+        data = (tmp_path / f"{i}.f32").read_bytes()
+        return torch.frombuffer(bytearray(data), dtype=F32).view(-1, 200)
+    ea, eb = expected(models, "mixed", a), expected(models, "mixed", b)
+    assert rel(read(0), ea[[20]]) < 2e-5
+    assert rel(read(1), eb[[0, 6]]) < 2e-5
+    assert not (tmp_path / "2.f32").exists()
+    assert rel(read(3), torch.stack([eb[19], ea[29], ea[25]])) < 2e-5
+    assert rel(read(4), eb[[5]]) < 2e-5
+
+
+def test_worker_serves_a_checkpoint(models):
+    import queue
+    from ollamamq_amd.engine.worker import Worker
+    from ollamamq_amd.models import PRESETS, register_checkpoint
+    if torch.cuda.is_available():
+        pytest.skip("CPU form of the worker test")
+    path = models["mixed"][0]
+    register_checkpoint(f"from-folder={path}")
+    try:
+        w = Worker(0, max_batch=2, default_ctx=128)
+        assert "from-folder" in w.available_models()
+        q = queue.Queue()
+        w.generate("from-folder", [1, 2, 3], GenParams(max_tokens=6),
+                   lambda t, done: q.put((t, done)))
+        out = []
+        while True:
+            t, done = q.get(timeout=60)
+            if done:
+                break
+            out.append(t)
+        assert len(out) == 6
+        assert w.unload("from-folder") is None
+    finally:
+        PRESETS.pop("from-folder")
