@@ -53,7 +53,7 @@ __global__ __launch_bounds__(256) void k_dyt(
     const int* __restrict__ row_seq,    // null: every row its own sequence
     const int* __restrict__ cu_q,
     const int64_t* __restrict__ rows,   // null, or the rows to compute
-    int n, int T_in, int W, int strip)
+    int n, int T_in, int W, int strip, int frag)   // frag: layout of h_out
 {
     const int c = (blockIdx.y * 256 + threadIdx.x) * VEC;
     if (c >= W) return;
@@ -89,6 +89,9 @@ __global__ __launch_bounds__(256) void k_dyt(
             h[i] = tanh_of<T>(pre.alpha * x[i]) * pw[i] + pb[i];
     };
 
+    auto h_at = [&](int r) {
+        return h_out + (frag ? frag_row_off(r, c, W) : (int64_t)r * W + c);
+    };
     const int r0 = blockIdx.x * strip;
     const int r1 = min(r0 + strip, n);
     float hp[VEC];
@@ -99,7 +102,7 @@ __global__ __launch_bounds__(256) void k_dyt(
         if (x_out) stv<VEC>(x_out + (int64_t)o * W + c, x);
         norm(x, h);
         if (!mix) {
-            stv<VEC>(h_out + (int64_t)o * W + c, h);
+            stv<VEC>(h_at(o), h);
             continue;
         }
         const int s = row_seq ? row_seq[r] : r;
@@ -129,7 +132,7 @@ __global__ __launch_bounds__(256) void k_dyt(
             out[i] = h[i] + (hp[i] - h[i]) * mx[i];
             hp[i] = h[i];
         }
-        stv<VEC>(h_out + (int64_t)o * W + c, out);
+        stv<VEC>(h_at(o), out);
     }
 }
 
@@ -139,7 +142,7 @@ static int dyt_launch(
     const void* tokens, const void* y, const void* y_part, int n_part,
     DyT post, DyT pre, const void* mix, void* prev, const void* slot,
     const void* pos, const void* row_seq, const void* cu_q,
-    const void* rows, int n, int T_in, int W, hipStream_t stream)
+    const void* rows, int n, int T_in, int W, int frag, hipStream_t stream)
 {
     const bool v4 = W % 4 == 0;
     const int per = 256 * (v4 ? 4 : 1);
@@ -155,7 +158,7 @@ static int dyt_launch(
             (const float*)y_part, n_part, post, pre, (const float*)mix,    \
             (float*)prev, (const int*)slot, (const int*)pos,               \
             (const int*)row_seq, (const int*)cu_q, (const int64_t*)rows,   \
-            n, T_in, W, strip)
+            n, T_in, W, strip, frag)
     if (v4) DYT_GO(4); else DYT_GO(1);
     #undef DYT_GO
     return (int)hipGetLastError();
@@ -168,14 +171,14 @@ extern "C" int dyt_residual(
     const void* pre_w, const void* pre_b, float pre_alpha,
     const void* mix, void* prev, const void* slot, const void* pos,
     const void* row_seq, const void* cu_q, const void* rows,
-    int n, int T_in, int W, hipStream_t stream)
+    int n, int T_in, int W, int frag, hipStream_t stream)
 {
     DyT post{(const float*)post_w, (const float*)post_b, post_alpha};
     DyT pre{(const float*)pre_w, (const float*)pre_b, pre_alpha};
     auto go = f32 ? dyt_launch<float> : dyt_launch<bf16>;
     return go(x_out, h_out, x_in, embed, tokens, y, y_part, n_part, post,
               pre, mix, prev, slot, pos, row_seq, cu_q, rows, n, T_in, W,
-              stream);
+              frag, stream);
 }
 
 // ---------------------------------------------------------------------------
@@ -187,7 +190,8 @@ template <typename T, int VEC, int NV>
 __global__ __launch_bounds__(256) void k_polynorm(
     T* __restrict__ out, const T* __restrict__ z,
     const float* __restrict__ z_part, int n_part, int64_t part_stride,
-    float ca, float cb, float cc, float ce, int F, float eps)
+    float ca, float cb, float cc, float ce, int F, float eps,
+    int frag)                           // layout of out
 {
     const int64_t row = blockIdx.x;
     const int tid = threadIdx.x;
@@ -242,7 +246,7 @@ __global__ __launch_bounds__(256) void k_polynorm(
         #pragma unroll
         for (int i = 0; i < VEC; i++)
             o[i] = v[i] * (a + v[i] * (b + v[i] * g)) + ce;
-        stv<VEC>(out + row * F + c, o);
+        stv<VEC>(out + (frag ? frag_row_off(row, c, F) : row * F + c), o);
     };
     if constexpr (NV > 0) {
         #pragma unroll
@@ -262,13 +266,13 @@ __global__ __launch_bounds__(256) void k_polynorm(
 extern "C" int polynorm(
     int f32, void* out, const void* z, const void* z_part, int n_part,
     float ca, float cb, float cc, float ce, int T_rows, int F, float eps,
-    hipStream_t stream)
+    int frag, hipStream_t stream)
 {
     const int64_t ps = (int64_t)T_rows * F;
     #define PN_GO(T, V, NV)                                                \
         k_polynorm<T, V, NV><<<T_rows, 256, 0, stream>>>(                  \
             (T*)out, (const T*)z, (const float*)z_part, n_part, ps,        \
-            ca, cb, cc, ce, F, eps)
+            ca, cb, cc, ce, F, eps, frag)
     #define PN_TYPE(T)                                                     \
         do {                                                               \
             if (F % 8) PN_GO(T, 1, 0);                                     \
@@ -289,7 +293,7 @@ extern "C" int polynorm(
 // Latent append: c = rmsnorm(d) * w into pool[page][offset][R].  One wave
 // per token.
 // ---------------------------------------------------------------------------
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void k_latent_append(
     T* __restrict__ pool, const T* __restrict__ d, int64_t ds,
     const float* __restrict__ w, const int* __restrict__ slot,
@@ -299,19 +303,25 @@ __global__ __launch_bounds__(256) void k_latent_append(
     const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
     const int lane = threadIdx.x & 63;
     if (t >= T_rows) return;
-    const T* src = d + (int64_t)t * ds;
-    float s = 0.f;
-    for (int i = lane; i < R; i += 64) {
-        const float v = ldf(src + i);
-        s += v * v;
-    }
-    s = wave_sum(s);
-    const float r = 1.f / sqrtf(s / R + eps);
     const int p = pos[t];
     const int pg = ptab[(int64_t)slot[t] * maxp + p / psz];
+    const T* src = d + (int64_t)t * ds;
     T* dst = pool + ((int64_t)pg * psz + p % psz) * R;
-    for (int i = lane; i < R; i += 64)
-        stf(dst + i, ldf(src + i) * r * w[i]);
+    float v[VEC], nw[VEC], s = 0.f;
+    const bool one = R <= 64 * VEC;         // the row fits the wave
+    for (int i = lane * VEC; i < R; i += 64 * VEC) {
+        ldv<VEC>(src + i, v);
+        #pragma unroll
+        for (int e = 0; e < VEC; e++) s += v[e] * v[e];
+    }
+    const float r = 1.f / sqrtf(wave_sum(s) / R + eps);
+    for (int i = lane * VEC; i < R; i += 64 * VEC) {
+        if (!one) ldv<VEC>(src + i, v);
+        ldv<VEC>(w + i, nw);
+        #pragma unroll
+        for (int e = 0; e < VEC; e++) v[e] *= r * nw[e];
+        stv<VEC>(dst + i, v);
+    }
 }
 
 extern "C" int latent_append(
@@ -320,15 +330,14 @@ extern "C" int latent_append(
     int psz, int maxp, float eps, hipStream_t stream)
 {
     const int g = (T_rows + 3) / 4;
-    if (f32)
-        k_latent_append<float><<<g, 256, 0, stream>>>(
-            (float*)pool, (const float*)d, ds, (const float*)w,
-            (const int*)slot, (const int*)pos, (const int*)ptab, T_rows, R,
-            psz, maxp, eps);
-    else
-        k_latent_append<bf16><<<g, 256, 0, stream>>>(
-            (bf16*)pool, (const bf16*)d, ds, (const float*)w,
-            (const int*)slot, (const int*)pos, (const int*)ptab, T_rows, R,
-            psz, maxp, eps);
+    const bool vec = R % 8 == 0 && ds % 8 == 0
+                     && (uintptr_t)d % (f32 ? 32 : 16) == 0;
+    #define AP_GO(T, V)                                                    \
+        k_latent_append<T, V><<<g, 256, 0, stream>>>(                      \
+            (T*)pool, (const T*)d, ds, (const float*)w, (const int*)slot,  \
+            (const int*)pos, (const int*)ptab, T_rows, R, psz, maxp, eps)
+    if (f32) { if (vec) AP_GO(float, 8); else AP_GO(float, 1); }
+    else { if (vec) AP_GO(bf16, 8); else AP_GO(bf16, 1); }
+    #undef AP_GO
     return (int)hipGetLastError();
 }

@@ -24,10 +24,12 @@ struct GlaIn {            // one row of the fused projection
     int rank;
 };
 
+// log(sigmoid(z)) / tau; the error of log(1 + e) is absolute, like that of
+// any exponent near zero
 DEV float log_alpha(float z, float inv_tau) {
-    return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau;
+    return (fminf(z, 0.f) - __logf(1.f + __expf(-fabsf(z)))) * inv_tau;
 }
-DEV float silu(float x) { return x / (1.f + expf(-x)); }
+DEV float silu(float x) { return x / (1.f + __expf(-x)); }
 
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void k_gla_step(
@@ -38,7 +40,8 @@ __global__ __launch_bounds__(256) void k_gla_step(
     float* __restrict__ state,          // [slots, H, D, V]
     const int* __restrict__ slot, const int* __restrict__ pos,
     const int* __restrict__ spans,      // [n, 2] first row, rows; null: 1 row
-    int H, int D, int V, float scale, float inv_tau, float eps)
+    int H, int D, int V, float scale, float inv_tau, float eps,
+    int frag)                           // layout of out
 {
     const int h = blockIdx.y, tid = threadIdx.x;
     const int t0 = spans ? spans[blockIdx.x * 2] : blockIdx.x;
@@ -64,7 +67,7 @@ __global__ __launch_bounds__(256) void k_gla_step(
             for (int r = 0; r < in.rank; r++)
                 z += ldf(a2 + (int64_t)c * in.rank + r)
                      * ldf(row + in.ou + r);
-            a_s[d] = expf(log_alpha(z, inv_tau));
+            a_s[d] = __expf(log_alpha(z, inv_tau));
         }
         __syncthreads();
         for (int vt = rg < RG ? tid % nv : V; vt * VEC < V; vt += nv) {
@@ -104,7 +107,8 @@ __global__ __launch_bounds__(256) void k_gla_step(
         const float ms = ((r_s[0] + r_s[1]) + (r_s[2] + r_s[3])) / V;
         const float rs = 1.f / sqrtf(ms + eps);
         for (int c = tid; c < V; c += 256)
-            stf(out + ((int64_t)t * H + h) * V + c,
+            stf(out + (frag ? frag_row_off(t, h * V + c, H * V)
+                            : ((int64_t)t * H + h) * V + c),
                 o_s[c] * rs * norm_w[c]
                     * silu(ldf(row + in.og + h * V + c)));
         __syncthreads();
@@ -116,7 +120,7 @@ extern "C" int gla_step(
     int og, int ou, int rank, const void* a2, const void* a2_b,
     const void* norm_w, void* state, const void* slot, const void* pos,
     const void* spans, int n, int H, int D, int V, float scale,
-    float inv_tau, float eps, hipStream_t stream)
+    float inv_tau, float eps, int frag, hipStream_t stream)
 {
     // a vector load of v needs aligned columns
     const bool v4 = V % 4 == 0 && ov % 4 == 0 && ld % 4 == 0;
@@ -132,7 +136,7 @@ extern "C" int gla_step(
             (T*)out, (const T*)p, in, (const T*)a2, (const float*)a2_b,    \
             (const float*)norm_w, (float*)state, (const int*)slot,         \
             (const int*)pos, (const int*)spans, H, D, V, scale, inv_tau,   \
-            eps)
+            eps, frag)
     if (f32) { if (v4) GS_GO(float, 4); else GS_GO(float, 1); }
     else { if (v4) GS_GO(bf16, 4); else GS_GO(bf16, 1); }
     #undef GS_GO
@@ -146,124 +150,174 @@ extern "C" int gla_step(
 #define DS (DB + 1)       // LDS row stride
 // largest sum of decay inside a part for which the part's own triangle may
 // be factored (e^{b_i} e^{-b_j}); beyond it the pairs are taken one by one
-#define SAFE 40.f
+#define SAFE 20.f
 
 // scratch per (chunk, head): qd [64][Dp], kd^T [Dp][64], A [64][64], eb [Dp]
 DEV int64_t gla_unit(int Dp) {
     return (int64_t)2 * CH * Dp + CH * CH + Dp;
 }
 
+// Wave w owns part w of the chunk.  z comes off the matrix cores with a
+// channel on a lane and four tokens in its registers, so the running sum
+// over the part is three adds and two cross-lane steps; only the factors
+// that other lanes need as matrix operands go through LDS.
 template <typename T>
 __global__ __launch_bounds__(256) void k_gla_prep(
     float* __restrict__ scr, const T* __restrict__ p, GlaIn in,
     const T* __restrict__ a2, const float* __restrict__ a2_b,
     const int* __restrict__ chunks,     // [n, 2] first row, rows
-    int H, int D, int Dp, float scale, float inv_tau)
+    int H, int D, int Dp, float scale, float inv_tau, int vec)
 {
     const int h = blockIdx.y, tid = threadIdx.x;
     const int lane = tid & 63, w = tid >> 6;
     const int lr = lane & 15, g = lane >> 4;
     const int t0 = chunks[blockIdx.x * 2], n = chunks[blockIdx.x * 2 + 1];
+    const int R4 = (in.rank + 3) & ~3, RS = R4 + 1;
     float* qd = scr + ((int64_t)blockIdx.x * H + h) * gla_unit(Dp);
     float* kdt = qd + CH * Dp;
     float* Ao = kdt + CH * Dp;
     float* eb = Ao + CH * CH;
     extern __shared__ __attribute__((aligned(16))) float sm[];
     float* q_s = sm;                    // [64][DS] scaled q
-    float* k_s = q_s + CH * DS;
+    float* k_s = q_s + CH * DS;         // k, or k e^{-b}
     float* b_s = k_s + CH * DS;         // running log decay inside a part
     float* qe_s = b_s + CH * DS;        // q e^{b}
     float* ke_s = qe_s + CH * DS;       // k e^{part total - b}
     float* et_s = ke_s + CH * DS;       // [4][DB] e^{part total}
-    float* u_s = et_s + 4 * DB;         // [64][rank]
+    float* w_s = et_s + 4 * DB;         // [DB][RS] rows of a2
+    float* u_s = w_s + DB * RS;         // [64][RS]
 
-    for (int i = tid; i < CH * in.rank; i += 256) {
-        const int t = i / in.rank;
-        u_s[i] = t < n ? ldf(p + (int64_t)(t0 + t) * in.ld + in.ou
-                             + i % in.rank) : 0.f;
+    for (int i = tid; i < CH * R4; i += 256) {
+        const int t = i / R4, r = i % R4;
+        u_s[t * RS + r] = t < n && r < in.rank
+            ? ldf(p + (int64_t)(t0 + t) * in.ld + in.ou + r) : 0.f;
     }
-    // this wave's tiles of A: its own diagonal, and of the six tiles below
-    // it (1,0) (2,1) (3,2) (2,0) (3,1) (3,0) numbers w and w + 4
+    // of the six tiles below the diagonal (1,0) (2,1) (3,2) (2,0) (3,1)
+    // (3,0) this wave makes numbers w and w + 4
     const int ti[6] = {1, 2, 3, 2, 3, 3}, tj[6] = {0, 1, 2, 0, 1, 0};
     f32x4 diag = {}, off[2] = {};
 
     for (int d0 = 0; d0 < Dp; d0 += DB) {
         __syncthreads();
-        for (int i = tid; i < CH * DB; i += 256) {
-            const int t = i / DB, d = i % DB;
-            const bool on = t < n && d0 + d < D;
+        for (int i = tid; i < DB * R4; i += 256) {
+            const int d = i / R4, r = i % R4;
+            w_s[d * RS + r] = d0 + d < D && r < in.rank
+                ? ldf(a2 + (int64_t)(h * D + d0 + d) * in.rank + r) : 0.f;
+        }
+        #pragma unroll
+        for (int x = 0; x < 2; x++) {       // 16 tokens x 32 channels by fours
+            const int i = lane + x * 64;
+            const int t = w * SUB + (i >> 3), d = (i & 7) * 4;
             const T* row = p + (int64_t)(t0 + t) * in.ld + h * D + d0 + d;
-            q_s[t * DS + d] = on ? ldf(row + in.oq) * scale : 0.f;
-            k_s[t * DS + d] = on ? ldf(row + in.ok) : 0.f;
-            float la = 0.f;
-            if (on) {
-                const int c = h * D + d0 + d;
-                float z = a2_b[c];
-                const T* wr = a2 + (int64_t)c * in.rank;
-                for (int r = 0; r < in.rank; r++)
-                    z += ldf(wr + r) * u_s[t * in.rank + r];
-                la = log_alpha(z, inv_tau);
+            float q4[4] = {}, k4[4] = {};
+            if (t < n) {
+                if (vec) {
+                    if (d0 + d < D) {
+                        ldv<4>(row + in.oq, q4);
+                        ldv<4>(row + in.ok, k4);
+                    }
+                } else
+                    for (int e = 0; e < 4; e++)
+                        if (d0 + d + e < D) {
+                            q4[e] = ldf(row + in.oq + e);
+                            k4[e] = ldf(row + in.ok + e);
+                        }
             }
-            b_s[t * DS + d] = la;
+            #pragma unroll
+            for (int e = 0; e < 4; e++) {
+                q_s[t * DS + d + e] = q4[e] * scale;
+                k_s[t * DS + d + e] = k4[e];
+            }
         }
         __syncthreads();
-        if (tid < 4 * DB) {
-            const int s = tid / DB, d = tid % DB;
-            float b = 0.f;
-            for (int t = s * SUB; t < (s + 1) * SUB; t++) {
-                b += b_s[t * DS + d];
-                b_s[t * DS + d] = b;
-                qe_s[t * DS + d] = q_s[t * DS + d] * expf(b);
+        f32x4 qe[2], ke[2];
+        bool safe = true;
+        float b[2][4];
+        #pragma unroll
+        for (int x = 0; x < 2; x++) {
+            f32x4 z = {};
+            for (int r = g; r < R4; r += 4)
+                z = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    u_s[(w * SUB + lr) * RS + r],
+                    w_s[(x * 16 + lr) * RS + r], z, 0, 0, 0);
+            const int d = x * 16 + lr;
+            const bool on = d0 + d < D;
+            const float bias = on ? a2_b[h * D + d0 + d] : 0.f;
+            float run = 0.f;
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int t = w * SUB + g * 4 + i;
+                if (on && t < n) run += log_alpha(z[i] + bias, inv_tau);
+                b[x][i] = run;
             }
-            for (int t = s * SUB; t < (s + 1) * SUB; t++)
-                ke_s[t * DS + d] = k_s[t * DS + d]
-                                   * expf(b - b_s[t * DS + d]);
-            et_s[s * DB + d] = expf(b);
+            float inc = run;                // over the lanes' four-token runs
+            const float u1 = __shfl_up(inc, 16, 64);
+            if (g >= 1) inc += u1;
+            const float u2 = __shfl_up(inc, 32, 64);
+            if (g >= 2) inc += u2;
+            float exc = __shfl_up(inc, 16, 64);
+            if (g == 0) exc = 0.f;
+            const float tot = __shfl(inc, 48 + lr, 64);
+            safe = safe && tot > -SAFE;
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                b[x][i] += exc;
+                const int o = (w * SUB + g * 4 + i) * DS + d;
+                qe[x][i] = q_s[o] * __expf(b[x][i]);
+                ke[x][i] = k_s[o] * __expf(tot - b[x][i]);
+                qe_s[o] = qe[x][i];
+                ke_s[o] = ke[x][i];
+            }
+            if (g == 0) et_s[w * DB + d] = __expf(tot);
         }
+        safe = __all(safe);
+        #pragma unroll
+        for (int x = 0; x < 2; x++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int o = (w * SUB + g * 4 + i) * DS + x * 16 + lr;
+                if (safe) k_s[o] *= __expf(-b[x][i]);
+                else b_s[o] = b[x][i];
+            }
         __syncthreads();
         // factors that meet the state
-        for (int i = tid; i < CH * DB; i += 256) {
-            const int t = i / DB, d = i % DB;
-            if (d0 + d < Dp) {
-                float f = qe_s[t * DS + d];
-                for (int s = 0; s < t / SUB; s++) f *= et_s[s * DB + d];
-                qd[t * Dp + d0 + d] = f;
-            }
+        #pragma unroll
+        for (int x = 0; x < 2; x++) {
+            const int d = x * 16 + lr;
+            if (d0 + d >= Dp) continue;
+            float before = 1.f, after = 1.f;
+            for (int s = 0; s < w; s++) before *= et_s[s * DB + d];
+            for (int s = w + 1; s < 4; s++) after *= et_s[s * DB + d];
+            #pragma unroll
+            for (int i = 0; i < 4; i++)
+                qd[(w * SUB + g * 4 + i) * Dp + d0 + d] = qe[x][i] * before;
+            *reinterpret_cast<f32x4*>(
+                kdt + (int64_t)(d0 + d) * CH + w * SUB + g * 4) =
+                ke[x] * after;
+            if (w == 3 && g == 0)
+                eb[d0 + d] = before * et_s[3 * DB + d];
         }
-        for (int i = tid; i < CH * DB; i += 256) {
-            const int d = i / CH, t = i % CH;
-            if (d0 + d < Dp) {
-                float f = ke_s[t * DS + d];
-                for (int s = t / SUB + 1; s < 4; s++) f *= et_s[s * DB + d];
-                kdt[(d0 + d) * CH + t] = f;
-            }
-        }
-        if (tid < DB && d0 + tid < Dp)
-            eb[d0 + tid] = et_s[tid] * et_s[DB + tid]
-                           * et_s[2 * DB + tid] * et_s[3 * DB + tid];
         // tiles below the diagonal
         #pragma unroll
         for (int x = 0; x < 2; x++) {
             const int id = w + x * 4;
             if (id >= 6) continue;
             const int I = ti[id], J = tj[id];
-            for (int d = g; d < DB; d += 4) {
-                float a = qe_s[(I * SUB + lr) * DS + d];
-                for (int s = J + 1; s < I; s++) a *= et_s[s * DB + d];
+            #pragma unroll
+            for (int d = 0; d < DB; d += 4) {
+                float a = qe_s[(I * SUB + lr) * DS + d + g];
+                for (int s = J + 1; s < I; s++) a *= et_s[s * DB + d + g];
                 off[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    a, ke_s[(J * SUB + lr) * DS + d], off[x], 0, 0, 0);
+                    a, ke_s[(J * SUB + lr) * DS + d + g], off[x], 0, 0, 0);
             }
         }
         // the part's own triangle
-        float mn = 0.f;
-        for (int d = lane; d < DB; d += 64)
-            mn = fminf(mn, b_s[(w * SUB + SUB - 1) * DS + d]);
-        const bool safe = wave_max(-mn) < SAFE;
         if (safe) {
-            for (int d = g; d < DB; d += 4) {
-                const int o = (w * SUB + lr) * DS + d;
+            #pragma unroll
+            for (int d = 0; d < DB; d += 4) {
+                const int o = (w * SUB + lr) * DS + d + g;
                 diag = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    qe_s[o], k_s[o] * expf(-b_s[o]), diag, 0, 0, 0);
+                    qe_s[o], k_s[o], diag, 0, 0, 0);
             }
         } else {
             // lane: column lr (the key), rows g*4 + i (the query)
@@ -274,7 +328,7 @@ __global__ __launch_bounds__(256) void k_gla_prep(
                 for (int i = 0; i < 4; i++) {
                     const int oi = (w * SUB + g * 4 + i) * DS + d;
                     diag[i] += q_s[oi] * kj
-                               * expf(fminf(b_s[oi] - bj, 0.f));
+                               * __expf(fminf(b_s[oi] - bj, 0.f));
                 }
             }
         }
@@ -294,7 +348,11 @@ __global__ __launch_bounds__(256) void k_gla_prep(
     }
 }
 
-// NS: 16-row state tiles per wave (D <= 64 * NS); VC: 16-column tiles
+// A sequence's chunks in order, one block per 16*VC value columns, the state
+// in registers (NS: 16-row tiles per wave, D <= 64 * NS).  Only the state
+// and v go through LDS; every other operand belongs to one wave and comes
+// straight from memory, loaded while the matrix cores work on what was
+// loaded before.
 template <typename T, int NS, int VC>
 __global__ __launch_bounds__(256) void k_gla_scan(
     float* __restrict__ o,              // [rows, H, V]
@@ -307,6 +365,8 @@ __global__ __launch_bounds__(256) void k_gla_scan(
     int H, int D, int Dp, int V)
 {
     constexpr int W = VC * 16, WS = W + (W % 64 == 16 ? 0 : 16);
+    constexpr int NQ = NS * 4;          // 16-channel steps over D
+    constexpr int NV = CH * W / 256;    // elements of v a thread
     const int h = blockIdx.y, v0 = blockIdx.z * W, tid = threadIdx.x;
     const int lane = tid & 63, w = tid >> 6;
     const int lr = lane & 15, g = lane >> 4;
@@ -331,17 +391,60 @@ __global__ __launch_bounds__(256) void k_gla_scan(
                                  ? 0.f : St[(int64_t)d * V + v];
             }
 
-    for (int ci = c0; ci < c0 + nc; ++ci) {
+    // operands in flight; a lane's k runs in fours, the same for both sides
+    f32x4 q4[NQ], a4[4], k4[NS][4], e4[NS];
+    float vv[NV];
+    auto unit = [&](int ci) {
+        return scr + ((int64_t)ci * H + h) * gla_unit(Dp);
+    };
+    auto load_qa = [&](int ci) {
+        const float* qr = unit(ci) + (w * 16 + lr) * Dp + g * 4;
+        #pragma unroll
+        for (int d = 0; d < NQ; d++)
+            q4[d] = d * 16 < Dp
+                ? *reinterpret_cast<const f32x4*>(qr + d * 16) : f32x4{};
+        const float* Ar = unit(ci) + 2 * CH * Dp + (w * 16 + lr) * CH + g * 4;
+        #pragma unroll
+        for (int j = 0; j < 4; j++)
+            a4[j] = j <= w
+                ? *reinterpret_cast<const f32x4*>(Ar + j * 16) : f32x4{};
+    };
+    auto load_k = [&](int ci) {
+        const float* kd = unit(ci) + CH * Dp;
+        const float* eb = unit(ci) + 2 * CH * Dp + CH * CH;
+        #pragma unroll
+        for (int x = 0; x < NS; x++) {
+            const int d = (w + x * 4) * 16;
+            const bool in_d = d < Dp;
+            e4[x] = in_d ? *reinterpret_cast<const f32x4*>(eb + d + g * 4)
+                         : f32x4{};
+            #pragma unroll
+            for (int t = 0; t < 4; t++)
+                k4[x][t] = in_d ? *reinterpret_cast<const f32x4*>(
+                    kd + (int64_t)(d + lr) * CH + t * 16 + g * 4) : f32x4{};
+        }
+    };
+    auto load_v = [&](int ci) {
         const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
-        const float* qd = scr + ((int64_t)ci * H + h) * gla_unit(Dp);
-        const float* kdt = qd + CH * Dp;
-        const float* A = kdt + CH * Dp;
-        const float* eb = A + CH * CH;
-        for (int i = tid; i < CH * W; i += 256) {
-            const int t = i / W, c = i % W;
-            v_s[t * WS + c] = (t < n && v0 + c < V)
+        #pragma unroll
+        for (int x = 0; x < NV; x++) {
+            const int i = tid + x * 256, t = i / W, c = i % W;
+            vv[x] = t < n && v0 + c < V
                 ? ldf(p + (int64_t)(t0 + t) * in.ld + in.ov + h * V + v0 + c)
                 : 0.f;
+        }
+    };
+    load_v(c0);
+    load_qa(c0);
+    load_k(c0);
+
+    for (int ci = c0; ci < c0 + nc; ++ci) {
+        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
+        const int nx = min(ci + 1, c0 + nc - 1);
+        #pragma unroll
+        for (int x = 0; x < NV; x++) {
+            const int i = tid + x * 256;
+            v_s[(i / W) * WS + i % W] = vv[x];
         }
         #pragma unroll
         for (int x = 0; x < NS; x++) {
@@ -355,31 +458,49 @@ __global__ __launch_bounds__(256) void k_gla_scan(
                             S[x][c][i];
         }
         __syncthreads();
-        // o tile of this wave's 16 tokens; a lane's k runs in fours, the
-        // same for both operands
+        load_v(nx);
+        // state: needs only v and registers
+        #pragma unroll
+        for (int x = 0; x < NS; x++) {
+            #pragma unroll
+            for (int c = 0; c < VC; c++) S[x][c] *= e4[x];
+            #pragma unroll
+            for (int t = 0; t < 4; t++)
+                #pragma unroll
+                for (int e = 0; e < 4; e++)
+                    #pragma unroll
+                    for (int c = 0; c < VC; c++)
+                        S[x][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                            k4[x][t][e],
+                            v_s[(t * 16 + g * 4 + e) * WS + c * 16 + lr],
+                            S[x][c], 0, 0, 0);
+        }
+        load_k(nx);
+        // o tile of this wave's 16 tokens
         f32x4 acc[VC] = {};
-        const float* qr = qd + (w * 16 + lr) * Dp + g * 4;
-        for (int d = 0; d < Dp; d += 16) {
-            const f32x4 a = *reinterpret_cast<const f32x4*>(qr + d);
-            #pragma unroll
-            for (int e = 0; e < 4; e++)
+        #pragma unroll
+        for (int d = 0; d < NQ; d++)
+            if (d * 16 < Dp)
                 #pragma unroll
-                for (int c = 0; c < VC; c++)
-                    acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                        a[e], S_s[(d + g * 4 + e) * WS + c * 16 + lr],
-                        acc[c], 0, 0, 0);
-        }
-        const float* Ar = A + (w * 16 + lr) * CH + g * 4;
-        for (int j = 0; j <= w; j++) {
-            const f32x4 a = *reinterpret_cast<const f32x4*>(Ar + j * 16);
-            #pragma unroll
-            for (int e = 0; e < 4; e++)
+                for (int e = 0; e < 4; e++)
+                    #pragma unroll
+                    for (int c = 0; c < VC; c++)
+                        acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                            q4[d][e],
+                            S_s[(d * 16 + g * 4 + e) * WS + c * 16 + lr],
+                            acc[c], 0, 0, 0);
+        #pragma unroll
+        for (int j = 0; j < 4; j++)
+            if (j <= w)
                 #pragma unroll
-                for (int c = 0; c < VC; c++)
-                    acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                        a[e], v_s[(j * 16 + g * 4 + e) * WS + c * 16 + lr],
-                        acc[c], 0, 0, 0);
-        }
+                for (int e = 0; e < 4; e++)
+                    #pragma unroll
+                    for (int c = 0; c < VC; c++)
+                        acc[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                            a4[j][e],
+                            v_s[(j * 16 + g * 4 + e) * WS + c * 16 + lr],
+                            acc[c], 0, 0, 0);
+        load_qa(nx);
         #pragma unroll
         for (int c = 0; c < VC; c++)
             #pragma unroll
@@ -389,28 +510,6 @@ __global__ __launch_bounds__(256) void k_gla_scan(
                     o[((int64_t)(t0 - row_base + t) * H + h) * V + v] =
                         acc[c][i];
             }
-        // state
-        #pragma unroll
-        for (int x = 0; x < NS; x++) {
-            const int d0 = (w + x * 4) * 16;
-            if (d0 >= Dp) continue;
-            const f32x4 e4 = *reinterpret_cast<const f32x4*>(
-                eb + d0 + g * 4);
-            #pragma unroll
-            for (int c = 0; c < VC; c++) S[x][c] *= e4;
-            const float* kr = kdt + (d0 + lr) * CH + g * 4;
-            #pragma unroll
-            for (int t = 0; t < CH; t += 16) {
-                const f32x4 a = *reinterpret_cast<const f32x4*>(kr + t);
-                #pragma unroll
-                for (int e = 0; e < 4; e++)
-                    #pragma unroll
-                    for (int c = 0; c < VC; c++)
-                        S[x][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                            a[e], v_s[(t + g * 4 + e) * WS + c * 16 + lr],
-                            S[x][c], 0, 0, 0);
-            }
-        }
         __syncthreads();
     }
     #pragma unroll
@@ -426,7 +525,7 @@ __global__ __launch_bounds__(256) void k_gla_scan(
 }
 
 // head norm and gate, one wave per (token, head)
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void k_gla_out(
     T* __restrict__ out, const float* __restrict__ o,
     const T* __restrict__ p, GlaIn in, const float* __restrict__ norm_w,
@@ -439,12 +538,24 @@ __global__ __launch_bounds__(256) void k_gla_out(
     const int h = (int)(u % H);
     const float* src = o + u * V;
     float sq = 0.f;
-    for (int c = lane; c < V; c += 64) sq += src[c] * src[c];
+    float x[VEC], gt[VEC], nw[VEC];
+    const bool one = V <= 64 * VEC;         // the row fits the wave
+    for (int c = lane * VEC; c < V; c += 64 * VEC) {
+        ldv<VEC>(src + c, x);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) sq += x[i] * x[i];
+    }
     const float rs = 1.f / sqrtf(wave_sum(sq) / V + eps);
     const T* gr = p + (row_base + t) * in.ld + in.og + h * V;
     T* dst = out + ((row_base + t) * H + h) * V;
-    for (int c = lane; c < V; c += 64)
-        stf(dst + c, src[c] * rs * norm_w[c] * silu(ldf(gr + c)));
+    for (int c = lane * VEC; c < V; c += 64 * VEC) {
+        if (!one) ldv<VEC>(src + c, x);
+        ldv<VEC>(gr + c, gt);
+        ldv<VEC>(norm_w + c, nw);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) x[i] *= rs * nw[i] * silu(gt[i]);
+        stv<VEC>(dst + c, x);
+    }
 }
 
 extern "C" int64_t gla_scratch_floats(int n_chunks, int H, int D)
@@ -468,9 +579,13 @@ extern "C" int gla_chunks(
         return (int)hipErrorInvalidValue;
     GlaIn in{ld, oq, ok, ov, og, ou, rank};
     const int Dp = (D + 15) & ~15;
-    const int lds_a = (5 * CH * DS + 4 * DB + CH * rank) * 4;
+    const int rs = ((rank + 3) & ~3) + 1;
+    const int lds_a = (5 * CH * DS + 4 * DB + (CH + DB) * rs) * 4;
     // wider column tiles re-read the factors less; narrow ones fill the chip
-    const int vc = (int64_t)n_seqs * H * ((V + 31) / 32) >= 256 ? 2 : 1;
+    const int vc = (int64_t)n_seqs * H * ((V + 31) / 32) >= 512
+                   && Dp <= 256 ? 2 : 1;
+    const int vec = D % 4 == 0 && oq % 4 == 0 && ok % 4 == 0 && ld % 4 == 0;
+    const bool vout = V % 4 == 0 && og % 4 == 0 && ld % 4 == 0;
     const int ws = vc == 1 ? 16 : 48;
     const int lds_b = (Dp + CH) * ws * 4;
     if (lds_a > 160 * 1024 || lds_b > 160 * 1024)
@@ -496,6 +611,10 @@ extern "C" int gla_chunks(
             else if (Dp <= 256) GC_SCAN(T, 4, VC);                         \
             else GC_SCAN(T, 8, VC);                                        \
         } while (0)
+    #define GC_OUT(T, VV)                                                  \
+        k_gla_out<T, VV><<<gc, 256, 0, stream>>>(                          \
+            (T*)out, (const float*)o_scr, (const T*)p, in,                 \
+            (const float*)norm_w, row_base, units, H, V, eps)
     #define GC_TYPE(T)                                                     \
         do {                                                               \
             (void)hipFuncSetAttribute(                                     \
@@ -504,14 +623,13 @@ extern "C" int gla_chunks(
             k_gla_prep<T><<<ga, 256, lds_a, stream>>>(                     \
                 (float*)scr, (const T*)p, in, (const T*)a2,                \
                 (const float*)a2_b, (const int*)chunks, H, D, Dp, scale,   \
-                inv_tau);                                                  \
+                inv_tau, vec);                                             \
             if (vc == 1) GC_NS(T, 1); else GC_NS(T, 2);                    \
-            k_gla_out<T><<<gc, 256, 0, stream>>>(                          \
-                (T*)out, (const float*)o_scr, (const T*)p, in,             \
-                (const float*)norm_w, row_base, units, H, V, eps);         \
+            if (vout) GC_OUT(T, 4); else GC_OUT(T, 1);                     \
         } while (0)
     if (f32) GC_TYPE(float); else GC_TYPE(bf16);
     #undef GC_TYPE
+    #undef GC_OUT
     #undef GC_NS
     #undef GC_SCAN
     return (int)hipGetLastError();

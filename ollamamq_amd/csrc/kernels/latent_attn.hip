@@ -21,20 +21,22 @@ template <typename T> DEV float exp_of(float x) {
 
 // ---------------------------------------------------------------------------
 // out[t][h][n] = sum_k x[t*xs + h*K + k] * w[h][n][k]
-// Grid (n / 64, t / (16*MT), H); a wave makes 16 n x 16*MT tokens.  The
-// product is transposed (A = w) so a lane stores four consecutive n.
+// Grid (n tiles, t / (16*MT), H); a tile is 16 n x 16*MT tokens.  KS == 1:
+// a block's four waves make four n tiles; KS == 4: they share one and deal
+// its k out (long k, few tiles).  The product is transposed (A = w) so a
+// lane stores four consecutive n.
 // ---------------------------------------------------------------------------
-template <typename T, int MT>
+template <typename T, int MT, int KS>
 __global__ __launch_bounds__(256) void k_head_gemm(
     T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ w,
-    int T_rows, int H, int N, int K, int64_t xs)
+    int T_rows, int H, int N, int K, int64_t xs, int frag)
 {
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int lr = lane & 15, g = lane >> 4;
     const int h = blockIdx.z;
-    const int n0 = (blockIdx.x * 4 + wid) * 16;
+    const int n0 = (KS == 1 ? blockIdx.x * 4 + wid : blockIdx.x) * 16;
     const int t0 = blockIdx.y * 16 * MT;
-    if (n0 >= N) return;
+    if (n0 >= N) return;                    // KS == 4: the whole block
     const T* wr = w + ((int64_t)h * N + min(n0 + lr, N - 1)) * K;
     const T* xr[MT];
     #pragma unroll
@@ -43,49 +45,66 @@ __global__ __launch_bounds__(256) void k_head_gemm(
                 + (int64_t)h * K;
     f32x4 acc[MT] = {};
     const bool vec = K % 8 == 0 && xs % 8 == 0;
-    for (int k0 = 0; k0 < K; k0 += 32) {
-        const int k = k0 + g * 8;
-        Frag<T> a, b[MT];
-        if (vec) {
-            const bool in = k < K;
-            a = in ? frag8(wr + k) : frag_zero<T>();
+    const int k_lo = (KS == 1 ? 0 : wid * 32) + g * 8;
+    if (vec) {
+        #pragma unroll 4
+        for (int k = k_lo; k - g * 8 < K; k += 32 * KS) {
+            const Frag<T> a = k < K ? frag8(wr + k) : frag_zero<T>();
             #pragma unroll
             for (int m = 0; m < MT; m++)
-                b[m] = in ? frag8(xr[m] + k) : frag_zero<T>();
-        } else {
-            a = frag_guard(wr, k, K);
-            #pragma unroll
-            for (int m = 0; m < MT; m++) b[m] = frag_guard(xr[m], k, K);
+                acc[m] = mma(a, k < K ? frag8(xr[m] + k) : frag_zero<T>(),
+                             acc[m]);
         }
+    } else {
+        for (int k = k_lo; k - g * 8 < K; k += 32 * KS) {
+            const Frag<T> a = frag_guard(wr, k, K);
+            #pragma unroll
+            for (int m = 0; m < MT; m++)
+                acc[m] = mma(a, frag_guard(xr[m], k, K), acc[m]);
+        }
+    }
+    if constexpr (KS == 4) {
+        __shared__ f32x4 red[4][MT][64];
         #pragma unroll
-        for (int m = 0; m < MT; m++) acc[m] = mma(a, b[m], acc[m]);
+        for (int m = 0; m < MT; m++) red[wid][m][lane] = acc[m];
+        __syncthreads();
+        if (wid >= MT) return;
+        acc[0] = (red[0][wid][lane] + red[1][wid][lane])
+                 + (red[2][wid][lane] + red[3][wid][lane]);
     }
     #pragma unroll
-    for (int m = 0; m < MT; m++) {
-        const int t = t0 + m * 16 + lr;
-        if (t >= T_rows) continue;
-        T* o = out + ((int64_t)t * H + h) * N + n0 + g * 4;
-        if (N % 4 == 0 && n0 + g * 4 + 4 <= N) {
+    for (int m = 0; m < (KS == 4 ? 1 : MT); m++) {
+        const int t = t0 + (KS == 4 ? wid : m) * 16 + lr;
+        const int n = n0 + g * 4;
+        if (t >= T_rows || n >= N) continue;
+        T* o = out + (frag ? frag_row_off(t, h * N + n, H * N)
+                           : ((int64_t)t * H + h) * N + n);
+        if (N % 4 == 0) {
             float v[4] = {acc[m][0], acc[m][1], acc[m][2], acc[m][3]};
             stv<4>(o, v);
         } else
             for (int i = 0; i < 4; i++)
-                if (n0 + g * 4 + i < N) stf(o + i, acc[m][i]);
+                if (n + i < N) stf(o + i, acc[m][i]);
     }
 }
 
+// frag: out in the activation-fragment layout (N % 8 == 0)
 extern "C" int head_gemm(int f32, void* out, const void* x, const void* w,
                          int T_rows, int H, int N, int K, int64_t xs,
-                         hipStream_t stream)
+                         int frag, hipStream_t stream)
 {
-    const bool wide = T_rows > 16;
-    dim3 grid((N + 63) / 64, (T_rows + (wide ? 31 : 15)) / (wide ? 32 : 16),
-              H);
-    #define HG_GO(T, M)                                                    \
-        k_head_gemm<T, M><<<grid, 256, 0, stream>>>(                       \
-            (T*)out, (const T*)x, (const T*)w, T_rows, H, N, K, xs)
-    if (f32) { if (wide) HG_GO(float, 2); else HG_GO(float, 1); }
-    else { if (wide) HG_GO(bf16, 2); else HG_GO(bf16, 1); }
+    if (frag && N % 8) return (int)hipErrorInvalidValue;
+    const bool wide = T_rows > 16, deal = K >= 256;
+    dim3 grid(deal ? (N + 15) / 16 : (N + 63) / 64,
+              (T_rows + (wide ? 31 : 15)) / (wide ? 32 : 16), H);
+    #define HG_GO(T, M, S)                                                 \
+        k_head_gemm<T, M, S><<<grid, 256, 0, stream>>>(                    \
+            (T*)out, (const T*)x, (const T*)w, T_rows, H, N, K, xs, frag)
+    #define HG_K(T, M) do { if (deal) HG_GO(T, M, 4); else HG_GO(T, M, 1); } \
+                       while (0)
+    if (f32) { if (wide) HG_K(float, 2); else HG_K(float, 1); }
+    else { if (wide) HG_K(bf16, 2); else HG_K(bf16, 1); }
+    #undef HG_K
     #undef HG_GO
     return (int)hipGetLastError();
 }
@@ -105,7 +124,7 @@ extern "C" int head_gemm(int f32, void* out, const void* x, const void* w,
 template <typename T, int MT, int KT, int NT>
 __global__ __launch_bounds__(256) void k_latent_attn(
     T* __restrict__ out,               // [rows, R]      (split == 1)
-    float* __restrict__ o_part,        // [split, rows, R]
+    T* __restrict__ o_part,            // [split, rows, R]
     float* __restrict__ ml_part,       // [split, rows, 2]
     const T* __restrict__ q,           // [rows, R]
     const T* __restrict__ pool,        // [pages, psz, R]
@@ -113,8 +132,8 @@ __global__ __launch_bounds__(256) void k_latent_attn(
     const int* __restrict__ pos,
     const int* __restrict__ items,     // [n, 2] first row, rows; null: decode
     int per_seq,                       // decode: items per sequence
-    int H, int R, int psz, int maxp, float scale, int64_t rows_total,
-    int split)
+    int H, int R, int pshift, int maxp, float scale, int64_t rows_total,
+    int split)                         // pages of 1 << pshift tokens
 {
     constexpr int M = 16 * MT;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -169,20 +188,43 @@ __global__ __launch_bounds__(256) void k_latent_attn(
         l_s[tid] = 0.f;
         lim_s[tid] = tid < n_rows ? pos[(row0 + tid) / H] + 1 : 0;
     }
+    // this thread's 8-element pieces of a chunk: (key, column) of each
+    constexpr int NP = KT * NT / 32;
+    Frag<T> piece[NP];
+    int where[NP];
+    #pragma unroll
+    for (int j = 0; j < NP; j++) {
+        const int u = tid + j * 256;
+        where[j] = u < KT * n8 ? (u / n8) << 16 | (u % n8) * 8 : -1;
+    }
+    const int pmask = (1 << pshift) - 1;
+    auto fetch = [&](int base) {
+        #pragma unroll
+        for (int j = 0; j < NP; j++) {
+            if (where[j] < 0) continue;
+            const int key = base + (where[j] >> 16), c = where[j] & 0xffff;
+            const T* src = pool + (((int64_t)pt[min(key, kv_len - 1)
+                                    >> pshift] << pshift)
+                                   + (key & pmask)) * R;
+            if (key >= kv_len) piece[j] = frag_zero<T>();
+            else if (vec) piece[j] = c < R ? frag8(src + c) : frag_zero<T>();
+            else piece[j] = frag_guard(src, c, R);
+        }
+    };
     f32x4 acc[MT][NT] = {};
     __syncthreads();               // a segment may hold no chunk at all
 
+    if (c_lo < c_hi) fetch(c_lo * KT);
     for (int ch = c_lo; ch < c_hi; ++ch) {
         const int base = ch * KT;
-        for (int u = tid; u < KT * n8; u += 256) {
-            const int k = u / n8, key = base + k;
-            stage(c_s + k * cs,
-                  key < kv_len
-                      ? pool + ((int64_t)pt[key / psz] * psz + key % psz) * R
-                      : nullptr,
-                  u % n8);
-        }
+        #pragma unroll
+        for (int j = 0; j < NP; j++)
+            if (where[j] >= 0)
+                *reinterpret_cast<Frag<T>*>(
+                    c_s + (where[j] >> 16) * cs + (where[j] & 0xffff))
+                    = piece[j];
         __syncthreads();
+        if (ch + 1 < c_hi) fetch(base + KT);
         #pragma unroll
         for (int i = 0; i < (MT * KT / 16 + 3) / 4; i++) {
             const int id = wid + i * 4;
@@ -273,19 +315,22 @@ __global__ __launch_bounds__(256) void k_latent_attn(
         if (row >= n_rows) continue;
         const int64_t gr = row0 + row;
         const float l = l_s[row];
-        const float inv = split > 1 ? 1.f : (l > 0.f ? 1.f / l : 0.f);
+        const float inv = l > 0.f ? 1.f / l : 0.f;
         #pragma unroll
         for (int n = 0; n < NT; n++) {
             const int c0 = (n * 4 + wid) * 16 + g * 4;
+            T* dst = split > 1
+                ? o_part + ((int64_t)blockIdx.y * rows_total + gr) * R + c0
+                : out + gr * R + c0;
+            float v[4];
             #pragma unroll
-            for (int i = 0; i < 4; i++)
-                if (c0 + i < R) {
-                    const float v = acc[mt][n][i] * inv;
-                    if (split > 1)
-                        o_part[((int64_t)blockIdx.y * rows_total + gr) * R
-                               + c0 + i] = v;
-                    else stf(out + gr * R + c0 + i, v);
-                }
+            for (int i = 0; i < 4; i++) v[i] = acc[mt][n][i] * inv;
+            if (R % 4 == 0) {
+                if (c0 < R) stv<4>(dst, v);
+            } else
+                #pragma unroll
+                for (int i = 0; i < 4; i++)
+                    if (c0 + i < R) stf(dst + i, v[i]);
         }
         if (split > 1 && wid == 0 && g == 0) {
             float* d = ml_part
@@ -296,28 +341,33 @@ __global__ __launch_bounds__(256) void k_latent_attn(
     }
 }
 
-template <typename T>
+// merge of the segments' normalised results, weights l e^{m - max}
+template <typename T, int VEC>
 __global__ __launch_bounds__(128) void k_latent_combine(
-    T* __restrict__ out, const float* __restrict__ o_part,
+    T* __restrict__ out, const T* __restrict__ o_part,
     const float* __restrict__ ml, int64_t row_base, int64_t rows_total,
-    int R, int split)
+    int R, int split)                   // split <= 64
 {
     const int64_t row = row_base + blockIdx.x;
-    float m = NEG;
-    for (int s = 0; s < split; s++)
-        m = fmaxf(m, ml[(s * rows_total + row) * 2]);
-    float l = 0.f;
-    for (int s = 0; s < split; s++) {
-        const float* d = ml + (s * rows_total + row) * 2;
-        l += d[1] * exp_of<T>(d[0] - m);
-    }
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    for (int i = threadIdx.x; i < R; i += 128) {
-        float v = 0.f;
-        for (int s = 0; s < split; s++)
-            v += o_part[(s * rows_total + row) * R + i]
-                 * exp_of<T>(ml[(s * rows_total + row) * 2] - m);
-        stf(out + row * R + i, v * inv);
+    const int lane = threadIdx.x & 63;
+    __shared__ float w_s[64];
+    const float* d = ml + (lane * rows_total + row) * 2;
+    const float m = lane < split ? d[0] : NEG;
+    const float top = wave_max(m);
+    const float e = lane < split ? d[1] * exp_of<T>(m - top) : 0.f;
+    const float l = wave_sum(e);
+    if (threadIdx.x < 64) w_s[lane] = l > 0.f ? e / l : 0.f;
+    __syncthreads();
+    for (int c = threadIdx.x * VEC; c < R; c += 128 * VEC) {
+        float v[VEC] = {};
+        #pragma unroll 4
+        for (int s = 0; s < split; s++) {
+            float u[VEC];
+            ldv<VEC>(o_part + (s * rows_total + row) * R + c, u);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) v[i] += w_s[s] * u[i];
+        }
+        stv<VEC>(out + row * R + c, v);
     }
 }
 
@@ -332,8 +382,8 @@ template <typename T, int MT, int KT, int NT>
 static int latent_go(
     void* out, void* op, void* mp, const void* q, const void* pool,
     const void* ptab, const void* slot, const void* pos, const void* items,
-    int n_items, int per_seq, int H, int R, int psz, int maxp, float scale,
-    int64_t rows_total, int split, hipStream_t stream)
+    int n_items, int per_seq, int H, int R, int pshift, int maxp,
+    float scale, int64_t rows_total, int split, hipStream_t stream)
 {
     const int lds = latent_lds(16 * MT, KT, R, sizeof(T));
     static bool once = false;
@@ -344,9 +394,9 @@ static int latent_go(
         once = true;
     }
     k_latent_attn<T, MT, KT, NT><<<dim3(n_items, split), 256, lds, stream>>>(
-        (T*)out, (float*)op, (float*)mp, (const T*)q, (const T*)pool,
+        (T*)out, (T*)op, (float*)mp, (const T*)q, (const T*)pool,
         (const int*)ptab, (const int*)slot, (const int*)pos,
-        (const int*)items, per_seq, H, R, psz, maxp, scale, rows_total,
+        (const int*)items, per_seq, H, R, pshift, maxp, scale, rows_total,
         split);
     return (int)hipGetLastError();
 }
@@ -369,6 +419,8 @@ extern "C" int latent_attn(
     int maxp, float scale, int64_t rows_total, int64_t row_base,
     int64_t rows_here, int split, hipStream_t stream)
 {
+    if (psz & (psz - 1) || split > 64) return (int)hipErrorInvalidValue;
+    const int pshift = __builtin_ctz(psz);
     const int esz = f32 ? 4 : 2;
     const int mt = latent_mt(f32, H, R);
     const int budget = 80 * 1024;            // two blocks a CU if possible
@@ -381,7 +433,8 @@ extern "C" int latent_attn(
     #define LA(T, M, K, N)                                                 \
         err = latent_go<T, M, K, N>(                                       \
             out, o_part, ml_part, q, pool, ptab, slot, pos, items,         \
-            n_items, per_seq, H, R, psz, maxp, scale, rows_total, split,   \
+            n_items, per_seq, H, R, pshift, maxp, scale, rows_total,       \
+            split,                                                         \
             stream)
     #define LA_N(T, M, K)                                                  \
         do {                                                               \
@@ -403,14 +456,13 @@ extern "C" int latent_attn(
     #undef LA_N
     #undef LA
     if (err || split == 1) return err;
-    if (f32)
-        k_latent_combine<float><<<(int)rows_here, 128, 0, stream>>>(
-            (float*)out, (const float*)o_part, (const float*)ml_part,
-            row_base, rows_total, R, split);
-    else
-        k_latent_combine<bf16><<<(int)rows_here, 128, 0, stream>>>(
-            (bf16*)out, (const float*)o_part, (const float*)ml_part,
-            row_base, rows_total, R, split);
+    #define LC_GO(T, V)                                                    \
+        k_latent_combine<T, V><<<(int)rows_here, 128, 0, stream>>>(        \
+            (T*)out, (const T*)o_part, (const float*)ml_part, row_base,    \
+            rows_total, R, split)
+    if (f32) { if (R % 4) LC_GO(float, 1); else LC_GO(float, 4); }
+    else { if (R % 4) LC_GO(bf16, 1); else LC_GO(bf16, 4); }
+    #undef LC_GO
     return (int)hipGetLastError();
 }
 
@@ -662,7 +714,7 @@ extern "C" int flash_attn(
     return err;
 }
 
-// Gather of several sequences' latents, 64 positions a block: groups
+// Gather of several sequences' latents in groups of 64 positions: groups
 // int32 [n, 3] (slot, first position, rows that exist); the rest is zero.
 template <typename T>
 __global__ __launch_bounds__(256) void k_latent_gather_groups(
@@ -674,7 +726,7 @@ __global__ __launch_bounds__(256) void k_latent_gather_groups(
     const int* row = ptab + (int64_t)gp[0] * maxp;
     const int base = gp[1], have = gp[2];
     const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    for (int j = wid; j < 64; j += 4) {
+    for (int j = blockIdx.y * 16 + wid; j < blockIdx.y * 16 + 16; j += 4) {
         T* dst = out + ((int64_t)blockIdx.x * 64 + j) * R;
         if (j >= have) {
             for (int i = lane; i < R; i += 64) stf(dst + i, 0.f);
@@ -695,11 +747,11 @@ extern "C" int latent_gather(
     const void* groups, int n, int R, int psz, int maxp, hipStream_t stream)
 {
     if (f32)
-        k_latent_gather_groups<float><<<n, 256, 0, stream>>>(
+        k_latent_gather_groups<float><<<dim3(n, 4), 256, 0, stream>>>(
             (float*)out, (const float*)pool, (const int*)ptab,
             (const int*)groups, R, psz, maxp);
     else
-        k_latent_gather_groups<bf16><<<n, 256, 0, stream>>>(
+        k_latent_gather_groups<bf16><<<dim3(n, 4), 256, 0, stream>>>(
             (bf16*)out, (const bf16*)pool, (const int*)ptab,
             (const int*)groups, R, psz, maxp);
     return (int)hipGetLastError();

@@ -70,6 +70,24 @@ DEV void stv(bf16* p, const float* o) {
     }
 }
 
+// Activation-fragment layout ("frag"): the SAME MFMA fragment order the
+// weight packs use, applied to a [32, K] activation: element (m, k) with
+// k = b*64 + j*16 + h*8 + e lives at 16-byte unit ((b*4 + j)*64 + h*32
+// + m), elem e.  Producers (GEMM epilogues, decode-attention combine,
+// the embedding fragify kernel) write it; consumers stream it LINEARLY
+// exactly like packed weights — the per-iteration x machinery (32-line
+// scattered loads or LDS staging, measured 15-30% on top of the pure
+// stream) disappears.  Buffers are always 32 rows; rows >= M hold
+// garbage that MFMA carries in dead accumulator rows (never stored).
+DEV int64_t frag_off(int m, int kcol) {
+    const int b = kcol >> 6, j = (kcol >> 4) & 3, h = (kcol >> 3) & 1;
+    return ((((int64_t)b * 4 + j) * 64) + h * 32 + m) * 8 + (kcol & 7);
+}
+// row r of a batch of up to 64: two halves of 32 rows, `cols` wide
+DEV int64_t frag_row_off(int r, int c, int cols) {
+    return (int64_t)(r >> 5) * 32 * cols + frag_off(r & 31, c);
+}
+
 DEV float wave_sum(float x) {
     #pragma unroll
     for (int o = 32; o; o >>= 1) x += __shfl_xor(x, o, 64);

@@ -27,30 +27,12 @@
 // any K%64==0, N%32==0, M<=64).  Wave partials meet in a single
 // end-of-kernel LDS reduce (the ONE barrier, after all streaming).
 // ksplit>1 writes fp32 partials; k_wstream_combine folds them (+bias).
-#include <hip/hip_runtime.h>
-#include <hip/hip_bf16.h>
-#include <cstdint>
+#include "tile_mma.h"
 
-typedef __hip_bfloat16 bf16;
-typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(16))) float f32x16;
 typedef __attribute__((ext_vector_type(4))) unsigned int u32x4;
 
 union u4bf8 { u32x4 u; bf16x8 v; };
-
-// Activation-fragment layout ("frag"): the SAME MFMA fragment order the
-// weight packs use, applied to a [32, K] activation: element (m, k) with
-// k = b*64 + j*16 + h*8 + e lives at 16-byte unit ((b*4 + j)*64 + h*32
-// + m), elem e.  Producers (GEMM epilogues, decode-attention combine,
-// the embedding fragify kernel) write it; consumers stream it LINEARLY
-// exactly like packed weights — the per-iteration x machinery (32-line
-// scattered loads or LDS staging, measured 15-30% on top of the pure
-// stream) disappears.  Buffers are always 32 rows; rows >= M hold
-// garbage that MFMA carries in dead accumulator rows (never stored).
-static __device__ __forceinline__ int64_t frag_off(int m, int kcol) {
-    const int b = kcol >> 6, j = (kcol >> 4) & 3, h = (kcol >> 3) & 1;
-    return ((((int64_t)b * 4 + j) * 64) + h * 32 + m) * 8 + (kcol & 7);
-}
 
 // Pure-stream diagnostic: same grid/geometry/addressing as the GEMM but
 // only the nt weight loads (no x, no MFMA) — measures this geometry's

@@ -269,6 +269,10 @@ class RinitarModel:
         self._pack_weights()
 
     def _pack_weights(self):
+        """Packed copies for the weight-streaming decode products.  When
+        every matrix has one, a decode step keeps its activations in the
+        fragment layout those products read (frag_decode)."""
+        self.embed_pk, self.frag_decode = None, False
         if self.device.type != "cuda" or self.dtype != torch.bfloat16 \
                 or os.environ.get("OLLAMAMQ_NO_PACK") == "1":
             return
@@ -278,6 +282,10 @@ class RinitarModel:
         for layer in self.layers:
             layer.packs = {n: ops.pack_weight(w)
                            for n, w in layer.matrices().items()}
+        self.embed_pk = ops.pack_weight(self.embed)
+        self.frag_decode = self.embed_pk is not None and all(
+            p is not None for layer in self.layers
+            for p in layer.packs.values())
 
     def weight_bytes(self) -> int:
         n = self.embed.numel()
@@ -285,19 +293,19 @@ class RinitarModel:
             n += sum(w.numel() for w in layer.matrices().values())
         return n * self.embed.element_size()
 
-    def _mixer(self, layer, run, h, cache, slot_ids, positions, meta):
+    def _mixer(self, layer, run, h, cache, slot_ids, positions, meta, frag):
         p = ops.linear(h, layer.w_in, packed=layer.packs.get("w_in"))
         s = layer.spec
         if s.type == "gla":
             o = ops.gla(p, layer.gla, cache.state[run]["gla"], slot_ids,
-                        positions, meta)
+                        positions, meta, frag)
         else:
             qk = s.heads * s.dim
             ops.latent_append(cache, run, p[:, qk:qk + s.kv_rank],
                               layer.dkv_norm, slot_ids, positions,
                               self.cfg.eps)
             o = ops.latent_attention(p[:, :qk], cache, run, layer.latent,
-                                     slot_ids, positions, meta)
+                                     slot_ids, positions, meta, frag)
         return ops.linear_parts(o, layer.w_o, layer.packs.get("w_o"))
 
     def forward(
@@ -312,27 +320,33 @@ class RinitarModel:
         """Logits (or final-norm hidden states) of the rows attn_meta
         selects."""
         meta, eps = attn_meta, self.cfg.eps
+        frag = (self.frag_decode and meta.one_each
+                and tokens.shape[0] <= 64)
         x = y = post = None
         for run, li in enumerate(self.cfg.runs):
             layer = self.layers[li]
             shift = ops.TokenShift(layer.shift, kv_cache.state[run]["prev"],
                                    slot_ids, positions, meta)
             x, h = ops.dyt_residual(x, y, post, layer.norm1, shift,
-                                    embed=self.embed, tokens=tokens)
+                                    embed=self.embed, tokens=tokens,
+                                    frag=frag)
             y = self._mixer(layer, run, h, kv_cache, slot_ids, positions,
-                            meta)
+                            meta, frag)
             post = layer.norm1b
             if layer.spec.ff:
                 x, h = ops.dyt_residual(x, y, post, layer.norm2,
-                                        embed=self.embed)
+                                        embed=self.embed, frag=frag)
                 z = ops.linear_parts(h, layer.w_up, layer.packs.get("w_up"))
-                a = ops.polynorm(z, layer.act, eps)
+                a = ops.polynorm(z, layer.act, eps, frag)
                 y = ops.linear_parts(a, layer.w_down,
                                      layer.packs.get("w_down"))
                 post = layer.norm2b
+        frag = frag and not return_hidden
         _, h = ops.dyt_residual(x, y, post, self.final_norm,
                                 embed=self.embed, tokens=tokens,
-                                rows=meta.logits_idx, need_x=False)
+                                rows=meta.logits_idx, need_x=False,
+                                frag=frag)
         if return_hidden:
             return h
-        return ops.linear(h, self.embed)
+        return ops.linear(h, self.embed,
+                          packed=self.embed_pk if frag else None)

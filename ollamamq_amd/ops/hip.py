@@ -14,7 +14,7 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .interface import AttnMeta, Partials
+from .interface import AttnMeta, FragRows, Partials
 
 _LIB_PATH = os.path.join(
     os.path.dirname(os.path.dirname(os.path.abspath(__file__))),
@@ -71,12 +71,12 @@ def _try_load():
                                           vp, vp, vp, i, i, i, i, i, vp]
     lib.dyt_residual.argtypes = [i, vp, vp, vp, vp, vp, vp, vp, i,
                                  vp, vp, f, vp, vp, f, vp, vp, vp, vp, vp,
-                                 vp, vp, i, i, i, vp]
-    lib.polynorm.argtypes = [i, vp, vp, vp, i, f, f, f, f, i, i, f, vp]
+                                 vp, vp, i, i, i, i, vp]
+    lib.polynorm.argtypes = [i, vp, vp, vp, i, f, f, f, f, i, i, f, i, vp]
     lib.latent_append.argtypes = [i, vp, vp, i64, vp, vp, vp, vp,
                                   i, i, i, i, f, vp]
     lib.latent_gather.argtypes = [i, vp, vp, vp, vp, i, i, i, i, vp]
-    lib.head_gemm.argtypes = [i, vp, vp, vp, i, i, i, i, i64, vp]
+    lib.head_gemm.argtypes = [i, vp, vp, vp, i, i, i, i, i64, i, vp]
     lib.latent_mt.argtypes = [i, i, i]
     lib.latent_attn.argtypes = [i, vp, vp, vp, vp, vp, vp, vp, vp, vp,
                                 i, i, i, i, i, i, f, i64, i64, i64, i, vp]
@@ -84,7 +84,7 @@ def _try_load():
     lib.flash_attn.argtypes = [i, vp, vp, vp, vp, vp, i, i, i, i, i64, i64,
                                f, vp]
     lib.gla_step.argtypes = [i, vp, vp, i64, i, i, i, i, i, i, vp, vp, vp,
-                             vp, vp, vp, vp, i, i, i, i, f, f, f, vp]
+                             vp, vp, vp, vp, i, i, i, i, f, f, f, i, vp]
     lib.gla_chunks.argtypes = [i, vp, vp, vp, vp, i64, i, i, i, i, i, i,
                                vp, vp, vp, vp, vp, vp, vp, i, vp, i, i, i,
                                i, i, i, f, f, f, vp]
@@ -685,6 +685,9 @@ def wstream_pure(packed, N, K, ks):
 
 
 def linear(x, weight, bias=None, packed=None):
+    if isinstance(x, FragRows):
+        assert bias is None
+        return _linear_frag(x, weight.shape[0], packed, False)
     M, K = x.shape
     N = weight.shape[0]
     if packed is not None and USE_WSTREAM and M <= 64 \
@@ -748,11 +751,37 @@ def _i32(t):
     return t if t.dtype == torch.int32 else t.int()
 
 
+def _frag_rows(M, cols, like):
+    """Buffer of an activation in fragment layout: 32-row halves."""
+    return FragRows(torch.empty(-(-M // 32) * 32 * cols,
+                                dtype=torch.bfloat16, device=like.device),
+                    M, cols)
+
+
+def _linear_frag(x, N, packed, parts):
+    """Weight-streaming product of an activation in fragment layout."""
+    M, K = x.rows, x.cols
+    ks = _wstream_ksplit(N, K)
+    y = part = None
+    if ks > 1:
+        part = torch.empty((ks, M, N), dtype=torch.float32,
+                           device=packed.device)
+    if ks == 1 or not parts:
+        y = torch.empty((M, N), dtype=torch.bfloat16, device=packed.device)
+    _check(_lib.wstream_gemm_bf16(
+        _p(y), _p(part), _p(x.buf), _p(packed), _p(None), M, N, K, 0, ks,
+        _WS_DEPTH, 2, _p(None), 0, 0.0, 0.0, _p(None), _p(None), 0,
+        _stream()), "wstream_gemm")
+    return y if y is not None else Partials(part)
+
+
 def linear_parts(x, weight, packed=None):
     """Decode: the weight-streaming product, left as split-K partial sums
     where it splits (the next kernel folds them in)."""
-    M, K = x.shape
     N = weight.shape[0]
+    if isinstance(x, FragRows):
+        return _linear_frag(x, N, packed, True)
+    M, K = x.shape
     if packed is not None and USE_WSTREAM and M <= 64 and N <= _WS_MAX_N \
             and x.dtype == torch.bfloat16 and x.stride(1) == 1:
         ks = int(_WS_KS) if _WS_KS else _wstream_ksplit(N, K)
@@ -780,7 +809,8 @@ def _row_seq(meta):
     return t
 
 
-def dyt_residual(x, y, post, pre, shift, embed, tokens, rows, need_x):
+def dyt_residual(x, y, post, pre, shift, embed, tokens, rows, need_x,
+                 frag=False):
     parts = y.parts if isinstance(y, Partials) else None
     yt = None if parts is not None else y
     W = pre.w.shape[0]
@@ -794,7 +824,12 @@ def dyt_residual(x, y, post, pre, shift, embed, tokens, rows, need_x):
                           and yt.dtype == dtype)
     assert parts is None or parts.shape[1:] == (T_in, W)
     n = T_in if rows is None else rows.shape[0]
-    h = torch.empty((n, W), dtype=dtype, device=pre.w.device)
+    if frag:
+        assert dtype == torch.bfloat16 and W % 64 == 0
+        res = _frag_rows(n, W, pre.w)
+        h = res.buf
+    else:
+        res = h = torch.empty((n, W), dtype=dtype, device=pre.w.device)
     if x is not None and y is None and rows is None:
         x_out, write = x, None               # nothing to add
     else:
@@ -812,28 +847,33 @@ def dyt_residual(x, y, post, pre, shift, embed, tokens, rows, need_x):
     tok = None if tokens is None else _i32(tokens)
     z = post if post is not None else pre
     if n == 0:
-        return x_out, h
+        return x_out, res
     _check(_lib.dyt_residual(
         _is_f32(h), _p(write), _p(h), _p(x), _p(embed), _p(tok), _p(yt),
         _p(parts), 0 if parts is None else parts.shape[0],
         _p(z.w), _p(z.b), z.alpha, _p(pre.w), _p(pre.b), pre.alpha,
         _p(mix), _p(prev), _p(slot), _p(pos), _p(row_seq), _p(cu), _p(rows),
-        n, T_in, W, _stream()), "dyt_residual")
-    return x_out, h
+        n, T_in, W, int(frag), _stream()), "dyt_residual")
+    return x_out, res
 
 
-def polynorm(z, coef, eps):
+def polynorm(z, coef, eps, frag=False):
     parts = z.parts if isinstance(z, Partials) else None
     T, F = (z if parts is None else parts[0]).shape
     dtype = torch.bfloat16 if parts is not None else z.dtype
-    out = torch.empty((T, F), dtype=dtype, device=(
-        z if parts is None else parts).device)
+    like = z if parts is None else parts
+    if frag:
+        assert dtype == torch.bfloat16 and F % 64 == 0
+        res = _frag_rows(T, F, like)
+        out = res.buf
+    else:
+        res = out = torch.empty((T, F), dtype=dtype, device=like.device)
     assert parts is not None or z.is_contiguous()
     _check(_lib.polynorm(
         _is_f32(out), _p(out), _p(None if parts is not None else z),
         _p(parts), 0 if parts is None else parts.shape[0], *coef, T, F,
-        float(eps), _stream()), "polynorm")
-    return out
+        float(eps), int(frag), _stream()), "polynorm")
+    return res
 
 
 def latent_append(cache, run, d, weight, slot_ids, positions, eps):
@@ -847,20 +887,23 @@ def latent_append(cache, run, d, weight, slot_ids, positions, eps):
         "latent_append")
 
 
-def head_gemm(x, w, out):
-    """out[t, h] = w[h] @ x[t, h]; x [T, H, K] (rows may be strided)."""
+def head_gemm(x, w, out, frag=False):
+    """out[t, h] = w[h] @ x[t, h]; x [T, H, K] (rows may be strided); frag:
+    out is the buffer of a FragRows."""
     T, H, K = x.shape
     N = w.shape[1]
     assert w.shape == (H, N, K) and w.is_contiguous() \
-        and out.shape == (T, H, N) and out.is_contiguous() \
+        and (frag or out.shape == (T, H, N)) and out.is_contiguous() \
         and x.stride(2) == 1 and (H == 1 or x.stride(1) == K)
     if T:
         _check(_lib.head_gemm(_is_f32(x), _p(out), _p(x), _p(w), T, H, N, K,
-                              x.stride(0), _stream()), "head_gemm")
+                              x.stride(0), int(frag), _stream()),
+               "head_gemm")
     return out
 
 
 LATENT_MAX_R = 1024       # absorbed kernel: latent width
+LATENT_SPLIT_MAX = 64     # and context segments
 FLASH_MAX = 256           # expanded kernel: key and value widths
 EXPAND_BYTES = 1 << 30    # expanded keys and values held at a time
 
@@ -932,12 +975,12 @@ def _latent_absorbed(o, q, cache, run, slots, pos, H, R, scale, items,
                      n_items, per_seq, row0, rows, max_kv):
     """One launch of the absorbed kernel over rows row0.. of q / o."""
     f32 = _is_f32(q)
-    split = int(max(1, min(512 // n_items, (max_kv + 127) // 128, 32)))
+    split = int(max(1, min(512 // n_items, (max_kv + 63) // 64,
+                           LATENT_SPLIT_MAX)))
     op = ml = None
     total = q.shape[0]
     if split > 1:
-        op = torch.empty((split, total, R), dtype=torch.float32,
-                         device=q.device)
+        op = torch.empty((split, total, R), dtype=q.dtype, device=q.device)
         ml = torch.empty((split, total, 2), dtype=torch.float32,
                          device=q.device)
     pool = cache.latent_pool[run]
@@ -949,7 +992,8 @@ def _latent_absorbed(o, q, cache, run, slots, pos, H, R, scale, items,
         row0, rows, split, _stream()), "latent_attn")
 
 
-def latent_attention(q, cache, run, w, slot_ids, positions, meta):
+def latent_attention(q, cache, run, w, slot_ids, positions, meta,
+                     frag=False):
     H, D, R = w.uk.shape
     V = w.uv.shape[1]
     T = q.shape[0]
@@ -957,7 +1001,12 @@ def latent_attention(q, cache, run, w, slot_ids, positions, meta):
     if R > LATENT_MAX_R and (max(D, V) > FLASH_MAX or meta.n_single):
         raise ValueError(f"latent attention with rank {R}, head widths "
                          f"{D}/{V}: no kernel")
-    out = torch.empty((T, H, V), dtype=q.dtype, device=q.device)
+    assert not frag or meta.one_each
+    if frag:
+        res = _frag_rows(T, H * V, q)
+        out = res.buf
+    else:
+        out = torch.empty((T, H, V), dtype=q.dtype, device=q.device)
     slots, pos = _i32(slot_ids), _i32(positions)
     nd = meta.n_single
     if meta.one_each:
@@ -979,7 +1028,10 @@ def latent_attention(q, cache, run, w, slot_ids, positions, meta):
             _latent_absorbed(o, lat, cache, run, slots, pos, H, R, w.scale,
                              items, items.shape[0], 1, nd * H,
                              (n_abs - nd) * H, kv_abs)
-        head_gemm(o.view(n_abs, H, R), w.uv, out[:n_abs])
+        head_gemm(o.view(n_abs, H, R), w.uv, out if frag else out[:n_abs],
+                  frag)
+        if frag:
+            return res
     pool = cache.latent_pool[run]
     for gather, tiles, kv in groups:
         c = torch.empty((kv, R), dtype=q.dtype, device=q.device)
@@ -1024,30 +1076,35 @@ def _gla_plan(meta, dev, step_tokens):
     return plan
 
 
-def gla(p, w, state, slot_ids, positions, meta):
+def gla(p, w, state, slot_ids, positions, meta, frag=False):
     T = p.shape[0]
     H, D, V = w.heads, w.dim, w.vdim
     assert p.stride(1) == 1 and state.dtype == torch.float32 \
         and state.shape[1:] == (H, D, V) and w.a2.dtype == p.dtype
     assert max(w.offsets) + w.rank <= p.shape[1]
-    out = torch.empty((T, H * V), dtype=p.dtype, device=p.device)
+    assert not frag or meta.one_each
+    if frag:
+        res = _frag_rows(T, H * V, p)
+        out = res.buf
+    else:
+        res = out = torch.empty((T, H * V), dtype=p.dtype, device=p.device)
     slots, pos = _i32(slot_ids), _i32(positions)
     f32 = _is_f32(p)
     head = (_p(p), p.stride(0), *w.offsets, w.rank, _p(w.a2), _p(w.a2_b),
             _p(w.norm), _p(state), _p(slots), _p(pos))
-    tail = (H, D, V, D ** -0.5, 1.0 / w.tau, float(w.eps), _stream())
+    tail = (H, D, V, D ** -0.5, 1.0 / w.tau, float(w.eps))
     nd = meta.n_single
     if nd:
-        _check(_lib.gla_step(f32, _p(out), *head, _p(None), nd, *tail),
-               "gla_step")
+        _check(_lib.gla_step(f32, _p(out), *head, _p(None), nd, *tail,
+                             int(frag), _stream()), "gla_step")
     if meta.one_each:
-        return out
+        return res
     chunked = D <= GLA_CHUNK_MAX[0] and w.rank <= GLA_CHUNK_MAX[1]
     spans, chunks, seqs, base, rows = _gla_plan(
         meta, p.device, GLA_STEP_TOKENS if chunked else 1 << 62)
     if spans is not None:
         _check(_lib.gla_step(f32, _p(out), *head, _p(spans),
-                             spans.shape[0], *tail), "gla_step")
+                             spans.shape[0], *tail, 0, _stream()), "gla_step")
     if chunks is not None:
         nc = chunks.shape[0]
         scr = torch.empty(_lib.gla_scratch_floats(nc, H, D),
@@ -1055,7 +1112,7 @@ def gla(p, w, state, slot_ids, positions, meta):
         o = torch.empty(rows * H * V, dtype=torch.float32, device=p.device)
         _check(_lib.gla_chunks(
             f32, _p(out), _p(scr), _p(o), *head, _p(chunks), nc, _p(seqs),
-            seqs.shape[0], base, rows, *tail), "gla_chunks")
+            seqs.shape[0], base, rows, *tail, _stream()), "gla_chunks")
     return out
 
 

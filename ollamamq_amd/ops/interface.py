@@ -100,6 +100,14 @@ class Partials(NamedTuple):
     parts: torch.Tensor
 
 
+class FragRows(NamedTuple):
+    """A bf16 activation [rows, cols] in the layout in which the
+    weight-streaming product reads it (GPU decode, up to 64 rows)."""
+    buf: torch.Tensor
+    rows: int
+    cols: int
+
+
 class LatentWeights(NamedTuple):
     """k = uk c, v = uv c per head; uk [H, D, R], uk_t [H, R, D] and
     uv [H, V, R] are views or copies of the same values."""
@@ -179,7 +187,7 @@ def linear(x, weight, bias=None, packed=None):
     decode path (M<=64) a hand-written weight-streaming MFMA kernel runs
     over the pre-packed copy when `packed` is provided (hipBLASLt measured
     1.8-4.6 TB/s vs the ~6.3 TB/s streaming roofline on these shapes)."""
-    if _use_hip(x):
+    if _use_hip(weight):
         from . import hip
         return hip.linear(x, weight, bias, packed)
     return torch.nn.functional.linear(x, weight, bias)
@@ -199,7 +207,7 @@ def pack_weight(w):
 
 def linear_parts(x, weight, packed=None) -> Union[torch.Tensor, Partials]:
     """As linear, but a split product may come back as its partial sums."""
-    if _use_hip(x):
+    if _use_hip(weight):
         from . import hip
         return hip.linear_parts(x, weight, packed)
     return torch.nn.functional.linear(x, weight)
@@ -207,25 +215,25 @@ def linear_parts(x, weight, packed=None) -> Union[torch.Tensor, Partials]:
 
 def dyt_residual(x, y, post: Optional[DyT], pre: DyT,
                  shift: Optional[TokenShift] = None, embed=None, tokens=None,
-                 rows=None, need_x=True):
+                 rows=None, need_x=True, frag=False):
     """One pass between two matrix products: x' = x + post(y), h = pre(x'),
     then the token shift.  x is fp32 [T, W], or None for the embedding rows
     of `tokens`; y a tensor, Partials or None; `rows` selects the rows to
-    compute.  Returns (x', h)."""
+    compute; frag returns h as FragRows.  Returns (x', h)."""
     if _use_hip(pre.w):
         from . import hip
         return hip.dyt_residual(x, y, post, pre, shift, embed, tokens, rows,
-                                need_x)
+                                need_x, frag)
     return ref.dyt_residual(x, y, post, pre, shift, embed, tokens, rows)
 
 
-def polynorm(z, coef, eps):
+def polynorm(z, coef, eps, frag=False):
     """a N(z) + b N(z^2) + c N(z^3) + e with coef = (a, b, c, e) and N the
     division by the row's root mean square."""
     t = z.parts if isinstance(z, Partials) else z
     if _use_hip(t):
         from . import hip
-        return hip.polynorm(z, coef, eps)
+        return hip.polynorm(z, coef, eps, frag)
     return ref.polynorm(z, coef, eps)
 
 
@@ -239,23 +247,24 @@ def latent_append(cache, run, d, weight, slot_ids, positions, eps):
 
 
 def latent_attention(q, cache, run, w: LatentWeights, slot_ids, positions,
-                     meta: AttnMeta):
+                     meta: AttnMeta, frag=False):
     """Causal softmax attention whose keys and values are linear in the
     cached latent.  q [T, H*D] (rows may be strided) -> [T, H*V]."""
     if _use_hip(q):
         from . import hip
         return hip.latent_attention(q, cache, run, w, slot_ids, positions,
-                                    meta)
+                                    meta, frag)
     return ref.latent_attention(q, cache, run, w, meta)
 
 
-def gla(p, w: GlaWeights, state, slot_ids, positions, meta: AttnMeta):
+def gla(p, w: GlaWeights, state, slot_ids, positions, meta: AttnMeta,
+        frag=False):
     """Gated linear attention over the fused projection p [T, ...]; state
     [slots, H, D, V] fp32 is read and advanced.  Head norm and output gate
     included.  -> [T, H*V]."""
     if _use_hip(p):
         from . import hip
-        return hip.gla(p, w, state, slot_ids, positions, meta)
+        return hip.gla(p, w, state, slot_ids, positions, meta, frag)
     return ref.gla(p, w, state, meta)
 
 

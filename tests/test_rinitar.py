@@ -79,7 +79,7 @@ MODELS = {
     "only-gla": config(64, 96, [gla_layer(2, 64, 64, 16.0, 64),
                                 gla_layer(4, 16, 32, 8.0)]),
     "only-latent": config(192, 96, [latent_layer(20, 64, 64, 128, 0.125, 128),
-                                    latent_layer(3, 72, 136, 40, 0.3)],
+                                    latent_layer(3, 72, 128, 40, 0.3)],
                           loop=(1, 2, 3)),
 }
 A1_RANK = {"mixed": 8, "odd": 5, "only-gla": 16, "only-latent": 1}
