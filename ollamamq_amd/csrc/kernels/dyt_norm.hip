@@ -37,7 +37,7 @@ template <typename T> DEV float tanh_of(float x) {
     else return tanh_fast(x);
 }
 
-template <typename T, int VEC>
+template <typename T, int VEC, bool FR>   // FR: h_out in fragment layout
 __global__ __launch_bounds__(256) void k_dyt(
     float* __restrict__ x_out,          // [n, W] or null
     T* __restrict__ h_out,              // [n, W]
@@ -53,7 +53,7 @@ __global__ __launch_bounds__(256) void k_dyt(
     const int* __restrict__ row_seq,    // null: every row its own sequence
     const int* __restrict__ cu_q,
     const int64_t* __restrict__ rows,   // null, or the rows to compute
-    int n, int T_in, int W, int strip, int frag)   // frag: layout of h_out
+    int n, int T_in, int W, int strip)
 {
     const int c = (blockIdx.y * 256 + threadIdx.x) * VEC;
     if (c >= W) return;
@@ -90,7 +90,7 @@ __global__ __launch_bounds__(256) void k_dyt(
     };
 
     auto h_at = [&](int r) {
-        return h_out + (frag ? frag_row_off(r, c, W) : (int64_t)r * W + c);
+        return h_out + (FR ? frag_row_off(r, c, W) : (int64_t)r * W + c);
     };
     const int r0 = blockIdx.x * strip;
     const int r1 = min(r0 + strip, n);
@@ -151,15 +151,18 @@ static int dyt_launch(
     int strip = 1;
     while (strip < 8 && (int64_t)n * cols / (strip * 2) >= 2048) strip *= 2;
     dim3 grid((n + strip - 1) / strip, cols);
-    #define DYT_GO(V)                                                      \
-        k_dyt<T, V><<<grid, 256, 0, stream>>>(                             \
+    #define DYT_GO(V, F)                                                   \
+        k_dyt<T, V, F><<<grid, 256, 0, stream>>>(                             \
             (float*)x_out, (T*)h_out, (const float*)x_in,                  \
             (const T*)embed, (const int*)tokens, (const T*)y,              \
             (const float*)y_part, n_part, post, pre, (const float*)mix,    \
             (float*)prev, (const int*)slot, (const int*)pos,               \
             (const int*)row_seq, (const int*)cu_q, (const int64_t*)rows,   \
-            n, T_in, W, strip, frag)
-    if (v4) DYT_GO(4); else DYT_GO(1);
+            n, T_in, W, strip)
+    if (frag && !v4) return (int)hipErrorInvalidValue;
+    if (frag) DYT_GO(4, true);
+    else if (v4) DYT_GO(4, false);
+    else DYT_GO(1, false);
     #undef DYT_GO
     return (int)hipGetLastError();
 }
@@ -183,19 +186,19 @@ extern "C" int dyt_residual(
 
 // ---------------------------------------------------------------------------
 // PolyNorm: out = a z/rms(z) + b z^2/rms(z^2) + c z^3/rms(z^3) + e, the rms
-// over the row.  One block per row; rows up to NV*256*VEC stay in registers
-// between the two passes (NV == 0: the second pass reads again).
+// over the row.  One block of BS threads per row; rows up to NV*BS*VEC stay
+// in registers between the two passes (NV == 0: the second pass reads
+// again).  FR: out in the activation-fragment layout.
 // ---------------------------------------------------------------------------
-template <typename T, int VEC, int NV>
-__global__ __launch_bounds__(256) void k_polynorm(
+template <typename T, int VEC, int NV, int BS, bool FR>
+__global__ __launch_bounds__(BS) void k_polynorm(
     T* __restrict__ out, const T* __restrict__ z,
     const float* __restrict__ z_part, int n_part, int64_t part_stride,
-    float ca, float cb, float cc, float ce, int F, float eps,
-    int frag)                           // layout of out
+    float ca, float cb, float cc, float ce, int F, float eps)
 {
     const int64_t row = blockIdx.x;
     const int tid = threadIdx.x;
-    __shared__ float red[3][4];
+    __shared__ float red[3][BS / 64];
     auto load = [&](int c, float* v) {
         if (z) { ldv<VEC>(z + row * F + c, v); return; }
         ldv<VEC>(z_part + row * F + c, v);
@@ -220,11 +223,11 @@ __global__ __launch_bounds__(256) void k_polynorm(
     if constexpr (NV > 0) {
         #pragma unroll
         for (int j = 0; j < NV; j++) {
-            const int c = (j * 256 + tid) * VEC;
+            const int c = (j * BS + tid) * VEC;
             if (c < F) { load(c, keep[j]); stat(keep[j]); }
         }
     } else {
-        for (int c = tid * VEC; c < F; c += 256 * VEC) {
+        for (int c = tid * VEC; c < F; c += BS * VEC) {
             float v[VEC];
             load(c, v);
             stat(v);
@@ -237,7 +240,9 @@ __global__ __launch_bounds__(256) void k_polynorm(
     __syncthreads();
     const float inv = 1.f / F;
     auto scale = [&](int k, float coef) {
-        const float s = (red[k][0] + red[k][1]) + (red[k][2] + red[k][3]);
+        float s = 0.f;
+        #pragma unroll
+        for (int i = 0; i < BS / 64; i++) s += red[k][i];
         return coef / sqrtf(s * inv + eps);
     };
     const float a = scale(0, ca), b = scale(1, cb), g = scale(2, cc);
@@ -246,16 +251,16 @@ __global__ __launch_bounds__(256) void k_polynorm(
         #pragma unroll
         for (int i = 0; i < VEC; i++)
             o[i] = v[i] * (a + v[i] * (b + v[i] * g)) + ce;
-        stv<VEC>(out + (frag ? frag_row_off(row, c, F) : row * F + c), o);
+        stv<VEC>(out + (FR ? frag_row_off(row, c, F) : row * F + c), o);
     };
     if constexpr (NV > 0) {
         #pragma unroll
         for (int j = 0; j < NV; j++) {
-            const int c = (j * 256 + tid) * VEC;
+            const int c = (j * BS + tid) * VEC;
             if (c < F) emit(c, keep[j]);
         }
     } else {
-        for (int c = tid * VEC; c < F; c += 256 * VEC) {
+        for (int c = tid * VEC; c < F; c += BS * VEC) {
             float v[VEC];
             load(c, v);
             emit(c, v);
@@ -269,21 +274,28 @@ extern "C" int polynorm(
     int frag, hipStream_t stream)
 {
     const int64_t ps = (int64_t)T_rows * F;
-    #define PN_GO(T, V, NV)                                                \
-        k_polynorm<T, V, NV><<<T_rows, 256, 0, stream>>>(                  \
+    #define PN_GO(T, V, NV, BS, FR)                                        \
+        k_polynorm<T, V, NV, BS, FR><<<T_rows, BS, 0, stream>>>(           \
             (T*)out, (const T*)z, (const float*)z_part, n_part, ps,        \
-            ca, cb, cc, ce, F, eps, frag)
-    #define PN_TYPE(T)                                                     \
+            ca, cb, cc, ce, F, eps)
+    // few rows: more threads on each
+    #define PN_TYPE(T, FR)                                                 \
         do {                                                               \
-            if (F % 8) PN_GO(T, 1, 0);                                     \
-            else if (F <= 2048) PN_GO(T, 8, 1);                            \
-            else if (F <= 4096) PN_GO(T, 8, 2);                            \
-            else if (F <= 8192) PN_GO(T, 8, 4);                            \
-            else if (F <= 16384) PN_GO(T, 8, 8);                           \
-            else if (F <= 24576) PN_GO(T, 8, 12);                          \
-            else PN_GO(T, 8, 0);                                           \
+            if (F % 8) PN_GO(T, 1, 0, 256, false);                         \
+            else if (F <= 2048) PN_GO(T, 8, 1, 256, FR);                   \
+            else if (T_rows <= 256 && F <= 8192) PN_GO(T, 8, 1, 1024, FR); \
+            else if (T_rows <= 256 && F <= 24576)                          \
+                PN_GO(T, 8, 3, 1024, FR);                                  \
+            else if (F <= 4096) PN_GO(T, 8, 2, 256, FR);                   \
+            else if (F <= 8192) PN_GO(T, 8, 4, 256, FR);                   \
+            else if (F <= 16384) PN_GO(T, 8, 8, 256, FR);                  \
+            else if (F <= 24576) PN_GO(T, 8, 12, 256, FR);                 \
+            else PN_GO(T, 8, 0, 256, FR);                                  \
         } while (0)
-    if (f32) PN_TYPE(float); else PN_TYPE(bf16);
+    if (frag && (f32 || F % 64)) return (int)hipErrorInvalidValue;
+    if (f32) PN_TYPE(float, false);
+    else if (frag) PN_TYPE(bf16, true);
+    else PN_TYPE(bf16, false);
     #undef PN_TYPE
     #undef PN_GO
     return (int)hipGetLastError();

@@ -32,7 +32,7 @@ DEV float log_alpha(float z, float inv_tau) {
 DEV float silu(float x) { return x / (1.f + __expf(-x)); }
 
 template <typename T, int VEC>
-__global__ __launch_bounds__(256) void k_gla_step(
+__global__ __launch_bounds__(256, 2) void k_gla_step(
     T* __restrict__ out,                // [T, H*V]
     const T* __restrict__ p, GlaIn in,
     const T* __restrict__ a2, const float* __restrict__ a2_b,
@@ -56,9 +56,25 @@ __global__ __launch_bounds__(256) void k_gla_step(
     float* o_s = a_s + D;               // [RG][V]
     float* r_s = o_s + RG * V;          // [4]
     float* Sh = state + ((int64_t)slot[t0] * H + h) * D * V;
+    const int vt0 = rg < RG ? tid % nv : V;
     bool fresh = pos[t0] == 0;
+    // state rows in flight: the first are asked for before the decays are
+    // worked out, then always one group ahead
+    constexpr int PF = 8;
+    float nxt[PF][VEC];
+    auto ahead = [&](const float* S, int d0) {
+        #pragma unroll
+        for (int j = 0; j < PF; j++) {
+            const int d = d0 + j * RG;
+            if (!fresh && d < D) ldv<VEC>(S + (int64_t)d * V, nxt[j]);
+            else
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) nxt[j][i] = 0.f;
+        }
+    };
     for (int t = t0; t < t0 + nt; ++t) {
         const T* row = p + (int64_t)t * in.ld;
+        if (vt0 * VEC < V) ahead(Sh + vt0 * VEC, rg);
         for (int d = tid; d < D; d += 256) {
             const int c = h * D + d;
             q_s[d] = ldf(row + in.oq + c) * scale;
@@ -70,25 +86,29 @@ __global__ __launch_bounds__(256) void k_gla_step(
             a_s[d] = __expf(log_alpha(z, inv_tau));
         }
         __syncthreads();
-        for (int vt = rg < RG ? tid % nv : V; vt * VEC < V; vt += nv) {
+        for (int vt = vt0; vt * VEC < V; vt += nv) {
             float* S = Sh + vt * VEC;
             float v[VEC], acc[VEC] = {};
+            if (vt != vt0) ahead(S, rg);
             ldv<VEC>(row + in.ov + h * V + vt * VEC, v);
-            #pragma unroll 8
-            for (int d = rg; d < D; d += RG) {
-                float s[VEC];
-                if (fresh) {
-                    #pragma unroll
-                    for (int i = 0; i < VEC; i++) s[i] = k_s[d] * v[i];
-                } else {
-                    ldv<VEC>(S + (int64_t)d * V, s);
-                    #pragma unroll
-                    for (int i = 0; i < VEC; i++)
-                        s[i] = a_s[d] * s[i] + k_s[d] * v[i];
-                }
-                stv<VEC>(S + (int64_t)d * V, s);
+            for (int d0 = rg; d0 < D; d0 += RG * PF) {
+                float s[PF][VEC];
                 #pragma unroll
-                for (int i = 0; i < VEC; i++) acc[i] += q_s[d] * s[i];
+                for (int j = 0; j < PF; j++)
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) s[j][i] = nxt[j][i];
+                if (d0 + RG * PF < D) ahead(S, d0 + RG * PF);
+                #pragma unroll
+                for (int j = 0; j < PF; j++) {
+                    const int d = d0 + j * RG;
+                    if (d >= D) break;
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) {
+                        s[j][i] = a_s[d] * s[j][i] + k_s[d] * v[i];
+                        acc[i] += q_s[d] * s[j][i];
+                    }
+                    stv<VEC>(S + (int64_t)d * V, s[j]);
+                }
             }
             stv<VEC>(o_s + rg * V + vt * VEC, acc);
         }

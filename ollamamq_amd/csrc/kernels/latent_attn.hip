@@ -197,24 +197,36 @@ __global__ __launch_bounds__(256) void k_latent_attn(
         const int u = tid + j * 256;
         where[j] = u < KT * n8 ? (u / n8) << 16 | (u % n8) * 8 : -1;
     }
+    // Loads are unconditional, with keys and columns clamped to valid ones:
+    // a key past the end has weight zero, a column past R meets zeros of q'
+    // or is not stored.  Page numbers are fetched a chunk ahead.
     const int pmask = (1 << pshift) - 1;
+    int page[NP];
+    auto key_of = [&](int j, int base) {
+        return min(base + (max(where[j], 0) >> 16), kv_len - 1);
+    };
+    auto pages = [&](int base) {
+        #pragma unroll
+        for (int j = 0; j < NP; j++) page[j] = pt[key_of(j, base) >> pshift];
+    };
     auto fetch = [&](int base) {
         #pragma unroll
         for (int j = 0; j < NP; j++) {
-            if (where[j] < 0) continue;
-            const int key = base + (where[j] >> 16), c = where[j] & 0xffff;
-            const T* src = pool + (((int64_t)pt[min(key, kv_len - 1)
-                                    >> pshift] << pshift)
-                                   + (key & pmask)) * R;
-            if (key >= kv_len) piece[j] = frag_zero<T>();
-            else if (vec) piece[j] = c < R ? frag8(src + c) : frag_zero<T>();
+            const int c = max(where[j], 0) & 0xffff;
+            const T* src = pool + (((int64_t)page[j] << pshift)
+                                   + (key_of(j, base) & pmask)) * R;
+            if (vec) piece[j] = frag8(src + min(c, R - 8));
             else piece[j] = frag_guard(src, c, R);
         }
     };
     f32x4 acc[MT][NT] = {};
     __syncthreads();               // a segment may hold no chunk at all
 
-    if (c_lo < c_hi) fetch(c_lo * KT);
+    if (c_lo < c_hi) {
+        pages(c_lo * KT);
+        fetch(c_lo * KT);
+        pages((c_lo + 1) * KT);
+    }
     for (int ch = c_lo; ch < c_hi; ++ch) {
         const int base = ch * KT;
         #pragma unroll
@@ -224,7 +236,10 @@ __global__ __launch_bounds__(256) void k_latent_attn(
                     c_s + (where[j] >> 16) * cs + (where[j] & 0xffff))
                     = piece[j];
         __syncthreads();
-        if (ch + 1 < c_hi) fetch(base + KT);
+        if (ch + 1 < c_hi) {
+            fetch(base + KT);
+            pages(base + 2 * KT);
+        }
         #pragma unroll
         for (int i = 0; i < (MT * KT / 16 + 3) / 4; i++) {
             const int id = wid + i * 4;
@@ -341,6 +356,238 @@ __global__ __launch_bounds__(256) void k_latent_attn(
     }
 }
 
+// ---------------------------------------------------------------------------
+// The same for bf16 with R <= 16 * NT, R % 8 == 0: every wave is a whole
+// attention of its own.  Wave (row tile rh, key group kh) holds its q' rows
+// as matrix operands and its [R, 16] result in registers and takes its own
+// keys of each 64-key chunk:
+//   S^T = C q'^T, so a lane holds one row's scores for keys 4g + i, which is
+//   the operand layout of the second product: P never leaves the lane;
+//   O^T += C^T P^T with C^T read through the LDS transpose load.
+// The waves meet only at the double-buffered chunk and in the last merge.
+// ---------------------------------------------------------------------------
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
+
+// lane (lr, g) <- column c0 + lr of rows r0 + 4g .. +3, 16 columns of a tile
+DEV s16x4 tr_read(const bf16* tile, int stride, int lane) {
+    const int lr = lane & 15, g = lane >> 4;
+    const bf16* p = tile + (4 * g + (lr >> 2)) * stride + (lr & 3) * 4;
+    return __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+        (lds_s16x4*)const_cast<bf16*>(p));
+}
+
+template <int NT, int RH>
+__global__ __launch_bounds__(256, 1) void k_latent_mq(
+    bf16* __restrict__ out, bf16* __restrict__ o_part,
+    float* __restrict__ ml_part, const bf16* __restrict__ q,
+    const bf16* __restrict__ pool, const int* __restrict__ ptab,
+    const int* __restrict__ slot, const int* __restrict__ pos,
+    const int* __restrict__ items, int per_seq, int H, int R, int pshift,
+    int maxp, float scale, int64_t rows_total, int split)
+{
+    constexpr int M = 16 * RH, KH = 4 / RH, NK = 4 / KH, KT = 64;
+    constexpr int Rp = NT * 16, CS = Rp + 8;
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    const int rh = wid % RH, kh = wid / RH;
+    int row0, n_rows;
+    if (items) {
+        row0 = items[blockIdx.x * 2];
+        n_rows = items[blockIdx.x * 2 + 1];
+    } else {
+        const int j = blockIdx.x % per_seq;
+        row0 = (blockIdx.x / per_seq) * H + j * M;
+        n_rows = min(M, H - j * M);
+    }
+    const int tok0 = row0 / H, tok1 = (row0 + n_rows - 1) / H;
+    const int kv_len = pos[tok1] + 1;
+    const int* pt = ptab + (int64_t)slot[tok0] * maxp;
+    const int n_chunks = (kv_len + KT - 1) / KT;
+    const int c_lo = (int)((int64_t)blockIdx.y * n_chunks / split);
+    const int c_hi = (int)((int64_t)(blockIdx.y + 1) * n_chunks / split);
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    bf16* c_s = reinterpret_cast<bf16*>(smem);    // [2][KT][CS]
+
+    const int row = rh * 16 + lr;
+    const int my_lim = row < n_rows ? pos[(row0 + row) / H] + 1 : 0;
+    bf16x8 qf[NT / 2];
+    {
+        const bf16* qr = q + (int64_t)(row0 + min(row, n_rows - 1)) * R;
+        #pragma unroll
+        for (int k = 0; k < NT / 2; k++) {
+            const int c = k * 32 + g * 8;
+            qf[k] = c < R ? frag8(qr + c) : frag_zero<bf16>();
+        }
+    }
+    // pieces of a chunk: a row is NT*2 of them, so a wave reads whole rows
+    constexpr int NP = KT * NT * 2 / 256;
+    bf16x8 piece[NP];
+    const int pmask = (1 << pshift) - 1;
+    int page[NP];
+    auto key_of = [&](int j, int base) {
+        return min(base + (tid + j * 256) / (NT * 2), kv_len - 1);
+    };
+    auto pages = [&](int base) {
+        #pragma unroll
+        for (int j = 0; j < NP; j++) page[j] = pt[key_of(j, base) >> pshift];
+    };
+    auto fetch = [&](int base) {
+        #pragma unroll
+        for (int j = 0; j < NP; j++) {
+            const int c = min((tid + j * 256) % (NT * 2) * 8, R - 8);
+            piece[j] = frag8(pool + (((int64_t)page[j] << pshift)
+                                     + (key_of(j, base) & pmask)) * R + c);
+        }
+    };
+    auto put = [&](int buf) {
+        #pragma unroll
+        for (int j = 0; j < NP; j++) {
+            const int u = tid + j * 256;
+            *reinterpret_cast<bf16x8*>(
+                c_s + (buf * KT + u / (NT * 2)) * CS + u % (NT * 2) * 8)
+                = piece[j];
+        }
+    };
+    f32x4 acc[NT] = {};
+    float m = NEG, l = 0.f;
+    if (c_lo < c_hi) {
+        pages(c_lo * KT);
+        fetch(c_lo * KT);
+        pages((c_lo + 1) * KT);
+        put(0);
+    }
+    __syncthreads();
+    for (int ch = c_lo; ch < c_hi; ++ch) {
+        const int base = ch * KT + kh * NK * 16;
+        const bf16* ct = c_s + (((ch - c_lo) & 1) * KT + kh * NK * 16) * CS;
+        if (ch + 1 < c_hi) {
+            fetch((ch + 1) * KT);
+            pages((ch + 2) * KT);
+        }
+        f32x4 s[NK] = {};
+        {
+            f32x4 odd[NK] = {};              // two chains per tile
+            #pragma unroll
+            for (int k = 0; k < NT / 2; k++)
+                #pragma unroll
+                for (int j = 0; j < NK; j++) {
+                    const bf16x8 a = frag8(ct + (j * 16 + lr) * CS + k * 32
+                                           + g * 8);
+                    if (k & 1) odd[j] = mma(a, qf[k], odd[j]);
+                    else s[j] = mma(a, qf[k], s[j]);
+                }
+            #pragma unroll
+            for (int j = 0; j < NK; j++) s[j] += odd[j];
+        }
+        float mx = NEG;
+        #pragma unroll
+        for (int j = 0; j < NK; j++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const float v = base + j * 16 + g * 4 + i < my_lim
+                                    ? s[j][i] * scale : NEG;
+                s[j][i] = v;
+                mx = fmaxf(mx, v);
+            }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float mn = fmaxf(m, mx);
+        const float f = __expf(m - mn);
+        float sum = 0.f;
+        #pragma unroll
+        for (int j = 0; j < NK; j++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const float p = s[j][i] > NEG ? __expf(s[j][i] - mn) : 0.f;
+                s[j][i] = p;
+                sum += p;
+            }
+        sum += __shfl_xor(sum, 16, 64);
+        sum += __shfl_xor(sum, 32, 64);
+        l = l * f + sum;
+        m = mn;
+        if (!__all(f == 1.f)) {
+            #pragma unroll
+            for (int n = 0; n < NT; n++) acc[n] *= f;
+        }
+        if constexpr (NK == 2) {
+            bf16x8 b;
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                b[i] = (__bf16)s[0][i];
+                b[i + 4] = (__bf16)s[1][i];
+            }
+            #pragma unroll
+            for (int n = 0; n < NT; n++) {
+                const s16x4 a0 = tr_read(ct + n * 16, CS, lane);
+                const s16x4 a1 = tr_read(ct + 16 * CS + n * 16, CS, lane);
+                typedef __attribute__((ext_vector_type(8))) short s16x8;
+                const s16x8 a = __builtin_shufflevector(a0, a1, 0, 1, 2, 3,
+                                                        4, 5, 6, 7);
+                acc[n] = mma(__builtin_bit_cast(bf16x8, a), b, acc[n]);
+            }
+        } else {
+            bf16x4 b4;
+            #pragma unroll
+            for (int i = 0; i < 4; i++) b4[i] = (__bf16)s[0][i];
+            const s16x4 b = __builtin_bit_cast(s16x4, b4);
+            #pragma unroll
+            for (int n = 0; n < NT; n++)
+                acc[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(
+                    tr_read(ct + n * 16, CS, lane), b, acc[n], 0, 0, 0);
+        }
+        if (ch + 1 < c_hi) put((ch + 1 - c_lo) & 1);
+        __syncthreads();
+    }
+    // merge the key groups: each wave's scaled result, then a share of the
+    // column tiles per wave
+    float* ml_s = reinterpret_cast<float*>(smem);           // [4][16][2]
+    f32x4* o_s = reinterpret_cast<f32x4*>(smem + 512);      // [4][NT][64]
+    if (g == 0) {
+        ml_s[(wid * 16 + lr) * 2] = m;
+        ml_s[(wid * 16 + lr) * 2 + 1] = l;
+    }
+    __syncthreads();
+    float top = NEG, den = 0.f;
+    #pragma unroll
+    for (int k = 0; k < KH; k++)
+        top = fmaxf(top, ml_s[((k * RH + rh) * 16 + lr) * 2]);
+    #pragma unroll
+    for (int k = 0; k < KH; k++) {
+        const float* d = ml_s + ((k * RH + rh) * 16 + lr) * 2;
+        den += d[1] * __expf(d[0] - top);
+    }
+    const float w = den > 0.f ? __expf(m - top) / den : 0.f;
+    #pragma unroll
+    for (int n = 0; n < NT; n++)
+        o_s[(wid * NT + n) * 64 + lane] = acc[n] * w;
+    __syncthreads();
+    if (row >= n_rows) return;
+    const int64_t gr = row0 + row;
+    bf16* dst = split > 1
+        ? o_part + ((int64_t)blockIdx.y * rows_total + gr) * R
+        : out + gr * R;
+    #pragma unroll
+    for (int n = 0; n < NT / KH; n++) {
+        const int t = kh * (NT / KH) + n;
+        f32x4 v = o_s[(rh * NT + t) * 64 + lane];
+        #pragma unroll
+        for (int k = 1; k < KH; k++)
+            v += o_s[((k * RH + rh) * NT + t) * 64 + lane];
+        const int c0 = t * 16 + g * 4;
+        if (c0 < R) {
+            float f4[4] = {v[0], v[1], v[2], v[3]};
+            stv<4>(dst + c0, f4);
+        }
+    }
+    if (split > 1 && kh == 0 && g == 0) {
+        float* d = ml_part + ((int64_t)blockIdx.y * rows_total + gr) * 2;
+        d[0] = top;
+        d[1] = den;
+    }
+}
+
 // merge of the segments' normalised results, weights l e^{m - max}
 template <typename T, int VEC>
 __global__ __launch_bounds__(128) void k_latent_combine(
@@ -430,6 +677,30 @@ extern "C" int latent_attn(
     if (latent_lds(16 * mt, kt, R, esz) > 160 * 1024 || R > 1024)
         return (int)hipErrorInvalidValue;
     int err = (int)hipErrorInvalidValue;
+    if (!f32 && R % 8 == 0 && R <= 512) {
+        auto go = [&](auto* kern, int nt) {
+            const int tile = 2 * 64 * (nt * 16 + 8) * 2;
+            const int merge = 512 + 4 * nt * 1024;
+            const int lds = tile > merge ? tile : merge;
+            (void)hipFuncSetAttribute(
+                (const void*)kern,
+                hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            kern<<<dim3(n_items, split), 256, lds, stream>>>(
+                (bf16*)out, (bf16*)o_part, (float*)ml_part, (const bf16*)q,
+                (const bf16*)pool, (const int*)ptab, (const int*)slot,
+                (const int*)pos, (const int*)items, per_seq, H, R, pshift,
+                maxp, scale, rows_total, split);
+            err = (int)hipGetLastError();
+        };
+        if (R <= 128)
+            mt == 2 ? go(k_latent_mq<8, 2>, 8) : go(k_latent_mq<8, 1>, 8);
+        else if (R <= 256)
+            mt == 2 ? go(k_latent_mq<16, 2>, 16)
+                    : go(k_latent_mq<16, 1>, 16);
+        else
+            mt == 2 ? go(k_latent_mq<32, 2>, 32)
+                    : go(k_latent_mq<32, 1>, 32);
+    } else {
     #define LA(T, M, K, N)                                                 \
         err = latent_go<T, M, K, N>(                                       \
             out, o_part, ml_part, q, pool, ptab, slot, pos, items,         \
@@ -451,6 +722,7 @@ extern "C" int latent_attn(
     #define LA_T(T)                                                        \
         do { if (mt == 2) LA_K(T, 2); else LA_K(T, 1); } while (0)
     if (f32) LA_T(float); else LA_T(bf16);
+    }
     #undef LA_T
     #undef LA_K
     #undef LA_N

@@ -208,9 +208,9 @@ class RinitarLayer:
                 uv=uv.contiguous(), scale=float(s.scale))
         # the input projections are one product; zero rows fill it up to the
         # 32-row tiles of the packed form
-        n = sum(c.shape[0] for c in cols)
-        if n % 32:
-            cols.append(torch.zeros(32 - n % 32, W, dtype=cols[0].dtype,
+        fill = -sum(c.shape[0] for c in cols) % 32
+        if fill:
+            cols.append(torch.zeros(fill, W, dtype=cols[0].dtype,
                                     device=cols[0].device))
         self.w_in = put(torch.cat(cols)).contiguous()
         self.w_o = put(get(mix + "o", (W, v))).contiguous()

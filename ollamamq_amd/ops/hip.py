@@ -758,10 +758,25 @@ def _frag_rows(M, cols, like):
                     M, cols)
 
 
+def _parts_ksplit(N, K):
+    """Split for a product whose consumer folds the partial sums: the one
+    that loads the 256 CUs most evenly, smaller if nearly as good."""
+    tiles, nb = N // 32, K // 64
+    best, best_eff = 1, 0.0
+    for ks in range(1, 9):
+        if nb < ks * 8:
+            break
+        n = tiles * ks
+        eff = n / (256 * -(-n // 256))
+        if eff > best_eff + 0.04:
+            best, best_eff = ks, eff
+    return best
+
+
 def _linear_frag(x, N, packed, parts):
     """Weight-streaming product of an activation in fragment layout."""
     M, K = x.rows, x.cols
-    ks = _wstream_ksplit(N, K)
+    ks = _parts_ksplit(N, K) if parts else _wstream_ksplit(N, K)
     y = part = None
     if ks > 1:
         part = torch.empty((ks, M, N), dtype=torch.float32,
@@ -975,7 +990,8 @@ def _latent_absorbed(o, q, cache, run, slots, pos, H, R, scale, items,
                      n_items, per_seq, row0, rows, max_kv):
     """One launch of the absorbed kernel over rows row0.. of q / o."""
     f32 = _is_f32(q)
-    split = int(max(1, min(512 // n_items, (max_kv + 63) // 64,
+    # one block a CU: more segments would only write more partial results
+    split = int(max(1, min(256 // n_items, (max_kv + 63) // 64,
                            LATENT_SPLIT_MAX)))
     op = ml = None
     total = q.shape[0]
