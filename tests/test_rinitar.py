@@ -114,7 +114,7 @@ def tokens_for(name, n, seed=0):
     return torch.randint(0, MODELS[name]["vocab"], (n,), generator=g).tolist()
 
 
-def run_portions(eng, tokens, portions, before=()):
+def run_portions(eng, tokens, portions):
     """Feed one stream in portions; logits at every place."""
     s = eng.open_stream()
     got, at = [], 0
