@@ -482,6 +482,27 @@ __global__ __launch_bounds__(256) void k_swiglu(
     }
 }
 
+__global__ __launch_bounds__(256) void k_swiglu_f32(
+    float* __restrict__ out, const float* __restrict__ gu, int64_t total,
+    int F)
+{
+    for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
+         i < total; i += (int64_t)gridDim.x * blockDim.x) {
+        const float* g = gu + i / F * 2 * F + i % F;
+        out[i] = g[0] / (1.f + expf(-g[0])) * g[F];
+    }
+}
+
+extern "C" int swiglu_f32(void* out, const void* gu, int T, int F,
+                          hipStream_t stream)
+{
+    const int64_t total = (int64_t)T * F;
+    const int64_t want = (total + 255) / 256;
+    k_swiglu_f32<<<(int)(want < 4096 ? (want > 0 ? want : 1) : 4096), 256, 0,
+                   stream>>>((float*)out, (const float*)gu, total, F);
+    return (int)hipGetLastError();
+}
+
 extern "C" int swiglu_bf16(void* out, const void* gu, int T, int F,
                             hipStream_t stream)
 {

@@ -1,50 +1,66 @@
-// gfx950 latent attention: a paged pool caches one latent row of R values
-// per token, keys and values are linear maps of it (k = W_uk c, v = W_uv c,
-// per head).  Two exact ways to attend, chosen per sequence by the caller:
+// gfx950 latent attention: a paged pool caches one row per token, the latent
+// c of R values and, if heads have a rotated part, the one rotated key part
+// r of Dr values that they share.  Keys and values are linear maps of the
+// latent (k = W_uk c, v = W_uv c, per head), the key followed by r.  Two
+// exact ways to attend, chosen per sequence by the caller:
 //
-// * absorbed (decode, short portions): q' = W_uk^T q makes the score
-//   q' . c, so all heads share the cached row — the pool is read once per
-//   token of context.  k_latent_attn streams the pool with the (token,
-//   head) rows on the matrix cores and returns the weighted latent per row,
-//   which k_head_gemm maps through W_uv.
-// * expanded (long portions): k and v of the whole context are made with
+// * absorbed (decode, short portions): q' = (W_uk^T q, rotated q) makes the
+//   score q' . (c, r), so all heads share the cached row — the pool is read
+//   once per token of context.  k_latent_attn streams the pool with the
+//   (token, head) rows on the matrix cores and returns the weighted latent
+//   per row, which k_head_gemm maps through W_uv.
+// * expanded (long portions): k and v of the visible context are made with
 //   one matrix product each, then k_flash is an ordinary causal flash
 //   attention with free key and value widths.
+//
+// In both a query may see a window of tokens only, itself included, and the
+// result may be gated by the sigmoid of a column of the fused projection.
+// Cached rows are KW wide, R + Dr filled up with zeros.
 #include "tile_mma.h"
 
 #define NEG (-3.0e38f)
 
-template <typename T> DEV float exp_of(float x) {
-    if constexpr (sizeof(T) == 4) return expf(x);
-    else return __expf(x);
-}
-
 // ---------------------------------------------------------------------------
-// out[t][h][n] = sum_k x[t*xs + h*K + k] * w[h][n][k]
+// out[t][h][n] = sum_k x[t*xs + h*hs + k] * w[h][n][k], times the sigmoid of
+// a gate column h*N + n.  Rows of `out` are os wide: what follows the N
+// columns is copied from behind the row's K inputs (`tail` of them), then
+// zeros.
 // Grid (n tiles, t / (16*MT), H); a tile is 16 n x 16*MT tokens.  KS == 1:
 // a block's four waves make four n tiles; KS == 4: they share one and deal
 // its k out (long k, few tiles).  The product is transposed (A = w) so a
 // lane stores four consecutive n.
 // ---------------------------------------------------------------------------
-template <typename T, int MT, int KS>
+template <typename T, typename P, int MT, int KS>
 __global__ __launch_bounds__(256) void k_head_gemm(
     T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ w,
-    int T_rows, int H, int N, int K, int64_t xs, int frag)
+    Rows<P> gate, int og, int T_rows, int H, int N, int K, int64_t xs,
+    int hs, int os, int tail, int frag)
 {
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int lr = lane & 15, g = lane >> 4;
     const int h = blockIdx.z;
     const int n0 = (KS == 1 ? blockIdx.x * 4 + wid : blockIdx.x) * 16;
     const int t0 = blockIdx.y * 16 * MT;
+    if (os > N && blockIdx.x == 0) {
+        const int more = os - N;
+        for (int i = threadIdx.x; i < 16 * MT * more; i += 256) {
+            const int64_t t = t0 + i / more;
+            const int j = i % more;
+            if (t < T_rows)
+                stf(out + (t * H + h) * os + N + j,
+                    j < tail ? ldf(x + t * xs + (int64_t)h * hs + K + j)
+                             : 0.f);
+        }
+    }
     if (n0 >= N) return;                    // KS == 4: the whole block
     const T* wr = w + ((int64_t)h * N + min(n0 + lr, N - 1)) * K;
     const T* xr[MT];
     #pragma unroll
     for (int m = 0; m < MT; m++)
         xr[m] = x + (int64_t)min(t0 + m * 16 + lr, T_rows - 1) * xs
-                + (int64_t)h * K;
+                + (int64_t)h * hs;
     f32x4 acc[MT] = {};
-    const bool vec = K % 8 == 0 && xs % 8 == 0;
+    const bool vec = K % 8 == 0 && xs % 8 == 0 && hs % 8 == 0;
     const int k_lo = (KS == 1 ? 0 : wid * 32) + g * 8;
     if (vec) {
         #pragma unroll 4
@@ -78,8 +94,17 @@ __global__ __launch_bounds__(256) void k_head_gemm(
         const int n = n0 + g * 4;
         if (t >= T_rows || n >= N) continue;
         T* o = out + (frag ? frag_row_off(t, h * N + n, H * N)
-                           : ((int64_t)t * H + h) * N + n);
-        if (N % 4 == 0) {
+                           : ((int64_t)t * H + h) * os + n);
+        if (gate.p) {
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                float z;
+                if (n + i >= N) break;
+                ldrow<1>(gate, t, og + h * N + n + i, &z);
+                acc[m][i] *= sigmoid_of<T>(z);
+            }
+        }
+        if (N % 4 == 0 && os % 4 == 0) {
             float v[4] = {acc[m][0], acc[m][1], acc[m][2], acc[m][3]};
             stv<4>(o, v);
         } else
@@ -88,22 +113,33 @@ __global__ __launch_bounds__(256) void k_head_gemm(
     }
 }
 
-// frag: out in the activation-fragment layout (N % 8 == 0)
+// frag: out in the activation-fragment layout (N % 8 == 0); gate may be null
 extern "C" int head_gemm(int f32, void* out, const void* x, const void* w,
-                         int T_rows, int H, int N, int K, int64_t xs,
-                         int frag, hipStream_t stream)
+                         const void* gate, int g32, int n_part,
+                         int64_t part_stride, int64_t gate_ld, int og,
+                         int T_rows, int H, int N, int K, int64_t xs, int hs,
+                         int os, int tail, int frag, hipStream_t stream)
 {
-    if (frag && N % 8) return (int)hipErrorInvalidValue;
+    if ((frag && (N % 8 || os != N)) || os < N || tail > os - N)
+        return (int)hipErrorInvalidValue;
     const bool wide = T_rows > 16, deal = K >= 256;
     dim3 grid(deal ? (N + 15) / 16 : (N + 63) / 64,
               (T_rows + (wide ? 31 : 15)) / (wide ? 32 : 16), H);
-    #define HG_GO(T, M, S)                                                 \
-        k_head_gemm<T, M, S><<<grid, 256, 0, stream>>>(                    \
-            (T*)out, (const T*)x, (const T*)w, T_rows, H, N, K, xs, frag)
-    #define HG_K(T, M) do { if (deal) HG_GO(T, M, 4); else HG_GO(T, M, 1); } \
-                       while (0)
-    if (f32) { if (wide) HG_K(float, 2); else HG_K(float, 1); }
-    else { if (wide) HG_K(bf16, 2); else HG_K(bf16, 1); }
+    #define HG_GO(T, P, M, S)                                              \
+        k_head_gemm<T, P, M, S><<<grid, 256, 0, stream>>>(                 \
+            (T*)out, (const T*)x, (const T*)w,                             \
+            Rows<P>{(const P*)gate, n_part, part_stride, gate_ld}, og,     \
+            T_rows, H, N, K, xs, hs, os, tail, frag)
+    #define HG_K(T, P, M)                                                  \
+        do {                                                               \
+            if (deal) HG_GO(T, P, M, 4); else HG_GO(T, P, M, 1);           \
+        } while (0)
+    #define HG_M(T, P)                                                     \
+        do { if (wide) HG_K(T, P, 2); else HG_K(T, P, 1); } while (0)
+    if (f32) HG_M(float, float);
+    else if (g32) HG_M(bf16, float);
+    else HG_M(bf16, bf16);
+    #undef HG_M
     #undef HG_K
     #undef HG_GO
     return (int)hipGetLastError();
@@ -126,14 +162,14 @@ __global__ __launch_bounds__(256) void k_latent_attn(
     T* __restrict__ out,               // [rows, R]      (split == 1)
     T* __restrict__ o_part,            // [split, rows, R]
     float* __restrict__ ml_part,       // [split, rows, 2]
-    const T* __restrict__ q,           // [rows, R]
-    const T* __restrict__ pool,        // [pages, psz, R]
+    const T* __restrict__ q,           // [rows, KW]
+    const T* __restrict__ pool,        // [pages, psz, KW]
     const int* __restrict__ ptab, const int* __restrict__ slot,
     const int* __restrict__ pos,
     const int* __restrict__ items,     // [n, 2] first row, rows; null: decode
     int per_seq,                       // decode: items per sequence
-    int H, int R, int pshift, int maxp, float scale, int64_t rows_total,
-    int split)                         // pages of 1 << pshift tokens
+    int H, int R, int KW, int pshift, int maxp, float scale, int window,
+    int64_t rows_total, int split)     // pages of 1 << pshift tokens
 {
     constexpr int M = 16 * MT;
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -150,11 +186,13 @@ __global__ __launch_bounds__(256) void k_latent_attn(
     const int tok0 = row0 / H, tok1 = (row0 + n_rows - 1) / H;
     const int kv_len = pos[tok1] + 1;
     const int* pt = ptab + (int64_t)slot[tok0] * maxp;
-    const int n_chunks = (kv_len + KT - 1) / KT;
-    const int c_lo = (int)((int64_t)blockIdx.y * n_chunks / split);
-    const int c_hi = (int)((int64_t)(blockIdx.y + 1) * n_chunks / split);
+    const int c_first = window > 0 ? max(0, pos[tok0] + 1 - window) / KT : 0;
+    const int n_chunks = (kv_len + KT - 1) / KT - c_first;
+    const int c_lo = c_first + (int)((int64_t)blockIdx.y * n_chunks / split);
+    const int c_hi = c_first
+        + (int)((int64_t)(blockIdx.y + 1) * n_chunks / split);
 
-    const int Rp = (R + 31) & ~31;
+    const int Rp = (KW + 31) & ~31;
     const int cs = Rp + 16 / (int)sizeof(T);      // LDS row strides
     constexpr int SS = KT + 4, PS = KT + 16 / (int)sizeof(T);
     extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -167,21 +205,21 @@ __global__ __launch_bounds__(256) void k_latent_attn(
     float* f_s = l_s + M;                         // [M] this chunk's rescale
     int* lim_s = reinterpret_cast<int*>(f_s + M); // [M] visible keys
 
-    const bool vec = R % 8 == 0;
-    // rows of the chunk or of q, zero beyond R
+    const bool vec = KW % 8 == 0;
+    // rows of the chunk or of q, zero beyond KW
     auto stage = [&](T* dst, const T* src_row, int c8) {
         const int k = c8 * 8;
         Frag<T> v;
         if (src_row == nullptr) v = frag_zero<T>();
-        else if (vec) v = k < R ? frag8(src_row + k) : frag_zero<T>();
-        else v = frag_guard(src_row, k, R);
+        else if (vec) v = k < KW ? frag8(src_row + k) : frag_zero<T>();
+        else v = frag_guard(src_row, k, KW);
         *reinterpret_cast<Frag<T>*>(dst + k) = v;
     };
     const int n8 = Rp / 8;
     for (int u = tid; u < M * n8; u += 256) {
         const int r = u / n8;
         stage(q_s + r * cs,
-              r < n_rows ? q + (int64_t)(row0 + r) * R : nullptr, u % n8);
+              r < n_rows ? q + (int64_t)(row0 + r) * KW : nullptr, u % n8);
     }
     if (tid < M) {
         m_s[tid] = NEG;
@@ -198,7 +236,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(
         where[j] = u < KT * n8 ? (u / n8) << 16 | (u % n8) * 8 : -1;
     }
     // Loads are unconditional, with keys and columns clamped to valid ones:
-    // a key past the end has weight zero, a column past R meets zeros of q'
+    // a key past the end has weight zero, a column past KW meets zeros of q'
     // or is not stored.  Page numbers are fetched a chunk ahead.
     const int pmask = (1 << pshift) - 1;
     int page[NP];
@@ -214,9 +252,9 @@ __global__ __launch_bounds__(256) void k_latent_attn(
         for (int j = 0; j < NP; j++) {
             const int c = max(where[j], 0) & 0xffff;
             const T* src = pool + (((int64_t)page[j] << pshift)
-                                   + (key_of(j, base) & pmask)) * R;
-            if (vec) piece[j] = frag8(src + min(c, R - 8));
-            else piece[j] = frag_guard(src, c, R);
+                                   + (key_of(j, base) & pmask)) * KW;
+            if (vec) piece[j] = frag8(src + min(c, KW - 8));
+            else piece[j] = frag_guard(src, c, KW);
         }
     };
     f32x4 acc[MT][NT] = {};
@@ -252,8 +290,11 @@ __global__ __launch_bounds__(256) void k_latent_attn(
                     s = mma(frag8(ar + k), frag8(br + k), s);
                 const int row = mt * 16 + lr, k0 = kt * 16 + g * 4;
                 #pragma unroll
-                for (int e = 0; e < 4; e++)
-                    s[e] = base + k0 + e < lim_s[row] ? s[e] * scale : NEG;
+                for (int e = 0; e < 4; e++) {
+                    const int d = lim_s[row] - (base + k0 + e);
+                    s[e] = d > 0 && (window <= 0 || d <= window)
+                               ? s[e] * scale : NEG;
+                }
                 *reinterpret_cast<f32x4*>(s_s + row * SS + k0) = s;
             }
         }
@@ -295,7 +336,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(
         #pragma unroll
         for (int n = 0; n < NT; n++) {
             const int col = (n * 4 + wid) * 16 + lr;
-            if ((n * 4 + wid) * 16 < Rp) {
+            if ((n * 4 + wid) * 16 < R) {
                 #pragma unroll
                 for (int mt = 0; mt < MT; mt++) acc[mt][n] *= f[mt];
                 #pragma unroll
@@ -357,8 +398,8 @@ __global__ __launch_bounds__(256) void k_latent_attn(
 }
 
 // ---------------------------------------------------------------------------
-// The same for bf16 with R <= 16 * NT, R % 8 == 0: every wave is a whole
-// attention of its own.  Wave (row tile rh, key group kh) holds its q' rows
+// The same for bf16 with KW <= 16 * NT, R <= 16 * NV, KW % 8 == 0 and
+// R % 4 == 0: every wave is a whole attention of its own.  Wave (row tile rh, key group kh) holds its q' rows
 // as matrix operands and its [R, 16] result in registers and takes its own
 // keys of each 64-key chunk:
 //   S^T = C q'^T, so a lane holds one row's scores for keys 4g + i, which is
@@ -366,14 +407,15 @@ __global__ __launch_bounds__(256) void k_latent_attn(
 //   O^T += C^T P^T with C^T read through the LDS transpose load.
 // The waves meet only at the double-buffered chunk and in the last merge.
 // ---------------------------------------------------------------------------
-template <int NT, int RH>
+template <int NT, int NV, int RH>
 __global__ __launch_bounds__(256, 1) void k_latent_mq(
     bf16* __restrict__ out, bf16* __restrict__ o_part,
     float* __restrict__ ml_part, const bf16* __restrict__ q,
     const bf16* __restrict__ pool, const int* __restrict__ ptab,
     const int* __restrict__ slot, const int* __restrict__ pos,
-    const int* __restrict__ items, int per_seq, int H, int R, int pshift,
-    int maxp, float scale, int64_t rows_total, int split)
+    const int* __restrict__ items, int per_seq, int H, int R, int KW,
+    int pshift, int maxp, float scale, int window, int64_t rows_total,
+    int split)
 {
     constexpr int M = 16 * RH, KH = 4 / RH, NK = 4 / KH, KT = 64;
     constexpr int Rp = NT * 16, CS = Rp + 8;
@@ -392,9 +434,11 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
     const int tok0 = row0 / H, tok1 = (row0 + n_rows - 1) / H;
     const int kv_len = pos[tok1] + 1;
     const int* pt = ptab + (int64_t)slot[tok0] * maxp;
-    const int n_chunks = (kv_len + KT - 1) / KT;
-    const int c_lo = (int)((int64_t)blockIdx.y * n_chunks / split);
-    const int c_hi = (int)((int64_t)(blockIdx.y + 1) * n_chunks / split);
+    const int c_first = window > 0 ? max(0, pos[tok0] + 1 - window) / KT : 0;
+    const int n_chunks = (kv_len + KT - 1) / KT - c_first;
+    const int c_lo = c_first + (int)((int64_t)blockIdx.y * n_chunks / split);
+    const int c_hi = c_first
+        + (int)((int64_t)(blockIdx.y + 1) * n_chunks / split);
     extern __shared__ __attribute__((aligned(16))) char smem[];
     bf16* c_s = reinterpret_cast<bf16*>(smem);    // [2][KT][CS]
 
@@ -402,11 +446,11 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
     const int my_lim = row < n_rows ? pos[(row0 + row) / H] + 1 : 0;
     bf16x8 qf[NT / 2];
     {
-        const bf16* qr = q + (int64_t)(row0 + min(row, n_rows - 1)) * R;
+        const bf16* qr = q + (int64_t)(row0 + min(row, n_rows - 1)) * KW;
         #pragma unroll
         for (int k = 0; k < NT / 2; k++) {
             const int c = k * 32 + g * 8;
-            qf[k] = c < R ? frag8(qr + c) : frag_zero<bf16>();
+            qf[k] = c < KW ? frag8(qr + c) : frag_zero<bf16>();
         }
     }
     // pieces of a chunk: a row is NT*2 of them, so a wave reads whole rows
@@ -424,9 +468,9 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
     auto fetch = [&](int base) {
         #pragma unroll
         for (int j = 0; j < NP; j++) {
-            const int c = min((tid + j * 256) % (NT * 2) * 8, R - 8);
+            const int c = min((tid + j * 256) % (NT * 2) * 8, KW - 8);
             piece[j] = frag8(pool + (((int64_t)page[j] << pshift)
-                                     + (key_of(j, base) & pmask)) * R + c);
+                                     + (key_of(j, base) & pmask)) * KW + c);
         }
     };
     auto put = [&](int buf) {
@@ -438,7 +482,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
                 = piece[j];
         }
     };
-    f32x4 acc[NT] = {};
+    f32x4 acc[NV] = {};
     float m = NEG, l = 0.f;
     if (c_lo < c_hi) {
         pages(c_lo * KT);
@@ -474,7 +518,8 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
         for (int j = 0; j < NK; j++)
             #pragma unroll
             for (int i = 0; i < 4; i++) {
-                const float v = base + j * 16 + g * 4 + i < my_lim
+                const int d = my_lim - (base + j * 16 + g * 4 + i);
+                const float v = d > 0 && (window <= 0 || d <= window)
                                     ? s[j][i] * scale : NEG;
                 s[j][i] = v;
                 mx = fmaxf(mx, v);
@@ -498,7 +543,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
         m = mn;
         if (!__all(f == 1.f)) {
             #pragma unroll
-            for (int n = 0; n < NT; n++) acc[n] *= f;
+            for (int n = 0; n < NV; n++) acc[n] *= f;
         }
         if constexpr (NK == 2) {
             bf16x8 b;
@@ -508,7 +553,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
                 b[i + 4] = (__bf16)s[1][i];
             }
             #pragma unroll
-            for (int n = 0; n < NT; n++) {
+            for (int n = 0; n < NV; n++) {
                 const s16x4 a0 = tr_read(ct + n * 16, CS, lane);
                 const s16x4 a1 = tr_read(ct + 16 * CS + n * 16, CS, lane);
                 const s16x8 a = __builtin_shufflevector(a0, a1, 0, 1, 2, 3,
@@ -521,7 +566,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
             for (int i = 0; i < 4; i++) b4[i] = (__bf16)s[0][i];
             const s16x4 b = __builtin_bit_cast(s16x4, b4);
             #pragma unroll
-            for (int n = 0; n < NT; n++)
+            for (int n = 0; n < NV; n++)
                 acc[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(
                     tr_read(ct + n * 16, CS, lane), b, acc[n], 0, 0, 0);
         }
@@ -531,7 +576,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
     // merge the key groups: each wave's scaled result, then a share of the
     // column tiles per wave
     float* ml_s = reinterpret_cast<float*>(smem);           // [4][16][2]
-    f32x4* o_s = reinterpret_cast<f32x4*>(smem + 512);      // [4][NT][64]
+    f32x4* o_s = reinterpret_cast<f32x4*>(smem + 512);      // [4][NV][64]
     if (g == 0) {
         ml_s[(wid * 16 + lr) * 2] = m;
         ml_s[(wid * 16 + lr) * 2 + 1] = l;
@@ -548,8 +593,8 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
     }
     const float w = den > 0.f ? __expf(m - top) / den : 0.f;
     #pragma unroll
-    for (int n = 0; n < NT; n++)
-        o_s[(wid * NT + n) * 64 + lane] = acc[n] * w;
+    for (int n = 0; n < NV; n++)
+        o_s[(wid * NV + n) * 64 + lane] = acc[n] * w;
     __syncthreads();
     if (row >= n_rows) return;
     const int64_t gr = row0 + row;
@@ -557,12 +602,12 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
         ? o_part + ((int64_t)blockIdx.y * rows_total + gr) * R
         : out + gr * R;
     #pragma unroll
-    for (int n = 0; n < NT / KH; n++) {
-        const int t = kh * (NT / KH) + n;
-        f32x4 v = o_s[(rh * NT + t) * 64 + lane];
+    for (int n = 0; n < NV / KH; n++) {
+        const int t = kh * (NV / KH) + n;
+        f32x4 v = o_s[(rh * NV + t) * 64 + lane];
         #pragma unroll
         for (int k = 1; k < KH; k++)
-            v += o_s[((k * RH + rh) * NT + t) * 64 + lane];
+            v += o_s[((k * RH + rh) * NV + t) * 64 + lane];
         const int c0 = t * 16 + g * 4;
         if (c0 < R) {
             float f4[4] = {v[0], v[1], v[2], v[3]};
@@ -606,9 +651,9 @@ __global__ __launch_bounds__(128) void k_latent_combine(
     }
 }
 
-static int latent_lds(int M, int KT, int R, int esz)
+static int latent_lds(int M, int KT, int KW, int esz)
 {
-    const int cs = ((R + 31) & ~31) + 16 / esz;
+    const int cs = ((KW + 31) & ~31) + 16 / esz;
     return (M + KT) * cs * esz + M * (KT + 16 / esz) * esz
            + M * (KT + 4) * 4 + 4 * M * 4;
 }
@@ -617,10 +662,11 @@ template <typename T, int MT, int KT, int NT>
 static int latent_go(
     void* out, void* op, void* mp, const void* q, const void* pool,
     const void* ptab, const void* slot, const void* pos, const void* items,
-    int n_items, int per_seq, int H, int R, int pshift, int maxp,
-    float scale, int64_t rows_total, int split, hipStream_t stream)
+    int n_items, int per_seq, int H, int R, int KW, int pshift, int maxp,
+    float scale, int window, int64_t rows_total, int split,
+    hipStream_t stream)
 {
-    const int lds = latent_lds(16 * MT, KT, R, sizeof(T));
+    const int lds = latent_lds(16 * MT, KT, KW, sizeof(T));
     static bool once = false;
     if (!once) {
         (void)hipFuncSetAttribute(
@@ -631,44 +677,58 @@ static int latent_go(
     k_latent_attn<T, MT, KT, NT><<<dim3(n_items, split), 256, lds, stream>>>(
         (T*)out, (T*)op, (float*)mp, (const T*)q, (const T*)pool,
         (const int*)ptab, (const int*)slot, (const int*)pos,
-        (const int*)items, per_seq, H, R, pshift, maxp, scale, rows_total,
-        split);
+        (const int*)items, per_seq, H, R, KW, pshift, maxp, scale, window,
+        rows_total, split);
     return (int)hipGetLastError();
 }
 
-// rows of an item: 16 * latent_mt(f32, H, R)
-extern "C" int latent_mt(int f32, int H, int R)
+// key tiles of k_latent_mq, 0 where it does not apply
+static int latent_mq_tiles(int f32, int R, int KW)
 {
-    const int esz = f32 ? 4 : 2;
-    if (H > 16 && latent_lds(32, 32, R, esz) <= 160 * 1024 && R <= 512)
-        return 2;
-    return 1;
+    if (f32 || KW % 8 || R % 4) return 0;
+    if (KW <= 128) return 8;
+    if (KW <= 256) return 16;
+    if (KW <= 288 && R <= 256) return 18;
+    if (KW <= 512) return 32;
+    return KW <= 576 && R <= 512 ? 36 : 0;
+}
+
+// rows of an item: 16 * latent_mt(f32, H, R, KW)
+extern "C" int latent_mt(int f32, int H, int R, int KW)
+{
+    if (H <= 16) return 1;
+    if (latent_mq_tiles(f32, R, KW)) return 2;
+    return KW <= 512 && latent_lds(32, 32, KW, f32 ? 4 : 2) <= 160 * 1024
+               ? 2 : 1;
 }
 
 // items: int32 [n_items, 2] (first row, rows <= 16 * latent_mt), each within
 // one sequence; null with per_seq = ceil(H / rows) for a decode batch.
+// window 0: all earlier keys.
 extern "C" int latent_attn(
     int f32, void* out, void* o_part, void* ml_part, const void* q,
     const void* pool, const void* ptab, const void* slot, const void* pos,
-    const void* items, int n_items, int per_seq, int H, int R, int psz,
-    int maxp, float scale, int64_t rows_total, int64_t row_base,
-    int64_t rows_here, int split, hipStream_t stream)
+    const void* items, int n_items, int per_seq, int H, int R, int KW,
+    int psz, int maxp, float scale, int window, int64_t rows_total,
+    int64_t row_base, int64_t rows_here, int split, hipStream_t stream)
 {
-    if (psz & (psz - 1) || split > 64) return (int)hipErrorInvalidValue;
+    if (psz & (psz - 1) || split > 64 || R > KW || KW > 1024)
+        return (int)hipErrorInvalidValue;
     const int pshift = __builtin_ctz(psz);
     const int esz = f32 ? 4 : 2;
-    const int mt = latent_mt(f32, H, R);
+    const int mt = latent_mt(f32, H, R, KW);
     const int budget = 80 * 1024;            // two blocks a CU if possible
     int kt = 64;
-    if (latent_lds(16 * mt, 64, R, esz) > budget) kt = 32;
-    if (latent_lds(16 * mt, kt, R, esz) > 160 * 1024) kt = 16;
-    if (latent_lds(16 * mt, kt, R, esz) > 160 * 1024 || R > 1024)
+    if (latent_lds(16 * mt, 64, KW, esz) > budget) kt = 32;
+    if (latent_lds(16 * mt, kt, KW, esz) > 160 * 1024) kt = 16;
+    const int nt = latent_mq_tiles(f32, R, KW);
+    if (!nt && latent_lds(16 * mt, kt, KW, esz) > 160 * 1024)
         return (int)hipErrorInvalidValue;
     int err = (int)hipErrorInvalidValue;
-    if (!f32 && R % 8 == 0 && R <= 512) {
-        auto go = [&](auto* kern, int nt) {
+    if (nt) {
+        auto go = [&](auto* kern, int nv) {
             const int tile = 2 * 64 * (nt * 16 + 8) * 2;
-            const int merge = 512 + 4 * nt * 1024;
+            const int merge = 512 + 4 * nv * 1024;
             const int lds = tile > merge ? tile : merge;
             (void)hipFuncSetAttribute(
                 (const void*)kern,
@@ -676,29 +736,29 @@ extern "C" int latent_attn(
             kern<<<dim3(n_items, split), 256, lds, stream>>>(
                 (bf16*)out, (bf16*)o_part, (float*)ml_part, (const bf16*)q,
                 (const bf16*)pool, (const int*)ptab, (const int*)slot,
-                (const int*)pos, (const int*)items, per_seq, H, R, pshift,
-                maxp, scale, rows_total, split);
+                (const int*)pos, (const int*)items, per_seq, H, R, KW,
+                pshift, maxp, scale, window, rows_total, split);
             err = (int)hipGetLastError();
         };
-        if (R <= 128)
-            mt == 2 ? go(k_latent_mq<8, 2>, 8) : go(k_latent_mq<8, 1>, 8);
-        else if (R <= 256)
-            mt == 2 ? go(k_latent_mq<16, 2>, 16)
-                    : go(k_latent_mq<16, 1>, 16);
-        else
-            mt == 2 ? go(k_latent_mq<32, 2>, 32)
-                    : go(k_latent_mq<32, 1>, 32);
+        #define MQ(N, V)                                                   \
+            (mt == 2 ? go(k_latent_mq<N, V, 2>, V)                         \
+                     : go(k_latent_mq<N, V, 1>, V))
+        if (nt == 8) MQ(8, 8);
+        else if (nt == 16) MQ(16, 16);
+        else if (nt == 18) MQ(18, 16);
+        else if (nt == 32) MQ(32, 32);
+        else MQ(36, 32);
+        #undef MQ
     } else {
     #define LA(T, M, K, N)                                                 \
         err = latent_go<T, M, K, N>(                                       \
             out, o_part, ml_part, q, pool, ptab, slot, pos, items,         \
-            n_items, per_seq, H, R, pshift, maxp, scale, rows_total,       \
-            split,                                                         \
-            stream)
+            n_items, per_seq, H, R, KW, pshift, maxp, scale, window,       \
+            rows_total, split, stream)
     #define LA_N(T, M, K)                                                  \
         do {                                                               \
-            if (R <= 128) LA(T, M, K, 2);                                  \
-            else if (R <= 512) LA(T, M, K, 8);                             \
+            if (KW <= 128) LA(T, M, K, 2);                                 \
+            else if (KW <= 512) LA(T, M, K, 8);                            \
             else LA(T, 1, K, 16);                                          \
         } while (0)
     #define LA_K(T, M)                                                     \
@@ -727,9 +787,10 @@ extern "C" int latent_attn(
 }
 
 // ---------------------------------------------------------------------------
-// Causal flash attention with free key width (<= 32*DT) and value width
-// (<= 16*VT), contiguous keys [kv, H, D] and TRANSPOSED values [H, V, kv]
-// (the caller's matrix product writes them that way).
+// Causal flash attention with free key width (D + Dr <= 32*DT) and value
+// width (<= 16*VT), contiguous keys [kv, H, D], a key part [kv, Dr] that all
+// heads share, and TRANSPOSED values [H, V, kv] (the caller's matrix product
+// writes them that way).
 //
 // Block: four waves of NQ 16-query tiles.  S^T = K Q^T puts a query on a
 // lane, so its softmax state is two scalars after two cross-lane steps; P
@@ -740,12 +801,18 @@ extern "C" int latent_attn(
 template <typename T, int DT, int VT, int NQ>
 __global__ __launch_bounds__(256) void k_flash(
     T* __restrict__ out,               // [T, H, V]
-    const T* __restrict__ q,           // [T, ..] row stride qs, head h at h*D
+    const T* __restrict__ q,           // [T, ..] row stride qs, head h at
+                                       // h * (D + Dr)
     const T* __restrict__ k,           // [kv, H*D]
+    const T* __restrict__ kr,          // [kv, ..] row stride krs
     const T* __restrict__ vt,          // [H*V, kv_ld]
-    const int* __restrict__ tiles,     // [n, 4] q row, pos, rows, kv offset
-    int H, int D, int V, int64_t qs, int64_t kv_ld, float scale)
+    Rows<T> gate, int og,              // gate columns og + h*V, or null
+    const int* __restrict__ tiles,     // [n, 4] q row, pos, rows, row of
+                                       // position 0 in k, kr and vt
+    int H, int D, int Dr, int V, int64_t qs, int64_t krs, int64_t kv_ld,
+    float scale, int window)
 {
+    const int DD = D + Dr;
     constexpr int KT = 64;
     constexpr int PAD = 16 / sizeof(T);
     constexpr int KS = DT * 32 + PAD, VS = KT + PAD;
@@ -759,7 +826,8 @@ __global__ __launch_bounds__(256) void k_flash(
     T* k_s = reinterpret_cast<T*>(smem);          // [KT][KS]
     T* v_s = k_s + KT * KS;                       // [VT*16][VS]
 
-    const bool vec = D % 8 == 0 && qs % 8 == 0;
+    const bool vec = D % 8 == 0 && Dr % 8 == 0 && qs % 8 == 0
+                     && (!Dr || (krs % 8 == 0 && (uintptr_t)kr % 16 == 0));
     Frag<T> qf[NQ][DT];
     int qpos[NQ];
     #pragma unroll
@@ -767,18 +835,20 @@ __global__ __launch_bounds__(256) void k_flash(
         const int r = (wid * NQ + n) * 16 + lr;
         qpos[n] = pos0 + r;
         const T* qr = q + (int64_t)(q0 + min(r, rows - 1)) * qs
-                      + (int64_t)h * D;
+                      + (int64_t)h * DD;
         #pragma unroll
         for (int d = 0; d < DT; d++) {
             const int c = d * 32 + g * 8;
-            if (vec) qf[n][d] = c < D ? frag8(qr + c) : frag_zero<T>();
-            else qf[n][d] = frag_guard(qr, c, D);
+            if (vec) qf[n][d] = c < DD ? frag8(qr + c) : frag_zero<T>();
+            else qf[n][d] = frag_guard(qr, c, DD);
         }
     }
     const T* kh = k + kv0 * H * D + (int64_t)h * D;
+    const T* krh = kr + kv0 * krs - D;
     const T* vh = vt + (int64_t)h * V * kv_ld + kv0;
     const int kv_len = pos0 + rows;
     const int n_chunks = (kv_len + KT - 1) / KT;
+    const int c_first = window > 0 ? max(0, pos0 + 1 - window) / KT : 0;
 
     constexpr int NK = DT;                        // 8-element pieces a thread
     constexpr int NV = VT / 2;
@@ -789,8 +859,15 @@ __global__ __launch_bounds__(256) void k_flash(
             const int u = tid + j * 256;
             const int key = u / (DT * 4), c = (u % (DT * 4)) * 8;
             const T* src = kh + (int64_t)(base + key) * H * D;
-            if (vec) kp[j] = c < D ? frag8(src + c) : frag_zero<T>();
-            else kp[j] = frag_guard(src, c, D);
+            const T* shared = krh + (base + key) * krs;
+            if (vec)
+                kp[j] = c < D ? frag8(src + c)
+                        : c < DD ? frag8(shared + c) : frag_zero<T>();
+            else
+                #pragma unroll
+                for (int e = 0; e < 8; e++)
+                    frag_set(kp[j], e, c + e < D ? ldf(src + c + e)
+                             : c + e < DD ? ldf(shared + c + e) : 0.f);
         }
         #pragma unroll
         for (int j = 0; j < NV; j++) {
@@ -820,8 +897,8 @@ __global__ __launch_bounds__(256) void k_flash(
     #pragma unroll
     for (int n = 0; n < NQ; n++) { m[n] = NEG; l[n] = 0.f; }
 
-    load(0);
-    for (int ch = 0; ch < n_chunks; ++ch) {
+    load(c_first * KT);
+    for (int ch = c_first; ch < n_chunks; ++ch) {
         const int base = ch * KT;
         store();
         __syncthreads();
@@ -838,7 +915,8 @@ __global__ __launch_bounds__(256) void k_flash(
                     s[n][kt] = mma(a, qf[n][d], s[n][kt]);
             }
         }
-        const bool edge = base + KT > pos0 + 1;   // some query sees less
+        const bool edge = base + KT > pos0 + 1    // some query sees less
+            || (window > 0 && base <= kv_len - 1 - window);
         #pragma unroll
         for (int n = 0; n < NQ; n++) {
             float mx = NEG;
@@ -847,23 +925,25 @@ __global__ __launch_bounds__(256) void k_flash(
                 #pragma unroll
                 for (int i = 0; i < 4; i++) {
                     float v = s[n][kt][i] * scale;
-                    if (edge && base + kt * 16 + g * 4 + i > qpos[n])
-                        v = NEG;
+                    if (edge) {
+                        const int d = qpos[n] - (base + kt * 16 + g * 4 + i);
+                        if (d < 0 || (window > 0 && d >= window)) v = NEG;
+                    }
                     s[n][kt][i] = v;
                     mx = fmaxf(mx, v);
                 }
             mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-            // key 0 is visible to every query, so the maximum is finite
-            // from the first chunk on and masked scores give exp() == 0
+            // a query that has seen no key yet: all its weights are zero
             const float mn = fmaxf(m[n], mx);
-            const float f = exp_of<T>(m[n] - mn);
+            const float ref = mn > NEG ? mn : 0.f;
+            const float f = exp_of<T>(m[n] - ref);
             float sum = 0.f;
             #pragma unroll
             for (int kt = 0; kt < 4; kt++)
                 #pragma unroll
                 for (int i = 0; i < 4; i++) {
-                    const float p = exp_of<T>(s[n][kt][i] - mn);
+                    const float p = exp_of<T>(s[n][kt][i] - ref);
                     s[n][kt][i] = p;
                     sum += p;
                 }
@@ -903,6 +983,15 @@ __global__ __launch_bounds__(256) void k_flash(
         #pragma unroll
         for (int v = 0; v < VT; v++) {
             const int c = v * 16 + g * 4;
+            if (gate.p) {
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    float z;
+                    if (c + i >= V) break;
+                    ldrow<1>(gate, q0 + r, og + h * V + c + i, &z);
+                    o[n][v][i] *= sigmoid_of<T>(z);
+                }
+            }
             if (V % 4 == 0) {
                 if (c < V) {
                     float w[4];
@@ -919,10 +1008,11 @@ __global__ __launch_bounds__(256) void k_flash(
 }
 
 template <typename T, int DT, int VT, int NQ>
-static int flash_go(void* out, const void* q, const void* k, const void* vt,
-                    const void* tiles, int n_tiles, int H, int D, int V,
-                    int64_t qs, int64_t kv_ld, float scale,
-                    hipStream_t stream)
+static int flash_go(void* out, const void* q, const void* k, const void* kr,
+                    const void* vt, const void* gate, int64_t gate_ld,
+                    int og, const void* tiles, int n_tiles, int H, int D,
+                    int Dr, int V, int64_t qs, int64_t krs, int64_t kv_ld,
+                    float scale, int window, hipStream_t stream)
 {
     const int pad = 16 / sizeof(T);
     const int lds = (64 * (DT * 32 + pad) + VT * 16 * (64 + pad))
@@ -935,26 +1025,30 @@ static int flash_go(void* out, const void* q, const void* k, const void* vt,
         once = true;
     }
     k_flash<T, DT, VT, NQ><<<dim3(H, n_tiles), 256, lds, stream>>>(
-        (T*)out, (const T*)q, (const T*)k, (const T*)vt, (const int*)tiles,
-        H, D, V, qs, kv_ld, scale);
+        (T*)out, (const T*)q, (const T*)k, (const T*)kr, (const T*)vt,
+        Rows<T>{(const T*)gate, 1, 0, gate_ld}, og, (const int*)tiles, H, D,
+        Dr, V, qs, krs, kv_ld, scale, window);
     return (int)hipGetLastError();
 }
 
-// queries per tile; tiles: int32 [n, 4] (first q row, its position, rows,
-// first row of the sequence in k / vt); k and vt hold every sequence padded
-// to a multiple of 64 positions; D, V <= 256
+// queries per tile; tiles: int32 [n, 4] (first q row, its position, rows, row
+// of position 0 in k / kr / vt); these hold every sequence from a multiple of
+// 64 positions on, no later than the first key any query sees, padded to
+// another; D + Dr, V <= 256; gate may be null
 extern "C" int flash_rows(int f32) { return f32 ? 64 : 128; }
 
 extern "C" int flash_attn(
-    int f32, void* out, const void* q, const void* k, const void* vt,
-    const void* tiles, int n_tiles, int H, int D, int V, int64_t qs,
-    int64_t kv_ld, float scale, hipStream_t stream)
+    int f32, void* out, const void* q, const void* k, const void* kr,
+    const void* vt, const void* gate, int64_t gate_ld, int og,
+    const void* tiles, int n_tiles, int H, int D, int Dr, int V, int64_t qs,
+    int64_t krs, int64_t kv_ld, float scale, int window, hipStream_t stream)
 {
-    if (D > 256 || V > 256) return (int)hipErrorInvalidValue;
+    if (D + Dr > 256 || V > 256) return (int)hipErrorInvalidValue;
     int err;
     #define FA(T, D_, V_, Q)                                               \
-        err = flash_go<T, D_, V_, Q>(out, q, k, vt, tiles, n_tiles, H, D,  \
-                                     V, qs, kv_ld, scale, stream)
+        err = flash_go<T, D_, V_, Q>(                                      \
+            out, q, k, kr, vt, gate, gate_ld, og, tiles, n_tiles, H, D,    \
+            Dr, V, qs, krs, kv_ld, scale, window, stream)
     #define FA_V(T, D_, Q)                                                 \
         do {                                                               \
             if (V <= 64) FA(T, D_, 4, Q);                                  \
@@ -963,8 +1057,9 @@ extern "C" int flash_attn(
         } while (0)
     #define FA_D(T, Q)                                                     \
         do {                                                               \
-            if (D <= 64) FA_V(T, 2, Q);                                    \
-            else if (D <= 128) FA_V(T, 4, Q);                              \
+            if (D + Dr <= 64) FA_V(T, 2, Q);                               \
+            else if (D + Dr <= 128) FA_V(T, 4, Q);                         \
+            else if (D + Dr <= 192) FA_V(T, 6, Q);                         \
             else FA_V(T, 8, Q);                                            \
         } while (0)
     if (f32) FA_D(float, 1); else FA_D(bf16, 2);

@@ -1,30 +1,22 @@
-// gfx950 row steps of blocks that norm what their sublayers return:
+// gfx950 row steps between the products of RMS-normed blocks:
 //
-//   x' = x + mult * N(y) * post      residual sum, fp32
-//   h  = N(x') * pre, or x' itself   next operand
+//   x' = x + mult * N(y) * post + shift   residual sum, fp32; without post
+//                                         mult * y itself is added
+//   h  = N(x') * pre, or x' itself        next operand
 //
-// N divides a row by its root mean square.  y may still be split: partial
-// sums of a split-K product, or a token's expert outputs with their shares,
-// are added up on the way in.  One block per row, the row in registers.  In
-// decode the row kernel can also route: with the new row at hand it takes the
-// few experts' logits and chooses.
+// N divides a row by its root mean square.  x may be the residual stream, the
+// scaled embedding rows or nothing.  y may still be split: partial sums of a
+// split-K product, or a token's expert outputs with their shares, are added
+// up on the way in.  h may be followed by the token's embedding row, as the
+// operand of a product over both.  One block per row, the row in registers.
+// In decode the row kernel can also route: with the new row at hand it takes
+// the few experts' logits and chooses.
 //
 // Also here: the split of a fused query/key/value projection with an RMS
 // norm over all queries and over all keys of a token, and the append of keys
-// and values to the paged pools.
+// and values to the paged pools; and the norm over all heads of a token with
+// a sigmoid gate.
 #include "route.h"
-
-// sum over the block; every thread gets it.  s: one float per wave
-template <int BS> DEV float block_sum(float v, float* s) {
-    v = wave_sum(v);
-    const int wid = threadIdx.x >> 6;
-    if ((threadIdx.x & 63) == 0) s[wid] = v;
-    __syncthreads();
-    float t = 0.f;
-    #pragma unroll
-    for (int i = 0; i < BS / 64; i++) t += s[i];
-    return t;
-}
 
 // sum_s share[s] * y[s * stride] (share null: all ones)
 template <int VEC, typename P>
@@ -64,7 +56,10 @@ __global__ __launch_bounds__(BS) void k_rms_residual(
     int n_part, int64_t part_stride, int64_t row_stride,
     const float* __restrict__ share,    // [T, n_part] or null
     const float* __restrict__ post, const float* __restrict__ pre,
+    const float* __restrict__ shift, // [W] or null
     float mult, float eps, const int64_t* __restrict__ rows, int W,
+    int tail,                           // h rows: [h, embedding row]
+    int bare,                           // no x at all
     Route rt)
 {
     const int o = blockIdx.x, tid = threadIdx.x;
@@ -77,6 +72,9 @@ __global__ __launch_bounds__(BS) void k_rms_residual(
         const int c = col(j);
         if (c >= W) break;
         if (x_in) ldv<VEC>(x_in + r * W + c, x[j]);
+        else if (bare)
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) x[j][i] = 0.f;
         else {
             ldv<VEC>(embed + (int64_t)tokens[r] * W + c, x[j]);
             #pragma unroll
@@ -94,17 +92,37 @@ __global__ __launch_bounds__(BS) void k_rms_residual(
             #pragma unroll
             for (int i = 0; i < VEC; i++) s += v[j][i] * v[j][i];
         }
-        const float f = mult / sqrtf(block_sum<BS>(s, red[0]) / W + eps);
+        const float f = post
+            ? mult / sqrtf(block_sum<BS>(s, red[0]) / W + eps) : mult;
         #pragma unroll
         for (int j = 0; j < NV; j++) {
             const int c = col(j);
             if (c >= W) break;
             float w[VEC];
-            ldv<VEC>(post + c, w);
+            if (post) ldv<VEC>(post + c, w);
+            else
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) w[i] = 1.f;
             #pragma unroll
             for (int i = 0; i < VEC; i++) x[j][i] += f * v[j][i] * w[i];
         }
     }
+    if (shift) {
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int c = col(j);
+            if (c >= W) break;
+            float w[VEC];
+            ldv<VEC>(shift + c, w);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) x[j][i] += w[i];
+        }
+    }
+    const int HW = tail ? 2 * W : W;
+    auto put = [&](int c, const float* v) {
+        stv<VEC>(h_out + (FR ? frag_row_off(o, c, HW) : (int64_t)o * HW + c),
+                 v);
+    };
     float f = 1.f;
     if (pre) {
         float s = 0.f;
@@ -127,8 +145,14 @@ __global__ __launch_bounds__(BS) void k_rms_residual(
             #pragma unroll
             for (int i = 0; i < VEC; i++) x[j][i] *= f * w[i];
         }
-        stv<VEC>(h_out + (FR ? frag_row_off(o, c, W) : (int64_t)o * W + c),
-                 x[j]);
+        put(c, x[j]);
+        if (tail) {
+            float e[VEC];
+            ldv<VEC>(embed + (int64_t)tokens[r] * W + c, e);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) e[i] *= embed_scale;
+            put(W + c, e);
+        }
     }
     if constexpr (RT) {
         __shared__ float part[BS / 64][8], z[ROUTE_MAX];
@@ -178,11 +202,14 @@ extern "C" int rms_residual(
     int f32, void* x_out, void* h_out, const void* x_in, const void* embed,
     const void* tokens, float embed_scale, const void* y, int y32,
     int n_part, int64_t part_stride, int64_t row_stride, const void* share,
-    const void* post, const void* pre, float mult, float eps,
-    const void* rows, int n, int W, int frag, const void* router,
+    const void* post, const void* pre, const void* shift, float mult,
+    float eps, const void* rows, int n, int W, int tail, int bare, int frag,
+    const void* router,
     void* chosen, void* route_share, int E, int top, hipStream_t stream)
 {
     const bool v4 = W % 4 == 0;
+    if ((bare && (x_in || !y)) || (tail && (!tokens || router)))
+        return (int)hipErrorInvalidValue;
     if (frag && (!v4 || f32)) return (int)hipErrorInvalidValue;
     if (router && (!frag || pre || E > ROUTE_MAX || top > E))
         return (int)hipErrorInvalidValue;
@@ -194,8 +221,8 @@ extern "C" int rms_residual(
             (float*)x_out, (T*)h_out, (const float*)x_in, (const T*)embed, \
             (const int*)tokens, embed_scale, (const P*)y, n_part,          \
             part_stride, row_stride, (const float*)share,                  \
-            (const float*)post, (const float*)pre, mult, eps,              \
-            (const int64_t*)rows, W, rt)
+            (const float*)post, (const float*)pre, (const float*)shift,    \
+            mult, eps, (const int64_t*)rows, W, tail, bare, rt)
     #define RR_N(T, P, V, F)                                               \
         do {                                                               \
             if (W <= 256 * V) RR(T, P, 256, 1, V, F);                      \
@@ -338,5 +365,96 @@ extern "C" int qk_norm_append(
     else QK_N(bf16, bf16);
     #undef QK_N
     #undef QK
+    return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// out = N(o) * w * sigmoid(gate), the norm over a token's whole row of N
+// columns; o fp32, the gate a column range of a projection that may still be
+// split.  One block per token.  NV > 0: the row stays in registers.
+// ---------------------------------------------------------------------------
+template <typename T, typename P, int BS, int NV, int VEC, bool FR>
+__global__ __launch_bounds__(BS) void k_rms_gate(
+    T* __restrict__ out, const float* __restrict__ o,
+    const float* __restrict__ w, Rows<P> gate, int og, int N, float eps)
+{
+    const int64_t t = blockIdx.x;
+    const int tid = threadIdx.x;
+    const float* row = o + t * N;
+    __shared__ float red[BS / 64];
+    constexpr int KEEP = NV > 0 ? NV : 1;
+    float v[KEEP][VEC], s = 0.f;
+    auto count = [&](const float* u) {
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) s += u[i] * u[i];
+    };
+    if constexpr (NV > 0) {
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int c = (j * BS + tid) * VEC;
+            if (c >= N) break;
+            ldv<VEC>(row + c, v[j]);
+            count(v[j]);
+        }
+    } else {
+        for (int c = tid * VEC; c < N; c += BS * VEC) {
+            ldv<VEC>(row + c, v[0]);
+            count(v[0]);
+        }
+    }
+    const float f = 1.f / sqrtf(block_sum<BS>(s, red) / N + eps);
+    auto emit = [&](int c, float* u) {
+        float a[VEC], g[VEC];
+        ldv<VEC>(w + c, a);
+        ldrow<VEC>(gate, t, og + c, g);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++)
+            u[i] *= f * a[i] * sigmoid_of<T>(g[i]);
+        stv<VEC>(out + (FR ? frag_row_off(t, c, N) : t * N + c), u);
+    };
+    if constexpr (NV > 0) {
+        #pragma unroll
+        for (int j = 0; j < NV; j++) {
+            const int c = (j * BS + tid) * VEC;
+            if (c >= N) break;
+            emit(c, v[j]);
+        }
+    } else {
+        for (int c = tid * VEC; c < N; c += BS * VEC) {
+            ldv<VEC>(row + c, v[0]);
+            emit(c, v[0]);
+        }
+    }
+}
+
+extern "C" int rms_gate(
+    int f32, void* out, const void* o, const void* w, const void* gate,
+    int p32, int n_part, int64_t part_stride, int64_t ld, int og, int T_rows,
+    int N, float eps, int frag, hipStream_t stream)
+{
+    const bool vec = N % 4 == 0 && og % 4 == 0 && ld % 4 == 0
+                     && part_stride % 4 == 0;
+    if (frag && (f32 || !vec || N % 64)) return (int)hipErrorInvalidValue;
+    #define RG(T, P, BS, NV, VE, FR)                                       \
+        k_rms_gate<T, P, BS, NV, VE, FR><<<T_rows, BS, 0, stream>>>(       \
+            (T*)out, (const float*)o, (const float*)w,                     \
+            Rows<P>{(const P*)gate, n_part, part_stride, ld}, og, N, eps)
+    #define RG_N(T, P, FR)                                                 \
+        do {                                                               \
+            if (!vec) RG(T, P, 256, 0, 1, false);                          \
+            else if (N <= 1024) RG(T, P, 256, 1, 4, FR);                   \
+            else if (T_rows <= 256 && N <= 4096) RG(T, P, 1024, 1, 4, FR); \
+            else if (N <= 2048) RG(T, P, 256, 2, 4, FR);                   \
+            else if (N <= 4096) RG(T, P, 256, 4, 4, FR);                   \
+            else if (N <= 8192) RG(T, P, 1024, 2, 4, FR);                  \
+            else RG(T, P, 1024, 0, 4, FR);                                 \
+        } while (0)
+    if (f32) RG_N(float, float, false);
+    else if (frag && p32) RG_N(bf16, float, true);
+    else if (frag) RG_N(bf16, bf16, true);
+    else if (p32) RG_N(bf16, float, false);
+    else RG_N(bf16, bf16, false);
+    #undef RG_N
+    #undef RG
     return (int)hipGetLastError();
 }

@@ -103,62 +103,6 @@ template <> struct RowRule<bf16> {
     }
 };
 
-// zero the keys a query does not see; dist0: distance of s[0][0]'s key
-template <int N>
-DEV void mask_keys(f32x4* s, int dist0, int window) {
-    #pragma unroll
-    for (int j = 0; j < N; j++)
-        #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int d = dist0 - j * 16 - i;
-            if (d < 0 || (window > 0 && d >= window)) s[j][i] = 0.f;
-        }
-}
-
-// operand of the value product: column lr of a tile of 32 keys, keys 4g + i
-// of its two halves, the order in which the lanes hold the weights
-DEV bf16x8 value_frag(const bf16* tile, int stride, int lane) {
-    const s16x4 a = tr_read(tile, stride, lane);
-    const s16x4 b = tr_read(tile + 16 * stride, stride, lane);
-    return __builtin_bit_cast(
-        bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
-}
-DEV f32x8s value_frag(const float* tile, int stride, int lane) {
-    const float* p = tile + (lane >> 4) * 4 * stride + (lane & 15);
-    f32x8s f;
-    #pragma unroll
-    for (int e = 0; e < 4; e++) {
-        f.lo[e] = p[e * stride];
-        f.hi[e] = p[(16 + e) * stride];
-    }
-    return f;
-}
-template <typename T> DEV Frag<T> weight_frag(const f32x4* s) {
-    Frag<T> b;
-    #pragma unroll
-    for (int e = 0; e < 4; e++) {
-        frag_set(b, e, s[0][e]);
-        frag_set(b, e + 4, s[1][e]);
-    }
-    return b;
-}
-
-// four columns c0.. of head h of token t; V values per head
-template <typename T>
-DEV void put_out(T* out, int t, int h, int c0, int H, int V, f32x4 v,
-                 bool frag) {
-    if (c0 >= V) return;
-    const int c = h * V + c0;
-    T* dst = out + (frag ? frag_row_off(t, c, H * V)
-                         : (int64_t)t * H * V + c);
-    float f[4] = {v[0], v[1], v[2], v[3]};
-    if (V % 4 == 0) stv<4>(dst, f);
-    else
-        #pragma unroll
-        for (int i = 0; i < 4; i++)
-            if (c0 + i < V) stf(dst + i, f[i]);
-}
-
 // ---------------------------------------------------------------------------
 // Portions of prompts.  Block: four waves of NQ 16-row tiles over 64-key
 // chunks.  S^T = K Q^T puts a row on a lane (16 keys per lane and chunk);

@@ -70,6 +70,35 @@ DEV void stv(bf16* p, const float* o) {
     }
 }
 
+// Rows of a matrix that may still be the partial sums of a split product:
+// n_part of them part_stride apart, rows ld apart.
+template <typename P> struct Rows {
+    const P* p;
+    int n_part;
+    int64_t part_stride, ld;
+};
+// VEC columns of row t from column c on
+template <int VEC, typename P>
+DEV void ldrow(const Rows<P>& r, int64_t t, int c, float* v) {
+    const P* p = r.p + t * r.ld + c;
+    ldv<VEC>(p, v);
+    for (int s = 1; s < r.n_part; s++) {
+        float u[VEC];
+        ldv<VEC>(p + s * r.part_stride, u);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) v[i] += u[i];
+    }
+}
+
+template <typename T> DEV float exp_of(float x) {
+    if constexpr (sizeof(T) == 4) return expf(x);
+    else return __expf(x);
+}
+template <typename T> DEV float sigmoid_of(float x) {
+    if constexpr (sizeof(T) == 4) return 1.f / (1.f + expf(-x));
+    else return __builtin_amdgcn_rcpf(1.f + __expf(-x));
+}
+
 // Activation-fragment layout ("frag"): the SAME MFMA fragment order the
 // weight packs use, applied to a [32, K] activation: element (m, k) with
 // k = b*64 + j*16 + h*8 + e lives at 16-byte unit ((b*4 + j)*64 + h*32
@@ -97,6 +126,18 @@ DEV float wave_max(float x) {
     #pragma unroll
     for (int o = 32; o; o >>= 1) x = fmaxf(x, __shfl_xor(x, o, 64));
     return x;
+}
+
+// sum over the block; every thread gets it.  s: one float per wave
+template <int BS> DEV float block_sum(float v, float* s) {
+    v = wave_sum(v);
+    const int wid = threadIdx.x >> 6;
+    if ((threadIdx.x & 63) == 0) s[wid] = v;
+    __syncthreads();
+    float t = 0.f;
+    #pragma unroll
+    for (int i = 0; i < BS / 64; i++) t += s[i];
+    return t;
 }
 
 // odd series, relative error below 4e-7 up to 0.25
@@ -162,6 +203,10 @@ DEV void frag_set(bf16x8& f, int e, float v) { f[e] = (__bf16)v; }
 DEV void frag_set(f32x8s& f, int e, float v) {
     if (e < 4) f.lo[e] = v; else f.hi[e - 4] = v;
 }
+DEV float frag_get(const bf16x8& f, int e) { return (float)f[e]; }
+DEV float frag_get(const f32x8s& f, int e) {
+    return e < 4 ? f.lo[e] : f.hi[e - 4];
+}
 // elements e with k0 + e < K; the rest are zero
 template <typename T>
 DEV Frag<T> frag_guard(const T* p, int k0, int K) {
@@ -189,4 +234,63 @@ DEV s16x4 tr_read(const bf16* tile, int stride, int lane) {
     const bf16* p = tile + (4 * g + (lr >> 2)) * stride + (lr & 3) * 4;
     return __builtin_amdgcn_ds_read_tr16_b64_v4i16(
         (lds_s16x4*)const_cast<bf16*>(p));
+}
+
+// Operand of a product over the rows of an LDS tile: column lr of 32 rows,
+// rows 4g + i of its two halves -- the order in which a 16x16 result holds
+// its rows, so that the result of one product is an operand of the next.
+DEV bf16x8 value_frag(const bf16* tile, int stride, int lane) {
+    const s16x4 a = tr_read(tile, stride, lane);
+    const s16x4 b = tr_read(tile + 16 * stride, stride, lane);
+    return __builtin_bit_cast(
+        bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
+}
+DEV f32x8s value_frag(const float* tile, int stride, int lane) {
+    const float* p = tile + (lane >> 4) * 4 * stride + (lane & 15);
+    f32x8s f;
+    #pragma unroll
+    for (int e = 0; e < 4; e++) {
+        f.lo[e] = p[e * stride];
+        f.hi[e] = p[(16 + e) * stride];
+    }
+    return f;
+}
+// and that operand from two results
+template <typename T> DEV Frag<T> weight_frag(const f32x4* s) {
+    Frag<T> b;
+    #pragma unroll
+    for (int e = 0; e < 4; e++) {
+        frag_set(b, e, s[0][e]);
+        frag_set(b, e + 4, s[1][e]);
+    }
+    return b;
+}
+
+// zero the weights of keys a query does not see; s[j][i] is the key
+// j * 16 + i after that of s[0][0], which is dist0 tokens back
+template <int N>
+DEV void mask_keys(f32x4* s, int dist0, int window) {
+    #pragma unroll
+    for (int j = 0; j < N; j++)
+        #pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int d = dist0 - j * 16 - i;
+            if (d < 0 || (window > 0 && d >= window)) s[j][i] = 0.f;
+        }
+}
+
+// four columns c0.. of head h of token t; V values per head
+template <typename T>
+DEV void put_out(T* out, int t, int h, int c0, int H, int V, f32x4 v,
+                 bool frag) {
+    if (c0 >= V) return;
+    const int c = h * V + c0;
+    T* dst = out + (frag ? frag_row_off(t, c, H * V)
+                         : (int64_t)t * H * V + c);
+    float f[4] = {v[0], v[1], v[2], v[3]};
+    if (V % 4 == 0) stv<4>(dst, f);
+    else
+        #pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (c0 + i < V) stf(dst + i, f[i]);
 }

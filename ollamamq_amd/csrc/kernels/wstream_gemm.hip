@@ -463,7 +463,7 @@ __global__ __launch_bounds__(512) void k_wstream_gemm(
                 #pragma unroll
                 for (int wv = 0; wv < 8; wv++)
                     s += red8[wv][mr][n];
-                if (ksplit == 1) {
+                if (ksplit == 1 && y) {
                     if (rstd_parts) s *= rstd_sh[m];
                     if (bias) s += __bfloat162float(bias[n0 + n]);
                     const int64_t yo =
@@ -607,7 +607,7 @@ __global__ __launch_bounds__(256) void k_wstream_combine_tiles(
     }
 }
 
-// y == null with ksplit > 1: the partial sums are the result
+// y == null: the partial sums, fp32, are the result
 extern "C" int wstream_gemm_bf16(
     void* y, void* part, const void* x, const void* wp, const void* bias,
     int M, int N, int K, int64_t xs, int ksplit, int depth, int xlds,

@@ -10,6 +10,7 @@ import os
 from typing import Dict, NamedTuple, Optional
 
 from .checkpoint import read_config
+from .kavedra import KAVEDRA_PRESETS, KavedraConfig, KavedraModel
 from .llama import PRESETS, LlamaConfig, LlamaModel
 from .revitar import REVITAR_PRESETS, RevitarConfig, RevitarModel
 from .rinitar import RINITAR_PRESETS, RinitarConfig, RinitarModel
@@ -24,9 +25,11 @@ ARCHITECTURES: Dict[str, Architecture] = {
     "Llama": Architecture(LlamaConfig, LlamaModel),
     "Rinitar": Architecture(RinitarConfig, RinitarModel),
     "Revitar": Architecture(RevitarConfig, RevitarModel),
+    "Kavedra": Architecture(KavedraConfig, KavedraModel),
 }
 PRESETS.update(RINITAR_PRESETS)
 PRESETS.update(REVITAR_PRESETS)
+PRESETS.update(KAVEDRA_PRESETS)
 
 
 def config_from_folder(path: str, name: Optional[str] = None):

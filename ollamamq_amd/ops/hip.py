@@ -14,7 +14,8 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .interface import AttnMeta, FragRows, Partials, Weighted
+from .interface import (LIGHTNING_CHUNK, AttnMeta, FragRows, Partials,
+                        Weighted)
 
 _LIB_PATH = os.path.join(
     os.path.dirname(os.path.dirname(os.path.abspath(__file__))),
@@ -43,6 +44,7 @@ def _try_load():
     lib.paged_attn_bf16.argtypes = [vp, vp, vp, vp, vp, vp, vp, vp, vp,
                                     i, i, i, i, i, i, f, i64, vp]
     lib.swiglu_bf16.argtypes = [vp, vp, i, i, vp]
+    lib.swiglu_f32.argtypes = lib.swiglu_bf16.argtypes
     lib.argmax_bf16.argtypes = [vp, vp, i, i, vp, vp, i, vp]
     lib.argmax_f32.argtypes = lib.argmax_bf16.argtypes
     lib.decode_attn_bf16.argtypes = [vp, vp, vp, vp, vp, vp, vp, vp, vp,
@@ -76,13 +78,32 @@ def _try_load():
     lib.latent_append.argtypes = [i, vp, vp, i64, vp, vp, vp, vp,
                                   i, i, i, i, f, vp]
     lib.latent_gather.argtypes = [i, vp, vp, vp, vp, i, i, i, i, vp]
-    lib.head_gemm.argtypes = [i, vp, vp, vp, i, i, i, i, i64, i, vp]
-    lib.latent_mt.argtypes = [i, i, i]
+    rows = [vp, i, i, i64, i64]      # pointer, fp32?, parts, strides
+    lib.head_gemm.argtypes = [i, vp, vp, vp, *rows, i, i, i, i, i, i64, i, i,
+                              i, i, vp]
+    lib.latent_mt.argtypes = [i, i, i, i]
     lib.latent_attn.argtypes = [i, vp, vp, vp, vp, vp, vp, vp, vp, vp,
-                                i, i, i, i, i, i, f, i64, i64, i64, i, vp]
+                                i, i, i, i, i, i, i, f, i, i64, i64, i64, i,
+                                vp]
+    lib.latent_rope_append.argtypes = [i, vp, vp, *rows, vp, vp, vp, vp, vp,
+                                       i, i, i, i, i, i, i, i, f, vp]
+    lib.rope_qkv_append.argtypes = [i, vp, vp, vp, *rows, vp, vp, i, vp, vp,
+                                    vp, i, i, i, i, i, i, i, i, i, vp]
+    lib.softmax_rows.argtypes = [i, i, i]
+    lib.softmax_step.argtypes = [i]
+    lib.softmax_attn.argtypes = [i, i, vp, vp, vp, vp, vp, vp, vp, vp, vp,
+                                 vp, i, i, i, i, i, i, i, i, i, i, i, i, i,
+                                 f, vp, i, vp]
+    lib.rms_gate.argtypes = [i, vp, vp, vp, *rows, i, i, i, f, i, vp]
+    lib.lightning_step.argtypes = [i, vp, *rows, i, i, i, vp, vp, vp, vp, vp,
+                                   i, i, i, i, vp]
+    lib.lightning_chunks.argtypes = [i, vp, vp, *rows, i, i, i, vp, vp, vp,
+                                     vp, vp, vp, i, i, i, i, i, i, vp]
+    lib.lightning_scratch.argtypes = [i, i, i, i]
+    lib.lightning_scratch.restype = i64
     lib.flash_rows.argtypes = [i]
-    lib.flash_attn.argtypes = [i, vp, vp, vp, vp, vp, i, i, i, i, i64, i64,
-                               f, vp]
+    lib.flash_attn.argtypes = [i, vp, vp, vp, vp, vp, vp, i64, i, vp, i, i,
+                               i, i, i, i64, i64, i64, f, i, vp]
     lib.gla_step.argtypes = [i, vp, vp, i64, i, i, i, i, i, i, vp, vp, vp,
                              vp, vp, vp, vp, i, i, i, i, f, f, f, i, vp]
     lib.gla_chunks.argtypes = [i, vp, vp, vp, vp, i64, i, i, i, i, i, i,
@@ -91,8 +112,8 @@ def _try_load():
     lib.gla_scratch_floats.argtypes = [i, i, i]
     lib.gla_scratch_floats.restype = i64
     lib.rms_residual.argtypes = [i, vp, vp, vp, vp, vp, f, vp, i, i, i64,
-                                 i64, vp, vp, vp, f, f, vp, i, i, i, vp, vp, vp,
-                                 i, i, vp]
+                                 i64, vp, vp, vp, vp, f, f, vp, i, i, i, i,
+                                 i, vp, vp, vp, i, i, vp]
     lib.qk_norm_append.argtypes = [i, vp, vp, vp, vp, i, i, i64, i64, vp, vp,
                                    vp, vp, vp, i, i, i, i, i, i, i, i, i, f,
                                    vp]
@@ -749,7 +770,10 @@ def swiglu(gate_up):
     T, F2 = gate_up.shape
     F = F2 // 2
     out = torch.empty((T, F), dtype=gate_up.dtype, device=gate_up.device)
-    _check(_lib.swiglu_bf16(_p(out), _p(gate_up), T, F, _stream()),
+    f32 = _is_f32(gate_up)
+    assert gate_up.is_contiguous() and (f32 or F % 8 == 0)
+    fn = _lib.swiglu_f32 if f32 else _lib.swiglu_bf16
+    _check(fn(_p(out), _p(gate_up), T, F, _stream()),
            "swiglu")
     return out
 
@@ -805,6 +829,30 @@ def _linear_frag(x, N, packed, parts):
         _WS_DEPTH, 2, _p(None), 0, 0.0, 0.0, _p(None), _p(None), 0,
         _stream()), "wstream_gemm")
     return y if y is not None else Partials(part)
+
+
+def linear_f32(x, weight, packed=None):
+    """A product whose consumer takes fp32: partial sums, also if there is
+    only one, or the library's fp32 result."""
+    N = weight.shape[0]
+    if isinstance(x, FragRows):
+        M, K = x.rows, x.cols
+        part = torch.empty((_parts_ksplit(N, K), M, N), dtype=torch.float32,
+                           device=weight.device)
+        _check(_lib.wstream_gemm_bf16(
+            _p(None), _p(part), _p(x.buf), _p(packed), _p(None), M, N, K, 0,
+            part.shape[0], _WS_DEPTH, 2, _p(None), 0, 0.0, 0.0, _p(None),
+            _p(None), 0, _stream()), "wstream_gemm")
+        return Partials(part)
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, weight)
+    return torch.mm(x, weight.t(), out_dtype=torch.float32)
+
+
+def linear_gu_frag(x, packed, N):
+    """linear_gu of an activation in fragment layout, and so its result."""
+    act = linear_gu(x.buf, packed, N, K=x.cols, yfrag=1, M_frag=x.rows)
+    return FragRows(act, x.rows, N // 2)
 
 
 def linear_parts(x, weight, packed=None):
@@ -919,18 +967,41 @@ def latent_append(cache, run, d, weight, slot_ids, positions, eps):
         "latent_append")
 
 
-def head_gemm(x, w, out, frag=False):
-    """out[t, h] = w[h] @ x[t, h]; x [T, H, K] (rows may be strided); frag:
-    out is the buffer of a FragRows."""
-    T, H, K = x.shape
-    N = w.shape[1]
-    assert w.shape == (H, N, K) and w.is_contiguous() \
-        and (frag or out.shape == (T, H, N)) and out.is_contiguous() \
-        and x.stride(2) == 1 and (H == 1 or x.stride(1) == K)
+def _rows(p):
+    """A projection, or the partial sums of one, as the kernels take it:
+    (pointer, fp32?, parts, stride of a part, stride of a row)."""
+    if p is None:
+        return _p(None), 0, 1, 0, 0
+    t = p.parts if isinstance(p, Partials) else p
+    assert t.stride(-1) == 1
+    f32 = int(t.dtype == torch.float32)
+    if isinstance(p, Partials):
+        return _p(t), f32, t.shape[0], t.stride(0), t.stride(1)
+    return _p(t), f32, 1, 0, t.stride(0)
+
+
+def _cols(p):
+    return (p.parts if isinstance(p, Partials) else p).shape[-1]
+
+
+def head_gemm(x, w, out, frag=False, tail=0, gate=None):
+    """out[t, h] = w[h] @ x[t, h, :K]; x [T, H, >= K] (rows may be strided);
+    frag: out is the buffer of a FragRows.  Wider rows of `out` end in `tail`
+    values from behind the inputs, then zeros; gate: Columns whose sigmoid
+    multiplies the result."""
+    T, H, wide = x.shape
+    N, K = w.shape[1:]
+    os = N if frag else out.shape[2]
+    assert w.shape[0] == H and w.is_contiguous() and wide >= K + tail \
+        and (frag or out.shape == (T, H, os)) and out.is_contiguous() \
+        and x.stride(2) == 1 and os >= N + tail
+    gp, og = (None, 0) if gate is None else gate
+    assert gp is None or og + H * N <= _cols(gp)
     if T:
-        _check(_lib.head_gemm(_is_f32(x), _p(out), _p(x), _p(w), T, H, N, K,
-                              x.stride(0), int(frag), _stream()),
-               "head_gemm")
+        _check(_lib.head_gemm(_is_f32(x), _p(out), _p(x), _p(w), *_rows(gp),
+                              og, T, H, N, K, x.stride(0),
+                              x.stride(1) if H > 1 else wide, os, tail,
+                              int(frag), _stream()), "head_gemm")
     return out
 
 
@@ -940,31 +1011,36 @@ FLASH_MAX = 256           # expanded kernel: key and value widths
 EXPAND_BYTES = 1 << 30    # expanded keys and values held at a time
 
 
-def _absorb_limit(H, D, V, R):
-    """Portions below this many tokens attend in latent space: the expanded
-    form pays R*(D+V) per key once, the absorbed one R+R instead of D+V per
-    (query, key)."""
-    if R > LATENT_MAX_R:
-        return 0
-    if max(D, V) > FLASH_MAX or 2 * R <= D + V:
-        return 1 << 62
-    return max(16, R * (D + V) // (2 * R - D - V))
+def _absorbs(n, kv, H, D, E, V, R, KW, window):
+    """Whether n queries after kv - n tokens attend in latent space: the
+    expanded form pays R*(D+V) once per key it needs, the absorbed one KW+R
+    instead of D+E+V for every (query, key).  D, E: unrotated and rotated key
+    width."""
+    if KW > LATENT_MAX_R:
+        return False
+    if max(D + E, V) > FLASH_MAX or n < 16:
+        return True
+    seen = min(kv, window) if window else kv
+    keys = min(kv, n + window - 1) if window else kv
+    return n * seen * (KW + R - D - E - V) < keys * R * (D + V)
 
 
-def _latent_plan(meta, H, D, V, R, f32, dev):
+def _latent_plan(meta, w, KW, f32, dev):
     """Batch layout for one attention shape, shared by the layers that have
     it: leading sequences attend in latent space, the rest expanded."""
-    key = f"_latent_{H}_{D}_{V}_{R}"
+    H, D, R = w.uk.shape
+    V, E, window = w.uv.shape[1], w.rot_dim, w.window
+    key = f"_latent_{H}_{D}_{E}_{V}_{R}_{window}"
     plan = getattr(meta, key, None)
     if plan is not None:
         return plan
     slots, q_lens, kv_lens = meta.layout()
-    limit = _absorb_limit(H, D, V, R)
-    M = 16 * _lib.latent_mt(f32, H, R)
+    M = 16 * _lib.latent_mt(f32, H, R, KW)
     nd = meta.n_single
     i, row, items = nd, nd, []
     kv_absorbed = 0
-    while i < len(slots) and q_lens[i] < limit:
+    while i < len(slots) and _absorbs(q_lens[i], kv_lens[i], H, D, E, V, R,
+                                      KW, window):
         lo, hi = row * H, (row + q_lens[i]) * H
         items += [(r, min(M, hi - r)) for r in range(lo, hi, M)]
         kv_absorbed = max(kv_absorbed, kv_lens[i])
@@ -986,12 +1062,14 @@ def _latent_plan(meta, H, D, V, R, f32, dev):
 
     while i < len(slots):
         n, kv = q_lens[i], kv_lens[i]
-        for b in range(0, kv, 64):
+        # whole groups of 64 positions from the first one a query sees
+        lo = max(0, kv - n + 1 - window) // 64 * 64 if window else 0
+        for b in range(lo, kv, 64):
             gather.append((slots[i], b, min(64, kv - b)))
         for t in range(0, n, QT):
-            tiles.append((row + t, kv - n + t, min(QT, n - t), kv0))
+            tiles.append((row + t, kv - n + t, min(QT, n - t), kv0 - lo))
         row += n
-        kv0 += (kv + 63) // 64 * 64
+        kv0 += (kv - lo + 63) // 64 * 64
         i += 1
         if kv0 * H * (D + V) * esz > EXPAND_BYTES:
             flush()
@@ -1003,37 +1081,42 @@ def _latent_plan(meta, H, D, V, R, f32, dev):
     return plan
 
 
-def _latent_absorbed(o, q, cache, run, slots, pos, H, R, scale, items,
-                     n_items, per_seq, row0, rows, max_kv):
+def _latent_absorbed(o, q, cache, run, slots, pos, H, w, items, n_items,
+                     per_seq, row0, rows, max_kv):
     """One launch of the absorbed kernel over rows row0.. of q / o."""
     f32 = _is_f32(q)
+    total, KW = q.shape
+    R = o.shape[1]
+    seen = min(max_kv, w.window + 63) if w.window else max_kv
     # one block a CU: more segments would only write more partial results
-    split = int(max(1, min(256 // n_items, (max_kv + 63) // 64,
+    split = int(max(1, min(256 // n_items, (seen + 63) // 64,
                            LATENT_SPLIT_MAX)))
     op = ml = None
-    total = q.shape[0]
     if split > 1:
         op = torch.empty((split, total, R), dtype=q.dtype, device=q.device)
         ml = torch.empty((split, total, 2), dtype=torch.float32,
                          device=q.device)
     pool = cache.latent_pool[run]
-    assert pool.dtype == q.dtype and pool.shape[2] == R
+    assert pool.dtype == q.dtype and pool.shape[2] == KW
     _check(_lib.latent_attn(
         f32, _p(o), _p(op), _p(ml), _p(q), _p(pool), _p(cache.page_table),
-        _p(slots), _p(pos), _p(items), n_items, per_seq, H, R,
-        cache.page_size, cache.page_table.shape[1], float(scale), total,
-        row0, rows, split, _stream()), "latent_attn")
+        _p(slots), _p(pos), _p(items), n_items, per_seq, H, R, KW,
+        cache.page_size, cache.page_table.shape[1], float(w.scale),
+        w.window, total, row0, rows, split, _stream()), "latent_attn")
 
 
 def latent_attention(q, cache, run, w, slot_ids, positions, meta,
-                     frag=False):
+                     frag=False, gate=None):
     H, D, R = w.uk.shape
-    V = w.uv.shape[1]
-    T = q.shape[0]
+    V, E = w.uv.shape[1], w.rot_dim
+    T, DD = q.shape[0], D + E
     f32 = _is_f32(q)
-    if R > LATENT_MAX_R and (max(D, V) > FLASH_MAX or meta.n_single):
+    pool = cache.latent_pool[run]
+    KW = pool.shape[2]
+    assert q.shape[1] == H * DD and KW >= R + E
+    if KW > LATENT_MAX_R and (max(DD, V) > FLASH_MAX or meta.n_single):
         raise ValueError(f"latent attention with rank {R}, head widths "
-                         f"{D}/{V}: no kernel")
+                         f"{DD}/{V}: no kernel")
     assert not frag or meta.one_each
     if frag:
         res = _frag_rows(T, H * V, q)
@@ -1045,48 +1128,76 @@ def latent_attention(q, cache, run, w, slot_ids, positions, meta,
     if meta.one_each:
         n_abs, items, kv_abs, groups = T, None, 0, []
     else:
-        n_abs, items, kv_abs, groups = _latent_plan(meta, H, D, V, R, f32,
+        n_abs, items, kv_abs, groups = _latent_plan(meta, w, KW, f32,
                                                     q.device)
     if n_abs:
-        qa = q[:n_abs].unflatten(1, (H, D))
-        lat = torch.empty((n_abs, H, R), dtype=q.dtype, device=q.device)
-        head_gemm(qa, w.uk_t, lat)
-        lat = lat.view(n_abs * H, R)
-        o = torch.empty_like(lat)
+        qa = q[:n_abs].unflatten(1, (H, DD))
+        lat = torch.empty((n_abs, H, KW), dtype=q.dtype, device=q.device)
+        head_gemm(qa, w.uk_t, lat, tail=E)
+        lat = lat.view(n_abs * H, KW)
+        o = torch.empty((n_abs * H, R), dtype=q.dtype, device=q.device)
         if nd:
-            per = -(-H // (16 * _lib.latent_mt(f32, H, R)))
-            _latent_absorbed(o, lat, cache, run, slots, pos, H, R, w.scale,
-                             None, nd * per, per, 0, nd * H, meta.max_kv)
+            per = -(-H // (16 * _lib.latent_mt(f32, H, R, KW)))
+            _latent_absorbed(o, lat, cache, run, slots, pos, H, w, None,
+                             nd * per, per, 0, nd * H, meta.max_kv)
         if items is not None:
-            _latent_absorbed(o, lat, cache, run, slots, pos, H, R, w.scale,
-                             items, items.shape[0], 1, nd * H,
-                             (n_abs - nd) * H, kv_abs)
+            _latent_absorbed(o, lat, cache, run, slots, pos, H, w, items,
+                             items.shape[0], 1, nd * H, (n_abs - nd) * H,
+                             kv_abs)
         head_gemm(o.view(n_abs, H, R), w.uv, out if frag else out[:n_abs],
-                  frag)
+                  frag, gate=gate)
         if frag:
             return res
-    pool = cache.latent_pool[run]
+    g, og = (None, 0) if gate is None else gate
+    if groups and isinstance(g, Partials):
+        g, og = g.parts[:, :, og:og + H * V].sum(0).to(q.dtype), 0
+    assert g is None or not groups or (g.dtype == q.dtype
+                                       and g.stride(1) == 1)
     for gather, tiles, kv in groups:
-        c = torch.empty((kv, R), dtype=q.dtype, device=q.device)
+        c = torch.empty((kv, KW), dtype=q.dtype, device=q.device)
         _check(_lib.latent_gather(
             f32, _p(c), _p(pool), _p(cache.page_table), _p(gather),
-            gather.shape[0], R, cache.page_size, cache.page_table.shape[1],
+            gather.shape[0], KW, cache.page_size, cache.page_table.shape[1],
             _stream()), "latent_gather")
-        k = torch.nn.functional.linear(c, w.uk.view(H * D, R))
-        vt = torch.mm(w.uv.view(H * V, R), c.t())
+        lat = c[:, :R]
+        k = torch.nn.functional.linear(lat, w.uk.view(H * D, R))
+        vt = torch.mm(w.uv.view(H * V, R), lat.t())
         _check(_lib.flash_attn(
-            f32, _p(out), _p(q), _p(k), _p(vt), _p(tiles), tiles.shape[0],
-            H, D, V, q.stride(0), kv, float(w.scale), _stream()),
-            "flash_attn")
+            f32, _p(out), _p(q), _p(k), _p(c[:, R:] if E else None), _p(vt),
+            _p(g), 0 if g is None else g.stride(0), og, _p(tiles),
+            tiles.shape[0], H, D, E, V, q.stride(0), KW, kv, float(w.scale),
+            w.window, _stream()), "flash_attn")
     return out.view(T, H * V)
+
+
+def latent_rope_append(p, cache, run, w, norm, eps, rope, slot_ids,
+                       positions):
+    H, D, R = w.uk.shape
+    E, pool, T = w.rot_dim, cache.latent_pool[run], slot_ids.shape[0]
+    assert rope.dims == E and rope.table.shape == (rope.table.shape[0], E) \
+        and rope.table.shape[0] >= cache.max_ctx and norm.numel() == R \
+        and _cols(p) >= H * (D + E) + R + E
+    q = torch.empty((T, H * (D + E)), dtype=pool.dtype, device=pool.device)
+    rows = _rows(p)
+    assert rows[1] or pool.dtype == torch.bfloat16
+    if T:
+        _check(_lib.latent_rope_append(
+            _is_f32(q), _p(q), _p(pool), *rows, _p(norm), _p(rope.table),
+            _p(_i32(slot_ids)), _p(_i32(positions)), _p(cache.page_table), T,
+            H, D, E, R, pool.shape[2], cache.page_size,
+            cache.page_table.shape[1], float(eps), _stream()),
+            "latent_rope_append")
+    return q
 
 
 GLA_STEP_TOKENS = 4       # portions up to this walk token by token
 GLA_CHUNK_MAX = (512, 256)   # key width and low rank the chunk kernels take
 
 
-def _gla_plan(meta, dev, step_tokens):
-    key = f"_gla_plan_{step_tokens}"
+def _chunk_plan(meta, dev, step_tokens):
+    """Layout of a recurrence: portions of up to `step_tokens` tokens at the
+    front walk token by token, the rest in chunks of 64."""
+    key = f"_chunk_plan_{step_tokens}"
     plan = getattr(meta, key, None)
     if plan is not None:
         return plan
@@ -1133,7 +1244,7 @@ def gla(p, w, state, slot_ids, positions, meta, frag=False):
     if meta.one_each:
         return res
     chunked = D <= GLA_CHUNK_MAX[0] and w.rank <= GLA_CHUNK_MAX[1]
-    spans, chunks, seqs, base, rows = _gla_plan(
+    spans, chunks, seqs, base, rows = _chunk_plan(
         meta, p.device, GLA_STEP_TOKENS if chunked else 1 << 62)
     if spans is not None:
         _check(_lib.gla_step(f32, _p(out), *head, _p(spans),
@@ -1149,19 +1260,76 @@ def gla(p, w, state, slot_ids, positions, meta, frag=False):
     return out
 
 
+LIGHTNING_STEP_TOKENS = 4    # portions up to this walk token by token
+LIGHTNING_MAX_D = 256        # key width the chunk kernels take
+
+
+def lightning(p, w, state, slot_ids, positions, meta, frag=False):
+    H, D, V = w.heads, w.dim, w.vdim
+    rows = _rows(p)
+    t = p.parts if isinstance(p, Partials) else p
+    T, dtype = t.shape[-2], torch.bfloat16 if isinstance(p, Partials) \
+        else p.dtype
+    f32 = int(dtype == torch.float32)
+    oq, ok, ov, og = w.offsets
+    assert state.dtype == torch.float32 and state.is_contiguous() \
+        and state.shape[1:] == (H, D, V) and w.norm.numel() == H * V \
+        and w.powers.shape == (H, LIGHTNING_CHUNK + 1) \
+        and w.powers.is_contiguous() \
+        and max(oq + H * D, ok + H * D, ov + H * V, og + H * V) <= t.shape[-1]
+    assert not frag or meta.one_each
+    o = torch.empty((T, H * V), dtype=torch.float32, device=t.device)
+    slots, pos = _i32(slot_ids), _i32(positions)
+    head = (*rows, oq, ok, ov, _p(w.powers), _p(state), _p(slots), _p(pos))
+    nd = meta.n_single
+    if nd:
+        _check(_lib.lightning_step(f32, _p(o), *head, _p(None), nd, H, D, V,
+                                   _stream()), "lightning_step")
+    if not meta.one_each:
+        spans, chunks, seqs, base, n = _chunk_plan(
+            meta, t.device,
+            LIGHTNING_STEP_TOKENS if D <= LIGHTNING_MAX_D else 1 << 62)
+        if spans is not None:
+            _check(_lib.lightning_step(
+                f32, _p(o), *head, _p(spans), spans.shape[0], H, D, V,
+                _stream()), "lightning_step")
+        if chunks is not None:
+            scr = torch.empty(_lib.lightning_scratch(n, H, D, V),
+                              dtype=dtype, device=t.device)
+            _check(_lib.lightning_chunks(
+                f32, _p(o), _p(scr), *head, _p(chunks), _p(seqs),
+                seqs.shape[0], base, n, H, D, V, _stream()),
+                "lightning_chunks")
+    N = H * V
+    if frag:
+        res = _frag_rows(T, N, t)
+        out = res.buf
+    else:
+        res = out = torch.empty((T, N), dtype=dtype, device=t.device)
+    if T:
+        _check(_lib.rms_gate(f32, _p(out), _p(o), _p(w.norm), *rows, og, T,
+                             N, float(w.eps), int(frag), _stream()),
+               "rms_gate")
+    return res
+
+
 # ---------------------------------------------------------------------------
 # norms on sublayer outputs, sigmoid attention, mixture of experts
 
 def rms_residual(x, y, post, pre, mult, eps, embed, tokens, embed_scale,
-                 rows, need_x, frag, route=None):
+                 rows, need_x, frag, route=None, shift=None, tail=False,
+                 bare=False):
     """route: MoeWeights whose router takes h on the way; then (x', h,
     (chosen, share))."""
     W = embed.shape[1]
     if x is not None:
         T = x.shape[0]
         assert x.dtype == torch.float32 and x.is_contiguous()
+    elif bare:
+        T = y.parts.shape[1] if isinstance(y, Partials) else y.shape[0]
     else:
         T = tokens.shape[0]
+    assert not tail or tokens.shape[0] == T
     n_part, part_stride, row_stride, share = 1, 0, W, None
     yt = y
     if isinstance(y, Partials):
@@ -1177,12 +1345,13 @@ def rms_residual(x, y, post, pre, mult, eps, embed, tokens, embed_scale,
     assert yt is None or (yt.is_contiguous() and yt.dtype in
                           (embed.dtype, torch.float32))
     n = T if rows is None else rows.shape[0]
+    HW = 2 * W if tail else W
     if frag:
         assert embed.dtype == torch.bfloat16 and W % 64 == 0
-        res = _frag_rows(n, W, embed)
+        res = _frag_rows(n, HW, embed)
         h = res.buf
     else:
-        res = h = torch.empty((n, W), dtype=embed.dtype, device=embed.device)
+        res = h = torch.empty((n, HW), dtype=embed.dtype, device=embed.device)
     x_out = torch.empty((n, W), dtype=torch.float32, device=embed.device) \
         if need_x else None
     chosen = route_share = None
@@ -1199,7 +1368,8 @@ def rms_residual(x, y, post, pre, mult, eps, embed, tokens, embed_scale,
             _p(None if tokens is None else _i32(tokens)), float(embed_scale),
             _p(yt), int(yt is not None and yt.dtype == torch.float32),
             n_part, part_stride, row_stride, _p(share), _p(post), _p(pre),
-            float(mult), float(eps), _p(rows), n, W, int(frag),
+            _p(shift), float(mult), float(eps), _p(rows), n, W, int(tail),
+            int(bare), int(frag),
             _p(None if route is None else route.router), _p(chosen),
             _p(route_share), E, top, _stream()), "rms_residual")
     if route is not None:
@@ -1246,25 +1416,25 @@ def qk_norm_append(p, cache, run, w, q_norm, k_norm, eps, slot_ids,
     return q
 
 
-SIGMOID_MAX = 256         # key and value widths
-SIGMOID_SHORT = 8         # portions up to this many tokens split the context
-SIGMOID_SPLIT_MAX = 16
-SIGMOID_LARGE = 128 * 1024   # (token, head) rows from which tiles are large:
+ATTN_MAX = 256         # key and value widths
+ATTN_SHORT = 8         # portions up to this many tokens split the context
+ATTN_SPLIT_MAX = 16
+ATTN_LARGE = 128 * 1024   # (token, head) rows from which tiles are large:
                              # they share staged keys, small ones share load
 
 
-def _sigmoid_plan(meta, R, rows, dev):
+def _tile_plan(meta, R, rows, dev):
     """Tiles of one attention shape: leading single tokens and short
     portions in 16-row tiles for the context-splitting kernel, the rest in
     `rows`-row tiles."""
-    key = f"_sigmoid_{R}_{rows}"
+    key = f"_tiles_{R}_{rows}"
     plan = getattr(meta, key, None)
     if plan is not None:
         return plan
     _, q_lens, kv_lens = meta.layout()
     i = row = kv = 0
     short, long_ = [], []
-    while i < len(q_lens) and q_lens[i] <= SIGMOID_SHORT:
+    while i < len(q_lens) and q_lens[i] <= ATTN_SHORT:
         lo, hi = row * R, (row + q_lens[i]) * R
         short += [(r, min(16, hi - r)) for r in range(lo, hi, 16)]
         kv = max(kv, kv_lens[i])
@@ -1287,7 +1457,7 @@ def sigmoid_attention(q, cache, run, w, slot_ids, positions, meta, frag):
     kp, vp = cache.key_pool[run], cache.value_pool[run]
     G, V, R = w.kv_heads, w.vdim, w.heads // w.kv_heads
     f32 = _is_f32(q)
-    if max(Dp, vp.shape[3]) > SIGMOID_MAX:
+    if max(Dp, vp.shape[3]) > ATTN_MAX:
         raise ValueError(f"sigmoid attention with head widths {w.dim}/"
                          f"{w.vdim}: no kernel")
     assert q.is_contiguous() and kp.dtype == q.dtype \
@@ -1304,8 +1474,8 @@ def sigmoid_attention(q, cache, run, w, slot_ids, positions, meta, frag):
         short = long_ = None
     else:
         rows = _lib.sigmoid_rows(f32, Dp, vp.shape[3]) \
-            if T * H >= SIGMOID_LARGE else 64
-        short, n_tok, kv, long_ = _sigmoid_plan(meta, R, rows, q.device)
+            if T * H >= ATTN_LARGE else 64
+        short, n_tok, kv, long_ = _tile_plan(meta, R, rows, q.device)
         n_items = 0 if short is None else short.shape[0]
 
     def launch(item_rows, items, n, t0, tokens, split, part):
@@ -1321,12 +1491,84 @@ def sigmoid_attention(q, cache, run, w, slot_ids, positions, meta, frag):
         seen = min(kv, w.window) if w.window else kv
         split = max(1, min(256 // (n_items * G),
                            -(-seen // _lib.sigmoid_step(f32)),
-                           SIGMOID_SPLIT_MAX))
+                           ATTN_SPLIT_MAX))
         part = torch.empty((split, T, H * V), dtype=torch.float32,
                            device=q.device) if split > 1 else None
         launch(16, short, n_items, 0, n_tok, split, part)
     if long_ is not None:
         launch(rows, long_, long_.shape[0], 0, T, 1, None)
+    return res
+
+
+def rope_qkv_append(p, bias, cache, run, w, rope, slot_ids, positions):
+    kp, vp = cache.key_pool[run], cache.value_pool[run]
+    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
+    T, n = slot_ids.shape[0], H * D + G * (D + V)
+    assert _cols(p) >= n and (bias is None or bias.numel() >= n)
+    assert kp.shape[1:3] == (G, cache.page_size) and kp.shape[3] >= D \
+        and vp.shape[3] >= V and rope.dims <= D
+    assert not rope.dims or (rope.table.shape[1] == rope.dims
+                             and rope.table.shape[0] >= cache.max_ctx)
+    q = torch.empty((T, H, kp.shape[3]), dtype=kp.dtype, device=kp.device)
+    rows = _rows(p)
+    assert rows[1] or kp.dtype == torch.bfloat16
+    if T:
+        _check(_lib.rope_qkv_append(
+            _is_f32(q), _p(q), _p(kp), _p(vp), *rows, _p(bias),
+            _p(rope.table), rope.dims, _p(_i32(slot_ids)),
+            _p(_i32(positions)), _p(cache.page_table), T, H, G, D, V,
+            kp.shape[3], vp.shape[3], cache.page_size,
+            cache.page_table.shape[1], _stream()), "rope_qkv_append")
+    return q
+
+
+def softmax_attention(q, cache, run, w, slot_ids, positions, meta, frag):
+    T, H, Dp = q.shape
+    kp, vp = cache.key_pool[run], cache.value_pool[run]
+    G, V, R = w.kv_heads, w.vdim, w.heads // w.kv_heads
+    Vp, f32 = vp.shape[3], _is_f32(q)
+    if max(Dp, Vp) > ATTN_MAX:
+        raise ValueError(f"softmax attention with head widths {w.dim}/"
+                         f"{w.vdim}: no kernel")
+    assert q.is_contiguous() and kp.dtype == q.dtype \
+        and kp.shape[1:] == (G, cache.page_size, Dp) and H == w.heads \
+        and (w.sink is None or w.sink.numel() == H)
+    assert not frag or meta.one_each
+    if frag:
+        res = _frag_rows(T, H * V, q)
+        out = res.buf
+    else:
+        res = out = torch.empty((T, H * V), dtype=q.dtype, device=q.device)
+    if meta.one_each:
+        n_items, n_tok, kv = T * -(-R // 16), T, meta.max_kv
+        short = long_ = None
+    else:
+        rows = _lib.softmax_rows(f32, Dp, Vp) if T * H >= ATTN_LARGE else 64
+        short, n_tok, kv, long_ = _tile_plan(meta, R, rows, q.device)
+        n_items = 0 if short is None else short.shape[0]
+
+    def launch(item_rows, items, n, tokens, split, part, ml):
+        _check(_lib.softmax_attn(
+            f32, item_rows, _p(out), _p(part), _p(ml), _p(q), _p(kp), _p(vp),
+            _p(cache.page_table), _p(_i32(slot_ids)), _p(_i32(positions)),
+            _p(items), n, 0, tokens, T, H, G, V, Dp, Vp, cache.page_size,
+            cache.page_table.shape[1], split, int(frag), w.scale, _p(w.sink),
+            w.window, _stream()), "softmax_attn")
+
+    if n_items:
+        seen = min(kv, w.window) if w.window else kv
+        split = max(1, min(256 // (n_items * G),
+                           -(-seen // _lib.softmax_step(f32)),
+                           ATTN_SPLIT_MAX))
+        part = ml = None
+        if split > 1:
+            part = torch.empty((split, T, H * V), dtype=torch.float32,
+                               device=q.device)
+            ml = torch.empty((split, T, H, 2), dtype=torch.float32,
+                             device=q.device)
+        launch(16, short, n_items, n_tok, split, part, ml)
+    if long_ is not None:
+        launch(rows, long_, long_.shape[0], T, 1, None, None)
     return res
 
 

@@ -116,13 +116,60 @@ class FragRows(NamedTuple):
     cols: int
 
 
+class Columns(NamedTuple):
+    """Columns of a fused projection from `first` on, as many as the consumer
+    needs; the projection may be Partials."""
+    p: object
+    first: int
+
+
+class Rope(NamedTuple):
+    """Rotary positions: table [positions, dims] fp32 holds (cos, sin) of
+    every pair (2i, 2i+1) of a head's first `dims` dimensions."""
+    table: torch.Tensor
+    dims: int
+
+
 class LatentWeights(NamedTuple):
     """k = uk c, v = uv c per head; uk [H, D, R], uk_t [H, R, D] and
-    uv [H, V, R] are views or copies of the same values."""
+    uv [H, V, R] are views or copies of the same values.  With rot_dim, query
+    heads are [D, rot_dim] and the cached row ends in a key part of that
+    width which all heads share.  A query sees `window` tokens, itself
+    included (0: all before it)."""
     uk: torch.Tensor
     uk_t: torch.Tensor
     uv: torch.Tensor
     scale: float
+    rot_dim: int = 0
+    window: int = 0
+
+
+class SoftmaxAttn(NamedTuple):
+    """Softmax attention over paged keys and values; `sink` (fp32 per query
+    head, or None) is one more logit of the denominator.  A query sees
+    `window` tokens, itself included (0: all before it)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    sink: Optional[torch.Tensor] = None
+    window: int = 0
+
+
+LIGHTNING_CHUNK = 64
+
+
+class LightningWeights(NamedTuple):
+    """Columns of the fused projection, and what the recurrence and the norm
+    over all heads read."""
+    heads: int
+    dim: int
+    vdim: int
+    offsets: tuple                # columns of q, k, v, gate
+    powers: torch.Tensor          # fp32 [heads, LIGHTNING_CHUNK + 1]
+    norm: torch.Tensor            # fp32 [heads * vdim]
+    eps: float
 
 
 class GlaWeights(NamedTuple):
@@ -286,6 +333,14 @@ def dyt_residual(x, y, post: Optional[DyT], pre: DyT,
     return ref.dyt_residual(x, y, post, pre, shift, embed, tokens, rows)
 
 
+def linear_f32(x, weight, packed=None) -> Union[torch.Tensor, Partials]:
+    """As linear_parts, the result fp32 whatever the operands' type."""
+    if _use_hip(weight):
+        from . import hip
+        return hip.linear_f32(x, weight, packed)
+    return torch.nn.functional.linear(x.float(), weight.float())
+
+
 def polynorm(z, coef, eps, frag=False):
     """a N(z) + b N(z^2) + c N(z^3) + e with coef = (a, b, c, e) and N the
     division by the row's root mean square."""
@@ -305,15 +360,69 @@ def latent_append(cache, run, d, weight, slot_ids, positions, eps):
     return ref.latent_append(cache, run, d, weight, slot_ids, positions, eps)
 
 
+def latent_rope_append(p, cache, run, w: LatentWeights, norm, eps,
+                       rope: Rope, slot_ids, positions):
+    """Split the projection p (columns q [H, D + rot_dim] | latent | shared
+    key part; a tensor or Partials), rotate, norm the latent, append latent
+    and key part to the run's pool.  -> queries [T, H * (D + rot_dim)]."""
+    t = p.parts if isinstance(p, Partials) else p
+    if _use_hip(t):
+        from . import hip
+        return hip.latent_rope_append(p, cache, run, w, norm, eps, rope,
+                                      slot_ids, positions)
+    return ref.latent_rope_append(p, cache, run, w, norm, eps, rope,
+                                  slot_ids, positions)
+
+
 def latent_attention(q, cache, run, w: LatentWeights, slot_ids, positions,
-                     meta: AttnMeta, frag=False):
+                     meta: AttnMeta, frag=False,
+                     gate: Optional[Columns] = None):
     """Causal softmax attention whose keys and values are linear in the
-    cached latent.  q [T, H*D] (rows may be strided) -> [T, H*V]."""
+    cached latent.  q [T, H*(D+rot_dim)] (rows may be strided) -> [T, H*V],
+    times the sigmoid of the gate's columns."""
     if _use_hip(q):
         from . import hip
         return hip.latent_attention(q, cache, run, w, slot_ids, positions,
-                                    meta, frag)
-    return ref.latent_attention(q, cache, run, w, meta)
+                                    meta, frag, gate)
+    return ref.latent_attention(q, cache, run, w, meta, gate)
+
+
+def rope_qkv_append(p, bias, cache, run, w: SoftmaxAttn, rope: Rope,
+                    slot_ids, positions):
+    """Split the projection p (columns q | k | v; a tensor or Partials), add
+    its bias (fp32, or None), rotate queries and keys, append keys and values
+    to the run's paged pools.  -> queries [T, H, D'], rows filled up with
+    zeros as the pool's are."""
+    t = p.parts if isinstance(p, Partials) else p
+    if _use_hip(t):
+        from . import hip
+        return hip.rope_qkv_append(p, bias, cache, run, w, rope, slot_ids,
+                                   positions)
+    return ref.rope_qkv_append(p, bias, cache, run, w, rope, slot_ids,
+                               positions)
+
+
+def softmax_attention(q, cache, run, w: SoftmaxAttn, slot_ids, positions,
+                      meta: AttnMeta, frag=False):
+    """Causal softmax attention over the run's paged keys and values; q as
+    rope_qkv_append returns it.  -> [T, H*V]."""
+    if _use_hip(q):
+        from . import hip
+        return hip.softmax_attention(q, cache, run, w, slot_ids, positions,
+                                     meta, frag)
+    return ref.softmax_attention(q, cache, run, w, meta)
+
+
+def lightning(p, w: LightningWeights, state, slot_ids, positions,
+              meta: AttnMeta, frag=False):
+    """Lightning attention over the fused projection p [T, ...] (a tensor or
+    Partials): silu of q, k and v, a recurrence with one decay per head;
+    state [slots, H, D, V] fp32 is read and advanced.  Norm over all heads
+    and output gate included.  -> [T, H*V]."""
+    if _use_hip(w.norm):
+        from . import hip
+        return hip.lightning(p, w, state, slot_ids, positions, meta, frag)
+    return ref.lightning(p, w, state, meta)
 
 
 def gla(p, w: GlaWeights, state, slot_ids, positions, meta: AttnMeta,
@@ -328,18 +437,23 @@ def gla(p, w: GlaWeights, state, slot_ids, positions, meta: AttnMeta,
 
 
 def rms_residual(x, y, post, pre, mult, eps, embed=None, tokens=None,
-                 embed_scale=1.0, rows=None, need_x=True, frag=False):
-    """One pass between two matrix products: x' = x + mult * N(y) * post,
+                 embed_scale=1.0, rows=None, need_x=True, frag=False,
+                 shift=None, tail=False, bare=False):
+    """One pass between two matrix products:
+    x' = x + mult * N(y) * post + shift, without `post` x + mult * y + shift;
     h = N(x') * pre, or x' itself without `pre`; N divides a row by its root
     mean square.  x is fp32 [T, W], or None for the scaled embedding rows of
-    `tokens`; y a tensor, Partials, Weighted or None; `rows` selects the
-    rows to compute; frag returns h as FragRows.  Returns (x', h)."""
+    `tokens` (for nothing if `bare`); y a tensor, Partials, Weighted or None;
+    shift fp32 [W] or None; `rows` selects the rows to compute; `tail`
+    appends the token's embedding row to h; frag returns h as FragRows.
+    Returns (x', h)."""
     if _use_hip(embed):
         from . import hip
         return hip.rms_residual(x, y, post, pre, mult, eps, embed, tokens,
-                                embed_scale, rows, need_x, frag)
+                                embed_scale, rows, need_x, frag, shift=shift,
+                                tail=tail, bare=bare)
     return ref.rms_residual(x, y, post, pre, mult, eps, embed, tokens,
-                            embed_scale, rows)
+                            embed_scale, rows, shift, tail, bare)
 
 
 def rms_residual_route(x, y, post, mult, eps, moe, embed=None, tokens=None,
@@ -411,7 +525,11 @@ def gateup_swiglu(x, weight, packed_gu=None):
     GU-packed copy this is ONE fused weight-streaming kernel; otherwise
     the library GEMM + the swiglu kernel.  (An MT2 variant for 33..64
     exists but measured BELOW the library at 64 users — its direct
-    fragment x-loads double the scattered line traffic; see NOTES.)"""
+    fragment x-loads double the scattered line traffic.)  FragRows go
+    through the fused kernel at any batch and stay FragRows."""
+    if isinstance(x, FragRows):
+        from . import hip
+        return hip.linear_gu_frag(x, packed_gu, weight.shape[0])
     if packed_gu is not None and x.shape[0] <= 32 and _use_hip(x):
         from . import hip
         if hip.USE_WSTREAM and x.dtype == torch.bfloat16 \

@@ -149,24 +149,128 @@ def latent_append(cache, run, d, weight, slot_ids, positions, eps):
     pool[pages.long(), (positions % ps).long()] = c.to(pool.dtype)
 
 
-def latent_attention(q, cache, run, w, meta):
+def whole(p):
+    """A projection in fp32, its partial sums added up."""
+    return p.parts.sum(0) if hasattr(p, "parts") else p.float()
+
+
+def _rotate(x, positions, rope):
+    """Pairs (2i, 2i+1) of x [T, H, dim], fp32."""
+    if not rope.dims:
+        return x
+    cs = rope.table[positions.long()].unsqueeze(1)       # [T, 1, dims]
+    c, s = cs[..., 0::2], cs[..., 1::2]
+    u, v = x[..., 0:rope.dims:2], x[..., 1:rope.dims:2]
+    turned = torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+    return torch.cat([turned, x[..., rope.dims:]], -1)
+
+
+def latent_rope_append(p, cache, run, w, norm, eps, rope, slot_ids,
+                       positions):
     H, D, R = w.uk.shape
-    T = q.shape[0]
+    E, f, T = w.rot_dim, whole(p), slot_ids.shape[0]
+    q, c, k = f[:, :H * (D + E) + R + E].split([H * (D + E), R, E], 1)
+    q = q.reshape(T, H, D + E)
+    q = torch.cat([q[..., :D], _rotate(q[..., D:], positions, rope)], -1)
+    pool, ps = cache.latent_pool[run], cache.page_size
+    pages = cache.page_table[slot_ids.long(), (positions // ps).long()]
+    row = torch.cat([_unit_rms(c, eps) * norm,
+                     _rotate(k.unsqueeze(1), positions, rope).squeeze(1)], -1)
+    pool[pages.long(), (positions % ps).long(), :R + E] = row.to(pool.dtype)
+    return q.reshape(T, -1).to(pool.dtype)
+
+
+def latent_attention(q, cache, run, w, meta, gate=None):
+    H, D, R = w.uk.shape
+    T, E = q.shape[0], w.rot_dim
     pool = cache.latent_pool[run]
     out = torch.empty(T, H, w.uv.shape[1], dtype=q.dtype, device=q.device)
     r = 0
     for slot, n, kv in zip(*meta.layout()):
         pages = cache.page_table[slot, :-(-kv // cache.page_size)].long()
-        c = pool[pages].reshape(-1, R)[:kv].float()
+        row = pool[pages].flatten(0, 1)[:kv].float()
+        c = row[:, :R]
         k = torch.einsum("tr,hdr->htd", c, w.uk.float())
+        k = torch.cat([k, row[:, R:R + E].expand(H, kv, E)], -1)
         v = torch.einsum("tr,hvr->htv", c, w.uv.float())
-        qi = q[r:r + n].float().view(n, H, D).transpose(0, 1)
+        qi = q[r:r + n].float().view(n, H, D + E).transpose(0, 1)
         s = qi @ k.transpose(1, 2) * w.scale
-        ahead = torch.arange(kv)[None] > torch.arange(kv - n, kv)[:, None]
-        s.masked_fill_(ahead, float("-inf"))
+        s.masked_fill_(~_seen(n, kv, w.window), float("-inf"))
         out[r:r + n] = (torch.softmax(s, -1) @ v).transpose(0, 1)
         r += n
-    return out.view(T, -1)
+    out = out.view(T, -1)
+    if gate is not None:
+        g = whole(gate.p)[:, gate.first:gate.first + out.shape[1]]
+        out = (out.float() * torch.sigmoid(g)).to(out.dtype)
+    return out
+
+
+def _seen(n, kv, window):
+    """Keys that the last n of kv tokens see."""
+    dist = torch.arange(kv - n, kv)[:, None] - torch.arange(kv)[None]
+    return (dist >= 0) & (dist < (window or kv))
+
+
+def rope_qkv_append(p, bias, cache, run, w, rope, slot_ids, positions):
+    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
+    T = slot_ids.shape[0]
+    f = whole(p)[:, :H * D + G * (D + V)]
+    if bias is not None:
+        f = f + bias
+    q, k, v = f.split([H * D, G * D, G * V], -1)
+    kp, vp = cache.key_pool[run], cache.value_pool[run]
+    ps = cache.page_size
+    pages = cache.page_table[slot_ids.long(), (positions // ps).long()].long()
+    offs = (positions % ps).long()
+    k = _rotate(k.reshape(T, G, D), positions, rope)
+    kp[pages, :, offs, :D] = k.to(kp.dtype)
+    vp[pages, :, offs, :V] = v.reshape(T, G, V).to(vp.dtype)
+    out = torch.zeros(T, H, kp.shape[3], dtype=kp.dtype, device=kp.device)
+    out[:, :, :D] = _rotate(q.reshape(T, H, D), positions, rope)
+    return out
+
+
+def softmax_attention(q, cache, run, w, meta):
+    T, H, G, V = q.shape[0], w.heads, w.kv_heads, w.vdim
+    kp, vp = cache.key_pool[run], cache.value_pool[run]
+    out = torch.empty(T, H, V, dtype=q.dtype, device=q.device)
+    r = 0
+    for slot, n, kv in zip(*meta.layout()):
+        pages = cache.page_table[slot, :-(-kv // cache.page_size)].long()
+        k, v = (pool[pages].transpose(1, 2).flatten(0, 1)[:kv].float()
+                .repeat_interleave(H // G, 1).transpose(0, 1)
+                for pool in (kp, vp))
+        s = q[r:r + n].float().transpose(0, 1) @ k.transpose(1, 2) * w.scale
+        s.masked_fill_(~_seen(n, kv, w.window), float("-inf"))
+        if w.sink is not None:
+            s = torch.cat([s, w.sink.view(H, 1, 1).expand(H, n, 1)], -1)
+        a = torch.softmax(s, -1)[..., :kv]
+        out[r:r + n] = (a @ v)[..., :V].transpose(0, 1)
+        r += n
+    return out.view(T, H * V)
+
+
+def lightning(p, w, state, meta):
+    H, D, V = w.heads, w.dim, w.vdim
+    oq, ok, ov, og = w.offsets
+    f = whole(p)
+    T = f.shape[0]
+    part = lambda at, n: torch.nn.functional.silu(
+        f[:, at:at + H * n]).view(T, H, n)
+    q, k, v = part(oq, D), part(ok, D), part(ov, V)
+    decay = w.powers[:, 1].view(H, 1, 1)
+    out = torch.empty(T, H, V)
+    r = 0
+    for slot, n, kv in zip(*meta.layout()):
+        S = state[slot] if kv > n else torch.zeros_like(state[slot])
+        for t in range(r, r + n):
+            S = decay * S + k[t].unsqueeze(-1) * v[t].unsqueeze(1)
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S
+        r += n
+    out = _unit_rms(out.view(T, H * V), w.eps) * w.norm
+    g = torch.sigmoid(f[:, og:og + H * V])
+    return (out * g).to(p.dtype if torch.is_tensor(p) else torch.bfloat16)
 
 
 def gla(p, w, state, meta):
@@ -197,16 +301,24 @@ def _unit_rms(x, eps):
 
 
 def rms_residual(x, y, post, pre, mult, eps, embed, tokens, embed_scale,
-                 rows):
+                 rows, shift=None, tail=False, bare=False):
     if x is None:
-        x = embed.index_select(0, tokens.long()).float() * embed_scale
+        x = 0.0 if bare else \
+            embed.index_select(0, tokens.long()).float() * embed_scale
     if y is not None:
         if hasattr(y, "share"):
             y = (y.parts.float() * y.share.unsqueeze(-1)).sum(1)
-        x = x + mult * _unit_rms(y.float(), eps) * post
+        y = whole(y)
+        x = x + mult * (y if post is None else _unit_rms(y, eps) * post)
+    if shift is not None:
+        x = x + shift
     if rows is not None:
         x = x[rows]
     h = x if pre is None else _unit_rms(x, eps) * pre
+    if tail:
+        at = tokens if rows is None else tokens[rows]
+        h = torch.cat([h, embed.index_select(0, at.long()).float()
+                       * embed_scale], -1)
     return x, h.to(embed.dtype)
 
 

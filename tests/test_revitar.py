@@ -276,7 +276,7 @@ def test_sigmoid_attention(where, size, window, form, monkeypatch):
     dev, dt = where
     if form == "large tiles":
         from ollamamq_amd.ops import hip
-        monkeypatch.setattr(hip, "SIGMOID_LARGE", 0)
+        monkeypatch.setattr(hip, "ATTN_LARGE", 0)
     H, G, D, V = size
     kv = 130 if form == "single" else 260
     g, w = attn_params(dev, H, G, D, V, window, seed=window)
