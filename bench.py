@@ -172,11 +172,14 @@ def layer_stacks(width, n_layers=4):
     the Llama layer's weights, its three feed-forward matrices against two
     wider ones.  So has "revitar", its feed-forward cut into eight experts of
     which a token uses two; "revitar work" has four times that, so that a
-    token's two experts do the Llama feed-forward's work."""
+    token's two experts do the Llama feed-forward's work.  The Kavedra layers
+    have the Llama layer's weights, the larger mixers against a narrower
+    feed-forward; "kavedra looped" runs two layers twice."""
     import dataclasses
     from ollamamq_amd.models import PRESETS
     size = "1b" if width <= 2048 else "8b"
     rin, rev = PRESETS[f"rinitar-{size}"], PRESETS[f"revitar-{size}"]
+    kav = PRESETS[f"kavedra-{size}"]
     gla = [s for s in rin.layers if s.type == "gla"][0]
     lat = [s for s in rin.layers if s.type != "gla"][0]
     llama = dataclasses.replace(
@@ -189,6 +192,14 @@ def layer_stacks(width, n_layers=4):
         return dataclasses.replace(base, name=f"{name}-{width}",
                                    width=width, vocab=32000,
                                    layers=layers)
+    # matrix rows of width `width` that a mixer has beyond Llama's 2.5
+    light, soft, lat_k = (
+        dataclasses.replace(s, ff=(llama.ffn - extra // 3) // 64 * 64)
+        for s, extra in zip(
+            (next(s for s in kav.layers if s.type == t) for t in
+             ("lightning", "attention", "latent_attention")),
+            (5 * width // 2, 0, width + 3 * 512 + 64)))
+    half = n_layers // 2
     return [("llama", llama),
             ("rinitar gla", stack(rin, "gla", [gla] * n_layers)),
             ("rinitar latent", stack(rin, "latent", [lat] * n_layers)),
@@ -196,7 +207,16 @@ def layer_stacks(width, n_layers=4):
                                     [gla, lat] * (n_layers // 2))),
             ("revitar", stack(rev, "experts", [att] * n_layers)),
             ("revitar work", stack(rev, "wide-experts", [
-                dataclasses.replace(att, ff=att.ff * 4)] * n_layers))]
+                dataclasses.replace(att, ff=att.ff * 4)] * n_layers)),
+            ("kavedra lightning", stack(kav, "lightning",
+                                        [light] * n_layers)),
+            ("kavedra attention", stack(kav, "softmax", [soft] * n_layers)),
+            ("kavedra latent", stack(kav, "rotated-latent",
+                                     [lat_k] * n_layers)),
+            ("kavedra mixed", stack(kav, "blend", [light, lat_k] * (half // 2)
+                                    + [light, soft] * (half // 2))),
+            ("kavedra looped", dataclasses.replace(
+                stack(kav, "loop", [light, soft]), loop=(0, 2, 2)))]
 
 
 def run_layers(args):
@@ -262,7 +282,7 @@ def run_layers(args):
             dt = time.monotonic() - t0
             table.append({
                 "stack": name, "width": width,
-                "layers": 4,
+                "layers": len(getattr(cfg, "runs", [0] * 4)),
                 "weights_mb": round(model.weight_bytes() / 2 ** 20),
                 "prefill_tokens_per_s": round(prefill),
                 "decode_tokens_per_s": round(users * args.steps / dt),
@@ -294,9 +314,9 @@ def main():
                          "(HTTP + scheduler + UDS workers) instead of "
                          "the engine-only kernel metric")
     ap.add_argument("--layers", action="store_true",
-                    help="prefill and decode throughput of Rinitar and "
-                         "Revitar layer stacks beside Llama stacks of equal "
-                         "size")
+                    help="prefill and decode throughput of Rinitar, Revitar "
+                         "and Kavedra layer stacks beside Llama stacks of "
+                         "equal size")
     ap.add_argument("--layer-sizes", type=str, default="2048,4096",
                     help="widths for --layers, of 2048, 4096")
     ap.add_argument("--stacks", type=str, default="",

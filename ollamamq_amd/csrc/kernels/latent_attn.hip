@@ -453,13 +453,26 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
             qf[k] = c < KW ? frag8(qr + c) : frag_zero<bf16>();
         }
     }
-    // pieces of a chunk: a row is NT*2 of them, so a wave reads whole rows
-    constexpr int NP = KT * NT * 2 / 256;
+    // pieces of a chunk, NT*2 in a row: the first MP of every row, a power of
+    // two, then the rest.  With 64 of them a wave reads one row, whose page
+    // is a scalar.
+    constexpr int MP = NT * 2 >= 64 ? 64 : NT * 2 >= 32 ? 32 : 16;
+    constexpr int XP = NT * 2 - MP, MJ = KT * MP / 256;
+    constexpr int NP = MJ + KT * XP / 256;
+    const int wave = __builtin_amdgcn_readfirstlane(wid);
+    auto row_of = [&](int j) {
+        if (j < MJ) return MP == 64 ? j * 4 + wave : (tid + j * 256) / MP;
+        return (tid + (j - MJ) * 256) / (XP ? XP : 1);
+    };
+    auto col_of = [&](int j) {
+        if (j < MJ) return tid % MP * 8;
+        return (MP + tid % (XP ? XP : 1)) * 8;
+    };
     bf16x8 piece[NP];
     const int pmask = (1 << pshift) - 1;
     int page[NP];
     auto key_of = [&](int j, int base) {
-        return min(base + (tid + j * 256) / (NT * 2), kv_len - 1);
+        return min(base + row_of(j), kv_len - 1);
     };
     auto pages = [&](int base) {
         #pragma unroll
@@ -468,19 +481,16 @@ __global__ __launch_bounds__(256, 1) void k_latent_mq(
     auto fetch = [&](int base) {
         #pragma unroll
         for (int j = 0; j < NP; j++) {
-            const int c = min((tid + j * 256) % (NT * 2) * 8, KW - 8);
+            const int c = min(col_of(j), KW - 8);
             piece[j] = frag8(pool + (((int64_t)page[j] << pshift)
                                      + (key_of(j, base) & pmask)) * KW + c);
         }
     };
     auto put = [&](int buf) {
         #pragma unroll
-        for (int j = 0; j < NP; j++) {
-            const int u = tid + j * 256;
+        for (int j = 0; j < NP; j++)
             *reinterpret_cast<bf16x8*>(
-                c_s + (buf * KT + u / (NT * 2)) * CS + u % (NT * 2) * 8)
-                = piece[j];
-        }
+                c_s + (buf * KT + row_of(j)) * CS + col_of(j)) = piece[j];
     };
     f32x4 acc[NV] = {};
     float m = NEG, l = 0.f;
@@ -799,7 +809,8 @@ extern "C" int latent_attn(
 // the lanes already hold P.
 // ---------------------------------------------------------------------------
 template <typename T, int DT, int VT, int NQ>
-__global__ __launch_bounds__(256) void k_flash(
+__global__ __launch_bounds__(256, sizeof(T) == 2 && DT <= 6 && VT <= 8
+                                      ? 2 : 1) void k_flash(
     T* __restrict__ out,               // [T, H, V]
     const T* __restrict__ q,           // [T, ..] row stride qs, head h at
                                        // h * (D + Dr)

@@ -208,15 +208,20 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int lr = lane & 15, g = lane >> 4;
     const int c0 = seqs[blockIdx.x * 2], nc = seqs[blockIdx.x * 2 + 1];
+    // a sequence's rows follow one another: every chunk but the last is full
     const int first = chunks[c0 * 2];
+    const int rows = (nc - 1) * CH + chunks[(c0 + nc - 1) * 2 + 1];
     const int64_t ld = (int64_t)H * (2 * Dp + Vp);
+    a += (first - row_base) * ld;
     float* St = state + ((int64_t)slot[first] * H + h) * D * V;
-    const float* pw = powers + h * PW;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     T* k_s = reinterpret_cast<T*>(smem);          // [CH][KS]
     T* v_s = k_s + CH * KS;                       // [CH][VS]
     T* d_s = v_s + CH * VS;                       // [NT][CH][VS] decayed v
     T* S_s = d_s + NT * CH * VS;                  // [NT][W][KS] state
+    float* pw = reinterpret_cast<float*>(S_s + NT * W * KS);    // [PW]
+    for (int i = tid; i < PW; i += 256) pw[i] = powers[h * PW + i];
+    __syncthreads();
 
     f32x4 S[NS][VC];
     const bool fresh = pos[first] == 0;
@@ -247,17 +252,16 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
     Frag<T> qf[DQ], kp[NK], vp[NV];
     float vw[NV];                       // factor of a piece of v
     // rows past the chunk's end repeat its last one and weigh nothing
-    auto load_q = [&](int ci) {
-        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
-        const T* r = a + (t0 - row_base + min(me, n - 1)) * ld
-                     + (int64_t)h * Dp + g * 8;
+    auto load_q = [&](int t0) {
+        const T* r = a + min(t0 + me, rows - 1) * ld + (int64_t)h * Dp
+                     + g * 8;
         #pragma unroll
         for (int d = 0; d < DQ; d++)
             qf[d] = d * 32 < Dp ? frag8(r + d * 32) : frag_zero<T>();
     };
-    auto load_kv = [&](int ci) {
-        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
-        const T* b = a + (int64_t)(t0 - row_base) * ld;
+    auto load_kv = [&](int t0) {
+        const int n = min(CH, rows - t0);
+        const T* b = a + t0 * ld;
         #pragma unroll
         for (int j = 0; j < NK; j++) {
             const int u = tid + j * 256;
@@ -279,12 +283,12 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
             }
         }
     };
-    load_kv(c0);
-    load_q(c0);
+    load_kv(0);
+    load_q(0);
 
-    for (int ci = c0; ci < c0 + nc; ++ci) {
-        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
-        const int nx = min(ci + 1, c0 + nc - 1);
+    for (int t0 = 0; t0 < rows; t0 += CH) {
+        const int n = min(CH, rows - t0);
+        const int nx = t0 + CH < rows ? t0 + CH : t0;
         #pragma unroll
         for (int j = 0; j < NK; j++) {
             const int u = tid + j * 256;
@@ -329,7 +333,7 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
                     stv<4>(S_s + (q * W + c * 16 + lr) * KS + d0, f[q]);
             }
         }
-        __syncthreads();
+        lds_barrier();
         load_kv(nx);
         // this wave's 16 queries: the state's part, then the chunk's own
         f32x4 acc[VC] = {}, s[4] = {};
@@ -379,7 +383,7 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
             }
         }
         if (me < n) {
-            float* dst = o + ((int64_t)(t0 + me) * H + h) * V;
+            float* dst = o + ((int64_t)(first + t0 + me) * H + h) * V;
             #pragma unroll
             for (int c = 0; c < VC; c++) {
                 const int v = v0 + c * 16 + g * 4;
@@ -420,7 +424,7 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
                         S[x][c] = mma(k, dv[q][c][hh], S[x][c]);
             }
         }
-        __syncthreads();
+        lds_barrier();
     }
     #pragma unroll
     for (int x = 0; x < NS; x++)
@@ -483,7 +487,7 @@ extern "C" int lightning_chunks(
             const int lds = ((CH + Terms<T>::N * VC * 16)                  \
                                  * (NS * 64 + pad)                         \
                              + (1 + Terms<T>::N) * CH * (VC * 16 + pad))   \
-                            * es;                                          \
+                            * es + PW * 4;                                 \
             (void)hipFuncSetAttribute(                                     \
                 (const void*)k_lightning_scan<T, NS, VC>,                  \
                 hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);   \

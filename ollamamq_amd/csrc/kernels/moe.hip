@@ -423,10 +423,6 @@ extern "C" int moe_gemm(
 // of the 16 served together no two share parity and that).  One barrier a stage, which waits for LDS
 // only: loads stay in flight across it.
 // ---------------------------------------------------------------------------
-DEV void lds_barrier() {
-    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-}
-
 template <bool GU>
 __global__ __launch_bounds__(256, 2) void k_moe_gemm_packed(
     bf16* __restrict__ out, const bf16* __restrict__ x,

@@ -128,6 +128,12 @@ DEV float wave_max(float x) {
     return x;
 }
 
+// Barrier for what goes through LDS: loads and stores to memory stay in
+// flight across it.
+DEV void lds_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+
 // sum over the block; every thread gets it.  s: one float per wave
 template <int BS> DEV float block_sum(float v, float* s) {
     v = wave_sum(v);
