@@ -145,23 +145,27 @@ extern "C" int lightning_step(
 
 // ---- chunks --------------------------------------------------------------
 
-// a [rows, H * (2 Dp + Vp)]: silu of q, k and v, heads filled up with zeros
+// a = q [H, rows, Dp], k [H, rows, Dp], v [H, rows, Vp]: their silu, filled up
+// with zeros
 template <typename T, typename P, int VEC>
 __global__ __launch_bounds__(256) void k_lightning_act(
-    T* __restrict__ a, Rows<P> p, Cols at, int row_base, int64_t total,
-    int H, int D, int V, int Dp, int Vp)
+    T* __restrict__ a, Rows<P> p, Cols at, int row_base, int rows,
+    int64_t total, int H, int D, int V, int Dp, int Vp)
 {
     const int64_t N = (int64_t)H * (2 * Dp + Vp);
     for (int64_t i = (blockIdx.x * (int64_t)256 + threadIdx.x) * VEC;
          i < total; i += (int64_t)gridDim.x * 256 * VEC) {
         const int64_t t = i / N;
         int c = (int)(i - t * N), off = at.q, wide = D, pad = Dp;
+        T* dst = a;
         if (c >= 2 * H * Dp) {
             c -= 2 * H * Dp;
             off = at.v, wide = V, pad = Vp;
+            dst += (int64_t)2 * H * rows * Dp;
         } else if (c >= H * Dp) {
             c -= H * Dp;
             off = at.k;
+            dst += (int64_t)H * rows * Dp;
         }
         const int h = c / pad, d = c % pad;
         float v[VEC] = {};
@@ -170,7 +174,7 @@ __global__ __launch_bounds__(256) void k_lightning_act(
             #pragma unroll
             for (int e = 0; e < VEC; e++) v[e] = silu_of<T>(v[e]);
         }
-        stv<VEC>(a + i, v);
+        stv<VEC>(dst + ((int64_t)h * rows + t) * pad + d, v);
     }
 }
 
@@ -196,7 +200,7 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
     const int* __restrict__ slot, const int* __restrict__ pos,
     const int* __restrict__ chunks,     // [n, 2] first row, rows
     const int* __restrict__ seqs,       // [m, 2] first chunk, chunks
-    int row_base, int H, int D, int V, int Dp, int Vp)
+    int row_base, int a_rows, int H, int D, int V, int Dp, int Vp)
 {
     constexpr int W = VC * 16, PAD = 16 / sizeof(T), NT = Terms<T>::N;
     constexpr int DM = NS * 64, KS = DM + PAD, VS = W + PAD;
@@ -211,8 +215,11 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
     // a sequence's rows follow one another: every chunk but the last is full
     const int first = chunks[c0 * 2];
     const int rows = (nc - 1) * CH + chunks[(c0 + nc - 1) * 2 + 1];
-    const int64_t ld = (int64_t)H * (2 * Dp + Vp);
-    a += (first - row_base) * ld;
+    const int64_t a0 = (int64_t)h * a_rows + first - row_base;
+    const int64_t a_qk = (int64_t)H * a_rows * Dp;
+    const T* aq = a + a0 * Dp;
+    const T* ak = aq + a_qk;
+    const T* av = a + 2 * a_qk + a0 * Vp + v0;
     float* St = state + ((int64_t)slot[first] * H + h) * D * V;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     T* k_s = reinterpret_cast<T*>(smem);          // [CH][KS]
@@ -253,21 +260,18 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
     float vw[NV];                       // factor of a piece of v
     // rows past the chunk's end repeat its last one and weigh nothing
     auto load_q = [&](int t0) {
-        const T* r = a + min(t0 + me, rows - 1) * ld + (int64_t)h * Dp
-                     + g * 8;
+        const T* r = aq + (int64_t)min(t0 + me, rows - 1) * Dp + g * 8;
         #pragma unroll
         for (int d = 0; d < DQ; d++)
             qf[d] = d * 32 < Dp ? frag8(r + d * 32) : frag_zero<T>();
     };
     auto load_kv = [&](int t0) {
         const int n = min(CH, rows - t0);
-        const T* b = a + t0 * ld;
         #pragma unroll
         for (int j = 0; j < NK; j++) {
             const int u = tid + j * 256;
             const int t = u / (DM / 8), c = u % (DM / 8) * 8;
-            kp[j] = c < Dp ? frag8(b + min(t, n - 1) * ld
-                                   + (int64_t)(H + h) * Dp + c)
+            kp[j] = c < Dp ? frag8(ak + (int64_t)(t0 + min(t, n - 1)) * Dp + c)
                            : frag_zero<T>();
         }
         #pragma unroll
@@ -277,8 +281,7 @@ __global__ __launch_bounds__(256) void k_lightning_scan(
             vp[j] = frag_zero<T>();
             vw[j] = 0.f;
             if (t < n && v0 + c < Vp) {
-                vp[j] = frag8(b + t * ld + (int64_t)2 * H * Dp
-                              + (int64_t)h * Vp + v0 + c);
+                vp[j] = frag8(av + (int64_t)(t0 + t) * Vp + c);
                 vw[j] = pw[n - 1 - t];
             }
         }
@@ -467,7 +470,7 @@ extern "C" int lightning_chunks(
     #define LA_GO(T, P, VE)                                                \
         k_lightning_act<T, P, VE><<<ga, 256, 0, stream>>>(                 \
             (T*)scr, Rows<P>{(const P*)p, n_part, part_stride, ld},        \
-            Cols{oq, ok, ov}, row_base, total, H, D, V, Dp, Vp)
+            Cols{oq, ok, ov}, row_base, rows, total, H, D, V, Dp, Vp)
     #define LA_V(T, P)                                                     \
         do { if (v8) LA_GO(T, P, 8); else LA_GO(T, P, 1); } while (0)
     if (f32) LA_V(float, float);
@@ -479,8 +482,9 @@ extern "C" int lightning_chunks(
     auto blocks = [&](int vc) {
         return (int64_t)n_seqs * H * ((V + vc * 16 - 1) / (vc * 16));
     };
-    const int vc = blocks(4) >= 512 && Dp <= 128 && !f32 ? 4
-                   : blocks(2) >= 256 ? 2 : 1;
+    const int vc = f32 ? (blocks(2) >= 512 ? 2 : 1)
+                   : Dp <= 128 && blocks(4) >= 2048 ? 4
+                   : blocks(2) >= 512 ? 2 : 1;
     #define SC(T, NS, VC)                                                  \
         do {                                                               \
             constexpr int es = sizeof(T), pad = 16 / es;                   \
@@ -496,8 +500,8 @@ extern "C" int lightning_chunks(
                    lds, stream>>>(                                         \
                     (float*)o, (const T*)scr, (const float*)powers,        \
                     (float*)state, (const int*)slot, (const int*)pos,      \
-                    (const int*)chunks, (const int*)seqs, row_base, H, D,  \
-                    V, Dp, Vp);                                            \
+                    (const int*)chunks, (const int*)seqs, row_base, rows,  \
+                    H, D, V, Dp, Vp);                                      \
         } while (0)
     #define SC_NS(T, VC)                                                   \
         do {                                                               \

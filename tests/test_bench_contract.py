@@ -78,14 +78,16 @@ def test_bench_stack_mode():
 
 
 def test_bench_layer_stacks():
-    """--layers is an option of its own: one JSON line, both designs."""
+    """--layers is an option of its own: one JSON line, all designs."""
     r = subprocess.run(
         [sys.executable, BENCH, "--layers", "--steps", "2", "--warmup", "1"],
         cwd=REPO, capture_output=True, text=True, timeout=300)
     assert r.returncode == 0, r.stderr[-2000:]
     out = last_json_line(r.stdout)
     stacks = {row["stack"] for row in out["results"]}
-    assert {"llama", "rinitar gla", "rinitar latent"} <= stacks
+    assert {"llama", "rinitar gla", "rinitar latent", "revitar",
+            "kavedra lightning", "kavedra attention", "kavedra latent",
+            "kavedra mixed", "kavedra looped"} <= stacks
     for row in out["results"]:
         assert row["prefill_tokens_per_s"] > 0
         assert row["decode_tokens_per_s"] > 0
