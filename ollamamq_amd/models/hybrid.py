@@ -21,8 +21,9 @@ from .checkpoint import CheckpointSource, RandomSource
 
 @dataclass(frozen=True)
 class RopeSpec:
-    """Rotary positions over the first `dims` dimensions of a head, pair
-    (2i, 2i+1) turning by base^(-2i/dims) per token.  scaling = (factor,
+    """Rotary positions over the first `dims` dimensions of a head, pair i
+    turning by base^(-2i/dims) per token: dimensions (2i, 2i+1), or
+    (i, i + dims/2) with `halves`.  scaling = (factor,
     original, fast, slow) is YaRN's: pairs that turn more than `fast` times
     over the original context keep their frequency, those below `slow` have
     it divided by `factor`, a linear ramp over the pairs between, and the
@@ -30,16 +31,18 @@ class RopeSpec:
     dims: int
     base: float
     scaling: Optional[Tuple[float, float, float, float]] = None
+    halves: bool = False
 
     def __post_init__(self):
         if self.dims < 0 or self.dims % 2:
             raise ValueError(f"{self.dims} rotated dimensions")
 
     @classmethod
-    def from_json(cls, d: dict) -> "RopeSpec":
+    def from_json(cls, d: dict, halves: bool = False) -> "RopeSpec":
         sc = d.get("scaling")
         return cls(int(d["dims"]), float(d["base"]), sc and tuple(
-            float(sc[k]) for k in ("factor", "original", "fast", "slow")))
+            float(sc[k]) for k in ("factor", "original", "fast", "slow")),
+            halves)
 
     def frequencies(self) -> torch.Tensor:
         """Angle per token of every pair, float64."""
@@ -80,7 +83,7 @@ class RopeTables:
             a = torch.outer(p, spec.frequencies().to(self.device))
             cs = torch.stack([a.cos(), a.sin()], -1) * spec.magnitude
             self._made[spec] = ops.Rope(cs.flatten(1).float().contiguous(),
-                                        spec.dims)
+                                        spec.dims, spec.halves)
         return self._made[spec]
 
 

@@ -246,15 +246,12 @@ class KavedraLayer(HybridLayer):
         self.norm1 = gain(pre + "norm1")
         if s.type == "lightning":
             cols = [mat("q", qk), mat("k", qk), mat("v", v), mat("g", v)]
-            steps = torch.arange(ops.LIGHTNING_CHUNK + 1,
-                                 dtype=torch.float64)
-            decay = torch.tensor(s.decay, dtype=torch.float64)
             norm = vec(mix + "norm", v, mean=1.0)
             self.mix = ops.LightningWeights(
                 heads=s.heads, dim=s.dim, vdim=s.vdim,
                 offsets=(0, qk, 2 * qk, 2 * qk + v),
-                powers=(decay[:, None] ** steps).float().to(norm.device)
-                .contiguous(), norm=norm, eps=eps)
+                powers=ops.decay_powers(s.decay, norm.device), norm=norm,
+                eps=eps)
         elif s.type == "attention":
             nk, nv = s.kv_heads * s.dim, s.kv_heads * s.vdim
             parts = (("q", qk), ("k", nk), ("v", nv))

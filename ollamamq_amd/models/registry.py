@@ -12,6 +12,7 @@ from typing import Dict, NamedTuple, Optional
 from .checkpoint import read_config
 from .kavedra import KAVEDRA_PRESETS, KavedraConfig, KavedraModel
 from .llama import PRESETS, LlamaConfig, LlamaModel
+from .pemidra import PEMIDRA_PRESETS, PemidraConfig, PemidraModel
 from .revitar import REVITAR_PRESETS, RevitarConfig, RevitarModel
 from .rinitar import RINITAR_PRESETS, RinitarConfig, RinitarModel
 
@@ -26,10 +27,12 @@ ARCHITECTURES: Dict[str, Architecture] = {
     "Rinitar": Architecture(RinitarConfig, RinitarModel),
     "Revitar": Architecture(RevitarConfig, RevitarModel),
     "Kavedra": Architecture(KavedraConfig, KavedraModel),
+    "Pemidra": Architecture(PemidraConfig, PemidraModel),
 }
 PRESETS.update(RINITAR_PRESETS)
 PRESETS.update(REVITAR_PRESETS)
 PRESETS.update(KAVEDRA_PRESETS)
+PRESETS.update(PEMIDRA_PRESETS)
 
 
 def config_from_folder(path: str, name: Optional[str] = None):

@@ -125,9 +125,25 @@ class Columns(NamedTuple):
 
 class Rope(NamedTuple):
     """Rotary positions: table [positions, dims] fp32 holds (cos, sin) of
-    every pair (2i, 2i+1) of a head's first `dims` dimensions."""
+    every pair of a head's first `dims` dimensions: (2i, 2i+1), or
+    (i, i + dims/2) with `halves`."""
     table: torch.Tensor
     dims: int
+    halves: bool = False
+
+
+class LayerNorm(NamedTuple):
+    """(x - mean) / sqrt(variance + eps) * w + b (w, b fp32)."""
+    w: torch.Tensor
+    b: torch.Tensor
+
+
+class Branches(NamedTuple):
+    """Results of sublayers side by side: share * sum N(y) * w over the
+    (y, w) pairs, N the division by a row's root mean square.  The consumer
+    norms them and adds them up."""
+    pairs: tuple
+    share: float
 
 
 class LatentWeights(NamedTuple):
@@ -147,7 +163,8 @@ class LatentWeights(NamedTuple):
 class SoftmaxAttn(NamedTuple):
     """Softmax attention over paged keys and values; `sink` (fp32 per query
     head, or None) is one more logit of the denominator.  A query sees
-    `window` tokens, itself included (0: all before it)."""
+    `window` tokens, itself included (0: all before it), or, with `chunk`,
+    the tokens of its own chunk of that many positions."""
     heads: int
     kv_heads: int
     dim: int
@@ -155,20 +172,81 @@ class SoftmaxAttn(NamedTuple):
     scale: float
     sink: Optional[torch.Tensor] = None
     window: int = 0
+    chunk: int = 0
+
+    def reach(self, kv: int) -> int:
+        """Most keys that a query of a context of kv tokens sees."""
+        return min(kv, self.window or self.chunk or kv)
+
+
+class HeadNorms(NamedTuple):
+    """What happens to each head of a projection before attention: RMS norm
+    with weights of the head's width (q, k, fp32), of the values without a
+    weight, and a factor per query head (fp32, or None)."""
+    q: torch.Tensor
+    k: torch.Tensor
+    values: bool
+    gain: Optional[torch.Tensor]
+    eps: float
 
 
 LIGHTNING_CHUNK = 64
 
 
+def decay_powers(decay, device) -> torch.Tensor:
+    """fp32 [heads, LIGHTNING_CHUNK + 1]: powers of every head's decay."""
+    steps = torch.arange(LIGHTNING_CHUNK + 1, dtype=torch.float64)
+    d = torch.tensor(decay, dtype=torch.float64)
+    return (d[:, None] ** steps).float().to(device).contiguous()
+
+
 class LightningWeights(NamedTuple):
-    """Columns of the fused projection, and what the recurrence and the norm
-    over all heads read."""
+    """Columns of the fused projection, and what the recurrence, the norm and
+    the output gate read."""
     heads: int
     dim: int
     vdim: int
     offsets: tuple                # columns of q, k, v, gate
-    powers: torch.Tensor          # fp32 [heads, LIGHTNING_CHUNK + 1]
-    norm: torch.Tensor            # fp32 [heads * vdim]
+    powers: torch.Tensor          # decay_powers
+    norm: Optional[torch.Tensor]  # fp32 [heads * vdim], None: no weight
+    eps: float
+    act: bool = True              # silu of q, k and v
+    key_scale: float = 1.0
+    per_head: bool = False        # norm of every head, not of all together
+    gate: str = "sigmoid"         # or "silu"
+
+
+UNIT_EPS = 1e-6       # inside the root of a unit vector
+
+
+class GatedDeltaWeights(NamedTuple):
+    """Gated delta rule with a decay per key channel.  Columns of the fused
+    projection (q, k and v follow one another), the short convolution over
+    them, the low-rank projections of decays and output gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    offsets: tuple                # columns of q|k|v, beta, decay, gate
+    conv: torch.Tensor            # fp32 [taps, channels], the current last
+    a2: torch.Tensor              # [heads * dim, rank]
+    rate: torch.Tensor            # fp32 [heads], exp of the stored logarithm
+    dt_bias: torch.Tensor         # fp32 [heads * dim]
+    g2: torch.Tensor              # [heads * vdim, rank]
+    norm: torch.Tensor            # fp32 [vdim]
+    eps: float
+
+
+class GeneralDeltaWeights(NamedTuple):
+    """Generalized delta rule: decay and removal rate per key channel.
+    Columns of the fused projection and the decays' low-rank projection."""
+    heads: int
+    dim: int
+    offsets: tuple                # columns of r, k, v, removal, gate, decay
+    w2: torch.Tensor              # [heads * dim, rank]
+    w0: torch.Tensor              # fp32 [heads * dim]
+    a_bias: torch.Tensor          # fp32 [heads * dim]
+    norm: torch.Tensor            # fp32 [heads * dim]
     eps: float
 
 
@@ -402,24 +480,40 @@ def rope_qkv_append(p, bias, cache, run, w: SoftmaxAttn, rope: Rope,
                                positions)
 
 
+def qkv_norm_rope_append(p, norms: HeadNorms, cache, run, w: SoftmaxAttn,
+                         rope: Rope, slot_ids, positions):
+    """Split the projection p (columns q | k | v; a tensor or Partials), norm
+    every head, rotate queries and keys, append keys and values to the run's
+    paged pools.  -> queries [T, H, D'], rows filled up with zeros as the
+    pool's are."""
+    t = p.parts if isinstance(p, Partials) else p
+    if _use_hip(t):
+        from . import hip
+        return hip.qkv_norm_rope_append(p, norms, cache, run, w, rope,
+                                        slot_ids, positions)
+    return ref.qkv_norm_rope_append(p, norms, cache, run, w, rope, slot_ids,
+                                    positions)
+
+
 def softmax_attention(q, cache, run, w: SoftmaxAttn, slot_ids, positions,
-                      meta: AttnMeta, frag=False):
+                      meta: AttnMeta, frag=False,
+                      gate: Optional[Columns] = None):
     """Causal softmax attention over the run's paged keys and values; q as
-    rope_qkv_append returns it.  -> [T, H*V]."""
+    rope_qkv_append returns it.  -> [T, H*V], a head's result times the
+    sigmoid of its gate column."""
     if _use_hip(q):
         from . import hip
         return hip.softmax_attention(q, cache, run, w, slot_ids, positions,
-                                     meta, frag)
-    return ref.softmax_attention(q, cache, run, w, meta)
+                                     meta, frag, gate)
+    return ref.softmax_attention(q, cache, run, w, meta, gate)
 
 
 def lightning(p, w: LightningWeights, state, slot_ids, positions,
               meta: AttnMeta, frag=False):
-    """Lightning attention over the fused projection p [T, ...] (a tensor or
-    Partials): silu of q, k and v, a recurrence with one decay per head;
-    state [slots, H, D, V] fp32 is read and advanced.  Norm over all heads
-    and output gate included.  -> [T, H*V]."""
-    if _use_hip(w.norm):
+    """Linear attention with one decay per head over the fused projection
+    p [T, ...] (a tensor or Partials); state [slots, H, D, V] fp32 is read
+    and advanced.  Norm and output gate included.  -> [T, H*V]."""
+    if _use_hip(w.powers):
         from . import hip
         return hip.lightning(p, w, state, slot_ids, positions, meta, frag)
     return ref.lightning(p, w, state, meta)
@@ -434,6 +528,52 @@ def gla(p, w: GlaWeights, state, slot_ids, positions, meta: AttnMeta,
         from . import hip
         return hip.gla(p, w, state, slot_ids, positions, meta, frag)
     return ref.gla(p, w, state, meta)
+
+
+def gated_delta(p, w: GatedDeltaWeights, state, conv_state, slot_ids,
+                positions, meta: AttnMeta, frag=False):
+    """Gated delta rule over the fused projection p [T, ...] (a tensor or
+    Partials):
+        S <- diag(g) S,  S <- S + k (beta (v - S^T k))^T,  o = S^T q.
+    state [slots, H, D, V] and conv_state [slots, taps - 1, channels], both
+    fp32, are read and advanced.  Head norm and output gate included.
+    -> [T, H*V]."""
+    if _use_hip(w.norm):
+        from . import hip
+        return hip.gated_delta(p, w, state, conv_state, slot_ids, positions,
+                               meta, frag)
+    return ref.gated_delta(p, w, state, conv_state, meta)
+
+
+def general_delta(p, w: GeneralDeltaWeights, state, slot_ids, positions,
+                  meta: AttnMeta, frag=False):
+    """Generalized delta rule over the fused projection p [T, ...] (a tensor
+    or Partials), u the unit key:
+        S <- diag(w) S - (a * u) (S^T u)^T + k v^T,  o = S^T r.
+    state [slots, H, D, D] fp32 is read and advanced.  Head norm and output
+    gate included.  -> [T, H*D]."""
+    if _use_hip(w.norm):
+        from . import hip
+        return hip.general_delta(p, w, state, slot_ids, positions, meta,
+                                 frag)
+    return ref.general_delta(p, w, state, meta)
+
+
+def ln_residual(x, y, norm: Optional[LayerNorm], mult, eps, scale=None,
+                embed=None, tokens=None, rows=None, need_x=True, frag=False,
+                then: Optional[LayerNorm] = None):
+    """One pass between two matrix products, the norm after the sum:
+    x' = norm(mult * x + scale * y), h = then(x'), or x' itself.  x is fp32
+    [T, W], or None for the embedding rows of `tokens`; y a tensor, Partials
+    or Branches of them, or None, and then x' = x; scale fp32 [W] or None;
+    `rows` selects the rows to compute; frag returns h as FragRows.
+    Returns (x', h)."""
+    if _use_hip(embed):
+        from . import hip
+        return hip.ln_residual(x, y, norm, mult, eps, scale, embed, tokens,
+                               rows, need_x, frag, then)
+    return ref.ln_residual(x, y, norm, mult, eps, scale, embed, tokens, rows,
+                           then)
 
 
 def rms_residual(x, y, post, pre, mult, eps, embed=None, tokens=None,
@@ -513,15 +653,16 @@ def moe_experts(h, w: MoeWeights, chosen, share, packs=None) -> Weighted:
     return ref.moe_experts(h, w, chosen, share)
 
 
-def swiglu(gate_up):
+def swiglu(gate_up, act="silu"):
+    """act(gate) * up with act "silu" or "gelu_tanh"."""
     if _use_hip(gate_up):
         from . import hip
-        return hip.swiglu(gate_up)
-    return ref.swiglu(gate_up)
+        return hip.swiglu(gate_up, act)
+    return ref.swiglu(gate_up, act)
 
 
-def gateup_swiglu(x, weight, packed_gu=None):
-    """act = swiglu(x @ Wgu^T).  On the decode path (M<=32) with a
+def gateup_swiglu(x, weight, packed_gu=None, act="silu"):
+    """act = swiglu(x @ Wgu^T), or with another activation of the gate.  On the decode path (M<=32) with a
     GU-packed copy this is ONE fused weight-streaming kernel; otherwise
     the library GEMM + the swiglu kernel.  (An MT2 variant for 33..64
     exists but measured BELOW the library at 64 users — its direct
@@ -529,13 +670,13 @@ def gateup_swiglu(x, weight, packed_gu=None):
     through the fused kernel at any batch and stay FragRows."""
     if isinstance(x, FragRows):
         from . import hip
-        return hip.linear_gu_frag(x, packed_gu, weight.shape[0])
+        return hip.linear_gu_frag(x, packed_gu, weight.shape[0], act)
     if packed_gu is not None and x.shape[0] <= 32 and _use_hip(x):
         from . import hip
         if hip.USE_WSTREAM and x.dtype == torch.bfloat16 \
                 and x.stride(1) == 1:
-            return hip.linear_gu(x, packed_gu, weight.shape[0])
-    return swiglu(linear(x, weight))
+            return hip.linear_gu(x, packed_gu, weight.shape[0], glu=act)
+    return swiglu(linear(x, weight), act)
 
 
 def pack_weight_gu(w):

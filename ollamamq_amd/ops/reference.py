@@ -7,6 +7,8 @@ reference's whole test strategy runs on loopback without real backends).
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 
@@ -103,12 +105,15 @@ def attention(q, cache, layer, meta):
     return out
 
 
-def swiglu(gate_up):
-    """[T, 2F] fused gate/up -> silu(gate) * up, fp32 math."""
+def swiglu(gate_up, act="silu"):
+    """[T, 2F] fused gate/up -> act(gate) * up, fp32 math."""
     f = gate_up.shape[-1] // 2
     g = gate_up[..., :f].float()
     u = gate_up[..., f:].float()
-    return (torch.nn.functional.silu(g) * u).to(gate_up.dtype)
+    g = {"silu": torch.nn.functional.silu,
+         "gelu_tanh": lambda t: torch.nn.functional.gelu(
+             t, approximate="tanh")}[act](g)
+    return (g * u).to(gate_up.dtype)
 
 
 def dyt_residual(x, y, post, pre, shift, embed, tokens, rows):
@@ -155,13 +160,18 @@ def whole(p):
 
 
 def _rotate(x, positions, rope):
-    """Pairs (2i, 2i+1) of x [T, H, dim], fp32."""
+    """The pairs of x [T, H, dim], fp32."""
     if not rope.dims:
         return x
     cs = rope.table[positions.long()].unsqueeze(1)       # [T, 1, dims]
     c, s = cs[..., 0::2], cs[..., 1::2]
-    u, v = x[..., 0:rope.dims:2], x[..., 1:rope.dims:2]
-    turned = torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+    if rope.halves:
+        u, v = x[..., :rope.dims].chunk(2, -1)
+    else:
+        u, v = x[..., 0:rope.dims:2], x[..., 1:rope.dims:2]
+    turned = [u * c - v * s, v * c + u * s]
+    turned = torch.cat(turned, -1) if rope.halves \
+        else torch.stack(turned, -1).flatten(-2)
     return torch.cat([turned, x[..., rope.dims:]], -1)
 
 
@@ -205,32 +215,55 @@ def latent_attention(q, cache, run, w, meta, gate=None):
     return out
 
 
-def _seen(n, kv, window):
+def _seen(n, kv, window, chunk=0):
     """Keys that the last n of kv tokens see."""
-    dist = torch.arange(kv - n, kv)[:, None] - torch.arange(kv)[None]
-    return (dist >= 0) & (dist < (window or kv))
+    i, j = torch.arange(kv - n, kv)[:, None], torch.arange(kv)[None]
+    seen = (j <= i) & (i - j < (window or kv))
+    return seen & (i // chunk == j // chunk) if chunk else seen
 
 
 def rope_qkv_append(p, bias, cache, run, w, rope, slot_ids, positions):
-    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
-    T = slot_ids.shape[0]
-    f = whole(p)[:, :H * D + G * (D + V)]
+    f = whole(p)[:, :w.heads * w.dim + w.kv_heads * (w.dim + w.vdim)]
     if bias is not None:
         f = f + bias
-    q, k, v = f.split([H * D, G * D, G * V], -1)
+    return _append(*_split_heads(f, w), cache, run, rope, slot_ids,
+                   positions)
+
+
+def _split_heads(f, w):
+    """Columns q | k | v as [T, heads, width] each."""
+    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
+    T = f.shape[0]
+    q, k, v = f[:, :H * D + G * (D + V)].split([H * D, G * D, G * V], -1)
+    return q.reshape(T, H, D), k.reshape(T, G, D), v.reshape(T, G, V)
+
+
+def _append(q, k, v, cache, run, rope, slot_ids, positions):
+    """Rotate queries and keys, append keys and values."""
+    D, V = k.shape[2], v.shape[2]
     kp, vp = cache.key_pool[run], cache.value_pool[run]
     ps = cache.page_size
     pages = cache.page_table[slot_ids.long(), (positions // ps).long()].long()
     offs = (positions % ps).long()
-    k = _rotate(k.reshape(T, G, D), positions, rope)
-    kp[pages, :, offs, :D] = k.to(kp.dtype)
-    vp[pages, :, offs, :V] = v.reshape(T, G, V).to(vp.dtype)
-    out = torch.zeros(T, H, kp.shape[3], dtype=kp.dtype, device=kp.device)
-    out[:, :, :D] = _rotate(q.reshape(T, H, D), positions, rope)
+    kp[pages, :, offs, :D] = _rotate(k, positions, rope).to(kp.dtype)
+    vp[pages, :, offs, :V] = v.to(vp.dtype)
+    out = torch.zeros(*q.shape[:2], kp.shape[3], dtype=kp.dtype,
+                      device=kp.device)
+    out[:, :, :D] = _rotate(q, positions, rope)
     return out
 
 
-def softmax_attention(q, cache, run, w, meta):
+def qkv_norm_rope_append(p, norms, cache, run, w, rope, slot_ids, positions):
+    q, k, v = _split_heads(whole(p), w)
+    q, k = _unit_rms(q, norms.eps) * norms.q, _unit_rms(k, norms.eps) * norms.k
+    if norms.gain is not None:
+        q = q * norms.gain[:, None]
+    if norms.values:
+        v = _unit_rms(v, norms.eps)
+    return _append(q, k, v, cache, run, rope, slot_ids, positions)
+
+
+def softmax_attention(q, cache, run, w, meta, gate=None):
     T, H, G, V = q.shape[0], w.heads, w.kv_heads, w.vdim
     kp, vp = cache.key_pool[run], cache.value_pool[run]
     out = torch.empty(T, H, V, dtype=q.dtype, device=q.device)
@@ -241,13 +274,33 @@ def softmax_attention(q, cache, run, w, meta):
                 .repeat_interleave(H // G, 1).transpose(0, 1)
                 for pool in (kp, vp))
         s = q[r:r + n].float().transpose(0, 1) @ k.transpose(1, 2) * w.scale
-        s.masked_fill_(~_seen(n, kv, w.window), float("-inf"))
+        s.masked_fill_(~_seen(n, kv, w.window, w.chunk), float("-inf"))
         if w.sink is not None:
             s = torch.cat([s, w.sink.view(H, 1, 1).expand(H, n, 1)], -1)
         a = torch.softmax(s, -1)[..., :kv]
         out[r:r + n] = (a @ v)[..., :V].transpose(0, 1)
         r += n
+    if gate is not None:
+        g = whole(gate.p)[:, gate.first:gate.first + H]
+        out = (out.float() * torch.sigmoid(g)[..., None]).to(out.dtype)
     return out.view(T, H * V)
+
+
+def _gated_heads(o, norm, gate, eps, dtype, per_head=True, act="sigmoid"):
+    """Norm of o [T, H, V], of every head or of all together, and the output
+    gate [T, H*V]."""
+    T, H, V = o.shape
+    o = _unit_rms(o if per_head else o.reshape(T, 1, H * V), eps) \
+        .reshape(T, H * V)
+    if norm is not None:
+        o = o * norm.repeat(H * V // norm.numel())
+    g = torch.sigmoid(gate) if act == "sigmoid" \
+        else torch.nn.functional.silu(gate)
+    return (o * g).to(dtype)
+
+
+def _type_of(p):
+    return p.dtype if torch.is_tensor(p) else torch.bfloat16
 
 
 def lightning(p, w, state, meta):
@@ -255,9 +308,9 @@ def lightning(p, w, state, meta):
     oq, ok, ov, og = w.offsets
     f = whole(p)
     T = f.shape[0]
-    part = lambda at, n: torch.nn.functional.silu(
-        f[:, at:at + H * n]).view(T, H, n)
-    q, k, v = part(oq, D), part(ok, D), part(ov, V)
+    act = torch.nn.functional.silu if w.act else lambda t: t
+    part = lambda at, n: act(f[:, at:at + H * n]).view(T, H, n)
+    q, k, v = part(oq, D), part(ok, D) * w.key_scale, part(ov, V)
     decay = w.powers[:, 1].view(H, 1, 1)
     out = torch.empty(T, H, V)
     r = 0
@@ -268,9 +321,100 @@ def lightning(p, w, state, meta):
             out[t] = torch.einsum("hdv,hd->hv", S, q[t])
         state[slot] = S
         r += n
-    out = _unit_rms(out.view(T, H * V), w.eps) * w.norm
-    g = torch.sigmoid(f[:, og:og + H * V])
-    return (out * g).to(p.dtype if torch.is_tensor(p) else torch.bfloat16)
+    return _gated_heads(out, w.norm, f[:, og:og + H * V], w.eps, _type_of(p),
+                        w.per_head, w.gate)
+
+
+def _delta(q, k, v, z, e, g, state, meta):
+    """S <- diag(g) S - e (z^T S) + k v^T with the old state on the right,
+    o = S^T q; everything [T, H, D] but v."""
+    out = torch.empty(v.shape)
+    r = 0
+    for slot, n, kv in zip(*meta.layout()):
+        S = state[slot] if kv > n else torch.zeros_like(state[slot])
+        for t in range(r, r + n):
+            read = torch.einsum("hdv,hd->hv", S, z[t])
+            S = g[t].unsqueeze(-1) * S - e[t].unsqueeze(-1) \
+                * read.unsqueeze(1) + k[t].unsqueeze(-1) * v[t].unsqueeze(1)
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S
+        r += n
+    return out
+
+
+def _unit(x):
+    from .interface import UNIT_EPS
+    return x * torch.rsqrt(x.pow(2).sum(-1, True) + UNIT_EPS)
+
+
+def _short_conv(x, w, state, meta):
+    """x [T, C], w [taps, C]; state [slots, taps - 1, C] holds a sequence's
+    last inputs."""
+    taps = w.shape[0]
+    out = torch.empty_like(x)
+    r = 0
+    for slot, n, kv in zip(*meta.layout()):
+        before = state[slot] if kv > n else torch.zeros_like(state[slot])
+        row = torch.cat([before, x[r:r + n]])
+        out[r:r + n] = sum(row[j:j + n] * w[j] for j in range(taps))
+        state[slot] = row[n:]
+        r += n
+    return out
+
+
+def gated_delta(p, w, state, conv_state, meta):
+    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
+    o_in, ob, oa, og = w.offsets
+    f = whole(p)
+    T, C = f.shape[0], w.conv.shape[1]
+    y = torch.nn.functional.silu(_short_conv(f[:, o_in:o_in + C], w.conv,
+                                             conv_state, meta))
+    q, k, v = y.split([G * D, G * D, H * V], -1)
+    heads = lambda t: _unit(t.reshape(T, G, D)).repeat_interleave(H // G, 1)
+    q, k, v = heads(q) * D ** -0.5, heads(k), v.reshape(T, H, V)
+    low = lambda at, m: f[:, at:at + m.shape[1]] @ m.float().T
+    z = torch.nn.functional.softplus(low(oa, w.a2) + w.dt_bias)
+    g = torch.exp(-w.rate[:, None] * z.view(T, H, D))
+    bk = torch.sigmoid(f[:, ob:ob + H]).unsqueeze(-1) * k
+    o = _delta(q, bk, v, g * k, bk, g, state, meta)
+    return _gated_heads(o, w.norm, low(og, w.g2), w.eps, _type_of(p))
+
+
+def general_delta(p, w, state, meta):
+    H, D = w.heads, w.dim
+    f = whole(p)
+    T = f.shape[0]
+    r, k, v, a, gate = (f[:, at:at + H * D] for at in w.offsets[:5])
+    heads = lambda t: t.reshape(T, H, D)
+    u = _unit(heads(k))
+    at = w.offsets[5]
+    z = torch.tanh(f[:, at:at + w.w2.shape[1]]) @ w.w2.float().T + w.w0
+    g = torch.exp(-math.exp(-0.5) * torch.sigmoid(z))
+    a = torch.sigmoid(a + w.a_bias)
+    o = _delta(heads(r), heads(k), heads(v), u, heads(a) * u, heads(g), state,
+               meta)
+    return _gated_heads(o, w.norm, gate, w.eps, _type_of(p))
+
+
+def _layer_norm(x, norm, eps):
+    return torch.nn.functional.layer_norm(x, x.shape[-1:], norm.w, norm.b,
+                                          eps)
+
+
+def ln_residual(x, y, norm, mult, eps, scale, embed, tokens, rows, then):
+    if x is None:
+        x = embed.index_select(0, tokens.long()).float()
+    if y is not None:
+        if hasattr(y, "pairs"):
+            y = y.share * sum(_unit_rms(whole(b), eps) * w
+                              for b, w in y.pairs)
+        y = whole(y)
+        x = _layer_norm(mult * x + (y if scale is None else scale * y), norm,
+                        eps)
+    if rows is not None:
+        x = x[rows]
+    h = x if then is None else _layer_norm(x, then, eps)
+    return x, h.to(embed.dtype)
 
 
 def gla(p, w, state, meta):
