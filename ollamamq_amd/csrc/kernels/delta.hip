@@ -1,0 +1,1322 @@
+// gfx950 delta rules: per head a [D, V] fp32 state that forgets per key
+// channel, removes along one vector what another reads, and writes,
+//
+//   S_t = diag(g_t) S_(t-1) - e_t (z_t^T S_(t-1)) + k_t v_t^T,
+//   o_t = S_t^T q_t.
+//
+// * the gated rule (GEN false), u the unit key and b the step size:
+//     S <- diag(g) S,  S <- S + u (b (v - S^T u))^T
+//   is z = g u and e = k = b u; queries, keys and values come through a short
+//   causal convolution and silu, queries and keys are unit vectors;
+// * the generalized rule (GEN true): z = u, e = a u and k the key itself.
+//
+// k_gated_rows / k_general_rows make what the recurrence reads and the
+// projection does not hold: convolved rows, scales that make unit vectors,
+// log decays and step sizes from low-rank projections, the gated rule's
+// output gate.  Then
+//
+// * k_delta_step: a token at a time (decode, portions of a few tokens), the
+//   state in registers;
+// * k_delta_prep / k_delta_scan: chunks of 64 tokens.  With c_i the sum of
+//   log decays up to token i of a chunk and w_i = z_i^T S_(i-1),
+//     w + A_ze w = Z S_0 + A_zk V,         Z_i = z_i e^{c_i} / g_i,
+//     o = Q S_0 + A_qk V - A_qe w,         Q_i = q_i e^{c_i},
+//     S' = diag(e^{c_n}) S_0 + K^T V - E^T w,   K_j = k_j e^{c_n - c_j},
+//   A_xy[i][j] = sum_d x_id y_jd e^{c_i - c_j} for j < i (j <= i for q, and
+//   for z with c_(i-1)).  In the gated rule e = k, so only u = V - w enters.
+//   prep makes the factors, the A and (I + A_ze)^-1 for all chunks at once;
+//   scan walks a sequence's chunks with the state in registers, a block per
+//   head and strip of value columns.  No exponent that meets data is
+//   positive: sums are kept per 16-token part, a pair of parts is joined by
+//   the decay between them.
+//
+// The results o [T, H, V] are fp32; the norm and gate that follow are
+// k_head_gate.  A sequence starts where its position is 0: state and earlier
+// inputs are then taken as zero and whatever the slot held is ignored.
+#include "tile_mma.h"
+
+template <typename T> DEV float silu_of(float x) {
+    return x * sigmoid_of<T>(x);
+}
+template <typename T> DEV float softplus_of(float x) {
+    return fmaxf(x, 0.f) + log1pf(exp_of<T>(-fabsf(x)));
+}
+#define UNIT_EPS 1e-6f                // inside the root of a unit vector
+#define LOG_ZERO (-104.f)             // e to this is zero in fp32
+#define HALF_DECAY 0.6065306597126334f   // e^{-1/2}
+
+// an fp32 value as matrix operand: two bf16 terms, or itself
+template <typename T> struct Terms;
+template <> struct Terms<bf16> {
+    static constexpr int N = 2;
+    static DEV void split(float x, bf16* t) {
+        t[0] = __float2bfloat16(x);
+        t[1] = __float2bfloat16(x - __bfloat162float(t[0]));
+    }
+};
+template <> struct Terms<float> {
+    static constexpr int N = 1;
+    static DEV void split(float x, float* t) { t[0] = x; }
+};
+
+// ---------------------------------------------------------------------------
+// z = W u for 16 tokens and 64 rows of W [N, rank], u the projection's columns
+// first.. of the lane's token t: z[j][i] is row n0 + 16 j + 4 g + i.
+// ---------------------------------------------------------------------------
+template <typename T, typename P, bool TANH>
+DEV void low_rank(const Rows<P>& p, int first, int rank,
+                  const T* __restrict__ w, int N, int n0, int64_t t,
+                  f32x4* z) {
+    constexpr int NT = Terms<T>::N;
+    const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
+    const bool v8 = p.ld % 8 == 0 && p.part_stride % 8 == 0 && first % 8 == 0
+                    && rank % 8 == 0;
+    for (int r0 = 0; r0 < rank; r0 += 32) {
+        const int k = r0 + g * 8;
+        float u[8] = {};
+        if (v8) {
+            if (k < rank) ldrow<8>(p, t, first + k, u);
+        } else
+            for (int e = 0; e < 8; e++)
+                if (k + e < rank) ldrow<1>(p, t, first + k + e, u + e);
+        Frag<T> uf[NT];
+        #pragma unroll
+        for (int e = 0; e < 8; e++) {
+            T y[NT];
+            Terms<T>::split(TANH ? tanh_of<T>(u[e]) : u[e], y);
+            #pragma unroll
+            for (int q = 0; q < NT; q++) frag_set(uf[q], e, ldf(&y[q]));
+        }
+        #pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int n = n0 + j * 16 + lr;
+            const T* row = w + (int64_t)n * rank;
+            Frag<T> wf = frag_zero<T>();
+            if (n < N) {
+                if (v8) { if (k < rank) wf = frag8(row + k); }
+                else wf = frag_guard(row, k, rank);
+            }
+            #pragma unroll
+            for (int q = 0; q < NT; q++) z[j] = mma(wf, uf[q], z[j]);
+        }
+    }
+}
+// four results from column n on
+template <typename T>
+DEV void put4(T* out, int64_t t, int n, int N, const float* v) {
+    if (N % 4 == 0) { if (n < N) stv<4>(out + t * N + n, v); }
+    else
+        #pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (n + i < N) stf(out + t * N + n + i, v[i]);
+}
+
+// ---------------------------------------------------------------------------
+// Waves of several roles, in this order: convolution of a strip of tokens of
+// one sequence (a group of L lanes per head), decays and gates of 16 tokens
+// and 64 channels, step sizes.
+// ---------------------------------------------------------------------------
+template <typename T, typename P> struct GatedRows {
+    Rows<P> p;
+    int T_rows, o_in, ob, oa, ra, og, rg;     // columns and ranks
+    int H, G, D, V, C, taps;
+    const float* conv;                // [taps, C], the current token's last
+    float* cstate;                    // [slots, taps - 1, C]
+    const int* slot; const int* pos;
+    const int* strips;                // [n, 4] first row, rows, the portion's
+                                      // first row and end; null: every row
+    int n_strips;
+    const T* a2; const float* rate; const float* dt; const T* g2;
+    T* y;                             // [T, C]
+    float* scales;                    // [T, 2G] of queries and keys
+    float* decay;                     // [T, H*D], logarithms
+    float* beta;                      // [T, H]
+    T* gate;                          // [T, H*V]
+    int L, n_conv, n_decay, n_gate;   // lanes per head; waves of a role
+};
+
+template <typename T, typename P, int VEC, int KEEP, int TAPS>
+DEV void conv_strip(const GatedRows<T, P>& a, int64_t item, int lane) {
+    const int U = 2 * a.G + a.H, unit = (int)(item % U);
+    const int s = (int)(item / U);
+    if (s >= a.n_strips) return;
+    int row = s, n = 1, p0 = s, p1 = s + 1;
+    if (a.strips) {
+        row = a.strips[s * 4], n = a.strips[s * 4 + 1];
+        p0 = a.strips[s * 4 + 2], p1 = a.strips[s * 4 + 3];
+    }
+    const bool is_v = unit >= 2 * a.G;
+    const int wide = is_v ? a.V : a.D;
+    const int c0 = is_v ? 2 * a.G * a.D + (unit - 2 * a.G) * a.V
+                        : unit * a.D;
+    const int taps = TAPS ? TAPS : a.taps, C = a.C;
+    const bool fresh = a.pos[p0] == 0;
+    float* st = a.cstate + (int64_t)a.slot[p0] * (taps - 1) * C + c0;
+    // the input of row r, which may lie before the portion
+    auto input = [&](int r, int c, float* v) {
+        if (r >= p0) ldrow<VEC>(a.p, r, a.o_in + c0 + c, v);
+        else if (!fresh) ldv<VEC>(st + (int64_t)(taps - 1 + r - p0) * C + c,
+                                  v);
+        else
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) v[i] = 0.f;
+    };
+    auto col = [&](int j) { return (j * a.L + lane) * VEC; };
+    constexpr int TM = TAPS ? TAPS : 1;
+    float x[TM][KEEP][VEC], wt[TM][KEEP][VEC];      // the last inputs
+    if constexpr (TAPS > 0) {
+        #pragma unroll
+        for (int j = 0; j < KEEP; j++) {
+            if (col(j) >= wide) break;
+            #pragma unroll
+            for (int m = 0; m < TAPS; m++)
+                ldv<VEC>(a.conv + m * C + c0 + col(j), wt[m][j]);
+            #pragma unroll
+            for (int m = 1; m < TAPS; m++)
+                input(row - TAPS + m, col(j), x[m][j]);
+        }
+    }
+    for (int r = row; r < row + n; r++) {
+        float sq = 0.f;
+        #pragma unroll
+        for (int j = 0; j < KEEP; j++) {
+            const int c = col(j);
+            if (c >= wide) break;
+            float v[VEC] = {};
+            if constexpr (TAPS > 0) {
+                #pragma unroll
+                for (int m = 0; m + 1 < TAPS; m++)
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) x[m][j][i] = x[m + 1][j][i];
+                input(r, c, x[TAPS - 1][j]);
+                #pragma unroll
+                for (int m = 0; m < TAPS; m++)
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++)
+                        v[i] += wt[m][j][i] * x[m][j][i];
+            } else
+                for (int m = 0; m < taps; m++) {
+                    float u[VEC], w[VEC];
+                    input(r - taps + 1 + m, c, u);
+                    ldv<VEC>(a.conv + m * C + c0 + c, w);
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) v[i] += w[i] * u[i];
+                }
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) {
+                v[i] = silu_of<T>(v[i]);
+                sq += v[i] * v[i];
+            }
+            stv<VEC>(a.y + (int64_t)r * C + c0 + c, v);
+        }
+        if (is_v) continue;
+        for (int o = a.L / 2; o; o >>= 1) sq += __shfl_xor(sq, o, 64);
+        if (lane == 0)
+            a.scales[(int64_t)r * 2 * a.G + unit] =
+                (unit < a.G ? 1.f / sqrtf((float)a.D) : 1.f)
+                / sqrtf(sq + UNIT_EPS);
+    }
+    // Every row that reads the state is in its portion's first strip, and
+    // this lane alone reads and writes these channels of it.
+    if (row != p0) return;
+    for (int m = 0; m < taps - 1; m++)
+        #pragma unroll
+        for (int j = 0; j < KEEP; j++) {
+            const int c = col(j);
+            if (c >= wide) break;
+            float v[VEC];
+            input(p1 - taps + 1 + m, c, v);
+            stv<VEC>(st + (int64_t)m * C + c, v);
+        }
+}
+
+template <typename T, typename P, int VEC, int KEEP, int TAPS>
+__global__ __launch_bounds__(256) void k_gated_rows(GatedRows<T, P> a)
+{
+    const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
+    int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (w < a.n_conv) {
+        conv_strip<T, P, VEC, KEEP, TAPS>(
+            a, w * (64 / a.L) + lane / a.L, lane & (a.L - 1));
+        return;
+    }
+    w -= a.n_conv;
+    if (w < a.n_decay) {
+        const int N = a.H * a.D, nc = (N + 63) / 64;
+        const int n0 = (int)(w % nc) * 64;
+        const int64_t t = w / nc * 16 + lr;
+        f32x4 z[4] = {};
+        low_rank<T, P, false>(a.p, a.oa, a.ra, a.a2, N, n0,
+                              min(t, (int64_t)a.T_rows - 1), z);
+        if (t >= a.T_rows) return;
+        #pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int n = n0 + j * 16 + g * 4;
+            float v[4];
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int m = min(n + i, N - 1);
+                v[i] = fmaxf(LOG_ZERO, -a.rate[m / a.D]
+                             * softplus_of<T>(z[j][i] + a.dt[m]));
+            }
+            put4(a.decay, t, n, N, v);
+        }
+        return;
+    }
+    w -= a.n_decay;
+    if (w < a.n_gate) {
+        const int N = a.H * a.V, nc = (N + 63) / 64;
+        const int n0 = (int)(w % nc) * 64;
+        const int64_t t = w / nc * 16 + lr;
+        f32x4 z[4] = {};
+        low_rank<T, P, false>(a.p, a.og, a.rg, a.g2, N, n0,
+                              min(t, (int64_t)a.T_rows - 1), z);
+        if (t >= a.T_rows) return;
+        #pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const float v[4] = {z[j][0], z[j][1], z[j][2], z[j][3]};
+            put4(a.gate, t, n0 + j * 16 + g * 4, N, v);
+        }
+        return;
+    }
+    w -= a.n_gate;
+    const int64_t i = w * 64 + lane;
+    if (i >= (int64_t)a.T_rows * a.H) return;
+    float x;
+    ldrow<1>(a.p, i / a.H, a.ob + (int)(i % a.H), &x);
+    a.beta[i] = sigmoid_of<T>(x);
+}
+
+static int waves_for(int64_t tokens, int channels) {
+    return (int)((tokens + 15) / 16 * ((channels + 63) / 64));
+}
+
+// strips int32 [n, 4] (first row, rows, the portion's first row and end), a
+// strip no shorter than taps - 1 unless its portion is; null: every row is a
+// portion of its own.
+extern "C" int gated_rows(
+    int f32, const void* p, int p32, int n_part, int64_t part_stride,
+    int64_t ld, int o_in, int ob, int oa, int ra, int og, int rg,
+    const void* conv, int taps, void* cstate, const void* slot,
+    const void* pos, const void* strips, int n_strips, const void* a2,
+    const void* rate, const void* dt, const void* g2, void* y, void* scales,
+    void* decay, void* beta, void* gate, int T_rows, int H, int G, int D,
+    int V, hipStream_t stream)
+{
+    const int C = 2 * G * D + H * V, wide = D > V ? D : V;
+    const bool v4 = D % 4 == 0 && V % 4 == 0 && o_in % 4 == 0 && ld % 4 == 0
+                    && part_stride % 4 == 0;
+    if (taps < 1 || ra < 1 || rg < 1 || wide > (v4 ? 1024 : 256))
+        return (int)hipErrorInvalidValue;
+    const bool one = v4 && wide <= 256;     // a head fits 64 lanes at once
+    int L = 64;
+    if (one) while (L > 1 && L / 2 * 4 >= wide) L /= 2;
+    const int64_t units = (int64_t)n_strips * (2 * G + H);
+    const int n_conv = (int)((units * L + 63) / 64);
+    const int n_decay = waves_for(T_rows, H * D);
+    const int n_gate = waves_for(T_rows, H * V);
+    const int64_t all = (int64_t)n_conv + n_decay + n_gate
+                        + ((int64_t)T_rows * H + 63) / 64;
+    const int grid = (int)((all + 3) / 4);
+    #define GR(T, P, VE, KE, TA)                                           \
+        k_gated_rows<T, P, VE, KE, TA><<<grid, 256, 0, stream>>>(          \
+            GatedRows<T, P>{                                               \
+                Rows<P>{(const P*)p, n_part, part_stride, ld}, T_rows,     \
+                o_in, ob, oa, ra, og, rg, H, G, D, V, C, taps,             \
+                (const float*)conv, (float*)cstate, (const int*)slot,      \
+                (const int*)pos, (const int*)strips, n_strips,             \
+                (const T*)a2, (const float*)rate, (const float*)dt,        \
+                (const T*)g2, (T*)y, (float*)scales, (float*)decay,        \
+                (float*)beta, (T*)gate, L, n_conv, n_decay, n_gate})
+    #define GR_V(T, P)                                                     \
+        do {                                                               \
+            if (one && taps == 4) GR(T, P, 4, 1, 4);                       \
+            else if (one) GR(T, P, 4, 1, 0);                               \
+            else if (v4) GR(T, P, 4, 4, 0);                                \
+            else GR(T, P, 1, 4, 0);                                        \
+        } while (0)
+    if (f32) GR_V(float, float);
+    else if (p32) GR_V(bf16, float);
+    else GR_V(bf16, bf16);
+    #undef GR_V
+    #undef GR
+    return (int)hipGetLastError();
+}
+
+// Roles of the generalized rule: scales of unit keys (a group of L lanes per
+// head), decays, and, for a projection in parts, its sum.
+template <typename T, typename P> struct GeneralRows {
+    Rows<P> p;
+    int T_rows, ok, ow, rank, H, D;
+    const T* w2; const float* w0;
+    float* scales;                    // [T, H]
+    float* decay;                     // [T, H*D], logarithms
+    T* y;                             // [T, cols] or null
+    int cols, L, n_key, n_decay;
+};
+
+template <typename T, typename P, int VEC>
+__global__ __launch_bounds__(256) void k_general_rows(GeneralRows<T, P> a)
+{
+    const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
+    int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (w < a.n_key) {
+        const int64_t u = w * (64 / a.L) + lane / a.L;
+        if (u >= (int64_t)a.T_rows * a.H) return;
+        const int l = lane & (a.L - 1), c0 = a.ok + (int)(u % a.H) * a.D;
+        float s = 0.f;
+        for (int c = l * VEC; c < a.D; c += a.L * VEC) {
+            float x[VEC];
+            ldrow<VEC>(a.p, u / a.H, c0 + c, x);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) s += x[i] * x[i];
+        }
+        for (int o = a.L / 2; o; o >>= 1) s += __shfl_xor(s, o, 64);
+        if (l == 0) a.scales[u] = 1.f / sqrtf(s + UNIT_EPS);
+        return;
+    }
+    w -= a.n_key;
+    if (w < a.n_decay) {
+        const int N = a.H * a.D, nc = (N + 63) / 64;
+        const int n0 = (int)(w % nc) * 64;
+        const int64_t t = w / nc * 16 + lr;
+        f32x4 z[4] = {};
+        low_rank<T, P, true>(a.p, a.ow, a.rank, a.w2, N, n0,
+                             min(t, (int64_t)a.T_rows - 1), z);
+        if (t >= a.T_rows) return;
+        #pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const int n = n0 + j * 16 + g * 4;
+            float v[4];
+            #pragma unroll
+            for (int i = 0; i < 4; i++)
+                v[i] = -HALF_DECAY
+                       * sigmoid_of<T>(z[j][i] + a.w0[min(n + i, N - 1)]);
+            put4(a.decay, t, n, N, v);
+        }
+        return;
+    }
+    if (!a.y) return;
+    w -= a.n_decay;
+    const int64_t i = (w * 64 + lane) * VEC;
+    if (i >= (int64_t)a.T_rows * a.cols) return;
+    float x[VEC];
+    ldrow<VEC>(a.p, i / a.cols, (int)(i % a.cols), x);
+    stv<VEC>(a.y + i, x);
+}
+
+extern "C" int general_rows(
+    int f32, const void* p, int p32, int n_part, int64_t part_stride,
+    int64_t ld, int ok, int ow, int rank, const void* w2, const void* w0,
+    void* scales, void* decay, void* y, int cols, int T_rows, int H, int D,
+    hipStream_t stream)
+{
+    const bool v4 = D % 4 == 0 && ok % 4 == 0 && ld % 4 == 0
+                    && part_stride % 4 == 0 && cols % 4 == 0;
+    if (rank < 1) return (int)hipErrorInvalidValue;
+    int L = 64;
+    while (L > 1 && L / 2 * (v4 ? 4 : 1) >= D) L /= 2;
+    const int n_key = (int)(((int64_t)T_rows * H * L + 63) / 64);
+    const int n_decay = waves_for(T_rows, H * D);
+    const int64_t n_sum = y ? ((int64_t)T_rows * cols / (v4 ? 4 : 1) + 63)
+                              / 64 : 0;
+    const int grid = (int)((n_key + n_decay + n_sum + 3) / 4);
+    #define GE(T, P, VE)                                                   \
+        k_general_rows<T, P, VE><<<grid, 256, 0, stream>>>(                \
+            GeneralRows<T, P>{                                             \
+                Rows<P>{(const P*)p, n_part, part_stride, ld}, T_rows, ok, \
+                ow, rank, H, D, (const T*)w2, (const float*)w0,            \
+                (float*)scales, (float*)decay, (T*)y, cols, L, n_key,      \
+                n_decay})
+    #define GE_V(T, P) do { if (v4) GE(T, P, 4); else GE(T, P, 1); } while (0)
+    if (f32) GE_V(float, float);
+    else if (p32) GE_V(bf16, float);
+    else GE_V(bf16, bf16);
+    #undef GE_V
+    #undef GE
+    return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// What the recurrence reads.  Rows of x hold q, k [G, D], v [H, V] and, for
+// the generalized rule, removal rates before their bias [H, D].
+// ---------------------------------------------------------------------------
+template <typename T> struct DeltaIn {
+    const T* x;
+    int64_t ld;
+    int oq, ok, ov, oa;
+    const float* qs;                  // scales of q [T, sld] or null
+    const float* ks;                  // and of unit keys
+    int sld;
+    const float* decay;               // [T, H*D], logarithms
+    const float* beta;                // [T, H], gated rule
+    const float* a_bias;              // [H*D], generalized rule
+    int H, G, D, V;
+};
+
+// One block per sequence, head and strip of VB value columns; a thread keeps
+// NR rows of VEC columns of the state.
+template <typename T, int VEC, int NR, bool GEN>
+__global__ __launch_bounds__(256) void k_delta_step(
+    float* __restrict__ o,              // [T, H, V]
+    DeltaIn<T> in, float* __restrict__ state,   // [slots, H, D, V]
+    const int* __restrict__ slot, const int* __restrict__ pos,
+    const int* __restrict__ spans,      // [n, 2] first row, rows; null: 1 row
+    int VB)
+{
+    const int H = in.H, D = in.D, V = in.V;
+    const int h = blockIdx.y, hk = h / (H / in.G), tid = threadIdx.x;
+    const int v0 = blockIdx.z * VB, nc = min(VB, V - v0);
+    const int t0 = spans ? spans[blockIdx.x * 2] : blockIdx.x;
+    const int nt = spans ? spans[blockIdx.x * 2 + 1] : 1;
+    const int nv = nc / VEC;            // threads across a state row
+    const int RG = 256 / nv;            // state rows side by side
+    const int rg = tid / nv;
+    const bool on = rg < RG;
+    const int vt = tid % nv * VEC;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    float* r_s = sm;                    // [RG][nc] what z reads
+    float* o_s = r_s + 256 * VEC;       // [RG][nc] what q reads
+    float* q_s = o_s + 256 * VEC;       // [D]
+    float* k_s = q_s + D;
+    float* z_s = k_s + D;
+    float* e_s = z_s + D;
+    float* g_s = e_s + D;
+    float* S = state + ((int64_t)slot[t0] * H + h) * D * V + v0 + vt;
+    float s[NR][VEC];
+    const bool fresh = pos[t0] == 0;
+    #pragma unroll
+    for (int j = 0; j < NR; j++) {
+        const int d = rg + j * RG;
+        if (on && !fresh && d < D) ldv<VEC>(S + (int64_t)d * V, s[j]);
+        else
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) s[j][i] = 0.f;
+    }
+    for (int t = t0; t < t0 + nt; ++t) {
+        const T* row = in.x + (int64_t)t * in.ld;
+        const float qs = in.qs ? in.qs[(int64_t)t * in.sld + hk] : 1.f;
+        const float ks = in.ks[(int64_t)t * in.sld + hk];
+        const float beta = GEN ? 0.f : in.beta[(int64_t)t * H + h];
+        for (int d = tid; d < D; d += 256) {
+            const int c = h * D + d;
+            const float k = ldf(row + in.ok + hk * D + d), u = k * ks;
+            const float g = exp_of<T>(in.decay[(int64_t)t * H * D + c]);
+            q_s[d] = ldf(row + in.oq + hk * D + d) * qs;
+            g_s[d] = g;
+            if (GEN) {
+                const float a = sigmoid_of<T>(ldf(row + in.oa + c)
+                                              + in.a_bias[c]);
+                k_s[d] = k;
+                z_s[d] = u;
+                e_s[d] = a * u;
+            } else {
+                k_s[d] = e_s[d] = beta * u;
+                z_s[d] = g * u;
+            }
+        }
+        __syncthreads();
+        float v[VEC], acc[VEC] = {};
+        if (on) {
+            ldv<VEC>(row + in.ov + h * V + v0 + vt, v);
+            #pragma unroll
+            for (int j = 0; j < NR; j++) {
+                const int d = rg + j * RG;
+                if (d >= D) break;
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) acc[i] += z_s[d] * s[j][i];
+            }
+            stv<VEC>(r_s + rg * nc + vt, acc);
+        }
+        __syncthreads();
+        if (on) {
+            float r[VEC] = {}, f[VEC] = {};
+            for (int y = 0; y < RG; y++) {
+                float x[VEC];
+                ldv<VEC>(r_s + y * nc + vt, x);
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) r[i] += x[i];
+            }
+            #pragma unroll
+            for (int j = 0; j < NR; j++) {
+                const int d = rg + j * RG;
+                if (d >= D) break;
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) {
+                    s[j][i] = g_s[d] * s[j][i] - e_s[d] * r[i]
+                              + k_s[d] * v[i];
+                    f[i] += q_s[d] * s[j][i];
+                }
+            }
+            stv<VEC>(o_s + rg * nc + vt, f);
+        }
+        __syncthreads();
+        for (int c = tid; c < nc; c += 256) {
+            float x = 0.f;
+            for (int y = 0; y < RG; y++) x += o_s[y * nc + c];
+            o[((int64_t)t * H + h) * V + v0 + c] = x;
+        }
+    }
+    #pragma unroll
+    for (int j = 0; j < NR; j++) {
+        const int d = rg + j * RG;
+        if (on && d < D) stv<VEC>(S + (int64_t)d * V, s[j]);
+    }
+}
+
+#define DELTA_IN(T)                                                        \
+    DeltaIn<T>{(const T*)x, ld, oq, ok, ov, oa, (const float*)qs,          \
+               (const float*)ks, sld, (const float*)decay,                 \
+               (const float*)beta, (const float*)a_bias, H, G, D, V}
+
+extern "C" int delta_step(
+    int f32, int gen, void* o, const void* x, int64_t ld, int oq, int ok,
+    int ov, int oa, const void* qs, const void* ks, int sld,
+    const void* decay, const void* beta, const void* a_bias, void* state,
+    const void* slot, const void* pos, const void* spans, int n, int H,
+    int G, int D, int V, hipStream_t stream)
+{
+    const bool v4 = V % 4 == 0 && ov % 4 == 0 && ld % 4 == 0;
+    const int vec = v4 ? 4 : 1;
+    if (D < 1 || V < 1 || D > 2048) return (int)hipErrorInvalidValue;
+    // threads across a strip: the rest of the block covers the rows, 16 a
+    // thread; narrower while there are few blocks
+    int nv = 256;
+    while (nv > 1 && 256 / nv * 16 < D) nv /= 2;
+    int vb = nv * vec < V ? nv * vec : V;
+    while (v4 && vb > 32 && vb % 8 == 0
+           && (int64_t)n * H * ((V + vb - 1) / vb) < 512) vb /= 2;
+    const int per = (D + 256 / (vb / vec) - 1) / (256 / (vb / vec));
+    const int lds = (2 * 256 * vec + 5 * D) * 4;
+    dim3 grid(n, H, (V + vb - 1) / vb);
+    #define DS_GO(T, VE, NR, GEN)                                          \
+        k_delta_step<T, VE, NR, GEN><<<grid, 256, lds, stream>>>(          \
+            (float*)o, DELTA_IN(T), (float*)state, (const int*)slot,       \
+            (const int*)pos, (const int*)spans, vb)
+    #define DS_N(T, VE, GEN)                                               \
+        do {                                                               \
+            if (per <= 4) DS_GO(T, VE, 4, GEN);                            \
+            else DS_GO(T, VE, 16, GEN);                                    \
+        } while (0)
+    #define DS_V(T, GEN)                                                   \
+        do { if (v4) DS_N(T, 4, GEN); else DS_N(T, 1, GEN); } while (0)
+    if (per > 16) return (int)hipErrorInvalidValue;
+    if (f32) { if (gen) DS_V(float, true); else DS_V(float, false); }
+    else { if (gen) DS_V(bf16, true); else DS_V(bf16, false); }
+    #undef DS_V
+    #undef DS_N
+    #undef DS_GO
+    return (int)hipGetLastError();
+}
+
+// ---- chunks --------------------------------------------------------------
+#define CH 64             // tokens of a chunk
+#define SUB 16            // tokens of a part
+#define DB 32             // key channels of a prep pass
+#define DS (DB + 4)       // LDS row strides
+#define AS (CH + 4)
+// largest sum of decay inside a part for which the part's own triangle may
+// be factored (e^{c_i} e^{-c_j}); beyond it the pairs are taken one by one
+#define SAFE 20.f
+
+// An fp32 matrix as operand of products: in bf16 models two planes of bf16
+// terms whose products leave out the smallest, else itself.
+template <typename T> struct Wide;
+template <> struct Wide<float> { f32x8s f; };
+template <> struct Wide<bf16> { bf16x8 hi, lo; };
+DEV Wide<float> ldw(const float* p, int64_t) { return {frag8(p)}; }
+DEV Wide<bf16> ldw(const bf16* p, int64_t plane) {
+    return {frag8(p), frag8(p + plane)};
+}
+template <typename T> DEV Wide<T> wide_zero() {
+    if constexpr (sizeof(T) == 4) return {frag_zero<float>()};
+    else return {frag_zero<bf16>(), frag_zero<bf16>()};
+}
+DEV f32x4 mma(const Wide<float>& a, const Wide<float>& b, f32x4 c) {
+    return mma(a.f, b.f, c);
+}
+DEV f32x4 mma(const Wide<bf16>& a, const Wide<bf16>& b, f32x4 c) {
+    c = mma(a.lo, b.hi, c);
+    c = mma(a.hi, b.lo, c);
+    return mma(a.hi, b.hi, c);
+}
+DEV void stw(float* p, int64_t, float v) { *p = v; }
+DEV void stw(bf16* p, int64_t plane, float v) {
+    bf16 t[2];
+    Terms<bf16>::split(v, t);
+    p[0] = t[0];
+    p[plane] = t[1];
+}
+template <typename T> DEV void stw4(T* p, int64_t plane, f32x4 v) {
+    float f[Terms<T>::N][4];
+    #pragma unroll
+    for (int i = 0; i < 4; i++) {
+        T t[Terms<T>::N];
+        Terms<T>::split(v[i], t);
+        #pragma unroll
+        for (int q = 0; q < Terms<T>::N; q++) f[q][i] = ldf(&t[q]);
+    }
+    #pragma unroll
+    for (int q = 0; q < Terms<T>::N; q++) stv<4>(p + q * plane, f[q]);
+}
+
+// Scratch per (chunk, head), each matrix of N planes: Q [64][Dp], Z [64][Dp],
+// K^T [Dp][64], (E^T), inverse [64][64], A_qk, (A_zk, A_qe); then the fp32
+// decay of the whole chunk [Dp].
+template <typename T, bool GEN> struct Unit {
+    static constexpr int NT = Terms<T>::N;
+    DEV static T* base(float* scr, int64_t i, int Dp) {
+        return (T*)(scr + i * floats(Dp));
+    }
+    static __host__ __device__ int64_t floats(int Dp) {
+        return (int64_t)(GEN ? 4 : 3) * CH * Dp + (GEN ? 4 : 2) * CH * CH
+               + Dp;
+    }
+    // offsets in elements; a plane follows its matrix
+    static __host__ __device__ int64_t tall(int m, int Dp) {
+        return (int64_t)m * NT * CH * Dp;
+    }
+    static __host__ __device__ int64_t square(int m, int Dp) {
+        return tall(GEN ? 4 : 3, Dp) + (int64_t)m * NT * CH * CH;
+    }
+    static __host__ __device__ int64_t fade(int Dp) {
+        return square(GEN ? 4 : 2, Dp);
+    }
+};
+enum { TALL_Q, TALL_Z, TALL_K, TALL_E };
+enum { SQ_INV, SQ_QK, SQ_ZK, SQ_QE };
+
+template <typename T, bool GEN>
+__global__ __launch_bounds__(256) void k_delta_prep(
+    float* __restrict__ scr, DeltaIn<T> in,
+    const int* __restrict__ chunks,     // [n, 2] first row, rows
+    int Dp, int vec)
+{
+    typedef Unit<T, GEN> Un;
+    const int H = in.H, D = in.D;
+    const int h = blockIdx.y, hk = h / (H / in.G), tid = threadIdx.x;
+    const int lane = tid & 63, w = tid >> 6;
+    const int lr = lane & 15, g = lane >> 4;
+    const int t0 = chunks[blockIdx.x * 2], n = chunks[blockIdx.x * 2 + 1];
+    T* un = Un::base(scr, (int64_t)blockIdx.x * H + h, Dp);
+    float* fade = (float*)(un + Un::fade(Dp));
+    const int64_t tp = (int64_t)CH * Dp, sp = CH * CH;      // planes
+    constexpr int PL = CH * DS;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    float* qe_s = sm;                   // [64][DS] q e^{c}, c from the part on
+    float* ze_s = qe_s + PL;            // z e^{c} / g
+    float* kt_s = ze_s + PL;            // k e^{part total - c}
+    float* kn_s = kt_s + PL;            // k e^{-c}, or k
+    float* x1_s = kn_s + PL;            // GEN: e e^{part total - c}; else q
+    float* x2_s = x1_s + PL;            // GEN: e e^{-c}; else u
+    float* c_s = x2_s + PL;             // gated rule: c
+    float* et_s = GEN ? c_s : c_s + PL; // [4][DB] e^{part total}
+    float* A_s = sm;                    // [64][AS] afterwards
+    float* I_s = A_s + CH * AS;
+
+    // a lane's token, and its eight channels of a pass
+    const int tk = w * SUB + (lane >> 2), c8 = (lane & 3) * 8;
+    const bool live = tk < n;
+    const int64_t t = t0 + min(tk, n - 1);
+    const T* row = in.x + t * in.ld;
+    const float on = live ? 1.f : 0.f;
+    const float qs = on * (in.qs ? in.qs[t * in.sld + hk] : 1.f);
+    const float ks = on * in.ks[t * in.sld + hk];
+    const float beta = GEN ? 0.f : in.beta[t * H + h];
+    // of the six tiles below the diagonal (1,0) (2,1) (3,2) (2,0) (3,1)
+    // (3,0) this wave makes numbers w and w + 4
+    const int ti[6] = {1, 2, 3, 2, 3, 3}, tj[6] = {0, 1, 2, 0, 1, 0};
+    // products of q and z with k (and e): the wave's diagonal tile, the
+    // tiles below the diagonal
+    f32x4 dqk = {}, dzk = {}, dqe = {}, dze = {};
+    f32x4 oqk[2] = {}, ozk[2] = {}, oqe[2] = {}, oze[2] = {};
+
+    for (int d0 = 0; d0 < Dp; d0 += DB) {
+        __syncthreads();
+        const int d = d0 + c8;
+        float q[8] = {}, k[8] = {}, c[8] = {}, a[8] = {};
+        if (vec) {
+            if (d < D) {
+                ldv<8>(row + in.oq + hk * D + d, q);
+                ldv<8>(row + in.ok + hk * D + d, k);
+                ldv<8>(in.decay + (t * H + h) * D + d, c);
+                if (GEN) ldv<8>(row + in.oa + h * D + d, a);
+            }
+        } else
+            for (int e = 0; e < 8; e++)
+                if (d + e < D) {
+                    q[e] = ldf(row + in.oq + hk * D + d + e);
+                    k[e] = ldf(row + in.ok + hk * D + d + e);
+                    c[e] = in.decay[(t * H + h) * D + d + e];
+                    if (GEN) a[e] = ldf(row + in.oa + h * D + d + e);
+                }
+        if (GEN)
+            #pragma unroll
+            for (int e = 0; e < 8; e++)
+                a[e] = d + e < D
+                    ? sigmoid_of<T>(a[e] + in.a_bias[h * D + d + e]) : 0.f;
+        float own[8], tot[8];
+        bool safe = true;
+        #pragma unroll
+        for (int e = 0; e < 8; e++) {
+            own[e] = c[e] = c[e] * on;
+            #pragma unroll
+            for (int s = 4; s < 64; s *= 2) {       // tokens are 4 lanes apart
+                const float y = __shfl_up(c[e], s, 64);
+                if (lane >= s) c[e] += y;
+            }
+            tot[e] = __shfl(c[e], 60 + (lane & 3), 64);
+            safe = safe && tot[e] > -SAFE;
+        }
+        safe = GEN || __all(safe);
+        float qe[8], ze[8], kt[8], kn[8], x1[8], x2[8];
+        #pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const float grow = exp_of<T>(c[e]);
+            const float left = exp_of<T>(tot[e] - c[e]);
+            const float back = safe ? exp_of<T>(-c[e]) : 1.f;
+            const float u = k[e] * ks;
+            const float kk = GEN ? k[e] * on : beta * u;
+            qe[e] = q[e] * qs * grow;
+            ze[e] = u * (GEN ? exp_of<T>(c[e] - own[e]) : grow);
+            kt[e] = kk * left;
+            kn[e] = kk * back;
+            x1[e] = GEN ? a[e] * u * left : q[e] * qs;
+            x2[e] = GEN ? a[e] * u * back : u;
+        }
+        const int at = tk * DS + c8;
+        stv<8>(qe_s + at, qe);
+        stv<8>(ze_s + at, ze);
+        stv<8>(kt_s + at, kt);
+        stv<8>(kn_s + at, kn);
+        if (GEN || !safe) {
+            stv<8>(x1_s + at, x1);
+            stv<8>(x2_s + at, x2);
+        }
+        if (!GEN && !safe) stv<8>(c_s + at, c);
+        if ((lane >> 2) == 0) {
+            #pragma unroll
+            for (int e = 0; e < 8; e++) tot[e] = exp_of<T>(tot[e]);
+            stv<8>(et_s + w * DB + c8, tot);
+        }
+        __syncthreads();
+        // factors that meet the state: the decay of the chunk before and
+        // after the part joins in
+        if (d < Dp) {
+            float before[8], after[8];
+            #pragma unroll
+            for (int e = 0; e < 8; e++) before[e] = after[e] = 1.f;
+            for (int s = 0; s < 4; s++) {
+                if (s == w) continue;
+                float f[8];
+                ldv<8>(et_s + s * DB + c8, f);
+                #pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    if (s < w) before[e] *= f[e];
+                    else after[e] *= f[e];
+                }
+            }
+            #pragma unroll
+            for (int e = 0; e < 8; e += 4) {
+                f32x4 y, z;
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    y[i] = qe[e + i] * before[e + i];
+                    z[i] = ze[e + i] * before[e + i];
+                }
+                stw4(un + Un::tall(TALL_Q, Dp) + (int64_t)tk * Dp + d + e, tp,
+                     y);
+                stw4(un + Un::tall(TALL_Z, Dp) + (int64_t)tk * Dp + d + e, tp,
+                     z);
+            }
+            #pragma unroll
+            for (int e = 0; e < 8; e++) {
+                stw(un + Un::tall(TALL_K, Dp) + (int64_t)(d + e) * CH + tk, tp,
+                    kt[e] * after[e]);
+                if (GEN)
+                    stw(un + Un::tall(TALL_E, Dp) + (int64_t)(d + e) * CH + tk,
+                        tp, x1[e] * after[e]);
+            }
+            if (w == 3 && (lane >> 2) == 0)
+                #pragma unroll
+                for (int e = 0; e < 8; e++)
+                    fade[d + e] = before[e] * et_s[3 * DB + c8 + e];
+        }
+        // tiles below the diagonal
+        #pragma unroll
+        for (int x = 0; x < 2; x++) {
+            const int id = w + x * 4;
+            if (id >= 6) continue;
+            const int I = ti[id], J = tj[id];
+            f32x8s qa = frag8(qe_s + (I * SUB + lr) * DS + g * 8);
+            f32x8s za = frag8(ze_s + (I * SUB + lr) * DS + g * 8);
+            for (int s = J + 1; s < I; s++) {
+                const f32x8s f = frag8(et_s + s * DB + g * 8);
+                qa.lo *= f.lo; qa.hi *= f.hi;
+                za.lo *= f.lo; za.hi *= f.hi;
+            }
+            const f32x8s kb = frag8(kt_s + (J * SUB + lr) * DS + g * 8);
+            oqk[x] = mma(qa, kb, oqk[x]);
+            ozk[x] = mma(za, kb, ozk[x]);
+            if (GEN) {
+                const f32x8s eb = frag8(x1_s + (J * SUB + lr) * DS + g * 8);
+                oqe[x] = mma(qa, eb, oqe[x]);
+                oze[x] = mma(za, eb, oze[x]);
+            }
+        }
+        // the part's own triangle
+        if (safe) {
+            const int r = (w * SUB + lr) * DS + g * 8;
+            const f32x8s qa = frag8(qe_s + r), za = frag8(ze_s + r);
+            const f32x8s kb = frag8(kn_s + r);
+            dqk = mma(qa, kb, dqk);
+            dzk = mma(za, kb, dzk);
+            if (GEN) {
+                const f32x8s eb = frag8(x2_s + r);
+                dqe = mma(qa, eb, dqe);
+                dze = mma(za, eb, dze);
+            }
+        } else {
+            // lane: column lr (the key), rows 4g + i (the query)
+            for (int e = 0; e < DB; e++) {
+                const int oj = (w * SUB + lr) * DS + e;
+                const float kj = kn_s[oj], cj = c_s[oj];
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int oi = (w * SUB + g * 4 + i) * DS + e;
+                    const float f = kj * exp_of<T>(fminf(c_s[oi] - cj, 0.f));
+                    dqk[i] += x1_s[oi] * f;
+                    dzk[i] += x2_s[oi] * f;
+                }
+            }
+        }
+    }
+    // A_ze to LDS, the others to memory; the gated rule's A_ze is A_zk
+    __syncthreads();
+    auto place = [&](int m, int I, int J, f32x4 v) {
+        #pragma unroll
+        for (int i = 0; i < 4; i++)
+            stw(un + Un::square(m, Dp) + (I * SUB + g * 4 + i) * CH
+                + J * SUB + lr, sp, v[i]);
+    };
+    auto keep = [&](int I, int J, f32x4 v) {
+        #pragma unroll
+        for (int i = 0; i < 4; i++)
+            A_s[(I * SUB + g * 4 + i) * AS + J * SUB + lr] = v[i];
+    };
+    #pragma unroll
+    for (int i = 0; i < 4; i++) {
+        if (lr > g * 4 + i) dqk[i] = dqe[i] = 0.f;
+        if (lr >= g * 4 + i) dzk[i] = dze[i] = 0.f;
+    }
+    const f32x4 none = {};
+    place(SQ_QK, w, w, dqk);
+    keep(w, w, GEN ? dze : dzk);
+    if (GEN) {
+        place(SQ_ZK, w, w, dzk);
+        place(SQ_QE, w, w, dqe);
+    }
+    if (w % 2 == 0) {       // products go 32 tokens at a time
+        place(SQ_QK, w, w + 1, none);
+        if (GEN) {
+            place(SQ_ZK, w, w + 1, none);
+            place(SQ_QE, w, w + 1, none);
+        }
+    }
+    #pragma unroll
+    for (int x = 0; x < 2; x++) {
+        const int id = w + x * 4;
+        if (id >= 6) continue;
+        place(SQ_QK, ti[id], tj[id], oqk[x]);
+        keep(ti[id], tj[id], GEN ? oze[x] : ozk[x]);
+        if (GEN) {
+            place(SQ_ZK, ti[id], tj[id], ozk[x]);
+            place(SQ_QE, ti[id], tj[id], oqe[x]);
+        }
+    }
+    __syncthreads();
+    // (I + A)^-1: a column a lane inside the diagonal blocks, then block by
+    // block below them
+    {
+        const float* A = A_s + w * SUB * AS + w * SUB;
+        float x[SUB];
+        #pragma unroll
+        for (int i = 0; i < SUB; i++) {
+            float y = i == lr ? 1.f : 0.f;
+            #pragma unroll
+            for (int j = 0; j < i; j++) y -= A[i * AS + j] * x[j];
+            x[i] = y;
+        }
+        #pragma unroll
+        for (int i = 0; i < SUB; i++)
+            if (i / 4 == g) I_s[(w * SUB + i) * AS + w * SUB + lr] = x[i];
+    }
+    __syncthreads();
+    auto below = [&](int I, int J) {
+        f32x4 y = {}, z = {};
+        for (int K = J; K < I; K++) {
+            const f32x4 a = *reinterpret_cast<const f32x4*>(
+                A_s + (I * SUB + lr) * AS + K * SUB + g * 4);
+            #pragma unroll
+            for (int e = 0; e < 4; e++)
+                y = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    a[e], I_s[(K * SUB + g * 4 + e) * AS + J * SUB + lr], y,
+                    0, 0, 0);
+        }
+        const f32x4 a = *reinterpret_cast<const f32x4*>(
+            I_s + (I * SUB + lr) * AS + I * SUB + g * 4);
+        #pragma unroll
+        for (int e = 0; e < 4; e++)
+            z = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], y[e], z, 0, 0, 0);
+        #pragma unroll
+        for (int i = 0; i < 4; i++)
+            I_s[(I * SUB + g * 4 + i) * AS + J * SUB + lr] = -z[i];
+    };
+    #pragma unroll
+    for (int s = 1; s < 4; s++) {
+        if (w + s < 4) below(w + s, w);
+        __syncthreads();
+    }
+    for (int i = tid; i < CH * CH / 4; i += 256) {
+        const int r = i / (CH / 4), c = i % (CH / 4) * 4;
+        f32x4 v = {};
+        if (c / SUB <= r / SUB)
+            v = *reinterpret_cast<const f32x4*>(I_s + r * AS + c);
+        stw4(un + Un::square(SQ_INV, Dp) + r * CH + c, sp, v);
+    }
+}
+
+// A sequence's chunks in order, one block per 16*VC value columns, the state
+// in registers (NS: 16-row tiles a wave, Dp <= 64 * NS); wave w has tokens
+// 16 w .. of a chunk.  What several waves need goes through LDS, transposed:
+// the state, v, what w is solved from and w itself.
+template <typename T, int NS, int VC, bool GEN>
+__global__ __launch_bounds__(256) void k_delta_scan(
+    float* __restrict__ o,              // [T, H, V]
+    float* __restrict__ scr, DeltaIn<T> in, float* __restrict__ state,
+    const int* __restrict__ slot, const int* __restrict__ pos,
+    const int* __restrict__ chunks,     // [n, 2]
+    const int* __restrict__ seqs,       // [m, 2] first chunk, chunks
+    int Dp, int vec)
+{
+    typedef Unit<T, GEN> Un;
+    constexpr int W = VC * 16, NT = Terms<T>::N, PAD = 16 / sizeof(T);
+    constexpr int KS = NS * 64 + PAD, TS = CH + PAD;
+    constexpr int NQ = NS * 2;          // 32-channel steps over D
+    constexpr int64_t SP = (int64_t)W * KS, VP = (int64_t)W * TS;   // planes
+    const int H = in.H, D = in.D, V = in.V;
+    const int h = blockIdx.y, v0 = blockIdx.z * W, tid = threadIdx.x;
+    const int lane = tid & 63;
+    const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int lr = lane & 15, g = lane >> 4;
+    const int c0 = seqs[blockIdx.x * 2], nc = seqs[blockIdx.x * 2 + 1];
+    const int first = chunks[c0 * 2];
+    float* St = state + ((int64_t)slot[first] * H + h) * D * V;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    T* S_s = reinterpret_cast<T*>(smem);      // [NT][W][KS] state
+    T* r_s = S_s + NT * SP;                   // [NT][W][TS] right-hand side
+    T* u_s = r_s + NT * VP;                   // [NT][W][TS] solution
+    T* v_s = u_s + NT * VP;                   // [GEN ? 2 : 1][NT][W][TS]
+
+    f32x4 S[NS][VC];
+    const bool fresh = pos[first] == 0;
+    #pragma unroll
+    for (int x = 0; x < NS; x++)
+        #pragma unroll
+        for (int c = 0; c < VC; c++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int d = (w + x * 4) * 16 + g * 4 + i;
+                const int v = v0 + c * 16 + lr;
+                S[x][c][i] = (fresh || d >= D || v >= V)
+                                 ? 0.f : St[(int64_t)d * V + v];
+            }
+
+    const int64_t tp = (int64_t)CH * Dp, sp = CH * CH;
+    Wide<T> zf[NQ], qf[NQ], inv[2], aqk[2], azk[2], aqe[2];
+    Wide<T> kf[NS][2], ef[NS][2];
+    f32x4 e4[NS];
+    float vv[VC * 4];
+    auto unit = [&](int ci) {
+        return Un::base(scr, (int64_t)ci * H + h, Dp);
+    };
+    auto load_zq = [&](int ci) {
+        const T* u = unit(ci) + (int64_t)(w * 16 + lr) * Dp + g * 8;
+        #pragma unroll
+        for (int d = 0; d < NQ; d++) {
+            zf[d] = d * 32 < Dp ? ldw(u + Un::tall(TALL_Z, Dp) + d * 32, tp)
+                                : wide_zero<T>();
+            qf[d] = d * 32 < Dp ? ldw(u + Un::tall(TALL_Q, Dp) + d * 32, tp)
+                                : wide_zero<T>();
+        }
+    };
+    auto load_square = [&](int ci, int m, Wide<T>* f) {
+        const T* u = unit(ci) + Un::square(m, Dp) + (w * 16 + lr) * CH
+                     + g * 8;
+        #pragma unroll
+        for (int j = 0; j < 2; j++)
+            f[j] = j * 2 <= w ? ldw(u + j * 32, sp) : wide_zero<T>();
+    };
+    auto load_k = [&](int ci) {
+        const T* u = unit(ci);
+        const float* fd = (const float*)(u + Un::fade(Dp));
+        #pragma unroll
+        for (int x = 0; x < NS; x++) {
+            const int d = (w + x * 4) * 16;
+            const bool in_d = d < Dp;
+            e4[x] = in_d ? *reinterpret_cast<const f32x4*>(fd + d + g * 4)
+                         : f32x4{};
+            #pragma unroll
+            for (int j = 0; j < 2; j++) {
+                const int64_t at = (int64_t)(d + lr) * CH + j * 32 + g * 8;
+                kf[x][j] = in_d ? ldw(u + Un::tall(TALL_K, Dp) + at, tp)
+                                : wide_zero<T>();
+                if (GEN)
+                    ef[x][j] = in_d ? ldw(u + Un::tall(TALL_E, Dp) + at, tp)
+                                    : wide_zero<T>();
+            }
+        }
+    };
+    // token lane of a chunk, columns (wave * VC + ..) * 4
+    auto load_v = [&](int ci) {
+        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
+        const T* r = in.x + (int64_t)(t0 + min(lane, n - 1)) * in.ld + in.ov
+                     + h * V + v0;
+        #pragma unroll
+        for (int q = 0; q < VC; q++) {
+            const int c = (w * VC + q) * 4;
+            #pragma unroll
+            for (int e = 0; e < 4; e++) vv[q * 4 + e] = 0.f;
+            if (lane >= n) continue;
+            if (vec) {
+                if (v0 + c < V) ldv<4>(r + c, vv + q * 4);
+            } else
+                #pragma unroll
+                for (int e = 0; e < 4; e++)
+                    if (v0 + c + e < V) vv[q * 4 + e] = ldf(r + c + e);
+        }
+    };
+    auto solve_operand = [&](const T* s, int c, int j) {
+        return ldw(s + (c * 16 + lr) * TS + j * 32 + g * 8, VP);
+    };
+    load_v(c0);
+    load_zq(c0);
+    load_square(c0, SQ_INV, inv);
+    load_square(c0, SQ_QK, aqk);
+    if (GEN) {
+        load_square(c0, SQ_ZK, azk);
+        load_square(c0, SQ_QE, aqe);
+    }
+    load_k(c0);
+
+    for (int ci = c0; ci < c0 + nc; ++ci) {
+        const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
+        const int nx = min(ci + 1, c0 + nc - 1);
+        T* vb = GEN && (ci & 1) ? v_s + NT * VP : v_s;
+        #pragma unroll
+        for (int e = 0; e < VC * 4; e++)
+            stw(vb + (w * VC * 4 + e) * TS + lane, VP, vv[e]);
+        #pragma unroll
+        for (int x = 0; x < NS; x++) {
+            const int d = (w + x * 4) * 16 + g * 4;
+            #pragma unroll
+            for (int c = 0; c < VC; c++)
+                stw4(S_s + (c * 16 + lr) * KS + d, SP, S[x][c]);
+        }
+        lds_barrier();
+        load_v(nx);
+        // what z and q read from the state before the chunk
+        f32x4 az[VC] = {}, ao[VC] = {};
+        #pragma unroll
+        for (int d = 0; d < NQ; d++) {
+            if (d * 32 >= Dp) continue;
+            #pragma unroll
+            for (int c = 0; c < VC; c++) {
+                const Wide<T> b = ldw(S_s + (c * 16 + lr) * KS + d * 32
+                                      + g * 8, SP);
+                az[c] = mma(zf[d], b, az[c]);
+                ao[c] = mma(qf[d], b, ao[c]);
+            }
+        }
+        load_zq(nx);
+        if (GEN) {
+            #pragma unroll
+            for (int j = 0; j < 2; j++) {
+                if (j * 2 > w) continue;
+                #pragma unroll
+                for (int c = 0; c < VC; c++) {
+                    const Wide<T> b = solve_operand(vb, c, j);
+                    az[c] = mma(azk[j], b, az[c]);
+                    ao[c] = mma(aqk[j], b, ao[c]);
+                }
+            }
+            load_square(nx, SQ_ZK, azk);
+            load_square(nx, SQ_QK, aqk);
+        }
+        #pragma unroll
+        for (int c = 0; c < VC; c++) {
+            const int at = (c * 16 + lr) * TS + w * 16 + g * 4;
+            if (!GEN) {
+                float f[4];
+                ldv<4>(vb + at, f);     // v itself: its first term
+                #pragma unroll
+                for (int i = 0; i < 4; i++) az[c][i] = f[i] - az[c][i];
+            }
+            stw4(r_s + at, VP, az[c]);
+        }
+        lds_barrier();
+        f32x4 u[VC] = {};
+        #pragma unroll
+        for (int j = 0; j < 2; j++) {
+            if (j * 2 > w) continue;
+            #pragma unroll
+            for (int c = 0; c < VC; c++)
+                u[c] = mma(inv[j], solve_operand(r_s, c, j), u[c]);
+        }
+        load_square(nx, SQ_INV, inv);
+        #pragma unroll
+        for (int c = 0; c < VC; c++)
+            stw4(u_s + (c * 16 + lr) * TS + w * 16 + g * 4, VP,
+                 GEN ? -u[c] : u[c]);
+        lds_barrier();
+        #pragma unroll
+        for (int j = 0; j < 2; j++) {
+            if (j * 2 > w) continue;
+            #pragma unroll
+            for (int c = 0; c < VC; c++)
+                ao[c] = mma(GEN ? aqe[j] : aqk[j],
+                            solve_operand(u_s, c, j), ao[c]);
+        }
+        load_square(nx, GEN ? SQ_QE : SQ_QK, GEN ? aqe : aqk);
+        #pragma unroll
+        for (int c = 0; c < VC; c++) {
+            const int v = v0 + c * 16 + lr;
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int t = w * 16 + g * 4 + i;
+                if (t < n && v < V)
+                    o[((int64_t)(t0 + t) * H + h) * V + v] = ao[c][i];
+            }
+        }
+        // the next state
+        #pragma unroll
+        for (int x = 0; x < NS; x++)
+            #pragma unroll
+            for (int c = 0; c < VC; c++) S[x][c] *= e4[x];
+        #pragma unroll
+        for (int j = 0; j < 2; j++)
+            #pragma unroll
+            for (int c = 0; c < VC; c++) {
+                const Wide<T> b = solve_operand(GEN ? vb : u_s, c, j);
+                #pragma unroll
+                for (int x = 0; x < NS; x++)
+                    if ((w + x * 4) * 16 < Dp)
+                        S[x][c] = mma(kf[x][j], b, S[x][c]);
+                if (GEN) {
+                    const Wide<T> b2 = solve_operand(u_s, c, j);
+                    #pragma unroll
+                    for (int x = 0; x < NS; x++)
+                        if ((w + x * 4) * 16 < Dp)
+                            S[x][c] = mma(ef[x][j], b2, S[x][c]);
+                }
+            }
+        load_k(nx);
+    }
+    #pragma unroll
+    for (int x = 0; x < NS; x++)
+        #pragma unroll
+        for (int c = 0; c < VC; c++)
+            #pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int d = (w + x * 4) * 16 + g * 4 + i;
+                const int v = v0 + c * 16 + lr;
+                if (d < D && v < V) St[(int64_t)d * V + v] = S[x][c][i];
+            }
+}
+
+static int delta_pad(int D) { return (D + DB - 1) / DB * DB; }
+
+extern "C" int64_t delta_scratch_floats(int gen, int n_chunks, int H, int D)
+{
+    const int Dp = delta_pad(D);
+    return (int64_t)n_chunks * H
+           * (gen ? Unit<float, true>::floats(Dp)
+                  : Unit<float, false>::floats(Dp));
+}
+
+template <typename T, int NS, int VC, bool GEN>
+static void scan_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
+                    const int* slot, const int* pos, const int* chunks,
+                    const int* seqs, int n_seqs, int Dp, int vec,
+                    hipStream_t stream)
+{
+    constexpr int W = VC * 16, PAD = 16 / sizeof(T), es = sizeof(T);
+    constexpr int lds = Terms<T>::N * es
+        * (W * (NS * 64 + PAD) + (GEN ? 4 : 3) * W * (CH + PAD));
+    static bool once = false;
+    if (!once) {
+        (void)hipFuncSetAttribute(
+            (const void*)k_delta_scan<T, NS, VC, GEN>,
+            hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        once = true;
+    }
+    k_delta_scan<T, NS, VC, GEN>
+        <<<dim3(n_seqs, in.H, (in.V + W - 1) / W), 256, lds, stream>>>(
+            o, scr, in, state, slot, pos, chunks, seqs, Dp, vec);
+}
+
+template <typename T, bool GEN>
+static int chunks_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
+                     const int* slot, const int* pos, const int* chunks,
+                     int n_chunks, const int* seqs, int n_seqs,
+                     hipStream_t stream)
+{
+    const int H = in.H, D = in.D, V = in.V, Dp = delta_pad(D);
+    if (D < 1 || V < 1 || D > 256) return (int)hipErrorInvalidValue;
+    const int v8 = D % 8 == 0 && in.oq % 8 == 0 && in.ok % 8 == 0
+                   && in.oa % 8 == 0 && in.ld % 8 == 0;
+    const int v4 = V % 4 == 0 && in.ov % 4 == 0 && in.ld % 4 == 0;
+    const int part = ((GEN ? 6 : 7) * CH * DS + 4 * DB) * 4;
+    const int solve = 2 * CH * AS * 4;
+    static bool once = false;
+    if (!once) {
+        (void)hipFuncSetAttribute(
+            (const void*)k_delta_prep<T, GEN>,
+            hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        once = true;
+    }
+    k_delta_prep<T, GEN><<<dim3(n_chunks, H), 256,
+                           part > solve ? part : solve, stream>>>(
+        scr, in, chunks, Dp, v8);
+    // wide strips share the loads of the factors, narrow ones fill the chip
+    const bool two = (int64_t)n_seqs * H * ((V + 31) / 32) >= 256;
+    #define DC(NS, VC)                                                     \
+        scan_go<T, NS, VC, GEN>(o, scr, in, state, slot, pos, chunks,      \
+                                seqs, n_seqs, Dp, v4, stream)
+    if (Dp <= 64) { if (two) DC(1, 2); else DC(1, 1); }
+    else if (Dp <= 128) { if (two) DC(2, 2); else DC(2, 1); }
+    else DC(4, 1);
+    #undef DC
+    return (int)hipGetLastError();
+}
+
+// Portions of whole sequences in chunks of 64 rows.  chunks int32 [n, 2]
+// (first row, rows), a sequence's chunks in a run; seqs int32 [m, 2] (first
+// chunk, chunks); D <= 256.
+extern "C" int delta_chunks(
+    int f32, int gen, void* o, void* scr, const void* x, int64_t ld, int oq,
+    int ok, int ov, int oa, const void* qs, const void* ks, int sld,
+    const void* decay, const void* beta, const void* a_bias, void* state,
+    const void* slot, const void* pos, const void* chunks, int n_chunks,
+    const void* seqs, int n_seqs, int H, int G, int D, int V,
+    hipStream_t stream)
+{
+    #define DC_GO(T, GEN)                                                  \
+        chunks_go<T, GEN>((float*)o, (float*)scr, DELTA_IN(T),             \
+                          (float*)state, (const int*)slot,                 \
+                          (const int*)pos, (const int*)chunks, n_chunks,   \
+                          (const int*)seqs, n_seqs, stream)
+    if (f32) return gen ? DC_GO(float, true) : DC_GO(float, false);
+    return gen ? DC_GO(bf16, true) : DC_GO(bf16, false);
+    #undef DC_GO
+}

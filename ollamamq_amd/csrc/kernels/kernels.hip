@@ -18,6 +18,7 @@
 #include <hip/hip_runtime.h>
 #include <hip/hip_bf16.h>
 #include <cstdint>
+#include "act.h"
 
 typedef __hip_bfloat16 bf16;
 typedef __hip_bfloat162 bf162;
@@ -459,8 +460,10 @@ extern "C" int paged_attn_bf16(
 }
 
 // ---------------------------------------------------------------------------
-// SwiGLU: [T, 2F] -> [T, F], silu(gate)*up, bf16 x8 vectorized, fp32 math.
+// Gated feed-forward: [T, 2F] -> [T, F], act(gate)*up, bf16 x8 vectorized,
+// fp32 math; act is silu or the tanh form of gelu.
 // ---------------------------------------------------------------------------
+template <int GELU>
 __global__ __launch_bounds__(256) void k_swiglu(
     bf16* __restrict__ out, const bf16* __restrict__ gu, int T, int F)
 {
@@ -475,13 +478,15 @@ __global__ __launch_bounds__(256) void k_swiglu(
         load8f(u, vu);
         #pragma unroll
         for (int e = 0; e < 8; e++) {
-            const float sig = 1.f / (1.f + __expf(-vg[e]));
+            const float z = GELU ? gelu_arg(vg[e]) : vg[e];
+            const float sig = 1.f / (1.f + __expf(-z));
             vg[e] = vg[e] * sig * vu[e];
         }
         store8bf(out + row * F + col8 * 8, vg);
     }
 }
 
+template <int GELU>
 __global__ __launch_bounds__(256) void k_swiglu_f32(
     float* __restrict__ out, const float* __restrict__ gu, int64_t total,
     int F)
@@ -489,27 +494,30 @@ __global__ __launch_bounds__(256) void k_swiglu_f32(
     for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
          i < total; i += (int64_t)gridDim.x * blockDim.x) {
         const float* g = gu + i / F * 2 * F + i % F;
-        out[i] = g[0] / (1.f + expf(-g[0])) * g[F];
+        const float z = GELU ? gelu_arg(g[0]) : g[0];
+        out[i] = g[0] / (1.f + expf(-z)) * g[F];
     }
 }
 
-extern "C" int swiglu_f32(void* out, const void* gu, int T, int F,
+extern "C" int swiglu_f32(void* out, const void* gu, int T, int F, int gelu,
                           hipStream_t stream)
 {
     const int64_t total = (int64_t)T * F;
     const int64_t want = (total + 255) / 256;
-    k_swiglu_f32<<<(int)(want < 4096 ? (want > 0 ? want : 1) : 4096), 256, 0,
-                   stream>>>((float*)out, (const float*)gu, total, F);
+    const int blocks = (int)(want < 4096 ? (want > 0 ? want : 1) : 4096);
+    auto go = gelu ? k_swiglu_f32<1> : k_swiglu_f32<0>;
+    go<<<blocks, 256, 0, stream>>>((float*)out, (const float*)gu, total, F);
     return (int)hipGetLastError();
 }
 
-extern "C" int swiglu_bf16(void* out, const void* gu, int T, int F,
+extern "C" int swiglu_bf16(void* out, const void* gu, int T, int F, int gelu,
                             hipStream_t stream)
 {
     const int64_t total = (int64_t)T * F / 8;
     const int64_t want = (total + 255) / 256;
     int blocks = (int)(want < 2048 ? (want > 0 ? want : 1) : 2048);
-    k_swiglu<<<blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gu, T, F);
+    auto go = gelu ? k_swiglu<1> : k_swiglu<0>;
+    go<<<blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gu, T, F);
     return (int)hipGetLastError();
 }
 

@@ -1,6 +1,6 @@
 // gfx950 lightning attention: per head a [D, V] fp32 state with one decay,
-//   S_t = r S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,   q, k, v = silu of their
-// columns in the fused projection.  The state and everything that enters it
+//   S_t = r S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,   q, k, v their columns in
+// the fused projection, or the silu of them.  The state and everything that enters it
 // beyond q, k and v is fp32: in bf16 models an fp32 operand of a matrix
 // product goes through the bf16 matrix cores as the sum of two bf16 terms.
 //
@@ -12,7 +12,7 @@
 //   the padded rows of q, k and v once; scan walks a sequence's chunks with
 //   the state in registers, a block per head and strip of value columns.
 // The results o [T, H, V] are fp32; the norm and gate that follow are
-// k_rms_gate.  A sequence starts where its position is 0: the state is then
+// k_rms_gate or k_head_gate.  A sequence starts where its position is 0: the state is then
 // taken as zero and whatever the slot held is ignored.
 #include "tile_mma.h"
 
@@ -20,7 +20,10 @@ template <typename T> DEV float silu_of(float x) {
     return x * sigmoid_of<T>(x);
 }
 
-struct Cols { int q, k, v; };         // first columns in the projection
+struct Cols { int q, k, v, act; };    // first columns in the projection
+template <typename T> DEV float act_of(const Cols& at, float x) {
+    return at.act ? silu_of<T>(x) : x;
+}
 
 #define CH 64                         // tokens of a chunk
 #define PW (CH + 1)                   // powers per head
@@ -69,16 +72,16 @@ __global__ __launch_bounds__(256, 2) void k_lightning_step(
         for (int d = tid; d < D; d += 256) {
             float x;
             ldrow<1>(p, t, at.q + h * D + d, &x);
-            q_s[d] = silu_of<T>(x);
+            q_s[d] = act_of<T>(at, x);
             ldrow<1>(p, t, at.k + h * D + d, &x);
-            k_s[d] = silu_of<T>(x);
+            k_s[d] = act_of<T>(at, x);
         }
         __syncthreads();
         if (on) {
             float v[VEC], acc[VEC] = {};
             ldrow<VEC>(p, t, at.v + h * V + v0 + vt, v);
             #pragma unroll
-            for (int i = 0; i < VEC; i++) v[i] = silu_of<T>(v[i]);
+            for (int i = 0; i < VEC; i++) v[i] = act_of<T>(at, v[i]);
             for (int d0 = rg; d0 < D; d0 += RG * PF) {
                 float s[PF][VEC];
                 #pragma unroll
@@ -113,7 +116,7 @@ __global__ __launch_bounds__(256, 2) void k_lightning_step(
 
 extern "C" int lightning_step(
     int f32, void* o, const void* p, int p32, int n_part,
-    int64_t part_stride, int64_t ld, int oq, int ok, int ov,
+    int64_t part_stride, int64_t ld, int oq, int ok, int ov, int act,
     const void* powers, void* state, const void* slot, const void* pos,
     const void* spans, int n, int H, int D, int V, hipStream_t stream)
 {
@@ -131,7 +134,7 @@ extern "C" int lightning_step(
     #define LS(T, P, VE)                                                   \
         k_lightning_step<T, P, VE><<<grid, 256, lds, stream>>>(            \
             (float*)o, Rows<P>{(const P*)p, n_part, part_stride, ld},      \
-            Cols{oq, ok, ov}, (const float*)powers, (float*)state,         \
+            Cols{oq, ok, ov, act}, (const float*)powers, (float*)state,         \
             (const int*)slot, (const int*)pos, (const int*)spans, H, D, V, \
             vb)
     #define LS_V(T, P) do { if (v4) LS(T, P, 4); else LS(T, P, 1); } while (0)
@@ -145,8 +148,8 @@ extern "C" int lightning_step(
 
 // ---- chunks --------------------------------------------------------------
 
-// a = q [H, rows, Dp], k [H, rows, Dp], v [H, rows, Vp]: their silu, filled up
-// with zeros
+// a = q [H, rows, Dp], k [H, rows, Dp], v [H, rows, Vp], activated and filled
+// up with zeros
 template <typename T, typename P, int VEC>
 __global__ __launch_bounds__(256) void k_lightning_act(
     T* __restrict__ a, Rows<P> p, Cols at, int row_base, int rows,
@@ -172,7 +175,7 @@ __global__ __launch_bounds__(256) void k_lightning_act(
         if (d < wide) {
             ldrow<VEC>(p, row_base + t, off + h * wide + d, v);
             #pragma unroll
-            for (int e = 0; e < VEC; e++) v[e] = silu_of<T>(v[e]);
+            for (int e = 0; e < VEC; e++) v[e] = act_of<T>(at, v[e]);
         }
         stv<VEC>(dst + ((int64_t)h * rows + t) * pad + d, v);
     }
@@ -455,7 +458,7 @@ extern "C" int64_t lightning_scratch(int rows, int H, int D, int V)
 // chunk, chunks); D <= 256.  Rows row_base .. row_base + rows - 1.
 extern "C" int lightning_chunks(
     int f32, void* o, void* scr, const void* p, int p32, int n_part,
-    int64_t part_stride, int64_t ld, int oq, int ok, int ov,
+    int64_t part_stride, int64_t ld, int oq, int ok, int ov, int act,
     const void* powers, void* state, const void* slot, const void* pos,
     const void* chunks, const void* seqs, int n_seqs, int row_base, int rows,
     int H, int D, int V, hipStream_t stream)
@@ -470,7 +473,7 @@ extern "C" int lightning_chunks(
     #define LA_GO(T, P, VE)                                                \
         k_lightning_act<T, P, VE><<<ga, 256, 0, stream>>>(                 \
             (T*)scr, Rows<P>{(const P*)p, n_part, part_stride, ld},        \
-            Cols{oq, ok, ov}, row_base, rows, total, H, D, V, Dp, Vp)
+            Cols{oq, ok, ov, act}, row_base, rows, total, H, D, V, Dp, Vp)
     #define LA_V(T, P)                                                     \
         do { if (v8) LA_GO(T, P, 8); else LA_GO(T, P, 1); } while (0)
     if (f32) LA_V(float, float);

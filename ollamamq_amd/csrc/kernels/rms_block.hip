@@ -14,8 +14,8 @@
 //
 // Also here: the split of a fused query/key/value projection with an RMS
 // norm over all queries and over all keys of a token, and the append of keys
-// and values to the paged pools; and the norm over all heads of a token with
-// a sigmoid gate.
+// and values to the paged pools; and the norm over all heads of a token, or
+// of every head by itself, with a gate.
 #include "route.h"
 
 // sum_s share[s] * y[s * stride] (share null: all ones)
@@ -456,5 +456,80 @@ extern "C" int rms_gate(
     else RG_N(bf16, bf16, false);
     #undef RG_N
     #undef RG
+    return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// out = N(mult * o) * w * gate, the norm over every head of V columns by
+// itself; w is shared by the heads (w_stride 0), per head (V) or null; the
+// gate the sigmoid or silu of a column range of a projection.  A group of L
+// lanes per head of a token.
+// ---------------------------------------------------------------------------
+template <typename T, typename P, int VEC, bool FR>
+__global__ __launch_bounds__(256) void k_head_gate(
+    T* __restrict__ out, const float* __restrict__ o, float mult,
+    const float* __restrict__ w, int w_stride, Rows<P> gate, int og,
+    int silu, int64_t units, int H, int V, int L, float eps)
+{
+    const int lane = threadIdx.x & (L - 1);
+    const int64_t u = ((int64_t)blockIdx.x * 256 + threadIdx.x) / L;
+    if (u >= units) return;
+    const int64_t t = u / H;
+    const int h = (int)(u % H);
+    const float* row = o + u * V;
+    const bool one = V <= L * VEC;          // the head fits the lanes
+    float x[VEC], s = 0.f;
+    for (int c = lane * VEC; c < V; c += L * VEC) {
+        ldv<VEC>(row + c, x);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) s += x[i] * x[i];
+    }
+    for (int k = L / 2; k; k >>= 1) s += __shfl_xor(s, k, 64);
+    const float f = mult / sqrtf(s * (mult * mult / V) + eps);
+    for (int c = lane * VEC; c < V; c += L * VEC) {
+        float g[VEC];
+        if (!one) ldv<VEC>(row + c, x);
+        ldrow<VEC>(gate, t, og + h * V + c, g);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++)
+            x[i] *= f * sigmoid_of<T>(g[i]) * (silu ? g[i] : 1.f);
+        if (w) {
+            ldv<VEC>(w + h * w_stride + c, g);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) x[i] *= g[i];
+        }
+        const int n = h * V + c;
+        stv<VEC>(out + (FR ? frag_row_off(t, n, H * V)
+                           : t * (int64_t)H * V + n), x);
+    }
+}
+
+extern "C" int head_gate(
+    int f32, void* out, const void* o, float mult, const void* w,
+    int w_stride, const void* gate, int p32, int n_part, int64_t part_stride,
+    int64_t ld, int og, int silu, int T_rows, int H, int V, float eps,
+    int frag, hipStream_t stream)
+{
+    const bool v4 = V % 4 == 0 && og % 4 == 0 && ld % 4 == 0
+                    && part_stride % 4 == 0;
+    if (frag && f32) return (int)hipErrorInvalidValue;
+    int L = 64;
+    while (L > 4 && L / 2 * (v4 ? 4 : 1) >= V) L /= 2;
+    const int64_t units = (int64_t)T_rows * H;
+    const int grid = (int)((units * L + 255) / 256);
+    #define HG(T, P, VE, FR)                                               \
+        k_head_gate<T, P, VE, FR><<<grid, 256, 0, stream>>>(               \
+            (T*)out, (const float*)o, mult, (const float*)w, w_stride,     \
+            Rows<P>{(const P*)gate, n_part, part_stride, ld}, og, silu,    \
+            units, H, V, L, eps)
+    #define HG_V(T, P, FR)                                                 \
+        do { if (v4) HG(T, P, 4, FR); else HG(T, P, 1, FR); } while (0)
+    if (f32) HG_V(float, float, false);
+    else if (frag && p32) HG_V(bf16, float, true);
+    else if (frag) HG_V(bf16, bf16, true);
+    else if (p32) HG_V(bf16, float, false);
+    else HG_V(bf16, bf16, false);
+    #undef HG_V
+    #undef HG
     return (int)hipGetLastError();
 }

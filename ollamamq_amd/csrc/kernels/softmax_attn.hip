@@ -4,8 +4,10 @@
 //   out = sum exp(score) v / (sum exp(score) + exp(sink))
 //
 // The sink, a number per query head, is one more term of the denominator and
-// is optional, as is the window.  Scores, maxima and sums are fp32; in bf16
-// models exponents are taken in base 2.
+// is optional, as is the window.  Instead of a window a query may see its own
+// chunk of positions, counted from the sequence's first.  A head's result may
+// be gated by the sigmoid of a projected number.  Scores, maxima and sums are
+// fp32; in bf16 models exponents are taken in base 2.
 //
 // All heads of a key/value head are rows of one tile: row = token * R + head
 // within the group, R = H / G, so a staged key serves the whole group.
@@ -17,8 +19,32 @@
 struct Soft {
     float scale;
     const float* sink;                // per query head, or null
-    int window;                       // 0: every earlier key
+    int window, chunk;                // both 0: every earlier key
 };
+// first key that a query at position p sees
+DEV int first_seen(const Soft& rule, int p) {
+    if (rule.window > 0) return max(0, p - rule.window + 1);
+    return rule.chunk > 0 ? p - p % rule.chunk : 0;
+}
+
+// Column `first` + head of a projection, or nothing
+struct HeadGate {
+    const void* p;
+    int f32, n_part;
+    int64_t part_stride, ld;
+    int first;
+};
+template <typename T> DEV float gate_of(const HeadGate& q, int64_t t, int h) {
+    if (!q.p) return 1.f;
+    float z;
+    if (sizeof(T) == 4 || q.f32)
+        ldrow<1>(Rows<float>{(const float*)q.p, q.n_part, q.part_stride, q.ld},
+                 t, q.first + h, &z);
+    else
+        ldrow<1>(Rows<T>{(const T*)q.p, q.n_part, q.part_stride, q.ld}, t,
+                 q.first + h, &z);
+    return sigmoid_of<T>(z);
+}
 
 // exponentials and the units of a score they take
 template <typename T> struct Expo;
@@ -32,10 +58,10 @@ template <> struct Expo<bf16> {
 };
 
 // Scores of N tiles of 16 keys become weights; m, l: the row's running
-// maximum and sum.  Returns what the row's earlier results are scaled by.
-// A row may have seen no key yet: its weights stay zero.
+// maximum and sum; the row sees `span` tokens, itself included.  Returns what
+// the row's earlier results are scaled by.  A row may have seen no key yet: its weights stay zero.
 template <typename T, int N>
-DEV float soften(f32x4* s, float c, bool masked, int dist0, int window,
+DEV float soften(f32x4* s, float c, bool masked, int dist0, int span,
                  float& m, float& l) {
     float mx = NEG;
     #pragma unroll
@@ -45,7 +71,7 @@ DEV float soften(f32x4* s, float c, bool masked, int dist0, int window,
             float v = s[j][i] * c;
             if (masked) {
                 const int d = dist0 - j * 16 - i;
-                if (d < 0 || (window > 0 && d >= window)) v = NEG;
+                if (d < 0 || d >= span) v = NEG;
             }
             s[j][i] = v;
             mx = fmaxf(mx, v);
@@ -95,7 +121,8 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 && DT <= 4 && VT <= 8
     const int* __restrict__ ptab, const int* __restrict__ slot,
     const int* __restrict__ pos,
     const int* __restrict__ items,     // [n, 2] first row, rows
-    int H, int G, int V, int Dp, int Vp, int pshift, int maxp, Soft rule)
+    int H, int G, int V, int Dp, int Vp, int pshift, int maxp, Soft rule,
+    HeadGate gate)
 {
     constexpr int KT = 64;
     constexpr int PAD = 16 / sizeof(T);
@@ -109,20 +136,22 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 && DT <= 4 && VT <= 8
     const int pos0 = pos[tok0], pos1 = pos[tok1];
     const int* pt = ptab + (int64_t)slot[tok0] * maxp;
     const int kv_len = pos1 + 1;
-    const int seen = rule.window > 0 ? max(0, pos0 - rule.window + 1) : 0;
+    const int seen = first_seen(rule, pos0);
+    const int last = first_seen(rule, pos1);
     const int c_lo = seen / KT, c_hi = (kv_len + KT - 1) / KT;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     T* k_s = reinterpret_cast<T*>(smem);          // [KT][KS]
     T* v_s = k_s + KT * KS;                       // [KT][VS]
 
     Frag<T> qf[NQ][DT];
-    int qpos[NQ], tok[NQ], head[NQ];
+    int qpos[NQ], tok[NQ], head[NQ], span[NQ];
     #pragma unroll
     for (int n = 0; n < NQ; n++) {
         const int f = row0 + min((wid * NQ + n) * 16 + lr, n_rows - 1);
         tok[n] = f / R;
         head[n] = kvh * R + f % R;
         qpos[n] = pos[tok[n]];
+        span[n] = qpos[n] - first_seen(rule, qpos[n]) + 1;
         const T* qr = q + ((int64_t)tok[n] * H + head[n]) * Dp;
         #pragma unroll
         for (int d = 0; d < DT; d++) {
@@ -209,13 +238,12 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 && DT <= 4 && VT <= 8
                         s[n][kt] = mma(a, qf[n][d], s[n][kt]);
                 }
             }
-            const bool inside = base + KT - 1 <= pos0
-                && (rule.window <= 0 || base > pos1 - rule.window);
+            const bool inside = base + KT - 1 <= pos0 && base >= last;
             #pragma unroll
             for (int n = 0; n < NQ; n++) {
                 const int dist0 = qpos[n] - base - g * 4;
                 const float f = soften<T, 4>(s[n], unit, !inside, dist0,
-                                             rule.window, m[n], l[n]);
+                                             span[n], m[n], l[n]);
                 if (!__all(f == 1.f)) {
                     #pragma unroll
                     for (int v = 0; v < VT; v++) o[n][v] *= f;
@@ -242,7 +270,8 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 && DT <= 4 && VT <= 8
     #pragma unroll
     for (int n = 0; n < NQ; n++) {
         if ((wid * NQ + n) * 16 + lr >= n_rows) continue;
-        const float f = finish<T>(m[n], l[n], rule.sink, head[n]);
+        const float f = finish<T>(m[n], l[n], rule.sink, head[n])
+                        * gate_of<T>(gate, tok[n], head[n]);
         #pragma unroll
         for (int v = 0; v < VT; v++)
             put_out(out, tok[n], head[n], v * 16 + g * 4, H, V, o[n][v] * f,
@@ -266,7 +295,7 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
     const int* __restrict__ slot, const int* __restrict__ pos,
     const int* __restrict__ items,     // null: decode, per_seq a token
     int per_seq, int T_rows, int H, int G, int V, int Dp, int Vp, int pshift,
-    int maxp, int split, int frag, Soft rule)
+    int maxp, int split, int frag, Soft rule, HeadGate gate)
 {
     constexpr int KT = 32, PAD = 16 / sizeof(T), VS = VT * 16 + PAD;
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
@@ -285,7 +314,7 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
     const int pos0 = pos[tok0], pos1 = pos[tok1];
     const int* pt = ptab + (int64_t)slot[tok0] * maxp;
     const int kv_len = pos1 + 1;
-    const int seen = rule.window > 0 ? max(0, pos0 - rule.window + 1) : 0;
+    const int seen = first_seen(rule, pos0);
     const int first = seen / KT;
     const int steps = (kv_len + KT - 1) / KT - first;
     // this wave's steps: every GW-th
@@ -297,6 +326,7 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
     const int f = row0 + min(lr, n_rows - 1);
     const int tok = f / R, head = kvh * R + f % R;
     const int qpos = pos[tok];
+    const int span = qpos - first_seen(rule, qpos) + 1;
     Frag<T> qf[DT], kf[2][DT], vr[VT];
     {
         const T* qr = q + ((int64_t)tok * H + head) * Dp;
@@ -367,8 +397,7 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
             pages(st + 2 * GW);
         }
         const int dist0 = qpos - base - g * 4;
-        const float f = soften<T, 2>(s, unit, true, dist0, rule.window, m,
-                                     l);
+        const float f = soften<T, 2>(s, unit, true, dist0, span, m, l);
         if (!__all(f == 1.f)) {
             #pragma unroll
             for (int v = 0; v < VT; v++) acc[v] *= f;
@@ -407,7 +436,8 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
         o_s[(wid * VT + v) * 64 + lane] = acc[v] * mine;
     __syncthreads();
     if (lr >= n_rows) return;
-    const float f0 = split > 1 ? 1.f : finish<T>(top, den, rule.sink, head);
+    const float f0 = split > 1 ? 1.f : finish<T>(top, den, rule.sink, head)
+                                       * gate_of<T>(gate, tok, head);
     for (int v = wid; v < VT; v += NW) {
         f32x4 t = o_s[v * 64 + lane];
         #pragma unroll
@@ -428,8 +458,9 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void k_softmax_combine(
     T* __restrict__ out, const float* __restrict__ part,
-    const float* __restrict__ ml, const float* __restrict__ sink, int t0,
-    int n, int T_rows, int H, int V, int split, int frag)
+    const float* __restrict__ ml, const float* __restrict__ sink,
+    HeadGate gate, int t0, int n, int T_rows, int H, int V, int split,
+    int frag)
 {
     const int N = H * V;
     const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * VEC;
@@ -449,7 +480,7 @@ __global__ __launch_bounds__(256) void k_softmax_combine(
         #pragma unroll
         for (int e = 0; e < VEC; e++) v[e] += w * u[e];
     }
-    const float f = finish<T>(top, den, sink, h);
+    const float f = finish<T>(top, den, sink, h) * gate_of<T>(gate, t, h);
     #pragma unroll
     for (int e = 0; e < VEC; e++) v[e] *= f;
     stv<VEC>(out + (frag ? frag_row_off(t, c, N) : (int64_t)t * N + c), v);
@@ -462,7 +493,7 @@ static int softmax_go(
     const void* vpool, const void* ptab, const void* slot, const void* pos,
     const void* items, int n_items, int per_seq, int T_rows, int H, int G,
     int V, int Dp, int Vp, int pshift, int maxp, int split, int frag,
-    Soft rule, hipStream_t stream)
+    Soft rule, HeadGate gate, hipStream_t stream)
 {
     constexpr int PAD = 16 / sizeof(T);
     if (item_rows == 16) {
@@ -482,7 +513,7 @@ static int softmax_go(
                 (T*)out, (float*)part, (float*)ml, (const T*)q,
                 (const T*)kpool, (const T*)vpool, (const int*)ptab, (const int*)slot,
                 (const int*)pos, (const int*)items, per_seq, T_rows, H, G, V,
-                Dp, Vp, pshift, maxp, split, frag, rule);
+                Dp, Vp, pshift, maxp, split, frag, rule, gate);
     } else {
         constexpr int NQ = sizeof(T) == 4 || DT == 8 || VT == 16 ? 1 : 2;
         auto go = item_rows > 64 ? k_softmax_flash<T, DT, VT, NQ>
@@ -501,7 +532,8 @@ static int softmax_go(
         go<<<dim3(G, n_items), 256, lds, stream>>>(
                 (T*)out, (const T*)q, (const T*)kpool, (const T*)vpool,
                 (const int*)ptab, (const int*)slot, (const int*)pos,
-                (const int*)items, H, G, V, Dp, Vp, pshift, maxp, rule);
+                (const int*)items, H, G, V, Dp, Vp, pshift, maxp, rule,
+                gate);
     }
     return (int)hipGetLastError();
 }
@@ -523,7 +555,8 @@ extern "C" int softmax_attn(
     const void* pos, const void* items, int n_items, int t0, int n_tok,
     int T_rows, int H, int G, int V, int Dp, int Vp, int psz, int maxp,
     int split, int frag, float scale, const void* sink, int window,
-    hipStream_t stream)
+    int chunk, const void* gate_p, int g32, int g_parts, int64_t g_stride,
+    int64_t g_ld, int og, hipStream_t stream)
 {
     if (psz & (psz - 1) || Dp % 8 || Vp % 8 || Dp > 256 || Vp > 256
         || (frag && (f32 || V % 4))
@@ -532,14 +565,15 @@ extern "C" int softmax_attn(
         return (int)hipErrorInvalidValue;
     const int pshift = __builtin_ctz(psz);
     const int per_seq = (H / G + 15) / 16;
-    Soft rule{scale, (const float*)sink, window};
+    Soft rule{scale, (const float*)sink, window, chunk};
+    const HeadGate gate{gate_p, g32, g_parts, g_stride, g_ld, og};
     int err;
     #define SA(T, D_, V_)                                                  \
         err = softmax_go<T, D_, V_>(                                       \
             item_rows, out, part, ml, q, kpool, vpool, ptab, slot, pos,    \
             items,                                                         \
             n_items, per_seq, T_rows, H, G, V, Dp, Vp, pshift, maxp,       \
-            split, frag, rule, stream)
+            split, frag, rule, gate, stream)
     #define SA_V(T, D_)                                                    \
         do {                                                               \
             if (Vp <= 64) SA(T, D_, 4);                                    \
@@ -564,7 +598,7 @@ extern "C" int softmax_attn(
         k_softmax_combine<T, VE>                                           \
             <<<(int)((all / VE + 255) / 256), 256, 0, stream>>>(           \
                 (T*)out, (const float*)part, (const float*)ml,             \
-                (const float*)sink, t0, n_tok, T_rows, H, V, split, frag)
+                (const float*)sink, gate, t0, n_tok, T_rows, H, V, split, frag)
     if (f32) { if (V % 4) SC(float, 1); else SC(float, 4); }
     else { if (V % 4) SC(bf16, 1); else SC(bf16, 4); }
     #undef SC

@@ -27,6 +27,7 @@
 // any K%64==0, N%32==0, M<=64).  Wave partials meet in a single
 // end-of-kernel LDS reduce (the ONE barrier, after all streaming).
 // ksplit>1 writes fp32 partials; k_wstream_combine folds them (+bias).
+#include "act.h"
 #include "tile_mma.h"
 
 typedef __attribute__((ext_vector_type(16))) float f32x16;
@@ -87,7 +88,7 @@ extern "C" int wstream_pure_bf16(void* sink, const void* wp, int N, int K,
 // packed with gate and up INTERLEAVED (tile t = 16 gate rows f=t*16..+16
 // then the 16 matching up rows — ops/hip.py pack_weight_gu), so each
 // block's 32-column output tile holds the (gate, up) pairs of 16 ffn
-// columns; the epilogue computes silu(g)*u and stores [M, 16] of the
+// columns; the epilogue computes silu(g)*u (GU == 2: gelu_tanh(g)*u) and stores [M, 16] of the
 // activation directly.  Kills the separate swiglu kernel (9.7 us x 32
 // layers/step in the r02 trace) and the gate_up intermediate round-trip.
 // Fused-rmsnorm chain extensions (all nullable; tp=1 decode path):
@@ -349,7 +350,8 @@ __global__ __launch_bounds__(512) void k_wstream_gemm(
                     sg *= rs;
                     su *= rs;
                 }
-                const float act = (sg / (1.f + __expf(-sg))) * su;
+                const float z = GU == 2 ? gelu_arg(sg) : sg;
+                const float act = (sg / (1.f + __expf(-z))) * su;
                 const int fc = t * 16 + c;
                 y[yfrag ? (int64_t)mt * 32 * F + frag_off(m, fc)
                         : (int64_t)gm * F + fc] = __float2bfloat16(act);
@@ -503,7 +505,8 @@ __global__ __launch_bounds__(512) void k_wstream_gemm(
 // Fused gate_up @ SwiGLU over GU-interleaved packed weights.
 // N = 2F total weight rows; output is the activation [M, F].
 // rstd_parts: optional fused-rmsnorm scale of the raw-residual input.
-extern "C" int wstream_gu_bf16(
+template <int GU>
+static int wstream_gu(
     void* act, const void* x, const void* wp, int M, int N, int K,
     int64_t xs, int xlds, const void* rstd_parts, int rstd_nt,
     float inv_h, float eps, int yfrag, hipStream_t stream)
@@ -512,37 +515,39 @@ extern "C" int wstream_gu_bf16(
     const int lds = (xlds == 1 ? 16 * 4096 : 8 * 32 * 32 * 4) + 256;
     if (M > 32) {
         if (xlds == 2) {       // frag chain at batches 33..64
-            k_wstream_gemm<2, 1, 2, 1><<<grid, 512, lds, stream>>>(
+            k_wstream_gemm<2, 1, 2, GU><<<grid, 512, lds, stream>>>(
                 (bf16*)act, nullptr, (const bf16*)x, (const u32x4*)wp,
                 nullptr, M, N, K, xs, 1, (const float*)rstd_parts,
                 rstd_nt, inv_h, eps, nullptr, nullptr, {}, yfrag);
             return (int)hipGetLastError();
         }
-        // generic-path fused gate_up+SwiGLU, direct x loads (unused by
-        // default: measured below lib at 64 users)
+        // generic-path fused product and activation, direct x loads (unused
+        // by default: measured below lib at 64 users)
         if (rstd_parts || yfrag) return -102;
-        k_wstream_gemm<2, 1, 0, 1><<<grid, 512, lds, stream>>>(
+        k_wstream_gemm<2, 1, 0, GU><<<grid, 512, lds, stream>>>(
             (bf16*)act, nullptr, (const bf16*)x, (const u32x4*)wp,
             nullptr, M, N, K, xs, 1, nullptr, 0, 0.f, 0.f,
             nullptr, nullptr, {}, 0);
         return (int)hipGetLastError();
     }
-    if (xlds == 2)
-        k_wstream_gemm<1, 1, 2, 1><<<grid, 512, lds, stream>>>(
-            (bf16*)act, nullptr, (const bf16*)x, (const u32x4*)wp,
-            nullptr, M, N, K, xs, 1, (const float*)rstd_parts, rstd_nt,
-            inv_h, eps, nullptr, nullptr, {}, yfrag);
-    else if (xlds == 1)
-        k_wstream_gemm<1, 1, 1, 1><<<grid, 512, lds, stream>>>(
-            (bf16*)act, nullptr, (const bf16*)x, (const u32x4*)wp,
-            nullptr, M, N, K, xs, 1, (const float*)rstd_parts, rstd_nt,
-            inv_h, eps, nullptr, nullptr, {}, yfrag);
-    else
-        k_wstream_gemm<1, 1, 0, 1><<<grid, 512, lds, stream>>>(
-            (bf16*)act, nullptr, (const bf16*)x, (const u32x4*)wp,
-            nullptr, M, N, K, xs, 1, (const float*)rstd_parts, rstd_nt,
-            inv_h, eps, nullptr, nullptr, {}, yfrag);
+    auto go = xlds == 2 ? k_wstream_gemm<1, 1, 2, GU>
+              : xlds == 1 ? k_wstream_gemm<1, 1, 1, GU>
+                          : k_wstream_gemm<1, 1, 0, GU>;
+    go<<<grid, 512, lds, stream>>>(
+        (bf16*)act, nullptr, (const bf16*)x, (const u32x4*)wp,
+        nullptr, M, N, K, xs, 1, (const float*)rstd_parts, rstd_nt,
+        inv_h, eps, nullptr, nullptr, {}, yfrag);
     return (int)hipGetLastError();
+}
+
+extern "C" int wstream_gu_bf16(
+    void* act, const void* x, const void* wp, int M, int N, int K,
+    int64_t xs, int xlds, const void* rstd_parts, int rstd_nt,
+    float inv_h, float eps, int yfrag, int gelu, hipStream_t stream)
+{
+    return (gelu ? wstream_gu<2> : wstream_gu<1>)(
+        act, x, wp, M, N, K, xs, xlds, rstd_parts, rstd_nt, inv_h, eps,
+        yfrag, stream);
 }
 
 

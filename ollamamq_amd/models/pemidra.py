@@ -295,7 +295,7 @@ class PemidraLayer(HybridLayer):
                 heads=m.heads, dim=m.dim, vdim=m.vdim,
                 offsets=tuple(_offsets([qk, qk, v, v])),
                 powers=ops.decay_powers(m.decay, self.ls1.device), norm=None,
-                eps=eps, act=False, key_scale=m.dim ** -0.5, per_head=True,
+                eps=eps, act=False, scale=m.dim ** -0.5, per_head=True,
                 gate="silu")
             outs = [("w_o", "o", v)]
         elif spec.type == "general_delta":

@@ -14,8 +14,8 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .interface import (LIGHTNING_CHUNK, AttnMeta, FragRows, Partials,
-                        Weighted)
+from .interface import (LIGHTNING_CHUNK, AttnMeta, Branches, FragRows,
+                        Partials, Weighted)
 
 _LIB_PATH = os.path.join(
     os.path.dirname(os.path.dirname(os.path.abspath(__file__))),
@@ -43,7 +43,7 @@ def _try_load():
                                    i, i, i, i, i, i64, vp]
     lib.paged_attn_bf16.argtypes = [vp, vp, vp, vp, vp, vp, vp, vp, vp,
                                     i, i, i, i, i, i, f, i64, vp]
-    lib.swiglu_bf16.argtypes = [vp, vp, i, i, vp]
+    lib.swiglu_bf16.argtypes = [vp, vp, i, i, i, vp]
     lib.swiglu_f32.argtypes = lib.swiglu_bf16.argtypes
     lib.argmax_bf16.argtypes = [vp, vp, i, i, vp, vp, i, vp]
     lib.argmax_f32.argtypes = lib.argmax_bf16.argtypes
@@ -61,7 +61,7 @@ def _try_load():
                                       i, i, vp, i, f, f, vp, vp, i, vp]
     lib.wstream_pure_bf16.argtypes = [vp, vp, i, i, i, vp]
     lib.wstream_gu_bf16.argtypes = [vp, vp, vp, i, i, i, i64, i,
-                                    vp, i, f, f, i, vp]
+                                    vp, i, f, f, i, i, vp]
     lib.row_sumsq_bf16.argtypes = [vp, vp, i, i, vp]
     lib.fragify_sumsq_bf16.argtypes = [vp, vp, vp, i, i, vp]
     lib.sample_gumbel_bf16.argtypes = [vp, vp, vp, vp, vp, vp, i, i,
@@ -93,11 +93,30 @@ def _try_load():
     lib.softmax_step.argtypes = [i]
     lib.softmax_attn.argtypes = [i, i, vp, vp, vp, vp, vp, vp, vp, vp, vp,
                                  vp, i, i, i, i, i, i, i, i, i, i, i, i, i,
-                                 f, vp, i, vp]
+                                 f, vp, i, i, *rows, i, vp]
+    lib.qkv_norm_rope.argtypes = [i, vp, vp, vp, *rows, vp, vp, vp, i, f, vp,
+                                  i, vp, vp, vp, i, i, i, i, i, i, i, i, i,
+                                  vp]
+    lib.head_gate.argtypes = [i, vp, vp, f, vp, i, *rows, i, i, i, i, i, f, i,
+                              vp]
+    lib.ln_residual.argtypes = [i, vp, vp, vp, vp, vp, vp, i, i, i64, vp, i,
+                                i, i64, vp, vp, f, vp, vp, vp, f, vp, vp, f,
+                                vp, i, i, i, vp]
+    lib.gated_rows.argtypes = [i, *rows, i, i, i, i, i, i, vp, i, vp, vp, vp,
+                               vp, i, vp, vp, vp, vp, vp, vp, vp, vp, vp, i,
+                               i, i, i, i, vp]
+    lib.general_rows.argtypes = [i, *rows, i, i, i, vp, vp, vp, vp, vp, i, i,
+                                 i, i, vp]
+    delta = [vp, i64, i, i, i, i, vp, vp, i, vp, vp, vp, vp, vp, vp]
+    lib.delta_step.argtypes = [i, i, vp, *delta, vp, i, i, i, i, i, vp]
+    lib.delta_chunks.argtypes = [i, i, vp, vp, *delta, vp, i, vp, i, i, i, i,
+                                 i, vp]
+    lib.delta_scratch_floats.argtypes = [i, i, i, i]
+    lib.delta_scratch_floats.restype = i64
     lib.rms_gate.argtypes = [i, vp, vp, vp, *rows, i, i, i, f, i, vp]
-    lib.lightning_step.argtypes = [i, vp, *rows, i, i, i, vp, vp, vp, vp, vp,
-                                   i, i, i, i, vp]
-    lib.lightning_chunks.argtypes = [i, vp, vp, *rows, i, i, i, vp, vp, vp,
+    lib.lightning_step.argtypes = [i, vp, *rows, i, i, i, i, vp, vp, vp, vp,
+                                   vp, i, i, i, i, vp]
+    lib.lightning_chunks.argtypes = [i, vp, vp, *rows, i, i, i, i, vp, vp, vp,
                                      vp, vp, vp, i, i, i, i, i, i, vp]
     lib.lightning_scratch.argtypes = [i, i, i, i]
     lib.lightning_scratch.restype = i64
@@ -521,9 +540,13 @@ def pack_weight_gu(w):
     return p.view(-1)
 
 
+GELU = {"silu": 0, "gelu_tanh": 1}      # activations of a gate
+
+
 def linear_gu(x, packed, N, rstd=None, rstd_nt=0, inv_h=0.0, eps=0.0,
-              K=None, yfrag=0, M_frag=32):
-    """act = swiglu(x @ Wgu^T) fused; N = 2F total weight rows.
+              K=None, yfrag=0, M_frag=32, glu="silu"):
+    """act = swiglu(x @ Wgu^T) fused; N = 2F total weight rows; glu names
+    the activation of the gate.
     With rstd: x is the raw residual and the epilogue applies the
     rmsnorm scale before SwiGLU (norm weight folded into the pack).
     K given => x is a frag-layout buffer (xlds=2); yfrag => the
@@ -540,7 +563,7 @@ def linear_gu(x, packed, N, rstd=None, rstd_nt=0, inv_h=0.0, eps=0.0,
                       dtype=x.dtype, device=x.device)
     _check(_lib.wstream_gu_bf16(
         _p(act), _p(x), _p(packed), M, N, K, xs, xlds,
-        _p(rstd), rstd_nt, float(inv_h), float(eps), yfrag,
+        _p(rstd), rstd_nt, float(inv_h), float(eps), yfrag, GELU[glu],
         _stream()), "wstream_gu")
     return act
 
@@ -766,14 +789,14 @@ def linear(x, weight, bias=None, packed=None):
     return torch.nn.functional.linear(x, weight, bias)
 
 
-def swiglu(gate_up):
+def swiglu(gate_up, act="silu"):
     T, F2 = gate_up.shape
     F = F2 // 2
     out = torch.empty((T, F), dtype=gate_up.dtype, device=gate_up.device)
     f32 = _is_f32(gate_up)
     assert gate_up.is_contiguous() and (f32 or F % 8 == 0)
     fn = _lib.swiglu_f32 if f32 else _lib.swiglu_bf16
-    _check(fn(_p(out), _p(gate_up), T, F, _stream()),
+    _check(fn(_p(out), _p(gate_up), T, F, GELU[act], _stream()),
            "swiglu")
     return out
 
@@ -849,9 +872,10 @@ def linear_f32(x, weight, packed=None):
     return torch.mm(x, weight.t(), out_dtype=torch.float32)
 
 
-def linear_gu_frag(x, packed, N):
+def linear_gu_frag(x, packed, N, glu="silu"):
     """linear_gu of an activation in fragment layout, and so its result."""
-    act = linear_gu(x.buf, packed, N, K=x.cols, yfrag=1, M_frag=x.rows)
+    act = linear_gu(x.buf, packed, N, K=x.cols, yfrag=1, M_frag=x.rows,
+                    glu=glu)
     return FragRows(act, x.rows, N // 2)
 
 
@@ -1273,14 +1297,16 @@ def lightning(p, w, state, slot_ids, positions, meta, frag=False):
     f32 = int(dtype == torch.float32)
     oq, ok, ov, og = w.offsets
     assert state.dtype == torch.float32 and state.is_contiguous() \
-        and state.shape[1:] == (H, D, V) and w.norm.numel() == H * V \
+        and state.shape[1:] == (H, D, V) \
+        and (w.norm is None or w.norm.numel() == H * V) \
         and w.powers.shape == (H, LIGHTNING_CHUNK + 1) \
         and w.powers.is_contiguous() \
         and max(oq + H * D, ok + H * D, ov + H * V, og + H * V) <= t.shape[-1]
     assert not frag or meta.one_each
     o = torch.empty((T, H * V), dtype=torch.float32, device=t.device)
     slots, pos = _i32(slot_ids), _i32(positions)
-    head = (*rows, oq, ok, ov, _p(w.powers), _p(state), _p(slots), _p(pos))
+    head = (*rows, oq, ok, ov, int(w.act), _p(w.powers), _p(state),
+            _p(slots), _p(pos))
     nd = meta.n_single
     if nd:
         _check(_lib.lightning_step(f32, _p(o), *head, _p(None), nd, H, D, V,
@@ -1300,6 +1326,11 @@ def lightning(p, w, state, slot_ids, positions, meta, frag=False):
                 f32, _p(o), _p(scr), *head, _p(chunks), _p(seqs),
                 seqs.shape[0], base, n, H, D, V, _stream()),
                 "lightning_chunks")
+    if w.per_head:
+        return head_gate(o, w.norm, p, og, w.gate, dtype, H, V, w.eps, frag,
+                         w.scale)
+    if w.gate != "sigmoid" or w.norm is None or w.scale != 1.0:
+        raise ValueError("norm over all heads: weight and sigmoid gate only")
     N = H * V
     if frag:
         res = _frag_rows(T, N, t)
@@ -1311,6 +1342,147 @@ def lightning(p, w, state, slot_ids, positions, meta, frag=False):
                              N, float(w.eps), int(frag), _stream()),
                "rms_gate")
     return res
+
+
+def head_gate(o, norm, gate, og, act, dtype, H, V, eps, frag, mult=1.0):
+    """Every head of mult * o [T, H*V] fp32 normed by itself, times the
+    weight (shared [V], [H*V] or None) and the sigmoid or silu of the gate's
+    columns og.."""
+    T = o.shape[0]
+    assert act in ("sigmoid", "silu") and _cols(gate) >= og + H * V \
+        and (norm is None or norm.numel() in (V, H * V))
+    if frag:
+        res = _frag_rows(T, H * V, o)
+        out = res.buf
+    else:
+        res = out = torch.empty((T, H * V), dtype=dtype, device=o.device)
+    stride = V if norm is not None and norm.numel() == H * V else 0
+    if T:
+        _check(_lib.head_gate(
+            int(dtype == torch.float32), _p(out), _p(o), float(mult),
+            _p(norm), stride, *_rows(gate), og, int(act == "silu"), T, H, V,
+            float(eps), int(frag), _stream()), "head_gate")
+    return res
+
+
+DELTA_STEP_TOKENS = 4    # portions up to this walk token by token
+DELTA_MAX_D = 256        # key width the chunk kernels take
+CONV_STRIP = 16          # tokens of a portion that one wave convolves
+
+
+def _conv_strips(meta, taps, dev):
+    """Strips of the portions, int32 [n, 4]: first row, rows, the portion's
+    first row and end.  No strip but a portion's first reads inputs from
+    before the portion."""
+    size = max(CONV_STRIP, taps - 1)
+    key = f"_strips_{size}"
+    t = getattr(meta, key, None)
+    if t is None:
+        strips, row = [], 0
+        for n in meta.layout()[1]:
+            strips += [(row + i, min(size, n - i), row, row + n)
+                       for i in range(0, n, size)]
+            row += n
+        t = torch.tensor(strips, dtype=torch.int32).to(dev)
+        setattr(meta, key, t)
+    return t
+
+
+def _delta(gen, x, offsets, qs, ks, decay, beta, a_bias, state, G, slots, pos,
+           meta):
+    """The recurrence over prepared rows -> o [T, H*V] fp32."""
+    H, D, V = state.shape[1:]
+    T, dev, f32 = x.shape[0], x.device, _is_f32(x)
+    assert state.dtype == torch.float32 and state.is_contiguous() \
+        and x.stride(1) == 1
+    o = torch.empty((T, H * V), dtype=torch.float32, device=dev)
+    head = (_p(x), x.stride(0), *offsets, _p(qs), _p(ks), ks.stride(0),
+            _p(decay), _p(beta), _p(a_bias), _p(state), _p(slots), _p(pos))
+    nd = meta.n_single
+
+    def step(spans, n):
+        _check(_lib.delta_step(f32, gen, _p(o), *head, _p(spans), n, H, G, D,
+                               V, _stream()), "delta_step")
+
+    if nd:
+        step(None, nd)
+    if not meta.one_each:
+        spans, chunks, seqs, _, _ = _chunk_plan(
+            meta, dev, DELTA_STEP_TOKENS if D <= DELTA_MAX_D else 1 << 62)
+        if spans is not None:
+            step(spans, spans.shape[0])
+        if chunks is not None:
+            n = chunks.shape[0]
+            scr = torch.empty(_lib.delta_scratch_floats(gen, n, H, D),
+                              dtype=torch.float32, device=dev)
+            _check(_lib.delta_chunks(
+                f32, gen, _p(o), _p(scr), *head, _p(chunks), n, _p(seqs),
+                seqs.shape[0], H, G, D, V, _stream()), "delta_chunks")
+    return o
+
+
+def gated_delta(p, w, state, conv_state, slot_ids, positions, meta, frag):
+    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
+    o_in, ob, oa, og = w.offsets
+    taps, C = w.conv.shape
+    ra, rg = w.a2.shape[1], w.g2.shape[1]
+    t = p.parts if isinstance(p, Partials) else p
+    T, dev, dtype = t.shape[-2], t.device, w.a2.dtype
+    assert C == 2 * G * D + H * V and state.shape[1:] == (H, D, V) \
+        and conv_state.shape[1:] == (taps - 1, C) \
+        and conv_state.dtype == torch.float32 \
+        and conv_state.is_contiguous() and w.conv.is_contiguous() \
+        and max(o_in + C, ob + H, oa + ra, og + rg) <= t.shape[-1] \
+        and w.a2.shape[0] == w.dt_bias.numel() == H * D \
+        and w.g2.shape == (H * V, rg) and w.rate.numel() == H \
+        and w.norm.numel() == V and w.a2.is_contiguous() \
+        and w.g2.is_contiguous()
+    assert isinstance(p, Partials) or p.dtype == dtype
+    assert not frag or meta.one_each
+    new = lambda *shape, dtype=torch.float32: torch.empty(
+        shape, dtype=dtype, device=dev)
+    y, gate = new(T, C, dtype=dtype), new(T, H * V, dtype=dtype)
+    scales, decay, beta = new(T, 2 * G), new(T, H * D), new(T, H)
+    slots, pos = _i32(slot_ids), _i32(positions)
+    strips = None if meta.one_each else _conv_strips(meta, taps, dev)
+    n = T if strips is None else strips.shape[0]
+    if T:
+        _check(_lib.gated_rows(
+            int(dtype == torch.float32), *_rows(p), o_in, ob, oa, ra, og, rg,
+            _p(w.conv), taps, _p(conv_state), _p(slots), _p(pos), _p(strips),
+            n, _p(w.a2), _p(w.rate), _p(w.dt_bias), _p(w.g2), _p(y),
+            _p(scales), _p(decay), _p(beta), _p(gate), T, H, G, D, V,
+            _stream()), "gated_rows")
+    o = _delta(0, y, (0, G * D, 2 * G * D, 0), scales, scales[:, G:], decay,
+               beta, None, state, G, slots, pos, meta)
+    return head_gate(o, w.norm, gate, 0, "sigmoid", dtype, H, V, w.eps, frag)
+
+
+def general_delta(p, w, state, slot_ids, positions, meta, frag):
+    H, D = w.heads, w.dim
+    o_r, ok, ov, oa, og, ow = w.offsets
+    rank = w.w2.shape[1]
+    t = p.parts if isinstance(p, Partials) else p
+    T, cols, dev, dtype = t.shape[-2], t.shape[-1], t.device, w.w2.dtype
+    assert state.shape[1:] == (H, D, D) and w.w2.shape[0] == H * D \
+        and w.w2.is_contiguous() and max(w.offsets[:5]) + H * D <= cols \
+        and ow + rank <= cols and w.w0.numel() == w.a_bias.numel() \
+        == w.norm.numel() == H * D
+    assert isinstance(p, Partials) or p.dtype == dtype
+    assert not frag or meta.one_each
+    scales = torch.empty((T, H), dtype=torch.float32, device=dev)
+    decay = torch.empty((T, H * D), dtype=torch.float32, device=dev)
+    whole = isinstance(p, Partials)
+    y = torch.empty((T, cols), dtype=dtype, device=dev) if whole else p
+    slots, pos = _i32(slot_ids), _i32(positions)
+    if T:
+        _check(_lib.general_rows(
+            int(dtype == torch.float32), *_rows(p), ok, ow, rank, _p(w.w2),
+            _p(w.w0), _p(scales), _p(decay), _p(y if whole else None), cols,
+            T, H, D, _stream()), "general_rows")
+    o = _delta(1, y, (o_r, ok, ov, oa), None, scales, decay, None, w.a_bias,
+               state, H, slots, pos, meta)
+    return head_gate(o, w.norm, y, og, "sigmoid", dtype, H, D, w.eps, frag)
 
 
 # ---------------------------------------------------------------------------
@@ -1374,6 +1546,55 @@ def rms_residual(x, y, post, pre, mult, eps, embed, tokens, embed_scale,
             _p(route_share), E, top, _stream()), "rms_residual")
     if route is not None:
         return x_out, res, (chosen, route_share)
+    return x_out, res
+
+
+def _src(y, T, W, dtype):
+    """A sublayer's result, whole or in parts: (pointer, fp32?, parts,
+    stride of a part)."""
+    if y is None:
+        return _p(None), 0, 1, 0
+    t = y.parts if isinstance(y, Partials) else y
+    assert t.is_contiguous() and t.shape[-2:] == (T, W) \
+        and t.dtype in (dtype, torch.float32)
+    return (_p(t), int(t.dtype == torch.float32),
+            t.shape[0] if isinstance(y, Partials) else 1, T * W)
+
+
+def ln_residual(x, y, norm, mult, eps, scale, embed, tokens, rows, need_x,
+                frag, then):
+    W, dtype = embed.shape[1], embed.dtype
+    T = (tokens if x is None else x).shape[0]
+    assert x is None or (x.dtype == torch.float32 and x.is_contiguous())
+    pairs, share = ((y, None),), 1.0
+    if isinstance(y, Branches):
+        pairs, share = y.pairs, y.share
+        if not 1 <= len(pairs) <= 2:
+            raise ValueError(f"{len(pairs)} branches: no kernel")
+    pairs = tuple(pairs) + ((None, None),) * (2 - len(pairs))
+    n = T if rows is None else rows.shape[0]
+    if frag:
+        assert dtype == torch.bfloat16 and W % 64 == 0
+        res = _frag_rows(n, W, embed)
+        h = res.buf
+    else:
+        res = h = torch.empty((n, W), dtype=dtype, device=embed.device)
+    if x is not None and y is None and rows is None:
+        x_out, write = x, None               # nothing to add
+    else:
+        x_out = write = torch.empty(
+            (n, W), dtype=torch.float32, device=embed.device) \
+            if need_x else None
+    nw, nb = norm if norm is not None else (None, None)
+    tw, tb = then if then is not None else (None, None)
+    if n:
+        _check(_lib.ln_residual(
+            _is_f32(h), _p(write), _p(h), _p(x), _p(embed),
+            _p(None if tokens is None else _i32(tokens)),
+            *_src(pairs[0][0], T, W, dtype), *_src(pairs[1][0], T, W, dtype),
+            _p(pairs[0][1]), _p(pairs[1][1]), float(share), _p(scale), _p(nw),
+            _p(nb), float(mult), _p(tw), _p(tb), float(eps), _p(rows), n, W,
+            int(frag), _stream()), "ln_residual")
     return x_out, res
 
 
@@ -1509,6 +1730,8 @@ def rope_qkv_append(p, bias, cache, run, w, rope, slot_ids, positions):
         and vp.shape[3] >= V and rope.dims <= D
     assert not rope.dims or (rope.table.shape[1] == rope.dims
                              and rope.table.shape[0] >= cache.max_ctx)
+    if rope.halves:
+        raise ValueError("rotation by halves without head norms: no kernel")
     q = torch.empty((T, H, kp.shape[3]), dtype=kp.dtype, device=kp.device)
     rows = _rows(p)
     assert rows[1] or kp.dtype == torch.bfloat16
@@ -1522,7 +1745,38 @@ def rope_qkv_append(p, bias, cache, run, w, rope, slot_ids, positions):
     return q
 
 
-def softmax_attention(q, cache, run, w, slot_ids, positions, meta, frag):
+def qkv_norm_rope_append(p, norms, cache, run, w, rope, slot_ids, positions):
+    kp, vp = cache.key_pool[run], cache.value_pool[run]
+    H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
+    T = slot_ids.shape[0]
+    if max(kp.shape[3], vp.shape[3]) > ATTN_MAX:
+        raise ValueError(f"softmax attention with head widths {D}/{V}: no "
+                         "kernel")
+    if rope.dims and not rope.halves:
+        raise ValueError("head norms with interleaved rotation: no kernel")
+    assert _cols(p) >= H * D + G * (D + V) and norms.q.numel() == D \
+        and norms.k.numel() == D \
+        and (norms.gain is None or norms.gain.numel() == H)
+    assert kp.shape[1:3] == (G, cache.page_size) and kp.shape[3] >= D \
+        and vp.shape[3] >= V and rope.dims <= D
+    assert not rope.dims or (rope.table.shape[1] == rope.dims
+                             and rope.table.shape[0] >= cache.max_ctx)
+    q = torch.empty((T, H, kp.shape[3]), dtype=kp.dtype, device=kp.device)
+    rows = _rows(p)
+    assert rows[1] or kp.dtype == torch.bfloat16
+    if T:
+        _check(_lib.qkv_norm_rope(
+            _is_f32(q), _p(q), _p(kp), _p(vp), *rows, _p(norms.q),
+            _p(norms.k), _p(norms.gain), int(norms.values), float(norms.eps),
+            _p(rope.table), rope.dims, _p(_i32(slot_ids)),
+            _p(_i32(positions)), _p(cache.page_table), T, H, G, D, V,
+            kp.shape[3], vp.shape[3], cache.page_size,
+            cache.page_table.shape[1], _stream()), "qkv_norm_rope")
+    return q
+
+
+def softmax_attention(q, cache, run, w, slot_ids, positions, meta, frag,
+                      gate=None):
     T, H, Dp = q.shape
     kp, vp = cache.key_pool[run], cache.value_pool[run]
     G, V, R = w.kv_heads, w.vdim, w.heads // w.kv_heads
@@ -1533,6 +1787,8 @@ def softmax_attention(q, cache, run, w, slot_ids, positions, meta, frag):
     assert q.is_contiguous() and kp.dtype == q.dtype \
         and kp.shape[1:] == (G, cache.page_size, Dp) and H == w.heads \
         and (w.sink is None or w.sink.numel() == H)
+    gp, og = (None, 0) if gate is None else gate
+    assert gp is None or og + H <= _cols(gp)
     assert not frag or meta.one_each
     if frag:
         res = _frag_rows(T, H * V, q)
@@ -1553,10 +1809,10 @@ def softmax_attention(q, cache, run, w, slot_ids, positions, meta, frag):
             _p(cache.page_table), _p(_i32(slot_ids)), _p(_i32(positions)),
             _p(items), n, 0, tokens, T, H, G, V, Dp, Vp, cache.page_size,
             cache.page_table.shape[1], split, int(frag), w.scale, _p(w.sink),
-            w.window, _stream()), "softmax_attn")
+            w.window, w.chunk, *_rows(gp), og, _stream()), "softmax_attn")
 
     if n_items:
-        seen = min(kv, w.window) if w.window else kv
+        seen = w.reach(kv)
         split = max(1, min(256 // (n_items * G),
                            -(-seen // _lib.softmax_step(f32)),
                            ATTN_SPLIT_MAX))

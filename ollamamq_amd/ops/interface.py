@@ -211,7 +211,7 @@ class LightningWeights(NamedTuple):
     norm: Optional[torch.Tensor]  # fp32 [heads * vdim], None: no weight
     eps: float
     act: bool = True              # silu of q, k and v
-    key_scale: float = 1.0
+    scale: float = 1.0            # of the results
     per_head: bool = False        # norm of every head, not of all together
     gate: str = "sigmoid"         # or "silu"
 

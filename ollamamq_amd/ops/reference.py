@@ -310,7 +310,7 @@ def lightning(p, w, state, meta):
     T = f.shape[0]
     act = torch.nn.functional.silu if w.act else lambda t: t
     part = lambda at, n: act(f[:, at:at + H * n]).view(T, H, n)
-    q, k, v = part(oq, D), part(ok, D) * w.key_scale, part(ov, V)
+    q, k, v = part(oq, D), part(ok, D), part(ov, V)
     decay = w.powers[:, 1].view(H, 1, 1)
     out = torch.empty(T, H, V)
     r = 0
@@ -321,8 +321,8 @@ def lightning(p, w, state, meta):
             out[t] = torch.einsum("hdv,hd->hv", S, q[t])
         state[slot] = S
         r += n
-    return _gated_heads(out, w.norm, f[:, og:og + H * V], w.eps, _type_of(p),
-                        w.per_head, w.gate)
+    return _gated_heads(out * w.scale, w.norm, f[:, og:og + H * V], w.eps,
+                        _type_of(p), w.per_head, w.gate)
 
 
 def _delta(q, k, v, z, e, g, state, meta):
