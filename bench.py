@@ -173,13 +173,14 @@ def layer_stacks(width, n_layers=4):
     wider ones.  So has "revitar", its feed-forward cut into eight experts of
     which a token uses two; "revitar work" has four times that, so that a
     token's two experts do the Llama feed-forward's work.  The Kavedra layers
-    have the Llama layer's weights, the larger mixers against a narrower
-    feed-forward; "kavedra looped" runs two layers twice."""
+    and the Pemidra layers have the Llama layer's weights, the larger mixers
+    against a narrower feed-forward; "kavedra looped" runs two layers
+    twice."""
     import dataclasses
     from ollamamq_amd.models import PRESETS
     size = "1b" if width <= 2048 else "8b"
     rin, rev = PRESETS[f"rinitar-{size}"], PRESETS[f"revitar-{size}"]
-    kav = PRESETS[f"kavedra-{size}"]
+    kav, pem = PRESETS[f"kavedra-{size}"], PRESETS[f"pemidra-{size}"]
     gla = [s for s in rin.layers if s.type == "gla"][0]
     lat = [s for s in rin.layers if s.type != "gla"][0]
     llama = dataclasses.replace(
@@ -200,6 +201,13 @@ def layer_stacks(width, n_layers=4):
              ("lightning", "attention", "latent_attention")),
             (5 * width // 2, 0, width + 3 * 512 + 64)))
     half = n_layers // 2
+    low = pem.low_rank
+    ret, gen, par = (
+        dataclasses.replace(next(s for s in pem.layers if s.type == t),
+                            ff=(llama.ffn - extra // 3) // 64 * 64)
+        for t, extra in (("retention", 5 * width // 2),
+                         ("general_delta", 7 * width // 2 + 2 * low),
+                         ("parallel", 2 * width + 3 * low)))
     return [("llama", llama),
             ("rinitar gla", stack(rin, "gla", [gla] * n_layers)),
             ("rinitar latent", stack(rin, "latent", [lat] * n_layers)),
@@ -216,7 +224,12 @@ def layer_stacks(width, n_layers=4):
             ("kavedra mixed", stack(kav, "blend", [light, lat_k] * (half // 2)
                                     + [light, soft] * (half // 2))),
             ("kavedra looped", dataclasses.replace(
-                stack(kav, "loop", [light, soft]), loop=(0, 2, 2)))]
+                stack(kav, "loop", [light, soft]), loop=(0, 2, 2))),
+            ("pemidra retention", stack(pem, "retention", [ret] * n_layers)),
+            ("pemidra delta", stack(pem, "delta", [gen] * n_layers)),
+            ("pemidra parallel", stack(pem, "parallel", [par] * n_layers)),
+            ("pemidra mixed", stack(pem, "medley", [par, ret, gen, par]
+                                    * (n_layers // 4)))]
 
 
 def run_layers(args):
@@ -314,9 +327,9 @@ def main():
                          "(HTTP + scheduler + UDS workers) instead of "
                          "the engine-only kernel metric")
     ap.add_argument("--layers", action="store_true",
-                    help="prefill and decode throughput of Rinitar, Revitar "
-                         "and Kavedra layer stacks beside Llama stacks of "
-                         "equal size")
+                    help="prefill and decode throughput of Rinitar, Revitar, "
+                         "Kavedra and Pemidra layer stacks beside Llama "
+                         "stacks of equal size")
     ap.add_argument("--layer-sizes", type=str, default="2048,4096",
                     help="widths for --layers, of 2048, 4096")
     ap.add_argument("--stacks", type=str, default="",
