@@ -39,7 +39,11 @@ template <typename T> DEV float silu_of(float x) {
     return x * sigmoid_of<T>(x);
 }
 template <typename T> DEV float softplus_of(float x) {
-    return fmaxf(x, 0.f) + log1pf(exp_of<T>(-fabsf(x)));
+    const float e = exp_of<T>(-fabsf(x));
+    if constexpr (sizeof(T) == 4) return fmaxf(x, 0.f) + log1pf(e);
+    // log(1 + e), with a series where 1 + e would lose e
+    const float s = e * (1.f + e * (-0.5f + e * (1.f / 3.f + e * -0.25f)));
+    return fmaxf(x, 0.f) + (e < 0.03f ? s : __logf(1.f + e));
 }
 #define UNIT_EPS 1e-6f                // inside the root of a unit vector
 #define LOG_ZERO (-104.f)             // e to this is zero in fp32
@@ -60,45 +64,66 @@ template <> struct Terms<float> {
 };
 
 // ---------------------------------------------------------------------------
-// z = W u for 16 tokens and 64 rows of W [N, rank], u the projection's columns
-// first.. of the lane's token t: z[j][i] is row n0 + 16 j + 4 g + i.
+// z = W u for 16 tokens and rows n0 .. n1 - 1 of W [N, rank], u (or its tanh)
+// the projection's columns first.. of the lane's token t; rank and first are
+// whole vectors of 8.  `emit` gets 16 rows at a time, four of them in a lane:
+// z[i] is row n + i.  The operand is made once for all rows while rank <= 128.
 // ---------------------------------------------------------------------------
-template <typename T, typename P, bool TANH>
+template <typename T, typename P, bool TANH, typename E>
 DEV void low_rank(const Rows<P>& p, int first, int rank,
-                  const T* __restrict__ w, int N, int n0, int64_t t,
-                  f32x4* z) {
+                  const T* __restrict__ w, int N, int n0, int n1, int64_t t,
+                  E emit) {
     constexpr int NT = Terms<T>::N;
     const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
-    const bool v8 = p.ld % 8 == 0 && p.part_stride % 8 == 0 && first % 8 == 0
-                    && rank % 8 == 0;
-    for (int r0 = 0; r0 < rank; r0 += 32) {
-        const int k = r0 + g * 8;
-        float u[8] = {};
-        if (v8) {
-            if (k < rank) ldrow<8>(p, t, first + k, u);
-        } else
-            for (int e = 0; e < 8; e++)
-                if (k + e < rank) ldrow<1>(p, t, first + k + e, u + e);
-        Frag<T> uf[NT];
-        #pragma unroll
-        for (int e = 0; e < 8; e++) {
-            T y[NT];
-            Terms<T>::split(TANH ? tanh_of<T>(u[e]) : u[e], y);
+    Frag<T> uf[4][NT];
+    auto operand = [&](int r0) {
+        float u[4][8] = {};
+        for (int q = 0; q < p.n_part; q++) {
+            const P* src = p.p + q * p.part_stride + t * p.ld + first;
+            float x[4][8];
             #pragma unroll
-            for (int q = 0; q < NT; q++) frag_set(uf[q], e, ldf(&y[q]));
+            for (int s = 0; s < 4; s++)
+                ldv<8>(src + min(r0 + s * 32 + g * 8, rank - 8), x[s]);
+            #pragma unroll
+            for (int s = 0; s < 4; s++)
+                #pragma unroll
+                for (int e = 0; e < 8; e++) u[s][e] += x[s][e];
         }
         #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const int n = n0 + j * 16 + lr;
-            const T* row = w + (int64_t)n * rank;
-            Frag<T> wf = frag_zero<T>();
-            if (n < N) {
-                if (v8) { if (k < rank) wf = frag8(row + k); }
-                else wf = frag_guard(row, k, rank);
+        for (int s = 0; s < 4; s++)
+            #pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const bool in = r0 + s * 32 + g * 8 < rank;
+                T y[NT];
+                Terms<T>::split(in ? TANH ? tanh_of<T>(u[s][e]) : u[s][e]
+                                   : 0.f, y);
+                #pragma unroll
+                for (int q = 0; q < NT; q++)
+                    frag_set(uf[s][q], e, ldf(&y[q]));
             }
+    };
+    if (rank <= 128) operand(0);
+    for (int n = n0; n < n1; n += 64) {
+        f32x4 z[4] = {};
+        for (int r0 = 0; r0 < rank; r0 += 128) {
+            if (rank > 128) operand(r0);
             #pragma unroll
-            for (int q = 0; q < NT; q++) z[j] = mma(wf, uf[q], z[j]);
+            for (int s = 0; s < 4; s++) {
+                const int k = r0 + s * 32 + g * 8;
+                if (r0 + s * 32 >= rank) continue;
+                #pragma unroll
+                for (int j = 0; j < 4; j++) {
+                    const int m = n + j * 16 + lr;
+                    const T* row = w + (int64_t)min(m, N - 1) * rank;
+                    const Frag<T> wf = frag8(row + min(k, rank - 8));
+                    #pragma unroll
+                    for (int q = 0; q < NT; q++)
+                        z[j] = mma(wf, uf[s][q], z[j]);
+                }
+            }
         }
+        #pragma unroll
+        for (int j = 0; j < 4; j++) emit(n + j * 16 + g * 4, z[j]);
     }
 }
 // four results from column n on
@@ -133,6 +158,7 @@ template <typename T, typename P> struct GatedRows {
     float* beta;                      // [T, H]
     T* gate;                          // [T, H*V]
     int L, n_conv, n_decay, n_gate;   // lanes per head; waves of a role
+    int wide;                         // columns of a low-rank wave
 };
 
 template <typename T, typename P, int VEC, int KEEP, int TAPS>
@@ -231,7 +257,7 @@ DEV void conv_strip(const GatedRows<T, P>& a, int64_t item, int lane) {
 }
 
 template <typename T, typename P, int VEC, int KEEP, int TAPS>
-__global__ __launch_bounds__(256) void k_gated_rows(GatedRows<T, P> a)
+__global__ __launch_bounds__(256, 4) void k_gated_rows(GatedRows<T, P> a)
 {
     const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
     int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -242,41 +268,38 @@ __global__ __launch_bounds__(256) void k_gated_rows(GatedRows<T, P> a)
     }
     w -= a.n_conv;
     if (w < a.n_decay) {
-        const int N = a.H * a.D, nc = (N + 63) / 64;
-        const int n0 = (int)(w % nc) * 64;
+        const int N = a.H * a.D, nc = (N + a.wide - 1) / a.wide;
+        const int n0 = (int)(w % nc) * a.wide;
         const int64_t t = w / nc * 16 + lr;
-        f32x4 z[4] = {};
-        low_rank<T, P, false>(a.p, a.oa, a.ra, a.a2, N, n0,
-                              min(t, (int64_t)a.T_rows - 1), z);
-        if (t >= a.T_rows) return;
-        #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const int n = n0 + j * 16 + g * 4;
-            float v[4];
-            #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int m = min(n + i, N - 1);
-                v[i] = fmaxf(LOG_ZERO, -a.rate[m / a.D]
-                             * softplus_of<T>(z[j][i] + a.dt[m]));
-            }
-            put4(a.decay, t, n, N, v);
-        }
+        low_rank<T, P, false>(
+            a.p, a.oa, a.ra, a.a2, N, n0, min(n0 + a.wide, N),
+            min(t, (int64_t)a.T_rows - 1), [&](int n, f32x4 z) {
+                if (t >= a.T_rows || n >= N) return;
+                const bool whole = a.D % 4 == 0;    // four of one head
+                float v[4], rate = a.rate[n / a.D];
+                #pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int m = min(n + i, N - 1);
+                    if (!whole) rate = a.rate[m / a.D];
+                    v[i] = fmaxf(LOG_ZERO,
+                                 -rate * softplus_of<T>(z[i] + a.dt[m]));
+                }
+                put4(a.decay, t, n, N, v);
+            });
         return;
     }
     w -= a.n_decay;
     if (w < a.n_gate) {
-        const int N = a.H * a.V, nc = (N + 63) / 64;
-        const int n0 = (int)(w % nc) * 64;
+        const int N = a.H * a.V, nc = (N + a.wide - 1) / a.wide;
+        const int n0 = (int)(w % nc) * a.wide;
         const int64_t t = w / nc * 16 + lr;
-        f32x4 z[4] = {};
-        low_rank<T, P, false>(a.p, a.og, a.rg, a.g2, N, n0,
-                              min(t, (int64_t)a.T_rows - 1), z);
-        if (t >= a.T_rows) return;
-        #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const float v[4] = {z[j][0], z[j][1], z[j][2], z[j][3]};
-            put4(a.gate, t, n0 + j * 16 + g * 4, N, v);
-        }
+        low_rank<T, P, false>(
+            a.p, a.og, a.rg, a.g2, N, n0, min(n0 + a.wide, N),
+            min(t, (int64_t)a.T_rows - 1), [&](int n, f32x4 z) {
+                if (t >= a.T_rows) return;
+                const float v[4] = {z[0], z[1], z[2], z[3]};
+                put4(a.gate, t, n, N, v);
+            });
         return;
     }
     w -= a.n_gate;
@@ -287,8 +310,14 @@ __global__ __launch_bounds__(256) void k_gated_rows(GatedRows<T, P> a)
     a.beta[i] = sigmoid_of<T>(x);
 }
 
-static int waves_for(int64_t tokens, int channels) {
-    return (int)((tokens + 15) / 16 * ((channels + 63) / 64));
+// columns of a low-rank wave: many share the operand, few fill the chip
+static int low_rank_cols(int T_rows) { return T_rows > 512 ? 256 : 64; }
+static bool low_rank_ok(int first, int rank, int64_t ld, int64_t stride) {
+    return rank >= 8 && rank % 8 == 0 && first % 8 == 0 && ld % 8 == 0
+           && stride % 8 == 0;
+}
+static int low_rank_waves(int64_t tokens, int channels, int wide) {
+    return (int)((tokens + 15) / 16 * ((channels + wide - 1) / wide));
 }
 
 // strips int32 [n, 4] (first row, rows, the portion's first row and end), a
@@ -306,15 +335,18 @@ extern "C" int gated_rows(
     const int C = 2 * G * D + H * V, wide = D > V ? D : V;
     const bool v4 = D % 4 == 0 && V % 4 == 0 && o_in % 4 == 0 && ld % 4 == 0
                     && part_stride % 4 == 0;
-    if (taps < 1 || ra < 1 || rg < 1 || wide > (v4 ? 1024 : 256))
+    if (taps < 1 || !low_rank_ok(oa, ra, ld, part_stride)
+        || !low_rank_ok(og, rg, ld, part_stride)
+        || wide > (v4 ? 1024 : 256))
         return (int)hipErrorInvalidValue;
     const bool one = v4 && wide <= 256;     // a head fits 64 lanes at once
     int L = 64;
     if (one) while (L > 1 && L / 2 * 4 >= wide) L /= 2;
     const int64_t units = (int64_t)n_strips * (2 * G + H);
     const int n_conv = (int)((units * L + 63) / 64);
-    const int n_decay = waves_for(T_rows, H * D);
-    const int n_gate = waves_for(T_rows, H * V);
+    const int cols = low_rank_cols(T_rows);
+    const int n_decay = low_rank_waves(T_rows, H * D, cols);
+    const int n_gate = low_rank_waves(T_rows, H * V, cols);
     const int64_t all = (int64_t)n_conv + n_decay + n_gate
                         + ((int64_t)T_rows * H + 63) / 64;
     const int grid = (int)((all + 3) / 4);
@@ -327,7 +359,7 @@ extern "C" int gated_rows(
                 (const int*)pos, (const int*)strips, n_strips,             \
                 (const T*)a2, (const float*)rate, (const float*)dt,        \
                 (const T*)g2, (T*)y, (float*)scales, (float*)decay,        \
-                (float*)beta, (T*)gate, L, n_conv, n_decay, n_gate})
+                (float*)beta, (T*)gate, L, n_conv, n_decay, n_gate, cols})
     #define GR_V(T, P)                                                     \
         do {                                                               \
             if (one && taps == 4) GR(T, P, 4, 1, 4);                       \
@@ -353,10 +385,11 @@ template <typename T, typename P> struct GeneralRows {
     float* decay;                     // [T, H*D], logarithms
     T* y;                             // [T, cols] or null
     int cols, L, n_key, n_decay;
+    int wide;                         // columns of a low-rank wave
 };
 
 template <typename T, typename P, int VEC>
-__global__ __launch_bounds__(256) void k_general_rows(GeneralRows<T, P> a)
+__global__ __launch_bounds__(256, 3) void k_general_rows(GeneralRows<T, P> a)
 {
     const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
     int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -377,23 +410,20 @@ __global__ __launch_bounds__(256) void k_general_rows(GeneralRows<T, P> a)
     }
     w -= a.n_key;
     if (w < a.n_decay) {
-        const int N = a.H * a.D, nc = (N + 63) / 64;
-        const int n0 = (int)(w % nc) * 64;
+        const int N = a.H * a.D, nc = (N + a.wide - 1) / a.wide;
+        const int n0 = (int)(w % nc) * a.wide;
         const int64_t t = w / nc * 16 + lr;
-        f32x4 z[4] = {};
-        low_rank<T, P, true>(a.p, a.ow, a.rank, a.w2, N, n0,
-                             min(t, (int64_t)a.T_rows - 1), z);
-        if (t >= a.T_rows) return;
-        #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const int n = n0 + j * 16 + g * 4;
-            float v[4];
-            #pragma unroll
-            for (int i = 0; i < 4; i++)
-                v[i] = -HALF_DECAY
-                       * sigmoid_of<T>(z[j][i] + a.w0[min(n + i, N - 1)]);
-            put4(a.decay, t, n, N, v);
-        }
+        low_rank<T, P, true>(
+            a.p, a.ow, a.rank, a.w2, N, n0, min(n0 + a.wide, N),
+            min(t, (int64_t)a.T_rows - 1), [&](int n, f32x4 z) {
+                if (t >= a.T_rows) return;
+                float v[4];
+                #pragma unroll
+                for (int i = 0; i < 4; i++)
+                    v[i] = -HALF_DECAY
+                           * sigmoid_of<T>(z[i] + a.w0[min(n + i, N - 1)]);
+                put4(a.decay, t, n, N, v);
+            });
         return;
     }
     if (!a.y) return;
@@ -413,11 +443,13 @@ extern "C" int general_rows(
 {
     const bool v4 = D % 4 == 0 && ok % 4 == 0 && ld % 4 == 0
                     && part_stride % 4 == 0 && cols % 4 == 0;
-    if (rank < 1) return (int)hipErrorInvalidValue;
+    if (!low_rank_ok(ow, rank, ld, part_stride))
+        return (int)hipErrorInvalidValue;
     int L = 64;
     while (L > 1 && L / 2 * (v4 ? 4 : 1) >= D) L /= 2;
     const int n_key = (int)(((int64_t)T_rows * H * L + 63) / 64);
-    const int n_decay = waves_for(T_rows, H * D);
+    const int wide = low_rank_cols(T_rows);
+    const int n_decay = low_rank_waves(T_rows, H * D, wide);
     const int64_t n_sum = y ? ((int64_t)T_rows * cols / (v4 ? 4 : 1) + 63)
                               / 64 : 0;
     const int grid = (int)((n_key + n_decay + n_sum + 3) / 4);
@@ -427,7 +459,7 @@ extern "C" int general_rows(
                 Rows<P>{(const P*)p, n_part, part_stride, ld}, T_rows, ok, \
                 ow, rank, H, D, (const T*)w2, (const float*)w0,            \
                 (float*)scales, (float*)decay, (T*)y, cols, L, n_key,      \
-                n_decay})
+                n_decay, wide})
     #define GE_V(T, P) do { if (v4) GE(T, P, 4); else GE(T, P, 1); } while (0)
     if (f32) GE_V(float, float);
     else if (p32) GE_V(bf16, float);
@@ -628,10 +660,6 @@ DEV Wide<float> ldw(const float* p, int64_t) { return {frag8(p)}; }
 DEV Wide<bf16> ldw(const bf16* p, int64_t plane) {
     return {frag8(p), frag8(p + plane)};
 }
-template <typename T> DEV Wide<T> wide_zero() {
-    if constexpr (sizeof(T) == 4) return {frag_zero<float>()};
-    else return {frag_zero<bf16>(), frag_zero<bf16>()};
-}
 DEV f32x4 mma(const Wide<float>& a, const Wide<float>& b, f32x4 c) {
     return mma(a.f, b.f, c);
 }
@@ -640,67 +668,68 @@ DEV f32x4 mma(const Wide<bf16>& a, const Wide<bf16>& b, f32x4 c) {
     c = mma(a.hi, b.lo, c);
     return mma(a.hi, b.hi, c);
 }
-DEV void stw(float* p, int64_t, float v) { *p = v; }
-DEV void stw(bf16* p, int64_t plane, float v) {
-    bf16 t[2];
-    Terms<bf16>::split(v, t);
-    p[0] = t[0];
-    p[plane] = t[1];
+// by a matrix of the model's type
+DEV f32x4 mma(const Wide<float>& a, const f32x8s& b, f32x4 c) {
+    return mma(a.f, b, c);
 }
-template <typename T> DEV void stw4(T* p, int64_t plane, f32x4 v) {
-    float f[Terms<T>::N][4];
+DEV f32x4 mma(const Wide<bf16>& a, bf16x8 b, f32x4 c) {
+    return mma(a.hi, b, mma(a.lo, b, c));
+}
+// VEC consecutive values
+template <typename T, int VEC>
+DEV void stw(T* p, int64_t plane, const float* v) {
+    float f[Terms<T>::N][VEC];
     #pragma unroll
-    for (int i = 0; i < 4; i++) {
+    for (int i = 0; i < VEC; i++) {
         T t[Terms<T>::N];
         Terms<T>::split(v[i], t);
         #pragma unroll
         for (int q = 0; q < Terms<T>::N; q++) f[q][i] = ldf(&t[q]);
     }
     #pragma unroll
-    for (int q = 0; q < Terms<T>::N; q++) stv<4>(p + q * plane, f[q]);
+    for (int q = 0; q < Terms<T>::N; q++) stv<VEC>(p + q * plane, f[q]);
 }
+template <typename T> DEV void stw4(T* p, int64_t plane, f32x4 v) {
+    const float f[4] = {v[0], v[1], v[2], v[3]};
+    stw<T, 4>(p, plane, f);
+}
+// four values of the model's type, as they are in memory
+template <typename T> struct Four;
+template <> struct Four<float> { typedef f32x4 type; };
+template <> struct Four<bf16> { typedef bf16x4 type; };
 
-// Scratch per (chunk, head), each matrix of N planes: Q [64][Dp], Z [64][Dp],
-// K^T [Dp][64], (E^T), inverse [64][64], A_qk, (A_zk, A_qe); then the fp32
-// decay of the whole chunk [Dp].
-template <typename T, bool GEN> struct Unit {
+// Scratch per (chunk, head), each matrix of NT planes: Q [64][DP],
+// Z [64][DP], K^T [DP][64], (E^T), inverse [64][64], A_qk, (A_zk, A_qe);
+// then the fp32 decay of the whole chunk [DP].  Offsets in elements of T.
+template <typename T, bool GEN, int DP> struct Unit {
     static constexpr int NT = Terms<T>::N;
-    DEV static T* base(float* scr, int64_t i, int Dp) {
-        return (T*)(scr + i * floats(Dp));
+    static constexpr int64_t TP = CH * DP, SP = CH * CH;    // planes
+    static constexpr int64_t tall(int m) { return m * NT * TP; }
+    static constexpr int64_t square(int m) {
+        return tall(GEN ? 4 : 3) + m * NT * SP;
     }
-    static __host__ __device__ int64_t floats(int Dp) {
-        return (int64_t)(GEN ? 4 : 3) * CH * Dp + (GEN ? 4 : 2) * CH * CH
-               + Dp;
-    }
-    // offsets in elements; a plane follows its matrix
-    static __host__ __device__ int64_t tall(int m, int Dp) {
-        return (int64_t)m * NT * CH * Dp;
-    }
-    static __host__ __device__ int64_t square(int m, int Dp) {
-        return tall(GEN ? 4 : 3, Dp) + (int64_t)m * NT * CH * CH;
-    }
-    static __host__ __device__ int64_t fade(int Dp) {
-        return square(GEN ? 4 : 2, Dp);
-    }
+    static constexpr int64_t fade = square(GEN ? 4 : 2);
+    static constexpr int64_t floats = (GEN ? 4 : 3) * TP + (GEN ? 4 : 2) * SP
+                                      + DP;
+    DEV T* at(float* scr, int64_t i) { return (T*)(scr + i * floats); }
 };
 enum { TALL_Q, TALL_Z, TALL_K, TALL_E };
 enum { SQ_INV, SQ_QK, SQ_ZK, SQ_QE };
 
-template <typename T, bool GEN>
+template <typename T, bool GEN, int DP>
 __global__ __launch_bounds__(256) void k_delta_prep(
     float* __restrict__ scr, DeltaIn<T> in,
     const int* __restrict__ chunks,     // [n, 2] first row, rows
-    int Dp, int vec)
+    int vec)
 {
-    typedef Unit<T, GEN> Un;
+    typedef Unit<T, GEN, DP> Un;
     const int H = in.H, D = in.D;
     const int h = blockIdx.y, hk = h / (H / in.G), tid = threadIdx.x;
     const int lane = tid & 63, w = tid >> 6;
     const int lr = lane & 15, g = lane >> 4;
     const int t0 = chunks[blockIdx.x * 2], n = chunks[blockIdx.x * 2 + 1];
-    T* un = Un::base(scr, (int64_t)blockIdx.x * H + h, Dp);
-    float* fade = (float*)(un + Un::fade(Dp));
-    const int64_t tp = (int64_t)CH * Dp, sp = CH * CH;      // planes
+    T* un = Un::at(scr, (int64_t)blockIdx.x * H + h);
+    float* fade = (float*)(un + Un::fade);
     constexpr int PL = CH * DS;
     extern __shared__ __attribute__((aligned(16))) float sm[];
     float* qe_s = sm;                   // [64][DS] q e^{c}, c from the part on
@@ -718,48 +747,58 @@ __global__ __launch_bounds__(256) void k_delta_prep(
     const int tk = w * SUB + (lane >> 2), c8 = (lane & 3) * 8;
     const bool live = tk < n;
     const int64_t t = t0 + min(tk, n - 1);
-    const T* row = in.x + t * in.ld;
+    const T* qr = in.x + t * in.ld + in.oq + hk * D;
+    const T* kr = in.x + t * in.ld + in.ok + hk * D;
+    const T* ar = in.x + t * in.ld + in.oa + h * D;
+    const float* cr = in.decay + (t * H + h) * D;
     const float on = live ? 1.f : 0.f;
     const float qs = on * (in.qs ? in.qs[t * in.sld + hk] : 1.f);
     const float ks = on * in.ks[t * in.sld + hk];
     const float beta = GEN ? 0.f : in.beta[t * H + h];
+    Frag<T> qn, kn, an;                 // the next pass
+    f32x8s cn;
+    auto load = [&](int d) {
+        if (vec) {
+            const int c = min(d, D - 8);
+            qn = frag8(qr + c);
+            kn = frag8(kr + c);
+            if (GEN) an = frag8(ar + c);
+            cn = frag8(cr + c);
+        } else {
+            qn = frag_guard(qr, d, D);
+            kn = frag_guard(kr, d, D);
+            if (GEN) an = frag_guard(ar, d, D);
+            cn = frag_guard(cr, d, D);
+        }
+    };
     // of the six tiles below the diagonal (1,0) (2,1) (3,2) (2,0) (3,1)
     // (3,0) this wave makes numbers w and w + 4
     const int ti[6] = {1, 2, 3, 2, 3, 3}, tj[6] = {0, 1, 2, 0, 1, 0};
-    // products of q and z with k (and e): the wave's diagonal tile, the
-    // tiles below the diagonal
+    // products of q and z with k (and e), a query on a lane: the wave's
+    // diagonal tile, the tiles below the diagonal
     f32x4 dqk = {}, dzk = {}, dqe = {}, dze = {};
     f32x4 oqk[2] = {}, ozk[2] = {}, oqe[2] = {}, oze[2] = {};
 
-    for (int d0 = 0; d0 < Dp; d0 += DB) {
-        __syncthreads();
+    load(c8);
+    for (int d0 = 0; d0 < DP; d0 += DB) {
         const int d = d0 + c8;
-        float q[8] = {}, k[8] = {}, c[8] = {}, a[8] = {};
-        if (vec) {
-            if (d < D) {
-                ldv<8>(row + in.oq + hk * D + d, q);
-                ldv<8>(row + in.ok + hk * D + d, k);
-                ldv<8>(in.decay + (t * H + h) * D + d, c);
-                if (GEN) ldv<8>(row + in.oa + h * D + d, a);
-            }
-        } else
-            for (int e = 0; e < 8; e++)
-                if (d + e < D) {
-                    q[e] = ldf(row + in.oq + hk * D + d + e);
-                    k[e] = ldf(row + in.ok + hk * D + d + e);
-                    c[e] = in.decay[(t * H + h) * D + d + e];
-                    if (GEN) a[e] = ldf(row + in.oa + h * D + d + e);
-                }
-        if (GEN)
-            #pragma unroll
-            for (int e = 0; e < 8; e++)
-                a[e] = d + e < D
-                    ? sigmoid_of<T>(a[e] + in.a_bias[h * D + d + e]) : 0.f;
+        float q[8], k[8], c[8], a[8];
+        #pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const float in_d = d + e < D ? 1.f : 0.f;
+            q[e] = in_d * frag_get(qn, e);
+            k[e] = in_d * frag_get(kn, e);
+            c[e] = in_d * on * frag_get(cn, e);
+            if (GEN)
+                a[e] = sigmoid_of<T>(frag_get(an, e)
+                                     + in.a_bias[h * D + min(d + e, D - 1)]);
+        }
+        if (d0 + DB < DP) load(d + DB);
         float own[8], tot[8];
         bool safe = true;
         #pragma unroll
         for (int e = 0; e < 8; e++) {
-            own[e] = c[e] = c[e] * on;
+            own[e] = c[e];
             #pragma unroll
             for (int s = 4; s < 64; s *= 2) {       // tokens are 4 lanes apart
                 const float y = __shfl_up(c[e], s, 64);
@@ -769,26 +808,27 @@ __global__ __launch_bounds__(256) void k_delta_prep(
             safe = safe && tot[e] > -SAFE;
         }
         safe = GEN || __all(safe);
-        float qe[8], ze[8], kt[8], kn[8], x1[8], x2[8];
+        float qe[8], ze[8], kt[8], kn2[8], x1[8], x2[8];
         #pragma unroll
         for (int e = 0; e < 8; e++) {
             const float grow = exp_of<T>(c[e]);
-            const float left = exp_of<T>(tot[e] - c[e]);
             const float back = safe ? exp_of<T>(-c[e]) : 1.f;
+            const float left = exp_of<T>(tot[e] - c[e]);
             const float u = k[e] * ks;
             const float kk = GEN ? k[e] * on : beta * u;
             qe[e] = q[e] * qs * grow;
             ze[e] = u * (GEN ? exp_of<T>(c[e] - own[e]) : grow);
             kt[e] = kk * left;
-            kn[e] = kk * back;
+            kn2[e] = kk * back;
             x1[e] = GEN ? a[e] * u * left : q[e] * qs;
             x2[e] = GEN ? a[e] * u * back : u;
         }
+        __syncthreads();                // the pass before is done with
         const int at = tk * DS + c8;
         stv<8>(qe_s + at, qe);
         stv<8>(ze_s + at, ze);
         stv<8>(kt_s + at, kt);
-        stv<8>(kn_s + at, kn);
+        stv<8>(kn_s + at, kn2);
         if (GEN || !safe) {
             stv<8>(x1_s + at, x1);
             stv<8>(x2_s + at, x2);
@@ -800,47 +840,44 @@ __global__ __launch_bounds__(256) void k_delta_prep(
             stv<8>(et_s + w * DB + c8, tot);
         }
         __syncthreads();
-        // factors that meet the state: the decay of the chunk before and
-        // after the part joins in
-        if (d < Dp) {
-            float before[8], after[8];
+        // factors that meet the state: the decay of the parts before joins
+        // q and z, that of the parts after k and e
+        {
+            float before[8];
             #pragma unroll
-            for (int e = 0; e < 8; e++) before[e] = after[e] = 1.f;
-            for (int s = 0; s < 4; s++) {
-                if (s == w) continue;
+            for (int e = 0; e < 8; e++) before[e] = 1.f;
+            for (int s = 0; s < w; s++) {
                 float f[8];
                 ldv<8>(et_s + s * DB + c8, f);
                 #pragma unroll
-                for (int e = 0; e < 8; e++) {
-                    if (s < w) before[e] *= f[e];
-                    else after[e] *= f[e];
-                }
-            }
-            #pragma unroll
-            for (int e = 0; e < 8; e += 4) {
-                f32x4 y, z;
-                #pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    y[i] = qe[e + i] * before[e + i];
-                    z[i] = ze[e + i] * before[e + i];
-                }
-                stw4(un + Un::tall(TALL_Q, Dp) + (int64_t)tk * Dp + d + e, tp,
-                     y);
-                stw4(un + Un::tall(TALL_Z, Dp) + (int64_t)tk * Dp + d + e, tp,
-                     z);
+                for (int e = 0; e < 8; e++) before[e] *= f[e];
             }
             #pragma unroll
             for (int e = 0; e < 8; e++) {
-                stw(un + Un::tall(TALL_K, Dp) + (int64_t)(d + e) * CH + tk, tp,
-                    kt[e] * after[e]);
-                if (GEN)
-                    stw(un + Un::tall(TALL_E, Dp) + (int64_t)(d + e) * CH + tk,
-                        tp, x1[e] * after[e]);
+                qe[e] *= before[e];
+                ze[e] *= before[e];
             }
-            if (w == 3 && (lane >> 2) == 0)
+            stw<T, 8>(un + Un::tall(TALL_Q) + tk * DP + d, Un::TP, qe);
+            stw<T, 8>(un + Un::tall(TALL_Z) + tk * DP + d, Un::TP, ze);
+            // transposed: eight tokens of a channel
+            const int tt = (tid & 7) * 8, ch = tid >> 3;
+            float after = 1.f, y[8];
+            for (int s = tt / SUB + 1; s < 4; s++) after *= et_s[s * DB + ch];
+            #pragma unroll
+            for (int i = 0; i < 8; i++)
+                y[i] = after * kt_s[(tt + i) * DS + ch];
+            stw<T, 8>(un + Un::tall(TALL_K) + (d0 + ch) * CH + tt, Un::TP,
+                      y);
+            if (GEN) {
                 #pragma unroll
-                for (int e = 0; e < 8; e++)
-                    fade[d + e] = before[e] * et_s[3 * DB + c8 + e];
+                for (int i = 0; i < 8; i++)
+                    y[i] = after * x1_s[(tt + i) * DS + ch];
+                stw<T, 8>(un + Un::tall(TALL_E) + (d0 + ch) * CH + tt,
+                          Un::TP, y);
+            }
+            if (tid < DB)
+                fade[d0 + tid] = et_s[tid] * et_s[DB + tid]
+                                 * et_s[2 * DB + tid] * et_s[3 * DB + tid];
         }
         // tiles below the diagonal
         #pragma unroll
@@ -856,12 +893,12 @@ __global__ __launch_bounds__(256) void k_delta_prep(
                 za.lo *= f.lo; za.hi *= f.hi;
             }
             const f32x8s kb = frag8(kt_s + (J * SUB + lr) * DS + g * 8);
-            oqk[x] = mma(qa, kb, oqk[x]);
-            ozk[x] = mma(za, kb, ozk[x]);
+            oqk[x] = mma(kb, qa, oqk[x]);
+            ozk[x] = mma(kb, za, ozk[x]);
             if (GEN) {
                 const f32x8s eb = frag8(x1_s + (J * SUB + lr) * DS + g * 8);
-                oqe[x] = mma(qa, eb, oqe[x]);
-                oze[x] = mma(za, eb, oze[x]);
+                oqe[x] = mma(eb, qa, oqe[x]);
+                oze[x] = mma(eb, za, oze[x]);
             }
         }
         // the part's own triangle
@@ -869,24 +906,25 @@ __global__ __launch_bounds__(256) void k_delta_prep(
             const int r = (w * SUB + lr) * DS + g * 8;
             const f32x8s qa = frag8(qe_s + r), za = frag8(ze_s + r);
             const f32x8s kb = frag8(kn_s + r);
-            dqk = mma(qa, kb, dqk);
-            dzk = mma(za, kb, dzk);
+            dqk = mma(kb, qa, dqk);
+            dzk = mma(kb, za, dzk);
             if (GEN) {
                 const f32x8s eb = frag8(x2_s + r);
-                dqe = mma(qa, eb, dqe);
-                dze = mma(za, eb, dze);
+                dqe = mma(eb, qa, dqe);
+                dze = mma(eb, za, dze);
             }
         } else {
-            // lane: column lr (the key), rows 4g + i (the query)
+            // lane: column lr (the query), rows 4g + i (the key)
             for (int e = 0; e < DB; e++) {
-                const int oj = (w * SUB + lr) * DS + e;
-                const float kj = kn_s[oj], cj = c_s[oj];
+                const int oi = (w * SUB + lr) * DS + e;
+                const float ci = c_s[oi], qi = x1_s[oi], zi = x2_s[oi];
                 #pragma unroll
                 for (int i = 0; i < 4; i++) {
-                    const int oi = (w * SUB + g * 4 + i) * DS + e;
-                    const float f = kj * exp_of<T>(fminf(c_s[oi] - cj, 0.f));
-                    dqk[i] += x1_s[oi] * f;
-                    dzk[i] += x2_s[oi] * f;
+                    const int oj = (w * SUB + g * 4 + i) * DS + e;
+                    const float f = kn_s[oj]
+                                    * exp_of<T>(fminf(ci - c_s[oj], 0.f));
+                    dqk[i] += qi * f;
+                    dzk[i] += zi * f;
                 }
             }
         }
@@ -894,33 +932,30 @@ __global__ __launch_bounds__(256) void k_delta_prep(
     // A_ze to LDS, the others to memory; the gated rule's A_ze is A_zk
     __syncthreads();
     auto place = [&](int m, int I, int J, f32x4 v) {
-        #pragma unroll
-        for (int i = 0; i < 4; i++)
-            stw(un + Un::square(m, Dp) + (I * SUB + g * 4 + i) * CH
-                + J * SUB + lr, sp, v[i]);
+        stw4(un + Un::square(m) + (I * SUB + lr) * CH + J * SUB + g * 4,
+             Un::SP, v);
     };
     auto keep = [&](int I, int J, f32x4 v) {
-        #pragma unroll
-        for (int i = 0; i < 4; i++)
-            A_s[(I * SUB + g * 4 + i) * AS + J * SUB + lr] = v[i];
+        *reinterpret_cast<f32x4*>(
+            A_s + (I * SUB + lr) * AS + J * SUB + g * 4) = v;
     };
     #pragma unroll
     for (int i = 0; i < 4; i++) {
-        if (lr > g * 4 + i) dqk[i] = dqe[i] = 0.f;
-        if (lr >= g * 4 + i) dzk[i] = dze[i] = 0.f;
+        if (g * 4 + i > lr) dqk[i] = dqe[i] = 0.f;
+        if (g * 4 + i >= lr) dzk[i] = dze[i] = 0.f;
     }
-    const f32x4 none = {};
     place(SQ_QK, w, w, dqk);
     keep(w, w, GEN ? dze : dzk);
     if (GEN) {
         place(SQ_ZK, w, w, dzk);
         place(SQ_QE, w, w, dqe);
     }
-    if (w % 2 == 0) {       // products go 32 tokens at a time
-        place(SQ_QK, w, w + 1, none);
+    for (int J = w + 1; J < 4; J++) {
+        const f32x4 none = {};
+        place(SQ_QK, w, J, none);
         if (GEN) {
-            place(SQ_ZK, w, w + 1, none);
-            place(SQ_QE, w, w + 1, none);
+            place(SQ_ZK, w, J, none);
+            place(SQ_QE, w, J, none);
         }
     }
     #pragma unroll
@@ -977,17 +1012,16 @@ __global__ __launch_bounds__(256) void k_delta_prep(
         if (w + s < 4) below(w + s, w);
         __syncthreads();
     }
-    for (int i = tid; i < CH * CH / 4; i += 256) {
-        const int r = i / (CH / 4), c = i % (CH / 4) * 4;
-        f32x4 v = {};
-        if (c / SUB <= r / SUB)
-            v = *reinterpret_cast<const f32x4*>(I_s + r * AS + c);
-        stw4(un + Un::square(SQ_INV, Dp) + r * CH + c, sp, v);
+    for (int i = tid; i < CH * CH / 8; i += 256) {
+        const int r = i / (CH / 8), c = i % (CH / 8) * 8;
+        float v[8] = {};
+        if (c / SUB <= r / SUB) ldv<8>(I_s + r * AS + c, v);
+        stw<T, 8>(un + Un::square(SQ_INV) + r * CH + c, Un::SP, v);
     }
 }
 
 // A sequence's chunks in order, one block per 16*VC value columns, the state
-// in registers (NS: 16-row tiles a wave, Dp <= 64 * NS); wave w has tokens
+// in registers (NS: 16-row tiles a wave, D <= 64 * NS); wave w has tokens
 // 16 w .. of a chunk.  What several waves need goes through LDS, transposed:
 // the state, v, what w is solved from and w itself.
 template <typename T, int NS, int VC, bool GEN>
@@ -997,13 +1031,15 @@ __global__ __launch_bounds__(256) void k_delta_scan(
     const int* __restrict__ slot, const int* __restrict__ pos,
     const int* __restrict__ chunks,     // [n, 2]
     const int* __restrict__ seqs,       // [m, 2] first chunk, chunks
-    int Dp, int vec)
+    int vec)
 {
-    typedef Unit<T, GEN> Un;
+    constexpr int DP = NS * 64;
+    typedef Unit<T, GEN, DP> Un;
+    typedef typename Four<T>::type Raw;
     constexpr int W = VC * 16, NT = Terms<T>::N, PAD = 16 / sizeof(T);
-    constexpr int KS = NS * 64 + PAD, TS = CH + PAD;
+    constexpr int KS = DP + PAD, TS = CH + PAD;
     constexpr int NQ = NS * 2;          // 32-channel steps over D
-    constexpr int64_t SP = (int64_t)W * KS, VP = (int64_t)W * TS;   // planes
+    constexpr int SP = W * KS, VP = W * TS;         // planes
     const int H = in.H, D = in.D, V = in.V;
     const int h = blockIdx.y, v0 = blockIdx.z * W, tid = threadIdx.x;
     const int lane = tid & 63;
@@ -1016,7 +1052,7 @@ __global__ __launch_bounds__(256) void k_delta_scan(
     T* S_s = reinterpret_cast<T*>(smem);      // [NT][W][KS] state
     T* r_s = S_s + NT * SP;                   // [NT][W][TS] right-hand side
     T* u_s = r_s + NT * VP;                   // [NT][W][TS] solution
-    T* v_s = u_s + NT * VP;                   // [GEN ? 2 : 1][NT][W][TS]
+    T* v_s = u_s + NT * VP;                   // [GEN ? 2 : 1][W][TS]
 
     f32x4 S[NS][VC];
     const bool fresh = pos[first] == 0;
@@ -1032,71 +1068,57 @@ __global__ __launch_bounds__(256) void k_delta_scan(
                                  ? 0.f : St[(int64_t)d * V + v];
             }
 
-    const int64_t tp = (int64_t)CH * Dp, sp = CH * CH;
+    // operands in flight, loaded as soon as those before are used
     Wide<T> zf[NQ], qf[NQ], inv[2], aqk[2], azk[2], aqe[2];
     Wide<T> kf[NS][2], ef[NS][2];
     f32x4 e4[NS];
-    float vv[VC * 4];
-    auto unit = [&](int ci) {
-        return Un::base(scr, (int64_t)ci * H + h, Dp);
-    };
+    Raw vv[VC];
+    auto unit = [&](int ci) { return Un::at(scr, (int64_t)ci * H + h); };
     auto load_zq = [&](int ci) {
-        const T* u = unit(ci) + (int64_t)(w * 16 + lr) * Dp + g * 8;
+        const T* u = unit(ci) + (w * 16 + lr) * DP + g * 8;
         #pragma unroll
         for (int d = 0; d < NQ; d++) {
-            zf[d] = d * 32 < Dp ? ldw(u + Un::tall(TALL_Z, Dp) + d * 32, tp)
-                                : wide_zero<T>();
-            qf[d] = d * 32 < Dp ? ldw(u + Un::tall(TALL_Q, Dp) + d * 32, tp)
-                                : wide_zero<T>();
+            zf[d] = ldw(u + Un::tall(TALL_Z) + d * 32, Un::TP);
+            qf[d] = ldw(u + Un::tall(TALL_Q) + d * 32, Un::TP);
         }
     };
     auto load_square = [&](int ci, int m, Wide<T>* f) {
-        const T* u = unit(ci) + Un::square(m, Dp) + (w * 16 + lr) * CH
-                     + g * 8;
+        const T* u = unit(ci) + Un::square(m) + (w * 16 + lr) * CH + g * 8;
         #pragma unroll
-        for (int j = 0; j < 2; j++)
-            f[j] = j * 2 <= w ? ldw(u + j * 32, sp) : wide_zero<T>();
+        for (int j = 0; j < 2; j++) f[j] = ldw(u + j * 32, Un::SP);
     };
     auto load_k = [&](int ci) {
         const T* u = unit(ci);
-        const float* fd = (const float*)(u + Un::fade(Dp));
+        const float* fd = (const float*)(u + Un::fade);
         #pragma unroll
         for (int x = 0; x < NS; x++) {
             const int d = (w + x * 4) * 16;
-            const bool in_d = d < Dp;
-            e4[x] = in_d ? *reinterpret_cast<const f32x4*>(fd + d + g * 4)
-                         : f32x4{};
+            e4[x] = *reinterpret_cast<const f32x4*>(fd + d + g * 4);
             #pragma unroll
             for (int j = 0; j < 2; j++) {
-                const int64_t at = (int64_t)(d + lr) * CH + j * 32 + g * 8;
-                kf[x][j] = in_d ? ldw(u + Un::tall(TALL_K, Dp) + at, tp)
-                                : wide_zero<T>();
-                if (GEN)
-                    ef[x][j] = in_d ? ldw(u + Un::tall(TALL_E, Dp) + at, tp)
-                                    : wide_zero<T>();
+                const int at = (d + lr) * CH + j * 32 + g * 8;
+                kf[x][j] = ldw(u + Un::tall(TALL_K) + at, Un::TP);
+                if (GEN) ef[x][j] = ldw(u + Un::tall(TALL_E) + at, Un::TP);
             }
         }
     };
-    // token lane of a chunk, columns (wave * VC + ..) * 4
+    // token `lane` of a chunk, columns (wave * VC + q) * 4
     auto load_v = [&](int ci) {
         const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
         const T* r = in.x + (int64_t)(t0 + min(lane, n - 1)) * in.ld + in.ov
-                     + h * V + v0;
+                     + h * V;
         #pragma unroll
         for (int q = 0; q < VC; q++) {
-            const int c = (w * VC + q) * 4;
-            #pragma unroll
-            for (int e = 0; e < 4; e++) vv[q * 4 + e] = 0.f;
-            if (lane >= n) continue;
-            if (vec) {
-                if (v0 + c < V) ldv<4>(r + c, vv + q * 4);
-            } else
+            const int c = v0 + (w * VC + q) * 4;
+            if (vec)
+                vv[q] = *reinterpret_cast<const Raw*>(r + min(c, V - 4));
+            else
                 #pragma unroll
                 for (int e = 0; e < 4; e++)
-                    if (v0 + c + e < V) vv[q * 4 + e] = ldf(r + c + e);
+                    vv[q][e] = ldf(r + min(c + e, V - 1));
         }
     };
-    auto solve_operand = [&](const T* s, int c, int j) {
+    auto wide_at = [&](const T* s, int c, int j) {
         return ldw(s + (c * 16 + lr) * TS + j * 32 + g * 8, VP);
     };
     load_v(c0);
@@ -1112,10 +1134,15 @@ __global__ __launch_bounds__(256) void k_delta_scan(
     for (int ci = c0; ci < c0 + nc; ++ci) {
         const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
         const int nx = min(ci + 1, c0 + nc - 1);
-        T* vb = GEN && (ci & 1) ? v_s + NT * VP : v_s;
+        T* vb = GEN && (ci & 1) ? v_s + VP : v_s;
         #pragma unroll
-        for (int e = 0; e < VC * 4; e++)
-            stw(vb + (w * VC * 4 + e) * TS + lane, VP, vv[e]);
+        for (int q = 0; q < VC; q++)
+            #pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int c = (w * VC + q) * 4 + e;
+                stf(vb + c * TS + lane, lane < n && v0 + c < V
+                                            ? (float)vv[q][e] : 0.f);
+            }
         #pragma unroll
         for (int x = 0; x < NS; x++) {
             const int d = (w + x * 4) * 16 + g * 4;
@@ -1128,8 +1155,7 @@ __global__ __launch_bounds__(256) void k_delta_scan(
         // what z and q read from the state before the chunk
         f32x4 az[VC] = {}, ao[VC] = {};
         #pragma unroll
-        for (int d = 0; d < NQ; d++) {
-            if (d * 32 >= Dp) continue;
+        for (int d = 0; d < NQ; d++)
             #pragma unroll
             for (int c = 0; c < VC; c++) {
                 const Wide<T> b = ldw(S_s + (c * 16 + lr) * KS + d * 32
@@ -1137,19 +1163,17 @@ __global__ __launch_bounds__(256) void k_delta_scan(
                 az[c] = mma(zf[d], b, az[c]);
                 ao[c] = mma(qf[d], b, ao[c]);
             }
-        }
         load_zq(nx);
         if (GEN) {
             #pragma unroll
-            for (int j = 0; j < 2; j++) {
-                if (j * 2 > w) continue;
+            for (int j = 0; j < 2; j++)
                 #pragma unroll
                 for (int c = 0; c < VC; c++) {
-                    const Wide<T> b = solve_operand(vb, c, j);
+                    const Frag<T> b = frag8(vb + (c * 16 + lr) * TS + j * 32
+                                            + g * 8);
                     az[c] = mma(azk[j], b, az[c]);
                     ao[c] = mma(aqk[j], b, ao[c]);
                 }
-            }
             load_square(nx, SQ_ZK, azk);
             load_square(nx, SQ_QK, aqk);
         }
@@ -1158,7 +1182,7 @@ __global__ __launch_bounds__(256) void k_delta_scan(
             const int at = (c * 16 + lr) * TS + w * 16 + g * 4;
             if (!GEN) {
                 float f[4];
-                ldv<4>(vb + at, f);     // v itself: its first term
+                ldv<4>(vb + at, f);
                 #pragma unroll
                 for (int i = 0; i < 4; i++) az[c][i] = f[i] - az[c][i];
             }
@@ -1167,27 +1191,40 @@ __global__ __launch_bounds__(256) void k_delta_scan(
         lds_barrier();
         f32x4 u[VC] = {};
         #pragma unroll
-        for (int j = 0; j < 2; j++) {
-            if (j * 2 > w) continue;
+        for (int j = 0; j < 2; j++)
             #pragma unroll
             for (int c = 0; c < VC; c++)
-                u[c] = mma(inv[j], solve_operand(r_s, c, j), u[c]);
-        }
+                u[c] = mma(inv[j], wide_at(r_s, c, j), u[c]);
         load_square(nx, SQ_INV, inv);
         #pragma unroll
         for (int c = 0; c < VC; c++)
             stw4(u_s + (c * 16 + lr) * TS + w * 16 + g * 4, VP,
                  GEN ? -u[c] : u[c]);
         lds_barrier();
+        // results and the next state
         #pragma unroll
-        for (int j = 0; j < 2; j++) {
-            if (j * 2 > w) continue;
+        for (int x = 0; x < NS; x++)
             #pragma unroll
-            for (int c = 0; c < VC; c++)
-                ao[c] = mma(GEN ? aqe[j] : aqk[j],
-                            solve_operand(u_s, c, j), ao[c]);
-        }
+            for (int c = 0; c < VC; c++) S[x][c] *= e4[x];
+        #pragma unroll
+        for (int j = 0; j < 2; j++)
+            #pragma unroll
+            for (int c = 0; c < VC; c++) {
+                const Wide<T> b = wide_at(u_s, c, j);
+                ao[c] = mma(GEN ? aqe[j] : aqk[j], b, ao[c]);
+                #pragma unroll
+                for (int x = 0; x < NS; x++)
+                    S[x][c] = mma(GEN ? ef[x][j] : kf[x][j], b, S[x][c]);
+                if (GEN) {
+                    const Frag<T> v = frag8(vb + (c * 16 + lr) * TS + j * 32
+                                            + g * 8);
+                    #pragma unroll
+                    for (int x = 0; x < NS; x++)
+                        S[x][c] = mma(kf[x][j], v, S[x][c]);
+                }
+            }
         load_square(nx, GEN ? SQ_QE : SQ_QK, GEN ? aqe : aqk);
+        load_k(nx);
         #pragma unroll
         for (int c = 0; c < VC; c++) {
             const int v = v0 + c * 16 + lr;
@@ -1198,29 +1235,6 @@ __global__ __launch_bounds__(256) void k_delta_scan(
                     o[((int64_t)(t0 + t) * H + h) * V + v] = ao[c][i];
             }
         }
-        // the next state
-        #pragma unroll
-        for (int x = 0; x < NS; x++)
-            #pragma unroll
-            for (int c = 0; c < VC; c++) S[x][c] *= e4[x];
-        #pragma unroll
-        for (int j = 0; j < 2; j++)
-            #pragma unroll
-            for (int c = 0; c < VC; c++) {
-                const Wide<T> b = solve_operand(GEN ? vb : u_s, c, j);
-                #pragma unroll
-                for (int x = 0; x < NS; x++)
-                    if ((w + x * 4) * 16 < Dp)
-                        S[x][c] = mma(kf[x][j], b, S[x][c]);
-                if (GEN) {
-                    const Wide<T> b2 = solve_operand(u_s, c, j);
-                    #pragma unroll
-                    for (int x = 0; x < NS; x++)
-                        if ((w + x * 4) * 16 < Dp)
-                            S[x][c] = mma(ef[x][j], b2, S[x][c]);
-                }
-            }
-        load_k(nx);
     }
     #pragma unroll
     for (int x = 0; x < NS; x++)
@@ -1234,25 +1248,25 @@ __global__ __launch_bounds__(256) void k_delta_scan(
             }
 }
 
-static int delta_pad(int D) { return (D + DB - 1) / DB * DB; }
+// key channels of the chunk kernels' tiles
+static int delta_tiles(int D) { return D <= 64 ? 64 : D <= 128 ? 128 : 256; }
 
 extern "C" int64_t delta_scratch_floats(int gen, int n_chunks, int H, int D)
 {
-    const int Dp = delta_pad(D);
-    return (int64_t)n_chunks * H
-           * (gen ? Unit<float, true>::floats(Dp)
-                  : Unit<float, false>::floats(Dp));
+    const int64_t dp = delta_tiles(D);
+    return (int64_t)n_chunks * H * ((gen ? 4 : 3) * CH * dp
+                                    + (gen ? 4 : 2) * CH * CH + dp);
 }
 
 template <typename T, int NS, int VC, bool GEN>
 static void scan_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
                     const int* slot, const int* pos, const int* chunks,
-                    const int* seqs, int n_seqs, int Dp, int vec,
-                    hipStream_t stream)
+                    const int* seqs, int n_seqs, int vec, hipStream_t stream)
 {
     constexpr int W = VC * 16, PAD = 16 / sizeof(T), es = sizeof(T);
-    constexpr int lds = Terms<T>::N * es
-        * (W * (NS * 64 + PAD) + (GEN ? 4 : 3) * W * (CH + PAD));
+    constexpr int NT = Terms<T>::N;
+    constexpr int lds = es * W * (NT * (NS * 64 + PAD)
+                                  + (2 * NT + (GEN ? 2 : 1)) * (CH + PAD));
     static bool once = false;
     if (!once) {
         (void)hipFuncSetAttribute(
@@ -1262,17 +1276,19 @@ static void scan_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
     }
     k_delta_scan<T, NS, VC, GEN>
         <<<dim3(n_seqs, in.H, (in.V + W - 1) / W), 256, lds, stream>>>(
-            o, scr, in, state, slot, pos, chunks, seqs, Dp, vec);
+            o, scr, in, state, slot, pos, chunks, seqs, vec);
 }
 
-template <typename T, bool GEN>
+template <typename T, bool GEN, int NS>
 static int chunks_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
                      const int* slot, const int* pos, const int* chunks,
                      int n_chunks, const int* seqs, int n_seqs,
                      hipStream_t stream)
 {
-    const int H = in.H, D = in.D, V = in.V, Dp = delta_pad(D);
-    if (D < 1 || V < 1 || D > 256) return (int)hipErrorInvalidValue;
+    static_assert(Unit<T, GEN, NS * 64>::floats
+                  == (GEN ? 4 : 3) * CH * NS * 64 + (GEN ? 4 : 2) * CH * CH
+                     + NS * 64, "scratch");
+    const int H = in.H, D = in.D, V = in.V;
     const int v8 = D % 8 == 0 && in.oq % 8 == 0 && in.ok % 8 == 0
                    && in.oa % 8 == 0 && in.ld % 8 == 0;
     const int v4 = V % 4 == 0 && in.ov % 4 == 0 && in.ld % 4 == 0;
@@ -1281,23 +1297,36 @@ static int chunks_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
     static bool once = false;
     if (!once) {
         (void)hipFuncSetAttribute(
-            (const void*)k_delta_prep<T, GEN>,
+            (const void*)k_delta_prep<T, GEN, NS * 64>,
             hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
         once = true;
     }
-    k_delta_prep<T, GEN><<<dim3(n_chunks, H), 256,
-                           part > solve ? part : solve, stream>>>(
-        scr, in, chunks, Dp, v8);
+    k_delta_prep<T, GEN, NS * 64><<<dim3(n_chunks, H), 256,
+                                    part > solve ? part : solve, stream>>>(
+        scr, in, chunks, v8);
     // wide strips share the loads of the factors, narrow ones fill the chip
-    const bool two = (int64_t)n_seqs * H * ((V + 31) / 32) >= 256;
-    #define DC(NS, VC)                                                     \
-        scan_go<T, NS, VC, GEN>(o, scr, in, state, slot, pos, chunks,      \
-                                seqs, n_seqs, Dp, v4, stream)
-    if (Dp <= 64) { if (two) DC(1, 2); else DC(1, 1); }
-    else if (Dp <= 128) { if (two) DC(2, 2); else DC(2, 1); }
-    else DC(4, 1);
-    #undef DC
+    const bool two = NS < 4 && (int64_t)n_seqs * H * ((V + 31) / 32) >= 256;
+    if (two)
+        scan_go<T, NS, NS < 4 ? 2 : 1, GEN>(o, scr, in, state, slot, pos,
+                                            chunks, seqs, n_seqs, v4, stream);
+    else
+        scan_go<T, NS, 1, GEN>(o, scr, in, state, slot, pos, chunks, seqs,
+                               n_seqs, v4, stream);
     return (int)hipGetLastError();
+}
+
+template <typename T, bool GEN>
+static int chunks_for(float* o, float* scr, const DeltaIn<T>& in,
+                      float* state, const int* slot, const int* pos,
+                      const int* chunks, int n_chunks, const int* seqs,
+                      int n_seqs, hipStream_t stream)
+{
+    if (in.D < 1 || in.V < 1 || in.D > 256) return (int)hipErrorInvalidValue;
+    const int dp = delta_tiles(in.D);
+    auto go = dp == 64 ? chunks_go<T, GEN, 1> : dp == 128
+              ? chunks_go<T, GEN, 2> : chunks_go<T, GEN, 4>;
+    return go(o, scr, in, state, slot, pos, chunks, n_chunks, seqs, n_seqs,
+              stream);
 }
 
 // Portions of whole sequences in chunks of 64 rows.  chunks int32 [n, 2]
@@ -1312,10 +1341,10 @@ extern "C" int delta_chunks(
     hipStream_t stream)
 {
     #define DC_GO(T, GEN)                                                  \
-        chunks_go<T, GEN>((float*)o, (float*)scr, DELTA_IN(T),             \
-                          (float*)state, (const int*)slot,                 \
-                          (const int*)pos, (const int*)chunks, n_chunks,   \
-                          (const int*)seqs, n_seqs, stream)
+        chunks_for<T, GEN>((float*)o, (float*)scr, DELTA_IN(T),            \
+                           (float*)state, (const int*)slot,                \
+                           (const int*)pos, (const int*)chunks, n_chunks,  \
+                           (const int*)seqs, n_seqs, stream)
     if (f32) return gen ? DC_GO(float, true) : DC_GO(float, false);
     return gen ? DC_GO(bf16, true) : DC_GO(bf16, false);
     #undef DC_GO

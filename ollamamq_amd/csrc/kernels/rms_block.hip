@@ -469,38 +469,40 @@ template <typename T, typename P, int VEC, bool FR>
 __global__ __launch_bounds__(256) void k_head_gate(
     T* __restrict__ out, const float* __restrict__ o, float mult,
     const float* __restrict__ w, int w_stride, Rows<P> gate, int og,
-    int silu, int64_t units, int H, int V, int L, float eps)
+    int silu, int H, int V, int L, float eps)
 {
     const int lane = threadIdx.x & (L - 1);
-    const int64_t u = ((int64_t)blockIdx.x * 256 + threadIdx.x) / L;
-    if (u >= units) return;
-    const int64_t t = u / H;
-    const int h = (int)(u % H);
-    const float* row = o + u * V;
+    const int64_t t = blockIdx.x;
+    const int per = 256 / L, step = gridDim.y * per;
     const bool one = V <= L * VEC;          // the head fits the lanes
-    float x[VEC], s = 0.f;
-    for (int c = lane * VEC; c < V; c += L * VEC) {
-        ldv<VEC>(row + c, x);
-        #pragma unroll
-        for (int i = 0; i < VEC; i++) s += x[i] * x[i];
-    }
-    for (int k = L / 2; k; k >>= 1) s += __shfl_xor(s, k, 64);
-    const float f = mult / sqrtf(s * (mult * mult / V) + eps);
-    for (int c = lane * VEC; c < V; c += L * VEC) {
-        float g[VEC];
-        if (!one) ldv<VEC>(row + c, x);
-        ldrow<VEC>(gate, t, og + h * V + c, g);
-        #pragma unroll
-        for (int i = 0; i < VEC; i++)
-            x[i] *= f * sigmoid_of<T>(g[i]) * (silu ? g[i] : 1.f);
-        if (w) {
-            ldv<VEC>(w + h * w_stride + c, g);
+    for (int h = blockIdx.y * per + threadIdx.x / L; h < H; h += step) {
+        const float* row = o + (t * H + h) * V;
+        float x[VEC], g[VEC], s = 0.f;
+        for (int c = lane * VEC; c < V; c += L * VEC) {
+            ldv<VEC>(row + c, x);
+            if (one) ldrow<VEC>(gate, t, og + h * V + c, g);
             #pragma unroll
-            for (int i = 0; i < VEC; i++) x[i] *= g[i];
+            for (int i = 0; i < VEC; i++) s += x[i] * x[i];
         }
-        const int n = h * V + c;
-        stv<VEC>(out + (FR ? frag_row_off(t, n, H * V)
-                           : t * (int64_t)H * V + n), x);
+        for (int k = L / 2; k; k >>= 1) s += __shfl_xor(s, k, 64);
+        const float f = mult / sqrtf(s * (mult * mult / V) + eps);
+        for (int c = lane * VEC; c < V; c += L * VEC) {
+            if (!one) {
+                ldv<VEC>(row + c, x);
+                ldrow<VEC>(gate, t, og + h * V + c, g);
+            }
+            #pragma unroll
+            for (int i = 0; i < VEC; i++)
+                x[i] *= f * sigmoid_of<T>(g[i]) * (silu ? g[i] : 1.f);
+            if (w) {
+                ldv<VEC>(w + h * w_stride + c, g);
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) x[i] *= g[i];
+            }
+            const int n = h * V + c;
+            stv<VEC>(out + (FR ? frag_row_off(t, n, H * V)
+                               : t * (int64_t)H * V + n), x);
+        }
     }
 }
 
@@ -515,13 +517,13 @@ extern "C" int head_gate(
     if (frag && f32) return (int)hipErrorInvalidValue;
     int L = 64;
     while (L > 4 && L / 2 * (v4 ? 4 : 1) >= V) L /= 2;
-    const int64_t units = (int64_t)T_rows * H;
-    const int grid = (int)((units * L + 255) / 256);
+    const int want = (H * L + 255) / 256;
+    const dim3 grid(T_rows, T_rows <= 256 ? want : (want + 1) / 2);
     #define HG(T, P, VE, FR)                                               \
         k_head_gate<T, P, VE, FR><<<grid, 256, 0, stream>>>(               \
             (T*)out, (const float*)o, mult, (const float*)w, w_stride,     \
             Rows<P>{(const P*)gate, n_part, part_stride, ld}, og, silu,    \
-            units, H, V, L, eps)
+            H, V, L, eps)
     #define HG_V(T, P, FR)                                                 \
         do { if (v4) HG(T, P, 4, FR); else HG(T, P, 1, FR); } while (0)
     if (f32) HG_V(float, float, false);

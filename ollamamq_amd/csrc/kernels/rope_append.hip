@@ -126,72 +126,68 @@ __global__ __launch_bounds__(256) void k_qkv_norm_rope(
     const float* __restrict__ gain, int vnorm, float eps,
     const float* __restrict__ table, int dims,
     const int* __restrict__ slot, const int* __restrict__ pos,
-    const int* __restrict__ ptab, int T_rows, int H, int G, int D, int V,
-    int Dp, int Vp, int psz, int maxp, int L)
+    const int* __restrict__ ptab, int H, int G, int D, int V, int Dp, int Vp,
+    int psz, int maxp, int L)
 {
     const int lane = threadIdx.x & (L - 1);
-    const int64_t u = ((int64_t)blockIdx.x * 256 + threadIdx.x) / L;
-    const int U = H + 2 * G;
-    const int64_t t = u / U;
-    if (t >= T_rows) return;
-    const int unit = (int)(u % U);
-    const bool is_q = unit < H, is_v = unit >= H + G;
-    const int wide = is_v ? V : D;
-    const int c0 = is_v ? (H + G) * D + (unit - H - G) * V : unit * D;
-    const float* wt = is_v ? nullptr : is_q ? qn : kn;
-    float x[KEEP][VEC], s = 0.f;
-    #pragma unroll
-    for (int j = 0; j < KEEP; j++) {
-        const int c = (j * L + lane) * VEC;
-        #pragma unroll
-        for (int i = 0; i < VEC; i++) x[j][i] = 0.f;
-        if (c < wide) ldrow<VEC>(p, t, c0 + c, x[j]);
-        #pragma unroll
-        for (int i = 0; i < VEC; i++) s += x[j][i] * x[j][i];
-    }
-    for (int o = L / 2; o; o >>= 1) s += __shfl_xor(s, o, 64);
-    const float f = is_v && !vnorm ? 1.f : 1.f / sqrtf(s / wide + eps);
+    const int64_t t = blockIdx.x;
     const int ps = pos[t], half = dims / 2;
+    const int64_t page = ptab[(int64_t)slot[t] * maxp + ps / psz];
+    const int off = ps % psz, step = gridDim.y * (256 / L);
     const float* cs = table + (int64_t)ps * dims;
-    const float up = is_q && gain ? gain[unit] : 1.f;
-    T* dst;
-    if (is_q) dst = q_out + (t * H + unit) * Dp;
-    else {
-        const int64_t page = ptab[(int64_t)slot[t] * maxp + ps / psz];
-        const int off = ps % psz;
-        dst = is_v ? vpool + ((page * G + unit - H - G) * psz + off) * Vp
-                   : kpool + ((page * G + unit - H) * psz + off) * Dp;
-    }
-    const int end = is_q ? Dp : wide;       // queries end in zeros
-    #pragma unroll
-    for (int j = 0; j < KEEP; j++) {
-        const int c = (j * L + lane) * VEC;
-        if (c >= end) continue;
-        if (c < wide) {
-            if (wt) {
-                float g[VEC];
-                ldv<VEC>(wt + c, g);
-                #pragma unroll
-                for (int i = 0; i < VEC; i++) x[j][i] *= g[i];
-            }
-            if (!is_v && c < dims) {
-                const bool low = c < half;
-                const int far = low ? c + half : c - half;
-                const int a = low ? c : far;
-                float y[VEC], g[VEC];
-                ldrow<VEC>(p, t, c0 + far, y);
-                ldv<VEC>(wt + far, g);
-                #pragma unroll
-                for (int i = 0; i < VEC; i++) {
-                    const float co = cs[2 * (a + i)], si = cs[2 * (a + i) + 1];
-                    x[j][i] = x[j][i] * co
-                              + (low ? -si : si) * y[i] * g[i];
-                }
-            }
+    for (int unit = blockIdx.y * (256 / L) + threadIdx.x / L;
+         unit < H + 2 * G; unit += step) {
+        const bool is_q = unit < H, is_v = unit >= H + G;
+        const int wide = is_v ? V : D;
+        const int c0 = is_v ? (H + G) * D + (unit - H - G) * V : unit * D;
+        const float* wt = is_v ? nullptr : is_q ? qn : kn;
+        float x[KEEP][VEC], s = 0.f;
+        #pragma unroll
+        for (int j = 0; j < KEEP; j++) {
+            const int c = (j * L + lane) * VEC;
             #pragma unroll
-            for (int i = 0; i < VEC; i++) x[j][i] *= f * up;
+            for (int i = 0; i < VEC; i++) x[j][i] = 0.f;
+            if (c < wide) ldrow<VEC>(p, t, c0 + c, x[j]);
+            #pragma unroll
+            for (int i = 0; i < VEC; i++) s += x[j][i] * x[j][i];
         }
-        stv<VEC>(dst + c, x[j]);
+        for (int o = L / 2; o; o >>= 1) s += __shfl_xor(s, o, 64);
+        const float f = is_v && !vnorm ? 1.f : 1.f / sqrtf(s / wide + eps);
+        const float up = is_q && gain ? gain[unit] : 1.f;
+        T* dst = is_q ? q_out + (t * H + unit) * Dp
+            : is_v ? vpool + ((page * G + unit - H - G) * psz + off) * Vp
+                   : kpool + ((page * G + unit - H) * psz + off) * Dp;
+        const int end = is_q ? Dp : wide;       // queries end in zeros
+        #pragma unroll
+        for (int j = 0; j < KEEP; j++) {
+            const int c = (j * L + lane) * VEC;
+            if (c >= end) continue;
+            if (c < wide) {
+                if (wt) {
+                    float g[VEC];
+                    ldv<VEC>(wt + c, g);
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) x[j][i] *= g[i];
+                }
+                if (!is_v && c < dims) {
+                    const bool low = c < half;
+                    const int far = low ? c + half : c - half;
+                    const int a = low ? c : far;
+                    float y[VEC], g[VEC];
+                    ldrow<VEC>(p, t, c0 + far, y);
+                    ldv<VEC>(wt + far, g);
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++) {
+                        const float co = cs[2 * (a + i)], si = cs[2 * (a + i) + 1];
+                        x[j][i] = x[j][i] * co
+                                  + (low ? -si : si) * y[i] * g[i];
+                    }
+                }
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) x[j][i] *= f * up;
+            }
+            stv<VEC>(dst + c, x[j]);
+        }
     }
 }
 
@@ -210,10 +206,18 @@ extern "C" int qkv_norm_rope(
                     && part_stride % 4 == 0;
     int L = 64;
     if (v4) while (L > 4 && L * 2 >= Dp && L * 2 >= Vp) L /= 2;
-    const int64_t lanes = (int64_t)T_rows * (H + 2 * G) * L;
-    const int grid = (int)((lanes + 255) / 256);
-    #define QN(T, P, VE, KE)                                                       k_qkv_norm_rope<T, P, VE, KE><<<grid, 256, 0, stream>>>(                       (T*)q_out, (T*)kpool, (T*)vpool,                                           Rows<P>{(const P*)p, n_part, part_stride, ld},                             (const float*)qn, (const float*)kn, (const float*)gain, vnorm,             eps, (const float*)table, dims, (const int*)slot,                          (const int*)pos, (const int*)ptab, T_rows, H, G, D, V, Dp, Vp,             psz, maxp, L)
-    #define QN_V(T, P)                                                             do { if (v4) QN(T, P, 4, 1); else QN(T, P, 1, 4); } while (0)
+    const int want = ((H + 2 * G) * L + 255) / 256;
+    const dim3 grid(T_rows, T_rows <= 256 ? want : (want + 2) / 3);
+    #define QN(T, P, VE, KE)                                               \
+        k_qkv_norm_rope<T, P, VE, KE><<<grid, 256, 0, stream>>>(           \
+            (T*)q_out, (T*)kpool, (T*)vpool,                               \
+            Rows<P>{(const P*)p, n_part, part_stride, ld},                 \
+            (const float*)qn, (const float*)kn, (const float*)gain, vnorm, \
+            eps, (const float*)table, dims, (const int*)slot,              \
+            (const int*)pos, (const int*)ptab, H, G, D, V, Dp, Vp, psz,    \
+            maxp, L)
+    #define QN_V(T, P)                                                     \
+        do { if (v4) QN(T, P, 4, 1); else QN(T, P, 1, 4); } while (0)
     if (f32) QN_V(float, float);
     else if (p32) QN_V(bf16, float);
     else QN_V(bf16, bf16);

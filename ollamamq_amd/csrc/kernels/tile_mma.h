@@ -82,7 +82,15 @@ template <int VEC, typename P>
 DEV void ldrow(const Rows<P>& r, int64_t t, int c, float* v) {
     const P* p = r.p + t * r.ld + c;
     ldv<VEC>(p, v);
-    for (int s = 1; s < r.n_part; s++) {
+    int s = 1;
+    for (; s + 1 < r.n_part; s += 2) {      // two at a time: half the waits
+        float u[VEC], w[VEC];
+        ldv<VEC>(p + s * r.part_stride, u);
+        ldv<VEC>(p + (s + 1) * r.part_stride, w);
+        #pragma unroll
+        for (int i = 0; i < VEC; i++) v[i] = v[i] + u[i] + w[i];
+    }
+    if (s < r.n_part) {
         float u[VEC];
         ldv<VEC>(p + s * r.part_stride, u);
         #pragma unroll

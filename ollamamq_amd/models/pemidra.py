@@ -266,13 +266,28 @@ PEMIDRA_PRESETS = {
 }
 
 
-def _offsets(sizes):
-    """First column of every part."""
+def _offsets(parts):
+    """First column of every part (a matrix or its rows)."""
     out, at = [], 0
-    for n in sizes:
+    for p in parts:
         out.append(at)
-        at += n
+        at += p if isinstance(p, int) else p.shape[0]
     return out
+
+
+def _whole(m, dim):
+    """A low-rank projection with its rank filled up to whole vectors."""
+    fill = -m.shape[dim] % 8
+    return torch.nn.functional.pad(m, (0, fill) if dim == 1
+                                   else (0, 0, 0, fill))
+
+
+def _aligned(cols, low):
+    """Wide projections, then low-rank ones from whole vectors on."""
+    fill = -sum(m.shape[0] for m in cols) % 8
+    if fill:
+        cols = cols + [low[0].new_zeros(fill, low[0].shape[1])]
+    return cols + [_whole(m, 0) for m in low]
 
 
 class PemidraLayer(HybridLayer):
@@ -293,19 +308,19 @@ class PemidraLayer(HybridLayer):
             cols = [mat("q", qk), mat("k", qk), mat("v", v), mat("g", v)]
             self.mix = ops.LightningWeights(
                 heads=m.heads, dim=m.dim, vdim=m.vdim,
-                offsets=tuple(_offsets([qk, qk, v, v])),
+                offsets=tuple(_offsets(cols)),
                 powers=ops.decay_powers(m.decay, self.ls1.device), norm=None,
                 eps=eps, act=False, scale=m.dim ** -0.5, per_head=True,
                 gate="silu")
             outs = [("w_o", "o", v)]
         elif spec.type == "general_delta":
             n = m.heads * m.dim
-            cols = [mat(c, n) for c in "rkvag"] + [mat("w1", None)]
-            rank = cols[-1].shape[0]
+            low = mat("w1", None)
+            cols = _aligned([mat(c, n) for c in "rkvag"], [low])
             self.mix = ops.GeneralDeltaWeights(
                 heads=m.heads, dim=m.dim,
-                offsets=tuple(_offsets([n] * 5 + [rank])),
-                w2=put(mat("w2", n, rank)).contiguous(),
+                offsets=(*_offsets(cols)[:5], _offsets(cols)[-1]),
+                w2=put(_whole(mat("w2", n, low.shape[0]), 1)).contiguous(),
                 w0=vec(mix + "w0", n), a_bias=vec(mix + "a.b", n),
                 norm=vec(mix + "norm", n, mean=1.0), eps=eps)
             outs = [("w_o", "o", n)]
@@ -329,18 +344,16 @@ class PemidraLayer(HybridLayer):
 
     def _parallel(self, m, mat, mix, vec, put, rope, eps):
         a, r = m.left, m.right
-        parts = [("left.q", a.heads * a.dim), ("left.k", a.kv_heads * a.dim),
-                 ("left.v", a.kv_heads * a.vdim),
-                 ("right.q", r.kv_heads * r.dim),
-                 ("right.k", r.kv_heads * r.dim),
-                 ("right.v", r.heads * r.vdim), ("right.a1", None),
-                 ("right.g1", None), ("left.g", a.heads),
-                 ("right.b", r.heads)]
-        cols = [mat(n, rows) for n, rows in parts]
-        at = dict(zip((n for n, _ in parts),
-                      _offsets([c.shape[0] for c in cols])))
-        rank = {n: c.shape[0] for (n, _), c in zip(parts, cols)}
-        self.gate_at = at["left.g"]
+        cols = [mat(n, rows) for n, rows in (
+            ("left.q", a.heads * a.dim), ("left.k", a.kv_heads * a.dim),
+            ("left.v", a.kv_heads * a.vdim), ("right.q", r.kv_heads * r.dim),
+            ("right.k", r.kv_heads * r.dim), ("right.v", r.heads * r.vdim),
+            ("left.g", a.heads), ("right.b", r.heads))]
+        a1, g1 = mat("right.a1", None), mat("right.g1", None)
+        at = _offsets(cols)
+        cols = _aligned(cols, [a1, g1])
+        at_a1, at_g1 = _offsets(cols)[-2:]
+        self.gate_at = at[6]
         self.rope = rope(a.rope)
         temp = vec(mix + "left.temp", a.heads, mean=1.0)
         self.heads = ops.HeadNorms(
@@ -356,14 +369,13 @@ class PemidraLayer(HybridLayer):
                            ("v", r.heads * r.vdim))])
         self.delta = ops.GatedDeltaWeights(
             heads=r.heads, kv_heads=r.kv_heads, dim=r.dim, vdim=r.vdim,
-            offsets=(at["right.q"], at["right.b"], at["right.a1"],
-                     at["right.g1"]),
+            offsets=(at[3], at[7], at_a1, at_g1),
             conv=taps.to(temp.device).float().t().contiguous(),
-            a2=put(mat("right.a2", r.heads * r.dim, rank["right.a1"]))
+            a2=put(_whole(mat("right.a2", r.heads * r.dim, a1.shape[0]), 1))
             .contiguous(),
             rate=vec(mix + "right.A_log", r.heads).exp(),
             dt_bias=vec(mix + "right.dt_bias", r.heads * r.dim),
-            g2=put(mat("right.g2", r.heads * r.vdim, rank["right.g1"]))
+            g2=put(_whole(mat("right.g2", r.heads * r.vdim, g1.shape[0]), 1))
             .contiguous(),
             norm=vec(mix + "right.norm", r.vdim, mean=1.0), eps=eps)
         W = cols[0].shape[1]
@@ -409,7 +421,7 @@ class PemidraModel(HybridModel):
         self._pack_weights()
 
     def _mixer(self, layer, run, h, cache, slot_ids, positions, meta, frag):
-        p = ops.linear_parts(h, layer.w_in, layer.packs.get("w_in"))
+        p = ops.linear_parts(h, layer.w_in, layer.packs.get("w_in"), most=3)
         state = cache.state[run]
 
         def out(name, o):

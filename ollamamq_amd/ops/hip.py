@@ -822,12 +822,12 @@ def _frag_rows(M, cols, like):
                     M, cols)
 
 
-def _parts_ksplit(N, K):
+def _parts_ksplit(N, K, most=8):
     """Split for a product whose consumer folds the partial sums: the one
     that loads the 256 CUs most evenly, smaller if nearly as good."""
     tiles, nb = N // 32, K // 64
     best, best_eff = 1, 0.0
-    for ks in range(1, 9):
+    for ks in range(1, most + 1):
         if nb < ks * 8:
             break
         n = tiles * ks
@@ -837,10 +837,10 @@ def _parts_ksplit(N, K):
     return best
 
 
-def _linear_frag(x, N, packed, parts):
+def _linear_frag(x, N, packed, parts, most=8):
     """Weight-streaming product of an activation in fragment layout."""
     M, K = x.rows, x.cols
-    ks = _parts_ksplit(N, K) if parts else _wstream_ksplit(N, K)
+    ks = _parts_ksplit(N, K, most) if parts else _wstream_ksplit(N, K)
     y = part = None
     if ks > 1:
         part = torch.empty((ks, M, N), dtype=torch.float32,
@@ -879,17 +879,17 @@ def linear_gu_frag(x, packed, N, glu="silu"):
     return FragRows(act, x.rows, N // 2)
 
 
-def linear_parts(x, weight, packed=None):
+def linear_parts(x, weight, packed=None, most=8):
     """Decode: the weight-streaming product, left as split-K partial sums
     where it splits (the next kernel folds them in)."""
     N = weight.shape[0]
     if isinstance(x, FragRows):
-        return _linear_frag(x, N, packed, True)
+        return _linear_frag(x, N, packed, True, most)
     M, K = x.shape
     if packed is not None and USE_WSTREAM and M <= 64 and N <= _WS_MAX_N \
             and x.dtype == torch.bfloat16 and x.stride(1) == 1:
         ks = int(_WS_KS) if _WS_KS else _wstream_ksplit(N, K)
-        if ks > 1:
+        if 1 < ks <= most:
             part = torch.empty((ks, M, N), dtype=torch.float32,
                                device=x.device)
             xlds = (_WS_XLDS if M <= 32 and N * K * 2 > (64 << 20) else 0)

@@ -239,7 +239,8 @@ class GatedDeltaWeights(NamedTuple):
 
 class GeneralDeltaWeights(NamedTuple):
     """Generalized delta rule: decay and removal rate per key channel.
-    Columns of the fused projection and the decays' low-rank projection."""
+    Columns of the fused projection and the decays' low-rank projection,
+    whose columns and rank are whole vectors of 8."""
     heads: int
     dim: int
     offsets: tuple                # columns of r, k, v, removal, gate, decay
@@ -389,11 +390,13 @@ def pack_weight(w):
     return None
 
 
-def linear_parts(x, weight, packed=None) -> Union[torch.Tensor, Partials]:
-    """As linear, but a split product may come back as its partial sums."""
+def linear_parts(x, weight, packed=None,
+                 most=8) -> Union[torch.Tensor, Partials]:
+    """As linear, but a split product may come back as its partial sums, at
+    most `most` of them (few where several consumers add them up)."""
     if _use_hip(weight):
         from . import hip
-        return hip.linear_parts(x, weight, packed)
+        return hip.linear_parts(x, weight, packed, most)
     return torch.nn.functional.linear(x, weight)
 
 
