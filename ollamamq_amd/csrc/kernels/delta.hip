@@ -66,15 +66,17 @@ template <> struct Terms<float> {
 // ---------------------------------------------------------------------------
 // z = W u for 16 tokens and rows n0 .. n1 - 1 of W [N, rank], u (or its tanh)
 // the projection's columns first.. of the lane's token t; rank and first are
-// whole vectors of 8.  `emit` gets 16 rows at a time, four of them in a lane:
+// whole vectors of 8.  W is stored as operands, 16 rows by 32 columns after
+// one another, rows filled up to 64 and columns to 32.  `emit` gets 16 rows at a time, four of them in a lane:
 // z[i] is row n + i.  The operand is made once for all rows while rank <= 128.
 // ---------------------------------------------------------------------------
 template <typename T, typename P, bool TANH, typename E>
 DEV void low_rank(const Rows<P>& p, int first, int rank,
-                  const T* __restrict__ w, int N, int n0, int n1, int64_t t,
+                  const T* __restrict__ w, int n0, int n1, int64_t t,
                   E emit) {
     constexpr int NT = Terms<T>::N;
-    const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
+    const int lane = threadIdx.x & 63, g = lane >> 4;
+    const int steps = (rank + 31) / 32;
     Frag<T> uf[4][NT];
     auto operand = [&](int r0) {
         float u[4][8] = {};
@@ -109,13 +111,12 @@ DEV void low_rank(const Rows<P>& p, int first, int rank,
             if (rank > 128) operand(r0);
             #pragma unroll
             for (int s = 0; s < 4; s++) {
-                const int k = r0 + s * 32 + g * 8;
                 if (r0 + s * 32 >= rank) continue;
                 #pragma unroll
                 for (int j = 0; j < 4; j++) {
-                    const int m = n + j * 16 + lr;
-                    const T* row = w + (int64_t)min(m, N - 1) * rank;
-                    const Frag<T> wf = frag8(row + min(k, rank - 8));
+                    const Frag<T> wf = frag8(
+                        w + ((int64_t)((n / 16 + j) * steps + r0 / 32 + s)
+                             * 64 + lane) * 8);
                     #pragma unroll
                     for (int q = 0; q < NT; q++)
                         z[j] = mma(wf, uf[s][q], z[j]);
@@ -202,45 +203,65 @@ DEV void conv_strip(const GatedRows<T, P>& a, int64_t item, int lane) {
                 input(row - TAPS + m, col(j), x[m][j]);
         }
     }
-    for (int r = row; r < row + n; r++) {
-        float sq = 0.f;
+    // rows a few at a time, so that their loads overlap
+    constexpr int NR = TAPS > 0 ? 4 : 1;
+    for (int r0 = row; r0 < row + n; r0 += NR) {
+        float ahead[NR][KEEP][VEC];
+        if constexpr (TAPS > 0) {
+            #pragma unroll
+            for (int y = 0; y < NR; y++)
+                #pragma unroll
+                for (int j = 0; j < KEEP; j++)
+                    if (col(j) < wide)
+                        ldrow<VEC>(a.p, min(r0 + y, row + n - 1),
+                                   a.o_in + c0 + col(j), ahead[y][j]);
+        }
         #pragma unroll
-        for (int j = 0; j < KEEP; j++) {
-            const int c = col(j);
-            if (c >= wide) break;
-            float v[VEC] = {};
-            if constexpr (TAPS > 0) {
-                #pragma unroll
-                for (int m = 0; m + 1 < TAPS; m++)
+        for (int y = 0; y < NR; y++) {
+            const int r = r0 + y;
+            if (r >= row + n) break;
+            float sq = 0.f;
+            #pragma unroll
+            for (int j = 0; j < KEEP; j++) {
+                const int c = col(j);
+                if (c >= wide) break;
+                float v[VEC] = {};
+                if constexpr (TAPS > 0) {
                     #pragma unroll
-                    for (int i = 0; i < VEC; i++) x[m][j][i] = x[m + 1][j][i];
-                input(r, c, x[TAPS - 1][j]);
-                #pragma unroll
-                for (int m = 0; m < TAPS; m++)
+                    for (int m = 0; m + 1 < TAPS; m++)
+                        #pragma unroll
+                        for (int i = 0; i < VEC; i++)
+                            x[m][j][i] = x[m + 1][j][i];
                     #pragma unroll
                     for (int i = 0; i < VEC; i++)
-                        v[i] += wt[m][j][i] * x[m][j][i];
-            } else
-                for (int m = 0; m < taps; m++) {
-                    float u[VEC], w[VEC];
-                    input(r - taps + 1 + m, c, u);
-                    ldv<VEC>(a.conv + m * C + c0 + c, w);
+                        x[TAPS - 1][j][i] = ahead[y][j][i];
                     #pragma unroll
-                    for (int i = 0; i < VEC; i++) v[i] += w[i] * u[i];
+                    for (int m = 0; m < TAPS; m++)
+                        #pragma unroll
+                        for (int i = 0; i < VEC; i++)
+                            v[i] += wt[m][j][i] * x[m][j][i];
+                } else
+                    for (int m = 0; m < taps; m++) {
+                        float u[VEC], w[VEC];
+                        input(r - taps + 1 + m, c, u);
+                        ldv<VEC>(a.conv + m * C + c0 + c, w);
+                        #pragma unroll
+                        for (int i = 0; i < VEC; i++) v[i] += w[i] * u[i];
+                    }
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) {
+                    v[i] = silu_of<T>(v[i]);
+                    sq += v[i] * v[i];
                 }
-            #pragma unroll
-            for (int i = 0; i < VEC; i++) {
-                v[i] = silu_of<T>(v[i]);
-                sq += v[i] * v[i];
+                stv<VEC>(a.y + (int64_t)r * C + c0 + c, v);
             }
-            stv<VEC>(a.y + (int64_t)r * C + c0 + c, v);
+            if (is_v) continue;
+            for (int o = a.L / 2; o; o >>= 1) sq += __shfl_xor(sq, o, 64);
+            if (lane == 0)
+                a.scales[(int64_t)r * 2 * a.G + unit] =
+                    (unit < a.G ? 1.f / sqrtf((float)a.D) : 1.f)
+                    / sqrtf(sq + UNIT_EPS);
         }
-        if (is_v) continue;
-        for (int o = a.L / 2; o; o >>= 1) sq += __shfl_xor(sq, o, 64);
-        if (lane == 0)
-            a.scales[(int64_t)r * 2 * a.G + unit] =
-                (unit < a.G ? 1.f / sqrtf((float)a.D) : 1.f)
-                / sqrtf(sq + UNIT_EPS);
     }
     // Every row that reads the state is in its portion's first strip, and
     // this lane alone reads and writes these channels of it.
@@ -272,7 +293,7 @@ __global__ __launch_bounds__(256, 4) void k_gated_rows(GatedRows<T, P> a)
         const int n0 = (int)(w % nc) * a.wide;
         const int64_t t = w / nc * 16 + lr;
         low_rank<T, P, false>(
-            a.p, a.oa, a.ra, a.a2, N, n0, min(n0 + a.wide, N),
+            a.p, a.oa, a.ra, a.a2, n0, min(n0 + a.wide, N),
             min(t, (int64_t)a.T_rows - 1), [&](int n, f32x4 z) {
                 if (t >= a.T_rows || n >= N) return;
                 const bool whole = a.D % 4 == 0;    // four of one head
@@ -294,7 +315,7 @@ __global__ __launch_bounds__(256, 4) void k_gated_rows(GatedRows<T, P> a)
         const int n0 = (int)(w % nc) * a.wide;
         const int64_t t = w / nc * 16 + lr;
         low_rank<T, P, false>(
-            a.p, a.og, a.rg, a.g2, N, n0, min(n0 + a.wide, N),
+            a.p, a.og, a.rg, a.g2, n0, min(n0 + a.wide, N),
             min(t, (int64_t)a.T_rows - 1), [&](int n, f32x4 z) {
                 if (t >= a.T_rows) return;
                 const float v[4] = {z[0], z[1], z[2], z[3]};
@@ -375,6 +396,7 @@ extern "C" int gated_rows(
     return (int)hipGetLastError();
 }
 
+#define KEY_ROWS 4
 // Roles of the generalized rule: scales of unit keys (a group of L lanes per
 // head), decays, and, for a projection in parts, its sum.
 template <typename T, typename P> struct GeneralRows {
@@ -394,18 +416,30 @@ __global__ __launch_bounds__(256, 3) void k_general_rows(GeneralRows<T, P> a)
     const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
     int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (w < a.n_key) {
+        // one head of up to KEY_ROWS tokens, their loads side by side
         const int64_t u = w * (64 / a.L) + lane / a.L;
-        if (u >= (int64_t)a.T_rows * a.H) return;
-        const int l = lane & (a.L - 1), c0 = a.ok + (int)(u % a.H) * a.D;
-        float s = 0.f;
+        const int64_t t0 = u / a.H * KEY_ROWS;
+        if (t0 >= a.T_rows) return;
+        const int l = lane & (a.L - 1), h = (int)(u % a.H);
+        float s[KEY_ROWS] = {};
         for (int c = l * VEC; c < a.D; c += a.L * VEC) {
-            float x[VEC];
-            ldrow<VEC>(a.p, u / a.H, c0 + c, x);
+            float x[KEY_ROWS][VEC];
             #pragma unroll
-            for (int i = 0; i < VEC; i++) s += x[i] * x[i];
+            for (int y = 0; y < KEY_ROWS; y++)
+                ldrow<VEC>(a.p, min(t0 + y, (int64_t)a.T_rows - 1),
+                           a.ok + h * a.D + c, x[y]);
+            #pragma unroll
+            for (int y = 0; y < KEY_ROWS; y++)
+                #pragma unroll
+                for (int i = 0; i < VEC; i++) s[y] += x[y][i] * x[y][i];
         }
-        for (int o = a.L / 2; o; o >>= 1) s += __shfl_xor(s, o, 64);
-        if (l == 0) a.scales[u] = 1.f / sqrtf(s + UNIT_EPS);
+        #pragma unroll
+        for (int y = 0; y < KEY_ROWS; y++) {
+            for (int o = a.L / 2; o; o >>= 1)
+                s[y] += __shfl_xor(s[y], o, 64);
+            if (l == 0 && t0 + y < a.T_rows)
+                a.scales[(t0 + y) * a.H + h] = 1.f / sqrtf(s[y] + UNIT_EPS);
+        }
         return;
     }
     w -= a.n_key;
@@ -414,7 +448,7 @@ __global__ __launch_bounds__(256, 3) void k_general_rows(GeneralRows<T, P> a)
         const int n0 = (int)(w % nc) * a.wide;
         const int64_t t = w / nc * 16 + lr;
         low_rank<T, P, true>(
-            a.p, a.ow, a.rank, a.w2, N, n0, min(n0 + a.wide, N),
+            a.p, a.ow, a.rank, a.w2, n0, min(n0 + a.wide, N),
             min(t, (int64_t)a.T_rows - 1), [&](int n, f32x4 z) {
                 if (t >= a.T_rows) return;
                 float v[4];
@@ -447,7 +481,8 @@ extern "C" int general_rows(
         return (int)hipErrorInvalidValue;
     int L = 64;
     while (L > 1 && L / 2 * (v4 ? 4 : 1) >= D) L /= 2;
-    const int n_key = (int)(((int64_t)T_rows * H * L + 63) / 64);
+    const int64_t keys = (int64_t)((T_rows + KEY_ROWS - 1) / KEY_ROWS) * H;
+    const int n_key = (int)((keys * L + 63) / 64);
     const int wide = low_rank_cols(T_rows);
     const int n_decay = low_rank_waves(T_rows, H * D, wide);
     const int64_t n_sum = y ? ((int64_t)T_rows * cols / (v4 ? 4 : 1) + 63)
@@ -644,12 +679,14 @@ extern "C" int delta_step(
 // ---- chunks --------------------------------------------------------------
 #define CH 64             // tokens of a chunk
 #define SUB 16            // tokens of a part
+#define XCDS 8
 #define DB 32             // key channels of a prep pass
 #define DS (DB + 4)       // LDS row strides
 #define AS (CH + 4)
 // largest sum of decay inside a part for which the part's own triangle may
-// be factored (e^{c_i} e^{-c_j}); beyond it the pairs are taken one by one
-#define SAFE 20.f
+// be factored (e^{c_i} e^{-c_j}, far inside the range of fp32); beyond it the
+// pairs are taken one by one
+#define SAFE 60.f
 
 // An fp32 matrix as operand of products: in bf16 models two planes of bf16
 // terms whose products leave out the smallest, else itself.
@@ -701,6 +738,8 @@ template <> struct Four<bf16> { typedef bf16x4 type; };
 // Scratch per (chunk, head), each matrix of NT planes: Q [64][DP],
 // Z [64][DP], K^T [DP][64], (E^T), inverse [64][64], A_qk, (A_zk, A_qe);
 // then the fp32 decay of the whole chunk [DP].  Offsets in elements of T.
+// A matrix is stored as the operands the scan reads, 16 rows by 32 columns
+// after one another, so that a wave's loads are linear.
 template <typename T, bool GEN, int DP> struct Unit {
     static constexpr int NT = Terms<T>::N;
     static constexpr int64_t TP = CH * DP, SP = CH * CH;    // planes
@@ -713,14 +752,19 @@ template <typename T, bool GEN, int DP> struct Unit {
                                       + DP;
     DEV T* at(float* scr, int64_t i) { return (T*)(scr + i * floats); }
 };
+// element (r, c) of a matrix with `steps` operands to a row of them
+DEV int oper_at(int r, int c, int steps) {
+    return ((r / 16 * steps + c / 32) * 64 + c % 32 / 8 * 16 + r % 16) * 8
+           + c % 8;
+}
 enum { TALL_Q, TALL_Z, TALL_K, TALL_E };
 enum { SQ_INV, SQ_QK, SQ_ZK, SQ_QE };
 
-template <typename T, bool GEN, int DP>
+// VEC: rows of x are whole vectors of 8 key channels
+template <typename T, bool GEN, int DP, bool VEC>
 __global__ __launch_bounds__(256) void k_delta_prep(
     float* __restrict__ scr, DeltaIn<T> in,
-    const int* __restrict__ chunks,     // [n, 2] first row, rows
-    int vec)
+    const int* __restrict__ chunks)     // [n, 2] first row, rows
 {
     typedef Unit<T, GEN, DP> Un;
     const int H = in.H, D = in.D;
@@ -758,7 +802,7 @@ __global__ __launch_bounds__(256) void k_delta_prep(
     Frag<T> qn, kn, an;                 // the next pass
     f32x8s cn;
     auto load = [&](int d) {
-        if (vec) {
+        if constexpr (VEC) {
             const int c = min(d, D - 8);
             qn = frag8(qr + c);
             kn = frag8(kr + c);
@@ -857,8 +901,10 @@ __global__ __launch_bounds__(256) void k_delta_prep(
                 qe[e] *= before[e];
                 ze[e] *= before[e];
             }
-            stw<T, 8>(un + Un::tall(TALL_Q) + tk * DP + d, Un::TP, qe);
-            stw<T, 8>(un + Un::tall(TALL_Z) + tk * DP + d, Un::TP, ze);
+            stw<T, 8>(un + Un::tall(TALL_Q) + oper_at(tk, d, DP / 32), Un::TP,
+                      qe);
+            stw<T, 8>(un + Un::tall(TALL_Z) + oper_at(tk, d, DP / 32), Un::TP,
+                      ze);
             // transposed: eight tokens of a channel
             const int tt = (tid & 7) * 8, ch = tid >> 3;
             float after = 1.f, y[8];
@@ -866,13 +912,13 @@ __global__ __launch_bounds__(256) void k_delta_prep(
             #pragma unroll
             for (int i = 0; i < 8; i++)
                 y[i] = after * kt_s[(tt + i) * DS + ch];
-            stw<T, 8>(un + Un::tall(TALL_K) + (d0 + ch) * CH + tt, Un::TP,
+            stw<T, 8>(un + Un::tall(TALL_K) + oper_at(d0 + ch, tt, 2), Un::TP,
                       y);
             if (GEN) {
                 #pragma unroll
                 for (int i = 0; i < 8; i++)
                     y[i] = after * x1_s[(tt + i) * DS + ch];
-                stw<T, 8>(un + Un::tall(TALL_E) + (d0 + ch) * CH + tt,
+                stw<T, 8>(un + Un::tall(TALL_E) + oper_at(d0 + ch, tt, 2),
                           Un::TP, y);
             }
             if (tid < DB)
@@ -932,7 +978,7 @@ __global__ __launch_bounds__(256) void k_delta_prep(
     // A_ze to LDS, the others to memory; the gated rule's A_ze is A_zk
     __syncthreads();
     auto place = [&](int m, int I, int J, f32x4 v) {
-        stw4(un + Un::square(m) + (I * SUB + lr) * CH + J * SUB + g * 4,
+        stw4(un + Un::square(m) + oper_at(I * SUB + lr, J * SUB + g * 4, 2),
              Un::SP, v);
     };
     auto keep = [&](int I, int J, f32x4 v) {
@@ -1016,22 +1062,27 @@ __global__ __launch_bounds__(256) void k_delta_prep(
         const int r = i / (CH / 8), c = i % (CH / 8) * 8;
         float v[8] = {};
         if (c / SUB <= r / SUB) ldv<8>(I_s + r * AS + c, v);
-        stw<T, 8>(un + Un::square(SQ_INV) + r * CH + c, Un::SP, v);
+        stw<T, 8>(un + Un::square(SQ_INV) + oper_at(r, c, 2), Un::SP, v);
     }
 }
+
+// memory accesses stay on their side
+DEV void keep_order() { asm volatile("" ::: "memory"); }
 
 // A sequence's chunks in order, one block per 16*VC value columns, the state
 // in registers (NS: 16-row tiles a wave, D <= 64 * NS); wave w has tokens
 // 16 w .. of a chunk.  What several waves need goes through LDS, transposed:
-// the state, v, what w is solved from and w itself.
-template <typename T, int NS, int VC, bool GEN>
+// the state, v, what w is solved from and w itself.  The strips of a head are
+// neighbours on one XCD, whose L2 they share the factors through.  VEC: rows
+// of x are whole vectors of 4 value columns.
+template <typename T, int NS, int VC, bool GEN, bool VEC>
 __global__ __launch_bounds__(256) void k_delta_scan(
     float* __restrict__ o,              // [T, H, V]
     float* __restrict__ scr, DeltaIn<T> in, float* __restrict__ state,
     const int* __restrict__ slot, const int* __restrict__ pos,
     const int* __restrict__ chunks,     // [n, 2]
     const int* __restrict__ seqs,       // [m, 2] first chunk, chunks
-    int vec)
+    int n_seqs)
 {
     constexpr int DP = NS * 64;
     typedef Unit<T, GEN, DP> Un;
@@ -1040,12 +1091,15 @@ __global__ __launch_bounds__(256) void k_delta_scan(
     constexpr int KS = DP + PAD, TS = CH + PAD;
     constexpr int NQ = NS * 2;          // 32-channel steps over D
     constexpr int SP = W * KS, VP = W * TS;         // planes
-    const int H = in.H, D = in.D, V = in.V;
-    const int h = blockIdx.y, v0 = blockIdx.z * W, tid = threadIdx.x;
+    const int H = in.H, D = in.D, V = in.V, tid = threadIdx.x;
+    const int strips = (V + W - 1) / W, place = blockIdx.x / XCDS;
+    const int head = place / strips * XCDS + blockIdx.x % XCDS;
+    if (head >= n_seqs * H) return;
+    const int seq = head / H, h = head % H, v0 = place % strips * W;
     const int lane = tid & 63;
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int lr = lane & 15, g = lane >> 4;
-    const int c0 = seqs[blockIdx.x * 2], nc = seqs[blockIdx.x * 2 + 1];
+    const int c0 = seqs[seq * 2], nc = seqs[seq * 2 + 1];
     const int first = chunks[c0 * 2];
     float* St = state + ((int64_t)slot[first] * H + h) * D * V;
     extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -1075,28 +1129,32 @@ __global__ __launch_bounds__(256) void k_delta_scan(
     Raw vv[VC];
     auto unit = [&](int ci) { return Un::at(scr, (int64_t)ci * H + h); };
     auto load_zq = [&](int ci) {
-        const T* u = unit(ci) + (w * 16 + lr) * DP + g * 8;
+        const T* u = unit(ci) + w * NQ * 512 + lane * 8;
         #pragma unroll
         for (int d = 0; d < NQ; d++) {
-            zf[d] = ldw(u + Un::tall(TALL_Z) + d * 32, Un::TP);
-            qf[d] = ldw(u + Un::tall(TALL_Q) + d * 32, Un::TP);
+            zf[d] = ldw(u + Un::tall(TALL_Z) + d * 512, Un::TP);
+            qf[d] = ldw(u + Un::tall(TALL_Q) + d * 512, Un::TP);
         }
     };
     auto load_square = [&](int ci, int m, Wide<T>* f) {
-        const T* u = unit(ci) + Un::square(m) + (w * 16 + lr) * CH + g * 8;
+        const T* u = unit(ci) + Un::square(m) + w * 1024 + lane * 8;
         #pragma unroll
-        for (int j = 0; j < 2; j++) f[j] = ldw(u + j * 32, Un::SP);
+        for (int j = 0; j < 2; j++) f[j] = ldw(u + j * 512, Un::SP);
+    };
+    auto load_fade = [&](int ci) {
+        const float* fd = (const float*)(unit(ci) + Un::fade) + w * 16
+                          + g * 4;
+        #pragma unroll
+        for (int x = 0; x < NS; x++)
+            e4[x] = *reinterpret_cast<const f32x4*>(fd + x * 64);
     };
     auto load_k = [&](int ci) {
-        const T* u = unit(ci);
-        const float* fd = (const float*)(u + Un::fade);
+        const T* u = unit(ci) + w * 1024 + lane * 8;
         #pragma unroll
         for (int x = 0; x < NS; x++) {
-            const int d = (w + x * 4) * 16;
-            e4[x] = *reinterpret_cast<const f32x4*>(fd + d + g * 4);
             #pragma unroll
             for (int j = 0; j < 2; j++) {
-                const int at = (d + lr) * CH + j * 32 + g * 8;
+                const int at = (x * 8 + j) * 512;
                 kf[x][j] = ldw(u + Un::tall(TALL_K) + at, Un::TP);
                 if (GEN) ef[x][j] = ldw(u + Un::tall(TALL_E) + at, Un::TP);
             }
@@ -1110,7 +1168,7 @@ __global__ __launch_bounds__(256) void k_delta_scan(
         #pragma unroll
         for (int q = 0; q < VC; q++) {
             const int c = v0 + (w * VC + q) * 4;
-            if (vec)
+            if constexpr (VEC)
                 vv[q] = *reinterpret_cast<const Raw*>(r + min(c, V - 4));
             else
                 #pragma unroll
@@ -1121,15 +1179,23 @@ __global__ __launch_bounds__(256) void k_delta_scan(
     auto wide_at = [&](const T* s, int c, int j) {
         return ldw(s + (c * 16 + lr) * TS + j * 32 + g * 8, VP);
     };
+    // in the order of the loop, so that its waits fit the first chunk too
     load_v(c0);
+    load_fade(c0);
+    keep_order();
     load_zq(c0);
-    load_square(c0, SQ_INV, inv);
-    load_square(c0, SQ_QK, aqk);
+    keep_order();
     if (GEN) {
         load_square(c0, SQ_ZK, azk);
-        load_square(c0, SQ_QE, aqe);
+        load_square(c0, SQ_QK, aqk);
+        keep_order();
     }
+    load_square(c0, SQ_INV, inv);
+    keep_order();
+    load_square(c0, GEN ? SQ_QE : SQ_QK, GEN ? aqe : aqk);
+    keep_order();
     load_k(c0);
+    keep_order();
 
     for (int ci = c0; ci < c0 + nc; ++ci) {
         const int t0 = chunks[ci * 2], n = chunks[ci * 2 + 1];
@@ -1150,8 +1216,14 @@ __global__ __launch_bounds__(256) void k_delta_scan(
             for (int c = 0; c < VC; c++)
                 stw4(S_s + (c * 16 + lr) * KS + d, SP, S[x][c]);
         }
+        #pragma unroll
+        for (int x = 0; x < NS; x++)
+            #pragma unroll
+            for (int c = 0; c < VC; c++) S[x][c] *= e4[x];
         lds_barrier();
         load_v(nx);
+        load_fade(nx);
+        keep_order();
         // what z and q read from the state before the chunk
         f32x4 az[VC] = {}, ao[VC] = {};
         #pragma unroll
@@ -1202,10 +1274,6 @@ __global__ __launch_bounds__(256) void k_delta_scan(
                  GEN ? -u[c] : u[c]);
         lds_barrier();
         // results and the next state
-        #pragma unroll
-        for (int x = 0; x < NS; x++)
-            #pragma unroll
-            for (int c = 0; c < VC; c++) S[x][c] *= e4[x];
         #pragma unroll
         for (int j = 0; j < 2; j++)
             #pragma unroll
@@ -1258,10 +1326,15 @@ extern "C" int64_t delta_scratch_floats(int gen, int n_chunks, int H, int D)
                                     + (gen ? 4 : 2) * CH * CH + dp);
 }
 
-template <typename T, int NS, int VC, bool GEN>
-static void scan_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
-                    const int* slot, const int* pos, const int* chunks,
-                    const int* seqs, int n_seqs, int vec, hipStream_t stream)
+struct Scan {
+    float* o; float* scr; float* state;
+    const int* slot; const int* pos; const int* chunks; int n_chunks;
+    const int* seqs; int n_seqs;
+    hipStream_t stream;
+};
+
+template <typename T, int NS, int VC, bool GEN, bool VEC>
+static void scan_go(const DeltaIn<T>& in, const Scan& a)
 {
     constexpr int W = VC * 16, PAD = 16 / sizeof(T), es = sizeof(T);
     constexpr int NT = Terms<T>::N;
@@ -1270,63 +1343,62 @@ static void scan_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
     static bool once = false;
     if (!once) {
         (void)hipFuncSetAttribute(
-            (const void*)k_delta_scan<T, NS, VC, GEN>,
+            (const void*)k_delta_scan<T, NS, VC, GEN, VEC>,
             hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
         once = true;
     }
-    k_delta_scan<T, NS, VC, GEN>
-        <<<dim3(n_seqs, in.H, (in.V + W - 1) / W), 256, lds, stream>>>(
-            o, scr, in, state, slot, pos, chunks, seqs, vec);
+    const int heads = (a.n_seqs * in.H + XCDS - 1) / XCDS * XCDS;
+    k_delta_scan<T, NS, VC, GEN, VEC>
+        <<<heads * ((in.V + W - 1) / W), 256, lds, a.stream>>>(
+            a.o, a.scr, in, a.state, a.slot, a.pos, a.chunks, a.seqs,
+            a.n_seqs);
+}
+
+template <typename T, bool GEN, int NS, bool VEC>
+static void prep_go(const DeltaIn<T>& in, const Scan& a)
+{
+    constexpr int part = ((GEN ? 6 : 7) * CH * DS + 4 * DB) * 4;
+    constexpr int solve = 2 * CH * AS * 4;
+    static bool once = false;
+    if (!once) {
+        (void)hipFuncSetAttribute(
+            (const void*)k_delta_prep<T, GEN, NS * 64, VEC>,
+            hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        once = true;
+    }
+    k_delta_prep<T, GEN, NS * 64, VEC>
+        <<<dim3(a.n_chunks, in.H), 256, part > solve ? part : solve,
+           a.stream>>>(a.scr, in, a.chunks);
 }
 
 template <typename T, bool GEN, int NS>
-static int chunks_go(float* o, float* scr, const DeltaIn<T>& in, float* state,
-                     const int* slot, const int* pos, const int* chunks,
-                     int n_chunks, const int* seqs, int n_seqs,
-                     hipStream_t stream)
+static int chunks_go(const DeltaIn<T>& in, const Scan& a)
 {
     static_assert(Unit<T, GEN, NS * 64>::floats
                   == (GEN ? 4 : 3) * CH * NS * 64 + (GEN ? 4 : 2) * CH * CH
                      + NS * 64, "scratch");
-    const int H = in.H, D = in.D, V = in.V;
-    const int v8 = D % 8 == 0 && in.oq % 8 == 0 && in.ok % 8 == 0
-                   && in.oa % 8 == 0 && in.ld % 8 == 0;
-    const int v4 = V % 4 == 0 && in.ov % 4 == 0 && in.ld % 4 == 0;
-    const int part = ((GEN ? 6 : 7) * CH * DS + 4 * DB) * 4;
-    const int solve = 2 * CH * AS * 4;
-    static bool once = false;
-    if (!once) {
-        (void)hipFuncSetAttribute(
-            (const void*)k_delta_prep<T, GEN, NS * 64>,
-            hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-        once = true;
-    }
-    k_delta_prep<T, GEN, NS * 64><<<dim3(n_chunks, H), 256,
-                                    part > solve ? part : solve, stream>>>(
-        scr, in, chunks, v8);
+    const int D = in.D, V = in.V;
+    if (D % 8 == 0 && in.oq % 8 == 0 && in.ok % 8 == 0 && in.oa % 8 == 0
+        && in.ld % 8 == 0)
+        prep_go<T, GEN, NS, true>(in, a);
+    else prep_go<T, GEN, NS, false>(in, a);
     // wide strips share the loads of the factors, narrow ones fill the chip
-    const bool two = NS < 4 && (int64_t)n_seqs * H * ((V + 31) / 32) >= 256;
-    if (two)
-        scan_go<T, NS, NS < 4 ? 2 : 1, GEN>(o, scr, in, state, slot, pos,
-                                            chunks, seqs, n_seqs, v4, stream);
-    else
-        scan_go<T, NS, 1, GEN>(o, scr, in, state, slot, pos, chunks, seqs,
-                               n_seqs, v4, stream);
+    constexpr int WIDE = NS < 4 ? 2 : 1;
+    const bool wide = (int64_t)a.n_seqs * in.H * ((V + 31) / 32) >= 256;
+    if (V % 4 || in.ov % 4 || in.ld % 4) scan_go<T, NS, 1, GEN, false>(in, a);
+    else if (wide) scan_go<T, NS, WIDE, GEN, true>(in, a);
+    else scan_go<T, NS, 1, GEN, true>(in, a);
     return (int)hipGetLastError();
 }
 
 template <typename T, bool GEN>
-static int chunks_for(float* o, float* scr, const DeltaIn<T>& in,
-                      float* state, const int* slot, const int* pos,
-                      const int* chunks, int n_chunks, const int* seqs,
-                      int n_seqs, hipStream_t stream)
+static int chunks_for(const DeltaIn<T>& in, const Scan& a)
 {
     if (in.D < 1 || in.V < 1 || in.D > 256) return (int)hipErrorInvalidValue;
     const int dp = delta_tiles(in.D);
-    auto go = dp == 64 ? chunks_go<T, GEN, 1> : dp == 128
-              ? chunks_go<T, GEN, 2> : chunks_go<T, GEN, 4>;
-    return go(o, scr, in, state, slot, pos, chunks, n_chunks, seqs, n_seqs,
-              stream);
+    return dp == 64 ? chunks_go<T, GEN, 1>(in, a)
+           : dp == 128 ? chunks_go<T, GEN, 2>(in, a)
+                       : chunks_go<T, GEN, 4>(in, a);
 }
 
 // Portions of whole sequences in chunks of 64 rows.  chunks int32 [n, 2]
@@ -1340,11 +1412,10 @@ extern "C" int delta_chunks(
     const void* seqs, int n_seqs, int H, int G, int D, int V,
     hipStream_t stream)
 {
-    #define DC_GO(T, GEN)                                                  \
-        chunks_for<T, GEN>((float*)o, (float*)scr, DELTA_IN(T),            \
-                           (float*)state, (const int*)slot,                \
-                           (const int*)pos, (const int*)chunks, n_chunks,  \
-                           (const int*)seqs, n_seqs, stream)
+    const Scan a{(float*)o, (float*)scr, (float*)state, (const int*)slot,
+                 (const int*)pos, (const int*)chunks, n_chunks,
+                 (const int*)seqs, n_seqs, stream};
+    #define DC_GO(T, GEN) chunks_for<T, GEN>(DELTA_IN(T), a)
     if (f32) return gen ? DC_GO(float, true) : DC_GO(float, false);
     return gen ? DC_GO(bf16, true) : DC_GO(bf16, false);
     #undef DC_GO

@@ -202,10 +202,14 @@ extern "C" int qkv_norm_rope(
     if (dims % 2 || dims > D || dims < 0 || Dp > 256 || Vp > 256 || D > Dp
         || V > Vp)
         return (int)hipErrorInvalidValue;
-    const bool v4 = D % 4 == 0 && V % 4 == 0 && dims % 8 == 0 && ld % 4 == 0
-                    && part_stride % 4 == 0;
+    auto whole = [&](int n) {
+        return D % n == 0 && V % n == 0 && dims % (2 * n) == 0 && ld % n == 0
+               && part_stride % n == 0;
+    };
+    const int vec = whole(8) ? 8 : whole(4) ? 4 : 1;
     int L = 64;
-    if (v4) while (L > 4 && L * 2 >= Dp && L * 2 >= Vp) L /= 2;
+    if (vec > 1)
+        while (L > 4 && L / 2 * vec >= Dp && L / 2 * vec >= Vp) L /= 2;
     const int want = ((H + 2 * G) * L + 255) / 256;
     const dim3 grid(T_rows, T_rows <= 256 ? want : (want + 2) / 3);
     #define QN(T, P, VE, KE)                                               \
@@ -217,7 +221,11 @@ extern "C" int qkv_norm_rope(
             (const int*)pos, (const int*)ptab, H, G, D, V, Dp, Vp, psz,    \
             maxp, L)
     #define QN_V(T, P)                                                     \
-        do { if (v4) QN(T, P, 4, 1); else QN(T, P, 1, 4); } while (0)
+        do {                                                               \
+            if (vec == 8) QN(T, P, 8, 1);                                  \
+            else if (vec == 4) QN(T, P, 4, 1);                             \
+            else QN(T, P, 1, 4);                                           \
+        } while (0)
     if (f32) QN_V(float, float);
     else if (p32) QN_V(bf16, float);
     else QN_V(bf16, bf16);

@@ -282,6 +282,10 @@ def _whole(m, dim):
                                    else (0, 0, 0, fill))
 
 
+def _low_rank(m):
+    return ops.low_rank(_whole(m, 1).contiguous())
+
+
 def _aligned(cols, low):
     """Wide projections, then low-rank ones from whole vectors on."""
     fill = -sum(m.shape[0] for m in cols) % 8
@@ -320,7 +324,7 @@ class PemidraLayer(HybridLayer):
             self.mix = ops.GeneralDeltaWeights(
                 heads=m.heads, dim=m.dim,
                 offsets=(*_offsets(cols)[:5], _offsets(cols)[-1]),
-                w2=put(_whole(mat("w2", n, low.shape[0]), 1)).contiguous(),
+                w2=_low_rank(put(mat("w2", n, low.shape[0]))),
                 w0=vec(mix + "w0", n), a_bias=vec(mix + "a.b", n),
                 norm=vec(mix + "norm", n, mean=1.0), eps=eps)
             outs = [("w_o", "o", n)]
@@ -371,12 +375,12 @@ class PemidraLayer(HybridLayer):
             heads=r.heads, kv_heads=r.kv_heads, dim=r.dim, vdim=r.vdim,
             offsets=(at[3], at[7], at_a1, at_g1),
             conv=taps.to(temp.device).float().t().contiguous(),
-            a2=put(_whole(mat("right.a2", r.heads * r.dim, a1.shape[0]), 1))
-            .contiguous(),
+            a2=_low_rank(put(mat("right.a2", r.heads * r.dim,
+                                 a1.shape[0]))),
             rate=vec(mix + "right.A_log", r.heads).exp(),
             dt_bias=vec(mix + "right.dt_bias", r.heads * r.dim),
-            g2=put(_whole(mat("right.g2", r.heads * r.vdim, g1.shape[0]), 1))
-            .contiguous(),
+            g2=_low_rank(put(mat("right.g2", r.heads * r.vdim,
+                                 g1.shape[0]))),
             norm=vec(mix + "right.norm", r.vdim, mean=1.0), eps=eps)
         W = cols[0].shape[1]
         self.left_out, self.right_out = (vec(f"{mix}{n}.out", W, mean=1.0)

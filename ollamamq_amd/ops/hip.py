@@ -1365,9 +1365,48 @@ def head_gate(o, norm, gate, og, act, dtype, H, V, eps, frag, mult=1.0):
     return res
 
 
+def pack_operand(w):
+    """[N, K] as operands of 16 rows by 32 columns (lane = column group * 16
+    + row, eight columns each) after one another; zeros fill up rows to 64
+    and columns to 32."""
+    N, K = w.shape
+    w = torch.nn.functional.pad(w, (0, -K % 32, 0, -N % 64))
+    return w.view(-1, 16, w.shape[1] // 32, 4, 8) \
+        .permute(0, 2, 3, 1, 4).contiguous().view(-1)
+
+
 DELTA_STEP_TOKENS = 4    # portions up to this walk token by token
 DELTA_MAX_D = 256        # key width the chunk kernels take
+DELTA_BYTES = 1 << 30    # chunk factors held at a time
 CONV_STRIP = 16          # tokens of a portion that one wave convolves
+
+
+def _chunk_groups(meta, dev, step_tokens, most):
+    """The chunks of _chunk_plan in groups of about `most`, the sequences'
+    chunks side by side: [(chunks, seqs)].  What a group needs in memory is
+    used again by the next, and stays near."""
+    key = f"_chunk_groups_{step_tokens}_{most}"
+    groups = getattr(meta, key, None)
+    if groups is None:
+        _, chunks, seqs, _, _ = _chunk_plan(meta, dev, step_tokens)
+        chunks, seqs = chunks.tolist(), seqs.tolist()
+        longest = max(n for _, n in seqs)
+        each = max(1, most // len(seqs))        # chunks of a sequence
+        n = -(-longest // each)
+        each = -(-longest // n)
+        groups = []
+        for lo in range(0, longest, each):
+            c, s = [], []
+            for first, count in seqs:
+                part = chunks[first + lo:first + min(count, lo + each)] \
+                    if lo < count else []
+                if part:
+                    s.append((len(c), len(part)))
+                    c += part
+            groups.append(tuple(torch.tensor(x, dtype=torch.int32).to(dev)
+                                for x in (c, s)))
+        setattr(meta, key, groups)
+    return groups
 
 
 def _conv_strips(meta, taps, dev):
@@ -1412,12 +1451,16 @@ def _delta(gen, x, offsets, qs, ks, decay, beta, a_bias, state, G, slots, pos,
         if spans is not None:
             step(spans, spans.shape[0])
         if chunks is not None:
-            n = chunks.shape[0]
-            scr = torch.empty(_lib.delta_scratch_floats(gen, n, H, D),
+            one = _lib.delta_scratch_floats(gen, 1, H, D)
+            groups = _chunk_groups(meta, dev, DELTA_STEP_TOKENS,
+                                   max(1, DELTA_BYTES // (4 * one)))
+            scr = torch.empty(max(c.shape[0] for c, _ in groups) * one,
                               dtype=torch.float32, device=dev)
-            _check(_lib.delta_chunks(
-                f32, gen, _p(o), _p(scr), *head, _p(chunks), n, _p(seqs),
-                seqs.shape[0], H, G, D, V, _stream()), "delta_chunks")
+            for chunks, seqs in groups:
+                _check(_lib.delta_chunks(
+                    f32, gen, _p(o), _p(scr), *head, _p(chunks),
+                    chunks.shape[0], _p(seqs), seqs.shape[0], H, G, D, V,
+                    _stream()), "delta_chunks")
     return o
 
 
@@ -1425,18 +1468,17 @@ def gated_delta(p, w, state, conv_state, slot_ids, positions, meta, frag):
     H, G, D, V = w.heads, w.kv_heads, w.dim, w.vdim
     o_in, ob, oa, og = w.offsets
     taps, C = w.conv.shape
-    ra, rg = w.a2.shape[1], w.g2.shape[1]
+    ra, rg = w.a2.rank, w.g2.rank
     t = p.parts if isinstance(p, Partials) else p
-    T, dev, dtype = t.shape[-2], t.device, w.a2.dtype
+    T, dev, dtype = t.shape[-2], t.device, w.a2.w.dtype
     assert C == 2 * G * D + H * V and state.shape[1:] == (H, D, V) \
         and conv_state.shape[1:] == (taps - 1, C) \
         and conv_state.dtype == torch.float32 \
         and conv_state.is_contiguous() and w.conv.is_contiguous() \
         and max(o_in + C, ob + H, oa + ra, og + rg) <= t.shape[-1] \
-        and w.a2.shape[0] == w.dt_bias.numel() == H * D \
-        and w.g2.shape == (H * V, rg) and w.rate.numel() == H \
-        and w.norm.numel() == V and w.a2.is_contiguous() \
-        and w.g2.is_contiguous()
+        and w.a2.w.shape[0] == w.dt_bias.numel() == H * D \
+        and w.g2.w.shape[0] == H * V and w.rate.numel() == H \
+        and w.norm.numel() == V
     assert isinstance(p, Partials) or p.dtype == dtype
     assert not frag or meta.one_each
     new = lambda *shape, dtype=torch.float32: torch.empty(
@@ -1450,7 +1492,8 @@ def gated_delta(p, w, state, conv_state, slot_ids, positions, meta, frag):
         _check(_lib.gated_rows(
             int(dtype == torch.float32), *_rows(p), o_in, ob, oa, ra, og, rg,
             _p(w.conv), taps, _p(conv_state), _p(slots), _p(pos), _p(strips),
-            n, _p(w.a2), _p(w.rate), _p(w.dt_bias), _p(w.g2), _p(y),
+            n, _p(w.a2.packed), _p(w.rate), _p(w.dt_bias), _p(w.g2.packed),
+            _p(y),
             _p(scales), _p(decay), _p(beta), _p(gate), T, H, G, D, V,
             _stream()), "gated_rows")
     o = _delta(0, y, (0, G * D, 2 * G * D, 0), scales, scales[:, G:], decay,
@@ -1461,11 +1504,11 @@ def gated_delta(p, w, state, conv_state, slot_ids, positions, meta, frag):
 def general_delta(p, w, state, slot_ids, positions, meta, frag):
     H, D = w.heads, w.dim
     o_r, ok, ov, oa, og, ow = w.offsets
-    rank = w.w2.shape[1]
+    rank = w.w2.rank
     t = p.parts if isinstance(p, Partials) else p
-    T, cols, dev, dtype = t.shape[-2], t.shape[-1], t.device, w.w2.dtype
-    assert state.shape[1:] == (H, D, D) and w.w2.shape[0] == H * D \
-        and w.w2.is_contiguous() and max(w.offsets[:5]) + H * D <= cols \
+    T, cols, dev, dtype = t.shape[-2], t.shape[-1], t.device, w.w2.w.dtype
+    assert state.shape[1:] == (H, D, D) and w.w2.w.shape[0] == H * D \
+        and max(w.offsets[:5]) + H * D <= cols \
         and ow + rank <= cols and w.w0.numel() == w.a_bias.numel() \
         == w.norm.numel() == H * D
     assert isinstance(p, Partials) or p.dtype == dtype
@@ -1477,8 +1520,8 @@ def general_delta(p, w, state, slot_ids, positions, meta, frag):
     slots, pos = _i32(slot_ids), _i32(positions)
     if T:
         _check(_lib.general_rows(
-            int(dtype == torch.float32), *_rows(p), ok, ow, rank, _p(w.w2),
-            _p(w.w0), _p(scales), _p(decay), _p(y if whole else None), cols,
+            int(dtype == torch.float32), *_rows(p), ok, ow, rank,
+            _p(w.w2.packed), _p(w.w0), _p(scales), _p(decay), _p(y if whole else None), cols,
             T, H, D, _stream()), "general_rows")
     o = _delta(1, y, (o_r, ok, ov, oa), None, scales, decay, None, w.a_bias,
                state, H, slots, pos, meta)

@@ -219,6 +219,24 @@ class LightningWeights(NamedTuple):
 UNIT_EPS = 1e-6       # inside the root of a unit vector
 
 
+class LowRank(NamedTuple):
+    """The second matrix [N, rank] of a low-rank projection and, on the GPU,
+    its copy in the order in which the matrix cores take it."""
+    w: torch.Tensor
+    packed: Optional[torch.Tensor] = None
+
+    @property
+    def rank(self) -> int:
+        return self.w.shape[1]
+
+
+def low_rank(w: torch.Tensor) -> LowRank:
+    if not w.is_cuda:
+        return LowRank(w)
+    from . import hip
+    return LowRank(w, hip.pack_operand(w))
+
+
 class GatedDeltaWeights(NamedTuple):
     """Gated delta rule with a decay per key channel.  Columns of the fused
     projection (q, k and v follow one another), the short convolution over
@@ -229,10 +247,10 @@ class GatedDeltaWeights(NamedTuple):
     vdim: int
     offsets: tuple                # columns of q|k|v, beta, decay, gate
     conv: torch.Tensor            # fp32 [taps, channels], the current last
-    a2: torch.Tensor              # [heads * dim, rank]
+    a2: LowRank                   # [heads * dim, rank]
     rate: torch.Tensor            # fp32 [heads], exp of the stored logarithm
     dt_bias: torch.Tensor         # fp32 [heads * dim]
-    g2: torch.Tensor              # [heads * vdim, rank]
+    g2: LowRank                   # [heads * vdim, rank]
     norm: torch.Tensor            # fp32 [vdim]
     eps: float
 
@@ -244,7 +262,7 @@ class GeneralDeltaWeights(NamedTuple):
     heads: int
     dim: int
     offsets: tuple                # columns of r, k, v, removal, gate, decay
-    w2: torch.Tensor              # [heads * dim, rank]
+    w2: LowRank                   # [heads * dim, rank]
     w0: torch.Tensor              # fp32 [heads * dim]
     a_bias: torch.Tensor          # fp32 [heads * dim]
     norm: torch.Tensor            # fp32 [heads * dim]

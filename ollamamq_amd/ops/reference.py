@@ -372,7 +372,7 @@ def gated_delta(p, w, state, conv_state, meta):
     q, k, v = y.split([G * D, G * D, H * V], -1)
     heads = lambda t: _unit(t.reshape(T, G, D)).repeat_interleave(H // G, 1)
     q, k, v = heads(q) * D ** -0.5, heads(k), v.reshape(T, H, V)
-    low = lambda at, m: f[:, at:at + m.shape[1]] @ m.float().T
+    low = lambda at, m: f[:, at:at + m.rank] @ m.w.float().T
     z = torch.nn.functional.softplus(low(oa, w.a2) + w.dt_bias)
     g = torch.exp(-w.rate[:, None] * z.view(T, H, D))
     bk = torch.sigmoid(f[:, ob:ob + H]).unsqueeze(-1) * k
@@ -388,7 +388,7 @@ def general_delta(p, w, state, meta):
     heads = lambda t: t.reshape(T, H, D)
     u = _unit(heads(k))
     at = w.offsets[5]
-    z = torch.tanh(f[:, at:at + w.w2.shape[1]]) @ w.w2.float().T + w.w0
+    z = torch.tanh(f[:, at:at + w.w2.rank]) @ w.w2.w.float().T + w.w0
     g = torch.exp(-math.exp(-0.5) * torch.sigmoid(z))
     a = torch.sigmoid(a + w.a_bias)
     o = _delta(heads(r), heads(k), heads(v), u, heads(a) * u, heads(g), state,
