@@ -521,15 +521,28 @@ template <typename T> struct DeltaIn {
     int H, G, D, V;
 };
 
+// What follows the recurrence: every head normed by itself, times the weight
+// and the sigmoid of the gate.
+template <typename T> struct HeadOut {
+    const float* w;
+    int w_stride;                     // 0: the heads share the weight
+    const T* gate;
+    int64_t ld;
+    int og;
+    float eps;
+    int frag;
+};
+
 // One block per sequence, head and strip of VB value columns; a thread keeps
-// NR rows of VEC columns of the state.
-template <typename T, int VEC, int NR, bool GEN>
+// NR rows of VEC columns of the state.  OUT: the strip is the whole head, its
+// norm and gate are in the same kernel.
+template <typename T, int VEC, int NR, bool GEN, bool OUT>
 __global__ __launch_bounds__(256) void k_delta_step(
-    float* __restrict__ o,              // [T, H, V]
+    void* __restrict__ out,             // [T, H, V] fp32; OUT: of type T
     DeltaIn<T> in, float* __restrict__ state,   // [slots, H, D, V]
     const int* __restrict__ slot, const int* __restrict__ pos,
     const int* __restrict__ spans,      // [n, 2] first row, rows; null: 1 row
-    int VB)
+    int VB, HeadOut<T> ho)
 {
     const int H = in.H, D = in.D, V = in.V;
     const int h = blockIdx.y, hk = h / (H / in.G), tid = threadIdx.x;
@@ -565,6 +578,13 @@ __global__ __launch_bounds__(256) void k_delta_step(
         const float qs = in.qs ? in.qs[(int64_t)t * in.sld + hk] : 1.f;
         const float ks = in.ks[(int64_t)t * in.sld + hk];
         const float beta = GEN ? 0.f : in.beta[(int64_t)t * H + h];
+        // this thread's first gate, asked for early
+        const T* gr = ho.gate + t * ho.ld + ho.og + h * V;
+        float z = 0.f, hw = 0.f;
+        if (OUT && tid < V) {
+            z = ldf(gr + tid);
+            hw = ho.w[h * ho.w_stride + tid];
+        }
         for (int d = tid; d < D; d += 256) {
             const int c = h * D + d;
             const float k = ldf(row + in.ok + hk * D + d), u = k * ks;
@@ -618,10 +638,28 @@ __global__ __launch_bounds__(256) void k_delta_step(
             stv<VEC>(o_s + rg * nc + vt, f);
         }
         __syncthreads();
+        float sq = 0.f;
         for (int c = tid; c < nc; c += 256) {
             float x = 0.f;
             for (int y = 0; y < RG; y++) x += o_s[y * nc + c];
-            o[((int64_t)t * H + h) * V + v0 + c] = x;
+            if (OUT) {
+                o_s[c] = x;             // only this thread reads column c
+                sq += x * x;
+            } else ((float*)out)[((int64_t)t * H + h) * V + v0 + c] = x;
+        }
+        if constexpr (OUT) {
+            __shared__ float red[4];
+            const float f = 1.f / sqrtf(block_sum<256>(sq, red) / V + ho.eps);
+            for (int c = tid; c < V; c += 256) {
+                const int m = h * V + c;
+                if (c != tid) {
+                    z = ldf(gr + c);
+                    hw = ho.w[h * ho.w_stride + c];
+                }
+                stf((T*)out + (ho.frag ? frag_row_off(t, m, H * V)
+                                       : (int64_t)t * H * V + m),
+                    o_s[c] * f * hw * sigmoid_of<T>(z));
+            }
         }
     }
     #pragma unroll
@@ -636,34 +674,65 @@ __global__ __launch_bounds__(256) void k_delta_step(
                (const float*)ks, sld, (const float*)decay,                 \
                (const float*)beta, (const float*)a_bias, H, G, D, V}
 
+// threads across a strip of the state: the rest of the block covers the rows,
+// 16 a thread
+static int step_threads(int D) {
+    int nv = 256;
+    while (nv > 1 && 256 / nv * 16 < D) nv /= 2;
+    return nv;
+}
+// value columns of a block, fewer while there are few blocks
+static int step_strip(int n, int H, int D, int V, bool v4) {
+    const int most = step_threads(D) * (v4 ? 4 : 1);
+    int vb = most < V ? most : V;
+    while (v4 && vb > 32 && vb % 8 == 0
+           && (int64_t)n * H * ((V + vb - 1) / vb) < 512) vb /= 2;
+    return vb;
+}
+// whether the step kernel takes whole heads and can norm and gate them
+extern "C" int delta_whole(int n, int H, int D, int V, int ov, int64_t ld)
+{
+    return V % 4 == 0 && ov % 4 == 0 && ld % 4 == 0
+           && step_strip(n, H, D, V, true) == V;
+}
+
+// whole: 0 leaves o [T, H, V] in fp32; 1 and 2 norm and gate it into o [T, H*V]
+// of the model's type, 2 in fragment layout.
 extern "C" int delta_step(
     int f32, int gen, void* o, const void* x, int64_t ld, int oq, int ok,
     int ov, int oa, const void* qs, const void* ks, int sld,
     const void* decay, const void* beta, const void* a_bias, void* state,
     const void* slot, const void* pos, const void* spans, int n, int H,
-    int G, int D, int V, hipStream_t stream)
+    int G, int D, int V, const void* norm, int norm_stride, const void* gate,
+    int64_t gate_ld, int og, float eps, int whole, hipStream_t stream)
 {
     const bool v4 = V % 4 == 0 && ov % 4 == 0 && ld % 4 == 0;
     const int vec = v4 ? 4 : 1;
     if (D < 1 || V < 1 || D > 2048) return (int)hipErrorInvalidValue;
-    // threads across a strip: the rest of the block covers the rows, 16 a
-    // thread; narrower while there are few blocks
-    int nv = 256;
-    while (nv > 1 && 256 / nv * 16 < D) nv /= 2;
-    int vb = nv * vec < V ? nv * vec : V;
-    while (v4 && vb > 32 && vb % 8 == 0
-           && (int64_t)n * H * ((V + vb - 1) / vb) < 512) vb /= 2;
-    const int per = (D + 256 / (vb / vec) - 1) / (256 / (vb / vec));
+    int vb = step_strip(n, H, D, V, v4);
+    if (whole) {
+        if (V > step_threads(D) * vec || (whole == 2 && f32))
+            return (int)hipErrorInvalidValue;
+        vb = V;
+    }
+    const int rows = 256 / (vb / vec), per = (D + rows - 1) / rows;
     const int lds = (2 * 256 * vec + 5 * D) * 4;
     dim3 grid(n, H, (V + vb - 1) / vb);
-    #define DS_GO(T, VE, NR, GEN)                                          \
-        k_delta_step<T, VE, NR, GEN><<<grid, 256, lds, stream>>>(          \
-            (float*)o, DELTA_IN(T), (float*)state, (const int*)slot,       \
-            (const int*)pos, (const int*)spans, vb)
+    #define DS_GO(T, VE, NR, GEN, OUT)                                     \
+        k_delta_step<T, VE, NR, GEN, OUT><<<grid, 256, lds, stream>>>(     \
+            o, DELTA_IN(T), (float*)state, (const int*)slot,               \
+            (const int*)pos, (const int*)spans, vb,                        \
+            HeadOut<T>{(const float*)norm, norm_stride, (const T*)gate,    \
+                       gate_ld, og, eps, whole == 2})
+    #define DS_O(T, VE, NR, GEN)                                           \
+        do {                                                               \
+            if (whole) DS_GO(T, VE, NR, GEN, true);                        \
+            else DS_GO(T, VE, NR, GEN, false);                             \
+        } while (0)
     #define DS_N(T, VE, GEN)                                               \
         do {                                                               \
-            if (per <= 4) DS_GO(T, VE, 4, GEN);                            \
-            else DS_GO(T, VE, 16, GEN);                                    \
+            if (per <= 4) DS_O(T, VE, 4, GEN);                             \
+            else DS_O(T, VE, 16, GEN);                                     \
         } while (0)
     #define DS_V(T, GEN)                                                   \
         do { if (v4) DS_N(T, 4, GEN); else DS_N(T, 1, GEN); } while (0)
@@ -672,6 +741,7 @@ extern "C" int delta_step(
     else { if (gen) DS_V(bf16, true); else DS_V(bf16, false); }
     #undef DS_V
     #undef DS_N
+    #undef DS_O
     #undef DS_GO
     return (int)hipGetLastError();
 }

@@ -378,7 +378,6 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
         load(gw);
         pages(gw + GW);
     }
-    const float gv = split > 1 ? 1.f : gate_of<T>(gate, tok, head);
     for (int st = gw; st < steps; st += GW) {
         const int base = (first + st) * KT;
         f32x4 s[2] = {};
@@ -438,7 +437,7 @@ __global__ __launch_bounds__(NW * 64) void k_softmax_decode(
     __syncthreads();
     if (lr >= n_rows) return;
     const float f0 = split > 1 ? 1.f : finish<T>(top, den, rule.sink, head)
-                                       * gv;
+                                       * gate_of<T>(gate, tok, head);
     for (int v = wid; v < VT; v += NW) {
         f32x4 t = o_s[v * 64 + lane];
         #pragma unroll

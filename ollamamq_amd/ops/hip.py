@@ -9,7 +9,7 @@ from __future__ import annotations
 
 import ctypes
 import os
-from typing import Optional
+from typing import NamedTuple, Optional
 
 import torch
 
@@ -108,7 +108,9 @@ def _try_load():
     lib.general_rows.argtypes = [i, *rows, i, i, i, vp, vp, vp, vp, vp, i, i,
                                  i, i, vp]
     delta = [vp, i64, i, i, i, i, vp, vp, i, vp, vp, vp, vp, vp, vp]
-    lib.delta_step.argtypes = [i, i, vp, *delta, vp, i, i, i, i, i, vp]
+    lib.delta_step.argtypes = [i, i, vp, *delta, vp, i, i, i, i, i, vp, i,
+                               vp, i64, i, f, i, vp]
+    lib.delta_whole.argtypes = [i, i, i, i, i, i64]
     lib.delta_chunks.argtypes = [i, i, vp, vp, *delta, vp, i, vp, i, i, i, i,
                                  i, vp]
     lib.delta_scratch_floats.argtypes = [i, i, i, i]
@@ -1427,29 +1429,50 @@ def _conv_strips(meta, taps, dev):
     return t
 
 
+class _HeadOut(NamedTuple):
+    """The norm and gate behind a recurrence: weight, gate rows, the gate's
+    first column, and the epsilon."""
+    norm: torch.Tensor
+    gate: torch.Tensor
+    og: int
+    eps: float
+
+
 def _delta(gen, x, offsets, qs, ks, decay, beta, a_bias, state, G, slots, pos,
-           meta):
-    """The recurrence over prepared rows -> o [T, H*V] fp32."""
+           meta, out: _HeadOut, frag):
+    """The recurrence over prepared rows, norm and gate -> [T, H*V]."""
     H, D, V = state.shape[1:]
     T, dev, f32 = x.shape[0], x.device, _is_f32(x)
     assert state.dtype == torch.float32 and state.is_contiguous() \
-        and x.stride(1) == 1
-    o = torch.empty((T, H * V), dtype=torch.float32, device=dev)
+        and x.stride(1) == 1 and out.gate.dtype == x.dtype \
+        and out.gate.stride(1) == 1 and out.norm.numel() in (V, H * V) \
+        and out.og + H * V <= out.gate.shape[1]
     head = (_p(x), x.stride(0), *offsets, _p(qs), _p(ks), ks.stride(0),
             _p(decay), _p(beta), _p(a_bias), _p(state), _p(slots), _p(pos))
     nd = meta.n_single
+    stride = V if out.norm.numel() == H * V else 0
 
-    def step(spans, n):
-        _check(_lib.delta_step(f32, gen, _p(o), *head, _p(spans), n, H, G, D,
-                               V, _stream()), "delta_step")
+    def step(o, spans, n, whole):
+        _check(_lib.delta_step(
+            f32, gen, _p(o), *head, _p(spans), n, H, G, D, V, _p(out.norm),
+            stride, _p(out.gate), out.gate.stride(0), out.og,
+            float(out.eps), 2 if whole and frag else int(whole), _stream()),
+            "delta_step")
 
+    if meta.one_each and T and _lib.delta_whole(
+            T, H, D, V, offsets[2], x.stride(0)):
+        res = _frag_rows(T, H * V, x) if frag else \
+            torch.empty((T, H * V), dtype=x.dtype, device=dev)
+        step(res.buf if frag else res, None, T, True)
+        return res
+    o = torch.empty((T, H * V), dtype=torch.float32, device=dev)
     if nd:
-        step(None, nd)
+        step(o, None, nd, False)
     if not meta.one_each:
         spans, chunks, seqs, _, _ = _chunk_plan(
             meta, dev, DELTA_STEP_TOKENS if D <= DELTA_MAX_D else 1 << 62)
         if spans is not None:
-            step(spans, spans.shape[0])
+            step(o, spans, spans.shape[0], False)
         if chunks is not None:
             one = _lib.delta_scratch_floats(gen, 1, H, D)
             groups = _chunk_groups(meta, dev, DELTA_STEP_TOKENS,
@@ -1461,7 +1484,8 @@ def _delta(gen, x, offsets, qs, ks, decay, beta, a_bias, state, G, slots, pos,
                     f32, gen, _p(o), _p(scr), *head, _p(chunks),
                     chunks.shape[0], _p(seqs), seqs.shape[0], H, G, D, V,
                     _stream()), "delta_chunks")
-    return o
+    return head_gate(o, out.norm, out.gate, out.og, "sigmoid", x.dtype, H, V,
+                     out.eps, frag)
 
 
 def gated_delta(p, w, state, conv_state, slot_ids, positions, meta, frag):
@@ -1496,9 +1520,9 @@ def gated_delta(p, w, state, conv_state, slot_ids, positions, meta, frag):
             _p(y),
             _p(scales), _p(decay), _p(beta), _p(gate), T, H, G, D, V,
             _stream()), "gated_rows")
-    o = _delta(0, y, (0, G * D, 2 * G * D, 0), scales, scales[:, G:], decay,
-               beta, None, state, G, slots, pos, meta)
-    return head_gate(o, w.norm, gate, 0, "sigmoid", dtype, H, V, w.eps, frag)
+    return _delta(0, y, (0, G * D, 2 * G * D, 0), scales, scales[:, G:],
+                  decay, beta, None, state, G, slots, pos, meta,
+                  _HeadOut(w.norm, gate, 0, w.eps), frag)
 
 
 def general_delta(p, w, state, slot_ids, positions, meta, frag):
@@ -1523,9 +1547,9 @@ def general_delta(p, w, state, slot_ids, positions, meta, frag):
             int(dtype == torch.float32), *_rows(p), ok, ow, rank,
             _p(w.w2.packed), _p(w.w0), _p(scales), _p(decay), _p(y if whole else None), cols,
             T, H, D, _stream()), "general_rows")
-    o = _delta(1, y, (o_r, ok, ov, oa), None, scales, decay, None, w.a_bias,
-               state, H, slots, pos, meta)
-    return head_gate(o, w.norm, y, og, "sigmoid", dtype, H, D, w.eps, frag)
+    return _delta(1, y, (o_r, ok, ov, oa), None, scales, decay, None,
+                  w.a_bias, state, H, slots, pos, meta,
+                  _HeadOut(w.norm, y, og, w.eps), frag)
 
 
 # ---------------------------------------------------------------------------
