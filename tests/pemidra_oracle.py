@@ -225,3 +225,89 @@ def run(cfg, weights, tokens):
     logits = layer_norm(x, w["final.norm"], w["final.norm.b"], eps) \
         @ w["head"].T
     return logits, torch.stack(layers)
+
+
+def random_weights(cfg, seed=0, ranks=(6, 13, 9)):
+    """bf16 weights with the checkpoint's names and shapes; ranks of the
+    gated rule's decays and gates and of the generalized rule's decays."""
+    g = torch.Generator().manual_seed(seed)
+    W = cfg["width"]
+    out = {}
+
+    def mat(name, n, k=W, s=1.0):
+        out[name] = (torch.randn(n, k, generator=g) * s / math.sqrt(k)) \
+            .to(torch.bfloat16)
+
+    def vec(name, n, mean=0.0, spread=0.2):
+        out[name] = (mean + spread * torch.randn(n, generator=g)) \
+            .to(torch.bfloat16)
+
+    def norm(name):
+        vec(name, W, 1.0)
+        vec(name + ".b", W)
+
+    def attention(x, m):
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        mat(x + "q", H * D)
+        mat(x + "k", G * D)
+        mat(x + "v", G * V)
+        vec(x + "q.norm", D, 1.3)
+        vec(x + "k.norm", D, 1.3)
+        vec(x + "temp", H, 1.0, 0.4)
+        mat(x + "g", H, s=2.0)
+        mat(x + "o", W, H * V)
+
+    def gated_delta(x, m):
+        H, G, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for n, rows in (("q", G * D), ("k", G * D), ("v", H * V)):
+            mat(x + n, rows)
+            mat(f"{x}{n}.conv", rows, m["conv"], 1.5)
+        mat(x + "b", H)
+        vec(x + "A_log", H, 0.0, 1.0)
+        vec(x + "norm", V, 1.0)
+        mat(x + "a1", ranks[0])
+        mat(x + "a2", H * D, ranks[0])
+        vec(x + "dt_bias", H * D, -2.0, 1.5)
+        mat(x + "g1", ranks[1])
+        mat(x + "g2", H * V, ranks[1])
+        mat(x + "o", W, H * V)
+
+    out["embed"] = torch.randn(cfg["vocab"], W, generator=g) \
+        .to(torch.bfloat16)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        x = p + "mix."
+        norm(p + "norm1")
+        vec(p + "ls1", W, 1.0)
+        if layer["type"] == "retention":
+            H, D, V = m["heads"], m["dim"], m["vdim"]
+            mat(x + "q", H * D)
+            mat(x + "k", H * D)
+            mat(x + "v", H * V)
+            mat(x + "g", H * V)
+            mat(x + "o", W, H * V)
+        elif layer["type"] == "general_delta":
+            n = m["heads"] * m["dim"]
+            for c in "rkvga":
+                mat(x + c, n)
+            vec(x + "a.b", n)
+            mat(x + "w1", ranks[2])
+            mat(x + "w2", n, ranks[2], 2.0)
+            vec(x + "w0", n, -1.0, 1.5)
+            vec(x + "norm", n, 1.0)
+            mat(x + "o", W, n)
+        else:
+            attention(x + "left.", m["left"])
+            gated_delta(x + "right.", m["right"])
+            vec(x + "left.out", W, 1.0)
+            vec(x + "right.out", W, 1.0)
+        if layer["mlp"]:
+            norm(p + "norm2")
+            vec(p + "ls2", W, 1.0)
+            F = layer["mlp"]["ff"]
+            mat(p + "mlp.gate", F)
+            mat(p + "mlp.up", F)
+            mat(p + "mlp.down", W, F)
+    norm("final.norm")
+    mat("head", cfg["vocab"])
+    return out
