@@ -35,9 +35,6 @@
 // inputs are then taken as zero and whatever the slot held is ignored.
 #include "tile_mma.h"
 
-template <typename T> DEV float silu_of(float x) {
-    return x * sigmoid_of<T>(x);
-}
 template <typename T> DEV float softplus_of(float x) {
     const float e = exp_of<T>(-fabsf(x));
     if constexpr (sizeof(T) == 4) return fmaxf(x, 0.f) + log1pf(e);
@@ -48,20 +45,6 @@ template <typename T> DEV float softplus_of(float x) {
 #define UNIT_EPS 1e-6f                // inside the root of a unit vector
 #define LOG_ZERO (-104.f)             // e to this is zero in fp32
 #define HALF_DECAY 0.6065306597126334f   // e^{-1/2}
-
-// an fp32 value as matrix operand: two bf16 terms, or itself
-template <typename T> struct Terms;
-template <> struct Terms<bf16> {
-    static constexpr int N = 2;
-    static DEV void split(float x, bf16* t) {
-        t[0] = __float2bfloat16(x);
-        t[1] = __float2bfloat16(x - __bfloat162float(t[0]));
-    }
-};
-template <> struct Terms<float> {
-    static constexpr int N = 1;
-    static DEV void split(float x, float* t) { t[0] = x; }
-};
 
 // ---------------------------------------------------------------------------
 // z = W u for 16 tokens and rows n0 .. n1 - 1 of W [N, rank], u (or its tanh)

@@ -1,8 +1,9 @@
 // gfx950 lightning attention: per head a [D, V] fp32 state with one decay,
 //   S_t = r S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,   q, k, v their columns in
-// the fused projection, or the silu of them.  The state and everything that enters it
-// beyond q, k and v is fp32: in bf16 models an fp32 operand of a matrix
-// product goes through the bf16 matrix cores as the sum of two bf16 terms.
+// the fused projection, or the silu of them.  The state and everything that
+// enters it beyond q, k and v is fp32: in bf16 models an fp32 operand of a
+// matrix product goes through the bf16 matrix cores as the sum of two bf16
+// terms.
 //
 // * k_lightning_step: a token at a time (decode, portions of a few tokens);
 // * k_lightning_act / k_lightning_scan: chunks of 64 tokens.  Inside a chunk
@@ -12,13 +13,9 @@
 //   the padded rows of q, k and v once; scan walks a sequence's chunks with
 //   the state in registers, a block per head and strip of value columns.
 // The results o [T, H, V] are fp32; the norm and gate that follow are
-// k_rms_gate or k_head_gate.  A sequence starts where its position is 0: the state is then
-// taken as zero and whatever the slot held is ignored.
+// k_rms_gate or k_head_gate.  A sequence starts where its position is 0: the
+// state is then taken as zero and whatever the slot held is ignored.
 #include "tile_mma.h"
-
-template <typename T> DEV float silu_of(float x) {
-    return x * sigmoid_of<T>(x);
-}
 
 struct Cols { int q, k, v, act; };    // first columns in the projection
 template <typename T> DEV float act_of(const Cols& at, float x) {
@@ -180,20 +177,6 @@ __global__ __launch_bounds__(256) void k_lightning_act(
         stv<VEC>(dst + ((int64_t)h * rows + t) * pad + d, v);
     }
 }
-
-// an fp32 value as matrix operand: two bf16 terms, or itself
-template <typename T> struct Terms;
-template <> struct Terms<bf16> {
-    static constexpr int N = 2;
-    static DEV void split(float x, bf16* t) {
-        t[0] = __float2bfloat16(x);
-        t[1] = __float2bfloat16(x - __bfloat162float(t[0]));
-    }
-};
-template <> struct Terms<float> {
-    static constexpr int N = 1;
-    static DEV void split(float x, float* t) { t[0] = x; }
-};
 
 template <typename T, int NS, int VC>
 __global__ __launch_bounds__(256) void k_lightning_scan(

@@ -20,11 +20,6 @@
 typedef __attribute__((ext_vector_type(4))) unsigned u32x4;
 typedef __attribute__((ext_vector_type(16))) float f32x16;
 
-template <typename T> DEV float silu_of(float z) {
-    if constexpr (sizeof(T) == 4) return z / (1.f + expf(-z));
-    else return z * __builtin_amdgcn_rcpf(1.f + __expf(-z));
-}
-
 // ---------------------------------------------------------------------------
 // Router.  Logits, softmax and choice in fp32; equal logits go to the lower
 // expert.

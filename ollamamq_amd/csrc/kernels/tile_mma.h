@@ -107,6 +107,10 @@ template <typename T> DEV float sigmoid_of(float x) {
     else return __builtin_amdgcn_rcpf(1.f + __expf(-x));
 }
 
+template <typename T> DEV float silu_of(float x) {
+    return x * sigmoid_of<T>(x);
+}
+
 // Activation-fragment layout ("frag"): the SAME MFMA fragment order the
 // weight packs use, applied to a [32, K] activation: element (m, k) with
 // k = b*64 + j*16 + h*8 + e lives at 16-byte unit ((b*4 + j)*64 + h*32
@@ -221,6 +225,20 @@ DEV float frag_get(const bf16x8& f, int e) { return (float)f[e]; }
 DEV float frag_get(const f32x8s& f, int e) {
     return e < 4 ? f.lo[e] : f.hi[e - 4];
 }
+// an fp32 value as matrix operand: two bf16 terms, or itself
+template <typename T> struct Terms;
+template <> struct Terms<bf16> {
+    static constexpr int N = 2;
+    static DEV void split(float x, bf16* t) {
+        t[0] = __float2bfloat16(x);
+        t[1] = __float2bfloat16(x - __bfloat162float(t[0]));
+    }
+};
+template <> struct Terms<float> {
+    static constexpr int N = 1;
+    static DEV void split(float x, float* t) { t[0] = x; }
+};
+
 // elements e with k0 + e < K; the rest are zero
 template <typename T>
 DEV Frag<T> frag_guard(const T* p, int k0, int K) {

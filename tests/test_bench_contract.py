@@ -87,7 +87,8 @@ def test_bench_layer_stacks():
     stacks = {row["stack"] for row in out["results"]}
     assert {"llama", "rinitar gla", "rinitar latent", "revitar",
             "kavedra lightning", "kavedra attention", "kavedra latent",
-            "kavedra mixed", "kavedra looped"} <= stacks
+            "kavedra mixed", "kavedra looped", "pemidra retention",
+            "pemidra delta", "pemidra parallel", "pemidra mixed"} <= stacks
     for row in out["results"]:
         assert row["prefill_tokens_per_s"] > 0
         assert row["decode_tokens_per_s"] > 0
