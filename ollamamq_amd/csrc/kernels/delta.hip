@@ -87,23 +87,36 @@ DEV void low_rank(const Rows<P>& p, int first, int rank,
                     frag_set(uf[s][q], e, ldf(&y[q]));
             }
     };
-    if (rank <= 128) operand(0);
+    // in decode the weights are as far away as the operand: ask for them first
+    constexpr bool EARLY = sizeof(P) > sizeof(T);
+    Frag<T> wf[4][4];
+    auto weights = [&](int n, int r0, int s) {
+        #pragma unroll
+        for (int j = 0; j < 4; j++)
+            wf[s][j] = frag8(w + ((int64_t)((n / 16 + j) * steps
+                                            + min(r0 / 32 + s, steps - 1))
+                                  * 64 + lane) * 8);
+    };
+    if (!EARLY && rank <= 128) operand(0);
     for (int n = n0; n < n1; n += 64) {
         f32x4 z[4] = {};
         for (int r0 = 0; r0 < rank; r0 += 128) {
-            if (rank > 128) operand(r0);
+            if constexpr (EARLY) {
+                #pragma unroll
+                for (int s = 0; s < 4; s++) weights(n, r0, s);
+            }
+            if (rank > 128 || (EARLY && n == n0)) operand(r0);
             #pragma unroll
             for (int s = 0; s < 4; s++) {
-                if (r0 + s * 32 >= rank) continue;
+                if constexpr (!EARLY) {
+                    if (r0 + s * 32 >= rank) continue;
+                    weights(n, r0, s);
+                }
                 #pragma unroll
-                for (int j = 0; j < 4; j++) {
-                    const Frag<T> wf = frag8(
-                        w + ((int64_t)((n / 16 + j) * steps + r0 / 32 + s)
-                             * 64 + lane) * 8);
+                for (int j = 0; j < 4; j++)
                     #pragma unroll
                     for (int q = 0; q < NT; q++)
-                        z[j] = mma(wf, uf[s][q], z[j]);
-                }
+                        z[j] = mma(wf[s][j], uf[s][q], z[j]);
             }
         }
         #pragma unroll
@@ -186,18 +199,29 @@ DEV void conv_strip(const GatedRows<T, P>& a, int64_t item, int lane) {
                 input(row - TAPS + m, col(j), x[m][j]);
         }
     }
-    // rows a few at a time, so that their loads overlap
+    // rows a few at a time, the next ones under way
     constexpr int NR = TAPS > 0 ? 4 : 1;
+    float next[NR][KEEP][VEC], ahead[NR][KEEP][VEC];
+    auto fetch = [&](int r0) {
+        #pragma unroll
+        for (int y = 0; y < NR; y++)
+            #pragma unroll
+            for (int j = 0; j < KEEP; j++)
+                if (col(j) < wide)
+                    ldrow<VEC>(a.p, min(r0 + y, row + n - 1),
+                               a.o_in + c0 + col(j), next[y][j]);
+    };
+    if constexpr (TAPS > 0) fetch(row);
     for (int r0 = row; r0 < row + n; r0 += NR) {
-        float ahead[NR][KEEP][VEC];
         if constexpr (TAPS > 0) {
             #pragma unroll
             for (int y = 0; y < NR; y++)
                 #pragma unroll
                 for (int j = 0; j < KEEP; j++)
-                    if (col(j) < wide)
-                        ldrow<VEC>(a.p, min(r0 + y, row + n - 1),
-                                   a.o_in + c0 + col(j), ahead[y][j]);
+                    #pragma unroll
+                    for (int i = 0; i < VEC; i++)
+                        ahead[y][j][i] = next[y][j][i];
+            if (r0 + NR < row + n) fetch(r0 + NR);
         }
         #pragma unroll
         for (int y = 0; y < NR; y++) {
@@ -261,7 +285,8 @@ DEV void conv_strip(const GatedRows<T, P>& a, int64_t item, int lane) {
 }
 
 template <typename T, typename P, int VEC, int KEEP, int TAPS>
-__global__ __launch_bounds__(256, 4) void k_gated_rows(GatedRows<T, P> a)
+__global__ __launch_bounds__(256, sizeof(P) > sizeof(T) ? 2 : 4)
+void k_gated_rows(GatedRows<T, P> a)
 {
     const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
     int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -394,7 +419,8 @@ template <typename T, typename P> struct GeneralRows {
 };
 
 template <typename T, typename P, int VEC>
-__global__ __launch_bounds__(256, 3) void k_general_rows(GeneralRows<T, P> a)
+__global__ __launch_bounds__(256, sizeof(P) > sizeof(T) ? 2 : 3)
+void k_general_rows(GeneralRows<T, P> a)
 {
     const int lane = threadIdx.x & 63, lr = lane & 15, g = lane >> 4;
     int64_t w = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
