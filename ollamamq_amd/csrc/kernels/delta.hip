@@ -50,8 +50,9 @@ template <typename T> DEV float softplus_of(float x) {
 // z = W u for 16 tokens and rows n0 .. n1 - 1 of W [N, rank], u (or its tanh)
 // the projection's columns first.. of the lane's token t; rank and first are
 // whole vectors of 8.  W is stored as operands, 16 rows by 32 columns after
-// one another, rows filled up to 64 and columns to 32.  `emit` gets 16 rows at a time, four of them in a lane:
-// z[i] is row n + i.  The operand is made once for all rows while rank <= 128.
+// one another, rows filled up to 64 and columns to 32.  `emit` gets 16 rows
+// at a time, four of them in a lane: z[i] is row n + i.  The operand is made
+// once for all rows while rank <= 128.
 // ---------------------------------------------------------------------------
 template <typename T, typename P, bool TANH, typename E>
 DEV void low_rank(const Rows<P>& p, int first, int rank,

@@ -683,8 +683,9 @@ def swiglu(gate_up, act="silu"):
 
 
 def gateup_swiglu(x, weight, packed_gu=None, act="silu"):
-    """act = swiglu(x @ Wgu^T), or with another activation of the gate.  On the decode path (M<=32) with a
-    GU-packed copy this is ONE fused weight-streaming kernel; otherwise
+    """act = swiglu(x @ Wgu^T), or with another activation of the gate.
+    On the decode path (M<=32) with a GU-packed copy this is ONE fused
+    weight-streaming kernel; otherwise
     the library GEMM + the swiglu kernel.  (An MT2 variant for 33..64
     exists but measured BELOW the library at 64 users — its direct
     fragment x-loads double the scattered line traffic.)  FragRows go
